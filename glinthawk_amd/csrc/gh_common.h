@@ -43,7 +43,8 @@ int ensure_init();
 // device the library was initialised on, -1 before initialisation (never initialises)
 int initialised_device();
 // gh_attn_decode.hip: looks up the address of this device's static split-partial array; called once by the initialisation, with `device` current
-int attn_static_scratch_init( int device );
+// (weak: a program that links only some of the translation units may come without the Llama2 attention)
+__attribute__( ( weak ) ) int attn_static_scratch_init( int device );
 // compute units of the device the library was initialised on (256 before initialisation)
 int cu_count();
 
@@ -88,7 +89,7 @@ public:
 // ---- library-owned device scratch ---------------------------------------------------------------
 // Grow-only buffer for purpose `which`, private to `stream`: work queued on different streams never
 // shares one.  Growing waits for that stream only.  `min_bytes` is the size of the first allocation.
-enum { SCRATCH_GEMM_PARTIALS = 0, SCRATCH_CONVERT = 1, SCRATCH_ATTN_PV = 2, SCRATCH_GATE_FACTOR = 3, SCRATCH_LIBRARY = 4, SCRATCH_PRODUCT = 5, SCRATCH_GEMM_PIECES = 6 };
+enum { SCRATCH_GEMM_PARTIALS = 0, SCRATCH_CONVERT = 1, SCRATCH_ATTN_PV = 2, SCRATCH_GATE_FACTOR = 3, SCRATCH_LIBRARY = 4, SCRATCH_PRODUCT = 5, SCRATCH_GEMM_PIECES = 6, SCRATCH_MIXER = 7 };
 int stream_scratch( hipStream_t stream, int which, uint64_t bytes, uint64_t min_bytes, void** out );
 // gh_gemm_lib.hip: a plain f16 product through the vendor's GEMM library; *done = false: declined, nothing queued
 int gemm_library( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, hipStream_t st, bool* done );
@@ -173,6 +174,12 @@ __device__ __forceinline__ float to_f32<__half>( __half v )
   return __half2float( v );
 }
 
+template<>
+__device__ __forceinline__ float to_f32<__bf16>( __bf16 v )
+{
+  return (float)v;
+}
+
 template<typename T>
 __device__ __forceinline__ T from_f32( float v );
 template<>
@@ -185,5 +192,31 @@ __device__ __forceinline__ __half from_f32<__half>( float v )
 {
   return __float2half_rn( v );
 }
+template<>
+__device__ __forceinline__ __bf16 from_f32<__bf16>( float v )
+{
+  return (__bf16)v; // to nearest even
+}
+
+// ---- matrix cores: operands of eight 16-bit elements a lane ------------------------------------
+// f16 and bf16 have the same operand layouts and the same rate; a kernel that is written over Mfma<E> serves both.
+typedef float mfma_f32x4 __attribute__( ( ext_vector_type( 4 ) ) );
+typedef float mfma_f32x16 __attribute__( ( ext_vector_type( 16 ) ) );
+template<typename E>
+struct Mfma;
+template<>
+struct Mfma<__half>
+{
+  typedef _Float16 x8 __attribute__( ( ext_vector_type( 8 ) ) );
+  static __device__ __forceinline__ mfma_f32x4 k32( x8 a, x8 b, mfma_f32x4 c ) { return __builtin_amdgcn_mfma_f32_16x16x32_f16( a, b, c, 0, 0, 0 ); }
+  static __device__ __forceinline__ mfma_f32x16 k16( x8 a, x8 b, mfma_f32x16 c ) { return __builtin_amdgcn_mfma_f32_32x32x16_f16( a, b, c, 0, 0, 0 ); }
+};
+template<>
+struct Mfma<__bf16>
+{
+  typedef __bf16 x8 __attribute__( ( ext_vector_type( 8 ) ) );
+  static __device__ __forceinline__ mfma_f32x4 k32( x8 a, x8 b, mfma_f32x4 c ) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16( a, b, c, 0, 0, 0 ); }
+  static __device__ __forceinline__ mfma_f32x16 k16( x8 a, x8 b, mfma_f32x16 c ) { return __builtin_amdgcn_mfma_f32_32x32x16_bf16( a, b, c, 0, 0, 0 ); }
+};
 
 } // namespace gh

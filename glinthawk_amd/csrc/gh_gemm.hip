@@ -1,11 +1,11 @@
 // Dense projection GEMM of the stage: xout(b, r) = sum_p w(r, p) * x(b, p), w row-major (r, s),
 // fp32 accumulate (Operations::matmul / untemplated_matmul, arch/amd64/common/ops.hh:74-93,212-271).
 //
-// f16: MFMA kernel.  The weight matrix is the streamed operand (read exactly once), the
+// f16, bf16: MFMA kernel.  The weight matrix is the streamed operand (read exactly once), the
 // activations are the small operand.  A work-group owns a 64-row slab of w and a 64-column slab of
 // the batch, walks K in steps of 128, stages both tiles in LDS with 16-byte chunks XOR-swizzled so
 // that the MFMA-operand reads are bank-conflict free, and keeps 4 x (16x16) fp32 accumulators per
-// wave (v_mfma_f32_16x16x32_f16).  When r / 64 is too small to fill the chip K is split across
+// wave (v_mfma_f32_16x16x32_f16 / _bf16).  When r / 64 is too small to fill the chip K is split across
 // work-groups and an fp32 partial buffer is reduced by a second kernel.
 //
 // f32: plain wave-per-row kernel (only the tiny fp32 configuration uses it).
@@ -13,13 +13,15 @@
 
 #include <cstdlib>
 #include <mutex>
+#include <type_traits>
 
 namespace gh {
 
 // streaming decode kernel (gh_gemm_stream.hip)
 bool gemm_stream_applicable( uint64_t s, uint64_t r, uint64_t b, const void* x, const void* w, const void* xout );
 void gemm_stream_plan( uint64_t s, uint64_t r, uint64_t b, uint32_t* splits_out, uint32_t* k_per_split_out, uint32_t* rows_per_wg_out );
-int gemm_stream_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits,
+template<typename E>
+int gemm_stream_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits,
                         uint32_t k_per_split, uint32_t rows_per_wg, bool write_partials, hipStream_t st );
 void gemm_stream_tuning( int target_wgs, int depth );
 void gemm_stream_gate_waves( int waves );
@@ -27,18 +29,28 @@ bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const
 int gemm_stream_gate_launch( __half* hb, const __half* x, const __half* w13, uint64_t s, uint64_t hidden, uint64_t b, hipStream_t st );
 // 256 x 256 tile kernel for products with enough tiles (gh_gemm_tile256.hip)
 bool gemm_tile256_applicable( uint64_t s, uint64_t r, uint64_t b, const void* x, const void* w, const void* xout );
-int gemm_tile256_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, int epilogue, hipStream_t st,
-                         uint32_t splits, uint32_t k_len, __half* xout2 = nullptr, uint64_t r_first = 0 );
+template<typename E>
+int gemm_tile256_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, int epilogue, hipStream_t st,
+                         uint32_t splits, uint32_t k_len, E* xout2 = nullptr, uint64_t r_first = 0 );
 uint64_t gemm_tile256_token_split( uint64_t s, uint64_t r, uint64_t b );
 void gemm_tile256_split_plan( uint64_t s, uint64_t r, uint64_t b, const void* x, const void* w, uint32_t* splits, uint32_t* k_len );
 void gemm_tile256_tuning( int rows );
 // large-batch (prefill) kernel (gh_gemm_tile.hip)
 bool gemm_tile_applicable( uint64_t s, uint64_t r, uint64_t b, const void* x, const void* w, const void* xout );
 void gemm_tile_plan( uint64_t s, uint64_t r, uint64_t b, uint32_t* splits_out, uint32_t* k_per_split_out );
-int gemm_tile_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits, uint32_t k_per_split,
+template<typename E>
+int gemm_tile_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits, uint32_t k_per_split,
                       hipStream_t st );
 
 namespace {
+
+// the 16-bit kernels by their storage type: `run` gets a null pointer of it
+template<typename F>
+int with_half_type( gh_dtype dt, F&& run )
+{
+  return dt == GH_BF16 ? run( static_cast<__bf16*>( nullptr ) ) : run( static_cast<__half*>( nullptr ) );
+}
+inline bool is_half_type( gh_dtype dt ) { return dt == GH_F16 || dt == GH_BF16; }
 
 int g_force_kernel = 0; // 0 auto, 1 small tiled kernel of this file, 2 streaming kernel, 3 large tile kernel
 // GLINT_LIBRARY_ROWS in the environment overrides the default (for the command-line profilers, which have no other way in)
@@ -49,7 +61,6 @@ uint64_t library_rows_default()
 }
 uint64_t g_library_rows = library_rows_default(); // 0: never; else plain products of this many rows and more go to the vendor's GEMM library (gh_gemm_set_library_rows)
 
-typedef _Float16 f16x8 __attribute__( ( ext_vector_type( 8 ) ) );
 typedef float f32x4 __attribute__( ( ext_vector_type( 4 ) ) );
 
 constexpr int BM = 64;  // weight rows per work-group
@@ -75,7 +86,8 @@ struct TileRegs
   uint4 v[4];
 };
 
-__device__ __forceinline__ TileRegs load_tile( const __half* __restrict__ mat, uint64_t ld, uint32_t row0, uint32_t n_rows, uint32_t k0, uint32_t k_end, bool k_vec_ok )
+template<typename E>
+__device__ __forceinline__ TileRegs load_tile( const E* __restrict__ mat, uint64_t ld, uint32_t row0, uint32_t n_rows, uint32_t k0, uint32_t k_end, bool k_vec_ok )
 {
   TileRegs t;
   const uint32_t chunk = threadIdx.x & 15;
@@ -85,14 +97,14 @@ __device__ __forceinline__ TileRegs load_tile( const __half* __restrict__ mat, u
     const uint32_t row = row0 + ( threadIdx.x >> 4 ) + 16 * i;
     uint4 v = make_uint4( 0, 0, 0, 0 );
     if ( row < n_rows && k < k_end ) {
-      const __half* p = mat + (uint64_t)row * ld + k;
+      const E* p = mat + (uint64_t)row * ld + k;
       if ( k_vec_ok && k + 8 <= k_end ) {
         v = *reinterpret_cast<const uint4*>( p );
       } else {
         union
         {
           uint4 raw;
-          __half h[8];
+          E h[8];
         } u;
         u.raw = make_uint4( 0, 0, 0, 0 );
         for ( int e = 0; e < 8; e++ ) {
@@ -119,11 +131,11 @@ __device__ __forceinline__ void store_tile( uint4* lds, const TileRegs& t )
 }
 
 // grid: (ceil(r / 64), ceil(b / 64), k_splits)
-template<bool SPLIT>
-__global__ __launch_bounds__( 256 ) void gemm_f16_kernel( __half* __restrict__ xout,
+template<typename E, bool SPLIT>
+__global__ __launch_bounds__( 256 ) void gemm_mfma_kernel( E* __restrict__ xout,
                                                           float* __restrict__ partial,
-                                                          const __half* __restrict__ x,
-                                                          const __half* __restrict__ w,
+                                                          const E* __restrict__ x,
+                                                          const E* __restrict__ w,
                                                           uint32_t s,
                                                           uint32_t r,
                                                           uint32_t b,
@@ -165,12 +177,12 @@ __global__ __launch_bounds__( 256 ) void gemm_f16_kernel( __half* __restrict__ x
 #pragma unroll
     for ( int kk = 0; kk < 4; kk++ ) {
       const uint32_t ch = 4 * kk + g4;
-      const f16x8 a = __builtin_bit_cast( f16x8, lw[arow * 16 + ( ch ^ ( arow & 15 ) )] );
+      const typename Mfma<E>::x8 a = __builtin_bit_cast( typename Mfma<E>::x8, lw[arow * 16 + ( ch ^ ( arow & 15 ) )] );
 #pragma unroll
       for ( int j = 0; j < 4; j++ ) {
         const uint32_t brow = 16 * j + c;
-        const f16x8 bb = __builtin_bit_cast( f16x8, lx[brow * 16 + ( ch ^ ( brow & 15 ) )] );
-        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_f16( a, bb, acc[j], 0, 0, 0 );
+        const typename Mfma<E>::x8 bb = __builtin_bit_cast( typename Mfma<E>::x8, lx[brow * 16 + ( ch ^ ( brow & 15 ) )] );
+        acc[j] = Mfma<E>::k32( a, bb, acc[j] );
       }
     }
     buf ^= 1; // the other buffer is free: its readers passed the barrier of this iteration
@@ -190,14 +202,15 @@ __global__ __launch_bounds__( 256 ) void gemm_f16_kernel( __half* __restrict__ x
         if ( SPLIT ) {
           partial[( (uint64_t)blockIdx.z * b + col ) * r + row] = acc[j][i];
         } else {
-          xout[(uint64_t)col * r + row] = __float2half_rn( acc[j][i] );
+          xout[(uint64_t)col * r + row] = from_f32<E>( acc[j][i] );
         }
       }
     }
   }
 }
 
-__global__ __launch_bounds__( 256 ) void gemm_reduce_kernel( __half* __restrict__ xout, const float* __restrict__ partial, uint64_t n, uint32_t splits )
+template<typename E>
+__global__ __launch_bounds__( 256 ) void gemm_reduce_kernel( E* __restrict__ xout, const float* __restrict__ partial, uint64_t n, uint32_t splits )
 {
   const uint64_t stride = (uint64_t)gridDim.x * blockDim.x;
   for ( uint64_t i = (uint64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += stride ) {
@@ -214,7 +227,7 @@ __global__ __launch_bounds__( 256 ) void gemm_reduce_kernel( __half* __restrict_
         sum += k0 + u < splits ? p[u] : 0.0f;
       }
     }
-    xout[i] = __float2half_rn( sum );
+    xout[i] = from_f32<E>( sum );
   }
 }
 
@@ -264,7 +277,7 @@ int gemm_gate_one_launch( void* hb, const void* x, const void* w13, uint64_t s, 
 // gemm_tile256_token_split), 0 otherwise.
 uint64_t gemm_token_split( uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, const void* x, const void* w, const void* xout )
 {
-  if ( dt != GH_F16 || g_force_kernel != 0 || !gemm_tile256_applicable( s, r, b, x, w, xout ) ) {
+  if ( !is_half_type( dt ) || g_force_kernel != 0 || !gemm_tile256_applicable( s, r, b, x, w, xout ) ) {
     return 0;
   }
   const uint64_t b1 = gemm_tile256_token_split( s, r, b );
@@ -276,7 +289,7 @@ uint64_t gemm_token_split( uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, cons
 // its other route.
 bool gemm_tile_epilogue_applicable( uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, const void* x, const void* w, const void* xout )
 {
-  return dt == GH_F16 && r % 8 == 0 && ( g_force_kernel == 0 || g_force_kernel == 4 ) && gemm_tile256_applicable( s, r, b, x, w, xout );
+  return is_half_type( dt ) && r % 8 == 0 && ( g_force_kernel == 0 || g_force_kernel == 4 ) && gemm_tile256_applicable( s, r, b, x, w, xout );
 }
 
 int gemm_tile_epilogue_launch( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, int epilogue, hipStream_t st,
@@ -287,30 +300,17 @@ int gemm_tile_epilogue_launch( void* xout, const void* x, const void* w, uint64_
     return GH_OK;
   }
   *done = true;
-  return gemm_tile256_launch( static_cast<__half*>( xout ), nullptr, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, epilogue, st, 1, 0 );
+  return with_half_type( dt, [&]( auto* e ) {
+    using E = std::remove_pointer_t<decltype( e )>;
+    return gemm_tile256_launch<E>( static_cast<E*>( xout ), nullptr, static_cast<const E*>( x ), static_cast<const E*>( w ), s, r, b, epilogue, st, 1, 0 );
+  } );
 }
 
-int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, hipStream_t st, bool want_partials,
-                   float** partial_out, uint32_t* splits_out )
+// the 16-bit part of gemm_partials()
+template<typename E>
+int gemm_half_partials( E* xout, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, hipStream_t st, bool want_partials, float** partial_out,
+                        uint32_t* splits_out )
 {
-  *partial_out = nullptr;
-  *splits_out = 0;
-  if ( dt == GH_F32 ) {
-    float* dst = static_cast<float*>( xout );
-    if ( want_partials ) {
-      if ( int rc = ensure_workspace( b * r * sizeof( float ), &dst, st ) ) {
-        return rc;
-      }
-      *partial_out = dst;
-      *splits_out = 1;
-    }
-    gemm_f32_kernel<<<(unsigned)( ( r + 3 ) / 4 ), 256, 0, st>>>( dst, static_cast<const float*>( x ), static_cast<const float*>( w ), (uint32_t)s, (uint32_t)r,
-                                                                 (uint32_t)b );
-    GH_LAUNCH_CHECK();
-    return GH_OK;
-  }
-  GH_REQUIRE( dt == GH_F16, "gh_matmul: unsupported dtype %d", (int)dt );
-
   // many tokens at once (prefill): the MFMA-bound tile kernel; few (decode): the weight-streaming one
   if ( ( g_force_kernel == 0 || g_force_kernel == 4 ) && gemm_tile256_applicable( s, r, b, x, w, xout ? xout : x ) ) {
     float* ws = nullptr;
@@ -321,7 +321,7 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
       *partial_out = ws;
       *splits_out = 1;
     }
-    return gemm_tile256_launch( static_cast<__half*>( xout ), ws, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, 0, st, 1, 0 );
+    return gemm_tile256_launch( xout, ws, x, w, s, r, b, 0, st, 1, 0 );
   }
   if ( g_force_kernel == 0 || g_force_kernel == 4 ) { // some hundred rows and few tiles: the same kernel with the K range split
     uint32_t splits = 0, k_len = 0;
@@ -333,7 +333,7 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
       }
       *partial_out = ws;
       *splits_out = splits;
-      return gemm_tile256_launch( nullptr, ws, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, 0, st, splits, k_len );
+      return gemm_tile256_launch<E>( nullptr, ws, x, w, s, r, b, 0, st, splits, k_len );
     }
   }
   GH_REQUIRE( g_force_kernel != 4, "gh_matmul: the 256 x 256 tile kernel needs b >= 192, at least 192 tiles with a last round that is not mostly empty, s %% 64 == 0 and 16-byte aligned operands" );
@@ -348,7 +348,7 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
       *partial_out = ws;
       *splits_out = splits;
     }
-    return gemm_tile_launch( static_cast<__half*>( xout ), ws, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, splits, k_per_split, st );
+    return gemm_tile_launch( xout, ws, x, w, s, r, b, splits, k_per_split, st );
   }
   GH_REQUIRE( g_force_kernel != 3, "gh_matmul: the tile kernel needs b > 64, s %% 8 == 0 and 16-byte aligned operands" );
 
@@ -364,7 +364,7 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
       *partial_out = ws;
       *splits_out = splits;
     }
-    return gemm_stream_launch( static_cast<__half*>( xout ), ws, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, splits, k_per_split,
+    return gemm_stream_launch( xout, ws, x, w, s, r, b, splits, k_per_split,
                                rows_per_wg, partial, st );
   }
   GH_REQUIRE( g_force_kernel != 2, "gh_matmul: the streaming kernel needs s %% 256 == 0, r %% 4 == 0 and 16-byte aligned operands" );
@@ -388,7 +388,7 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
 
   const dim3 grid( grid_m, grid_n, splits );
   if ( splits == 1 && !want_partials ) {
-    gemm_f16_kernel<false><<<grid, 256, 0, st>>>( static_cast<__half*>( xout ), nullptr, static_cast<const __half*>( x ), static_cast<const __half*>( w ),
+    gemm_mfma_kernel<E, false><<<grid, 256, 0, st>>>( xout, nullptr, x, w,
                                                  (uint32_t)s, (uint32_t)r, (uint32_t)b, k_per_split, k_vec_ok );
     GH_LAUNCH_CHECK();
     return GH_OK;
@@ -397,12 +397,38 @@ int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_
   if ( int rc = ensure_workspace( (uint64_t)splits * b * r * sizeof( float ), &ws, st ) ) {
     return rc;
   }
-  gemm_f16_kernel<true><<<grid, 256, 0, st>>>( nullptr, ws, static_cast<const __half*>( x ), static_cast<const __half*>( w ), (uint32_t)s, (uint32_t)r,
+  gemm_mfma_kernel<E, true><<<grid, 256, 0, st>>>( nullptr, ws, x, w, (uint32_t)s, (uint32_t)r,
                                               (uint32_t)b, k_per_split, k_vec_ok );
   GH_LAUNCH_CHECK();
   *partial_out = ws;
   *splits_out = splits;
   return GH_OK;
+}
+
+int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, hipStream_t st, bool want_partials,
+                   float** partial_out, uint32_t* splits_out )
+{
+  *partial_out = nullptr;
+  *splits_out = 0;
+  if ( dt == GH_F32 ) {
+    float* dst = static_cast<float*>( xout );
+    if ( want_partials ) {
+      if ( int rc = ensure_workspace( b * r * sizeof( float ), &dst, st ) ) {
+        return rc;
+      }
+      *partial_out = dst;
+      *splits_out = 1;
+    }
+    gemm_f32_kernel<<<(unsigned)( ( r + 3 ) / 4 ), 256, 0, st>>>( dst, static_cast<const float*>( x ), static_cast<const float*>( w ), (uint32_t)s, (uint32_t)r,
+                                                                 (uint32_t)b );
+    GH_LAUNCH_CHECK();
+    return GH_OK;
+  }
+  GH_REQUIRE( is_half_type( dt ), "gh_matmul: unsupported dtype %d", (int)dt );
+  return with_half_type( dt, [&]( auto* e ) {
+    using E = std::remove_pointer_t<decltype( e )>;
+    return gemm_half_partials<E>( static_cast<E*>( xout ), static_cast<const E*>( x ), static_cast<const E*>( w ), s, r, b, st, want_partials, partial_out, splits_out );
+  } );
 }
 
 } // namespace gh
@@ -481,8 +507,8 @@ int gh_matmul_pair( void* xout_a, void* xout_b, const void* x, const void* w, ui
     return GH_OK;
   }
   GH_REQUIRE( xout_a && xout_b && x && w, "gh_matmul_pair: NULL pointer" );
-  GH_REQUIRE( dt == GH_F16 || dt == GH_F32, "gh_matmul_pair: unsupported dtype %d", (int)dt );
-  const uint64_t elem = dt == GH_F16 ? 2 : 4;
+  GH_REQUIRE( is_half_type( dt ) || dt == GH_F32, "gh_matmul_pair: unsupported dtype %d", (int)dt );
+  const uint64_t elem = dtype_size( dt );
   const uint64_t r = r_a + r_b;
   GH_REQUIRE( s > 0 && s <= 0x7fffffffull && r <= 0x7fffffffull && b <= 0x7fffffffull, "gh_matmul_pair: bad shape" );
   if ( r_a > 0 && r_b > 0 && gemm_library_wanted( s, r_a, b, dt, x, w, xout_a ) && gemm_library_wanted( s, r_b, b, dt, x, w, xout_b ) ) {
@@ -493,7 +519,7 @@ int gh_matmul_pair( void* xout_a, void* xout_b, const void* x, const void* w, ui
   }
   // many rows: one launch of the large tile kernel whose work-groups store to the matrix their rows belong to, so that the two
   // products fill their rounds together (a product of 2048 rows alone leaves most of the chip idle)
-  if ( dt == GH_F16 && g_force_kernel == 0 && r_a > 0 && r_b > 0 && r_a % 8 == 0 && r_b % 8 == 0 && gemm_tile256_applicable( s, r, b, x, w, xout_a )
+  if ( is_half_type( dt ) && g_force_kernel == 0 && r_a > 0 && r_b > 0 && r_a % 8 == 0 && r_b % 8 == 0 && gemm_tile256_applicable( s, r, b, x, w, xout_a )
        && ( reinterpret_cast<uintptr_t>( xout_b ) & 15u ) == 0 ) {
     if ( const uint64_t b1 = gemm_token_split( s, r, b, dt, x, w, xout_a ) ) {
       if ( ( b1 * r_a * elem ) % 16 == 0 && ( b1 * r_b * elem ) % 16 == 0 ) {
@@ -504,8 +530,11 @@ int gh_matmul_pair( void* xout_a, void* xout_b, const void* x, const void* w, ui
                                static_cast<const char*>( x ) + b1 * s * elem, w, s, r_a, r_b, b - b1, dt, stream );
       }
     }
-    return gemm_tile256_launch( static_cast<__half*>( xout_a ), nullptr, static_cast<const __half*>( x ), static_cast<const __half*>( w ), s, r, b, 0,
-                                as_stream( stream ), 1, 0, static_cast<__half*>( xout_b ), r_a );
+    return with_half_type( dt, [&]( auto* e ) {
+      using E = std::remove_pointer_t<decltype( e )>;
+      return gemm_tile256_launch<E>( static_cast<E*>( xout_a ), nullptr, static_cast<const E*>( x ), static_cast<const E*>( w ), s, r, b, 0, as_stream( stream ), 1,
+                                     0, static_cast<E*>( xout_b ), r_a );
+    } );
   }
   if ( int rc = gh_matmul( xout_a, x, w, s, r_a, b, dt, stream ) ) {
     return rc;
@@ -545,11 +574,15 @@ int gh_matmul( void* xout, const void* x, const void* w, uint64_t s, uint64_t r,
   if ( int rc = gemm_partials( xout, x, w, s, r, b, dt, st, false, &partial, &splits ) ) {
     return rc;
   }
-  if ( splits > 0 ) { // only the f16 kernels leave partials when not asked to
+  if ( splits > 0 ) { // only the 16-bit kernels leave partials when not asked to
     const uint64_t n = b * r;
     const unsigned blocks = (unsigned)std::min<uint64_t>( ( n + 255 ) / 256, 4096 );
-    gemm_reduce_kernel<<<blocks, 256, 0, st>>>( static_cast<__half*>( xout ), partial, n, splits );
-    GH_LAUNCH_CHECK();
+    return with_half_type( dt, [&]( auto* e ) -> int {
+      using E = std::remove_pointer_t<decltype( e )>;
+      gemm_reduce_kernel<E><<<blocks, 256, 0, st>>>( static_cast<E*>( xout ), partial, n, splits );
+      GH_LAUNCH_CHECK();
+      return GH_OK;
+    } );
   }
   return GH_OK;
 }

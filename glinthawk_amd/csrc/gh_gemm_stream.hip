@@ -1,5 +1,5 @@
 // Weight-streaming GEMM for decode: xout(b, r) = sum_p w(r, p) * x(b, p) with a small batch
-// (64 columns per column slab), f16 storage, fp32 accumulate.  Every weight element is read from HBM
+// (64 columns per column slab), f16 or bf16 storage, fp32 accumulate.  Every weight element is read from HBM
 // exactly once, so the kernel is built like a streaming read:
 //
 //   work-group = 4 waves = up to 128 weight rows x one K range; wave = up to 32 rows x all 64 batch
@@ -29,7 +29,6 @@
 
 namespace gh {
 
-typedef _Float16 f16x8 __attribute__( ( ext_vector_type( 8 ) ) );
 typedef float f32x16 __attribute__( ( ext_vector_type( 16 ) ) );
 
 namespace {
@@ -109,6 +108,7 @@ __device__ __forceinline__ void stage_x_half( uint4* tile, const XSlab<W>& t, in
 }
 
 // 128 k of math for a wave: 8 steps of k = 16
+template<typename E>
 __device__ __forceinline__ void half_mfma( f32x16 acc[2], const uint4* wtile, const uint4* xtile )
 {
   const uint32_t lane = threadIdx.x & 63;
@@ -116,12 +116,12 @@ __device__ __forceinline__ void half_mfma( f32x16 acc[2], const uint4* wtile, co
 #pragma unroll
   for ( int s = 0; s < 8; s++ ) {
     const uint32_t ch = 2 * s + g2;
-    const f16x8 a = __builtin_bit_cast( f16x8, wtile[r * 16 + ( ch ^ ( r & 15 ) )] );
+    const typename Mfma<E>::x8 a = __builtin_bit_cast( typename Mfma<E>::x8, wtile[r * 16 + ( ch ^ ( r & 15 ) )] );
 #pragma unroll
     for ( int t = 0; t < 2; t++ ) {
       const uint32_t col = 32 * t + r;
-      const f16x8 b = __builtin_bit_cast( f16x8, xtile[col * 16 + ( ch ^ ( col & 15 ) )] );
-      acc[t] = __builtin_amdgcn_mfma_f32_32x32x16_f16( a, b, acc[t], 0, 0, 0 );
+      const typename Mfma<E>::x8 b = __builtin_bit_cast( typename Mfma<E>::x8, xtile[col * 16 + ( ch ^ ( col & 15 ) )] );
+      acc[t] = Mfma<E>::k16( a, b, acc[t] );
     }
   }
 }
@@ -135,11 +135,11 @@ constexpr int MODE_GATE = 2;  // w = [w1 rows | w3 rows], r = rows of each: stor
 // MODE_GATE: a work-group takes 64 output rows; waves 0, 1 stream them from w1, waves 2, 3 the same
 // rows from w3, so that the two factors of an output element sit in the same lane and accumulator
 // register of a wave pair and meet through LDS after the K loop (no K split in this mode).
-template<int MODE, int W = 4>
-__global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( __half* __restrict__ xout,
+template<typename E, int MODE, int W = 4>
+__global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( E* __restrict__ xout,
                                                              float* __restrict__ partial,
-                                                             const __half* __restrict__ x,
-                                                             const __half* __restrict__ w,
+                                                             const E* __restrict__ x,
+                                                             const E* __restrict__ w,
                                                              uint32_t s,
                                                              uint32_t r,
                                                              uint32_t b,
@@ -177,8 +177,8 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
   // descriptors bounded to the wave's rows / the work-group's columns: anything past the matrix reads as zero
   const uint32_t w_rows = row0 < r ? min( rows_per_wave, r - row0 ) : 0u;
   const uint32_t x_cols = col0 < b ? min( (uint32_t)COLS, b - col0 ) : 0u;
-  const __amdgpu_buffer_rsrc_t w_rsrc = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( w + (uint64_t)w_row0 * s ), 0, (int)( w_rows * ld_bytes ), 0x00020000 );
-  const __amdgpu_buffer_rsrc_t x_rsrc = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( x + (uint64_t)col0 * s ), 0, (int)( x_cols * ld_bytes ), 0x00020000 );
+  const __amdgpu_buffer_rsrc_t w_rsrc = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( w + (uint64_t)w_row0 * s ), 0, (int)( w_rows * ld_bytes ), 0x00020000 );
+  const __amdgpu_buffer_rsrc_t x_rsrc = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( x + (uint64_t)col0 * s ), 0, (int)( x_cols * ld_bytes ), 0x00020000 );
   const uint32_t w_lane = ( lane >> 4 ) * ld_bytes + ( lane & 15 ) * 16;
   const uint32_t x_lane = ( threadIdx.x >> 4 ) * ld_bytes + ( threadIdx.x & 15 ) * 16;
 
@@ -226,7 +226,7 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
       stage_w_half( wtile, wr[set], h );
       load_x_half( xr, x_rsrc, x_lane, ld_bytes, kb, h ); // same registers, next slab
       __syncthreads();
-      half_mfma( acc, wtile, s_x[h] );
+      half_mfma<E>( acc, wtile, s_x[h] );
     }
   };
   for ( ;; ) { // exits are uniform across the work-group
@@ -250,7 +250,7 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
       for ( int t = 0; t < 2; t++ ) {
 #pragma unroll
         for ( int v = 0; v < 16; v++ ) {
-          gate[( ( ( wave % HALF_W ) * 2 + t ) * 16 + v ) * 64 + lane] = __half2float( __float2half_rn( acc[t][v] ) );
+          gate[( ( ( wave % HALF_W ) * 2 + t ) * 16 + v ) * 64 + lane] = to_f32<E>( from_f32<E>( acc[t][v] ) );
         }
       }
     }
@@ -267,16 +267,16 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
         union
         {
           uint2 raw;
-          __half h[4];
+          E h[4];
         } o;
 #pragma unroll
         for ( int i = 0; i < 4; i++ ) {
-          const float y1 = __half2float( __float2half_rn( acc[t][4 * q4 + i] ) );
+          const float y1 = to_f32<E>( from_f32<E>( acc[t][4 * q4 + i] ) );
           const float y3 = gate[( ( wave * 2 + t ) * 16 + 4 * q4 + i ) * 64 + lane];
-          o.h[i] = __float2half_rn( y1 / ( 1.0f + __expf( -y1 ) ) * y3 );
+          o.h[i] = from_f32<E>( y1 / ( 1.0f + __expf( -y1 ) ) * y3 );
         }
         if ( col < b && 8 * q4 + 4 * g2 < rows_per_wave ) {
-          __half* dst = xout + (uint64_t)col * r + row;
+          E* dst = xout + (uint64_t)col * r + row;
           if ( row + 3 < r ) {
             *reinterpret_cast<uint2*>( dst ) = o.raw;
           } else {
@@ -315,22 +315,22 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
           }
         }
       } else {
-        __half* dst = xout + (uint64_t)col * r + row;
+        E* dst = xout + (uint64_t)col * r + row;
         if ( row + 3 < r ) {
           union
           {
             uint2 raw;
-            __half h[4];
+            E h[4];
           } o;
 #pragma unroll
           for ( int i = 0; i < 4; i++ ) {
-            o.h[i] = __float2half_rn( acc[t][4 * q4 + i] );
+            o.h[i] = from_f32<E>( acc[t][4 * q4 + i] );
           }
           *reinterpret_cast<uint2*>( dst ) = o.raw;
         } else {
           for ( int i = 0; i < 4; i++ ) {
             if ( row + i < r ) {
-              dst[i] = __float2half_rn( acc[t][4 * q4 + i] );
+              dst[i] = from_f32<E>( acc[t][4 * q4 + i] );
             }
           }
         }
@@ -342,13 +342,14 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
 int g_target_wgs = 0; // tuning override of the CU count the plan balances for (0: the device's)
 int g_gate_waves = 0;  // tuning override of the waves per work-group of the one-launch gate product (0: by the rule in its launcher; 4, 8)
 
-void launch( dim3 grid, hipStream_t st, bool split, __half* xout, float* partial, const __half* x, const __half* w, uint32_t s, uint32_t r, uint32_t b,
+template<typename E>
+void launch( dim3 grid, hipStream_t st, bool split, E* xout, float* partial, const E* x, const E* w, uint32_t s, uint32_t r, uint32_t b,
              uint32_t k_per_split, uint32_t n_col_slabs, uint32_t rows_per_wave )
 {
   if ( split ) {
-    gemm_stream_kernel<MODE_SPLIT><<<grid, 256, 0, st>>>( xout, partial, x, w, s, r, b, k_per_split, n_col_slabs, rows_per_wave );
+    gemm_stream_kernel<E, MODE_SPLIT><<<grid, 256, 0, st>>>( xout, partial, x, w, s, r, b, k_per_split, n_col_slabs, rows_per_wave );
   } else {
-    gemm_stream_kernel<MODE_PLAIN><<<grid, 256, 0, st>>>( xout, partial, x, w, s, r, b, k_per_split, n_col_slabs, rows_per_wave );
+    gemm_stream_kernel<E, MODE_PLAIN><<<grid, 256, 0, st>>>( xout, partial, x, w, s, r, b, k_per_split, n_col_slabs, rows_per_wave );
   }
 }
 
@@ -406,7 +407,8 @@ void gemm_stream_plan( uint64_t s, uint64_t r, uint64_t b, uint32_t* splits_out,
   *rows_per_wg_out = best_rows;
 }
 
-int gemm_stream_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits,
+template<typename E>
+int gemm_stream_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits,
                         uint32_t k_per_split, uint32_t rows_per_wg, bool write_partials, hipStream_t st )
 {
   GH_REQUIRE( rows_per_wg % 16 == 0 && rows_per_wg >= 16 && rows_per_wg <= WG_ROWS, "gh_matmul: bad row tile %u", rows_per_wg );
@@ -449,15 +451,20 @@ int gemm_stream_gate_launch( __half* hb, const __half* x, const __half* w13, uin
   const uint64_t gx = col_slabs == 1 ? row_blocks : ( row_blocks + 7 ) / 8 * 8 * col_slabs;
   GH_REQUIRE( gx < ( 1ull << 31 ), "gh_matmul_silu_gate: grid too large" );
   if ( waves == 8 ) {
-    gemm_stream_kernel<MODE_GATE, 8><<<dim3( (unsigned)gx, 1, 1 ), 512, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
+    gemm_stream_kernel<__half, MODE_GATE, 8><<<dim3( (unsigned)gx, 1, 1 ), 512, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
                                                                               (uint32_t)col_slabs, rows_per_wave );
   } else {
-    gemm_stream_kernel<MODE_GATE><<<dim3( (unsigned)gx, 1, 1 ), 256, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
+    gemm_stream_kernel<__half, MODE_GATE><<<dim3( (unsigned)gx, 1, 1 ), 256, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
                                                                            (uint32_t)col_slabs, rows_per_wave );
   }
   GH_LAUNCH_CHECK();
   return GH_OK;
 }
+
+template int gemm_stream_launch<__half>( __half*, float*, const __half*, const __half*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, uint32_t, bool,
+                                         hipStream_t );
+template int gemm_stream_launch<__bf16>( __bf16*, float*, const __bf16*, const __bf16*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, uint32_t, bool,
+                                         hipStream_t );
 
 void gemm_stream_tuning( int target_wgs, int depth )
 {

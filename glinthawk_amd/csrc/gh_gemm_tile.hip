@@ -1,5 +1,5 @@
 // Large-batch GEMM for prefill: xout(b, r) = sum_p w(r, p) * x(b, p) with b in the hundreds or
-// thousands (all prompt tokens of a batch at once), f16 storage, fp32 accumulate.  This regime is
+// thousands (all prompt tokens of a batch at once), f16 or bf16 storage, fp32 accumulate.  This regime is
 // MFMA-bound, not HBM-bound: both operands are re-used across a 128 x 128 output tile.
 //
 //   work-group = 4 waves (2 x 2), tile 128 weight rows x 128 tokens, K in steps of 64
@@ -24,7 +24,6 @@
 
 namespace gh {
 
-typedef _Float16 f16x8 __attribute__( ( ext_vector_type( 8 ) ) );
 typedef float f32x16 __attribute__( ( ext_vector_type( 16 ) ) );
 
 namespace {
@@ -38,7 +37,8 @@ struct Frag
   uint4 v[4]; // thread t: row t/8 + 32*i, chunk t%8
 };
 
-__device__ __forceinline__ void load_frag( Frag& f, const __half* __restrict__ mat, uint64_t ld, uint32_t row0, uint32_t n_rows, uint32_t k0, uint32_t k_end )
+template<typename E>
+__device__ __forceinline__ void load_frag( Frag& f, const E* __restrict__ mat, uint64_t ld, uint32_t row0, uint32_t n_rows, uint32_t k0, uint32_t k_end )
 {
   const uint32_t chunk = threadIdx.x & 7;
   const uint32_t k = k0 + 8 * chunk;
@@ -71,11 +71,11 @@ struct TileOrder
 };
 
 // grid: (8 * padded tiles per XCD, 1, k splits).  s % 8 == 0, 16-byte aligned operands.
-template<bool SPLIT>
-__global__ __launch_bounds__( 256 ) void gemm_tile_kernel( __half* __restrict__ xout,
+template<typename E, bool SPLIT>
+__global__ __launch_bounds__( 256 ) void gemm_tile_kernel( E* __restrict__ xout,
                                                            float* __restrict__ partial,
-                                                           const __half* __restrict__ x,
-                                                           const __half* __restrict__ w,
+                                                           const E* __restrict__ x,
+                                                           const E* __restrict__ w,
                                                            uint32_t s,
                                                            uint32_t r,
                                                            uint32_t b,
@@ -135,17 +135,17 @@ __global__ __launch_bounds__( 256 ) void gemm_tile_kernel( __half* __restrict__ 
 #pragma unroll
     for ( int st = 0; st < 4; st++ ) {
       const uint32_t ch = 2 * st + g2;
-      f16x8 a[2], bb[2];
+      typename Mfma<E>::x8 a[2], bb[2];
 #pragma unroll
       for ( int i = 0; i < 2; i++ ) {
-        a[i] = __builtin_bit_cast( f16x8, lw[swz( wm * 64 + 32 * i + lr, ch )] );
-        bb[i] = __builtin_bit_cast( f16x8, lx[swz( wn * 64 + 32 * i + lr, ch )] );
+        a[i] = __builtin_bit_cast( typename Mfma<E>::x8, lw[swz( wm * 64 + 32 * i + lr, ch )] );
+        bb[i] = __builtin_bit_cast( typename Mfma<E>::x8, lx[swz( wn * 64 + 32 * i + lr, ch )] );
       }
 #pragma unroll
       for ( int i = 0; i < 2; i++ ) {
 #pragma unroll
         for ( int j = 0; j < 2; j++ ) {
-          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_f16( a[i], bb[j], acc[i][j], 0, 0, 0 );
+          acc[i][j] = Mfma<E>::k16( a[i], bb[j], acc[i][j] );
         }
       }
     }
@@ -199,11 +199,11 @@ __global__ __launch_bounds__( 256 ) void gemm_tile_kernel( __half* __restrict__ 
           union
           {
             uint2 raw;
-            __half h[4];
+            E h[4];
           } o;
 #pragma unroll
           for ( int e = 0; e < 4; e++ ) {
-            o.h[e] = __float2half_rn( acc[i][j][4 * q4 + e] );
+            o.h[e] = from_f32<E>( acc[i][j][4 * q4 + e] );
           }
           const uint32_t chunk = 8 * wm + 4 * i + q4; // 8 rows each; g2 picks the half of the chunk
           out[( token * 16 + ( chunk ^ ( token & 15 ) ) ) * 2 + g2] = o.raw;
@@ -247,22 +247,22 @@ __global__ __launch_bounds__( 256 ) void gemm_tile_kernel( __half* __restrict__ 
           }
           continue;
         }
-        __half* dst = xout + (uint64_t)col * r + row;
+        E* dst = xout + (uint64_t)col * r + row;
         if ( row + 3 < r && ( r & 3 ) == 0 ) {
           union
           {
             uint2 raw;
-            __half h[4];
+            E h[4];
           } o;
 #pragma unroll
           for ( int e = 0; e < 4; e++ ) {
-            o.h[e] = __float2half_rn( acc[i][j][4 * q4 + e] );
+            o.h[e] = from_f32<E>( acc[i][j][4 * q4 + e] );
           }
           *reinterpret_cast<uint2*>( dst ) = o.raw;
         } else {
           for ( int e = 0; e < 4; e++ ) {
             if ( row + e < r ) {
-              dst[e] = __float2half_rn( acc[i][j][4 * q4 + e] );
+              dst[e] = from_f32<E>( acc[i][j][4 * q4 + e] );
             }
           }
         }
@@ -296,7 +296,8 @@ void gemm_tile_plan( uint64_t s, uint64_t r, uint64_t b, uint32_t* splits_out, u
 }
 
 // `partial` != nullptr: fp32 partial sums (splits, b, r) instead of xout
-int gemm_tile_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits, uint32_t k_per_split,
+template<typename E>
+int gemm_tile_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, uint32_t splits, uint32_t k_per_split,
                       hipStream_t st )
 {
   TileOrder ord;
@@ -313,12 +314,15 @@ int gemm_tile_launch( __half* xout, float* partial, const __half* x, const __hal
   GH_REQUIRE( partial != nullptr || splits == 1, "gh_matmul: split K needs a partials buffer" );
   const dim3 grid( (unsigned)gx, 1, splits );
   if ( partial != nullptr ) {
-    gemm_tile_kernel<true><<<grid, 256, 0, st>>>( xout, partial, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, k_per_split, ord );
+    gemm_tile_kernel<E, true><<<grid, 256, 0, st>>>( xout, partial, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, k_per_split, ord );
   } else {
-    gemm_tile_kernel<false><<<grid, 256, 0, st>>>( xout, partial, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, k_per_split, ord );
+    gemm_tile_kernel<E, false><<<grid, 256, 0, st>>>( xout, partial, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, k_per_split, ord );
   }
   GH_LAUNCH_CHECK();
   return GH_OK;
 }
+
+template int gemm_tile_launch<__half>( __half*, float*, const __half*, const __half*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, hipStream_t );
+template int gemm_tile_launch<__bf16>( __bf16*, float*, const __bf16*, const __bf16*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, hipStream_t );
 
 } // namespace gh

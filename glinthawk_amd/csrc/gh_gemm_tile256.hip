@@ -61,7 +61,6 @@
 
 namespace gh {
 
-typedef _Float16 f16x8 __attribute__( ( ext_vector_type( 8 ) ) );
 typedef float f32x16 __attribute__( ( ext_vector_type( 16 ) ) );
 typedef __attribute__( ( address_space( 3 ) ) ) void* lds_ptr;
 
@@ -121,16 +120,16 @@ constexpr int EPI_STORE = 0, EPI_ACCUM = 1, EPI_PARTIAL = 3;
 // grid: 8 x (padded tiles of one XCD) by K splits (more than one only with EPI_PARTIAL: split z leaves its sums in
 // partial[z]).  s % 64 == 0, k_len % 64 == 0, 16-byte aligned operands.
 // NA: 32-row accumulator tiles per wave, 2 (256 weight rows per work-group) or 3 (384).
-template<int EPI, int NA>
-__global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half* __restrict__ xout,
+template<typename E, int EPI, int NA>
+__global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( E* __restrict__ xout,
                                                                         float* __restrict__ partial,
-                                                                        const __half* __restrict__ x,
-                                                                        const __half* __restrict__ w,
+                                                                        const E* __restrict__ x,
+                                                                        const E* __restrict__ w,
                                                                         uint32_t s,
                                                                         uint32_t r,
                                                                         uint32_t b,
                                                                         uint32_t k_len, // k per split
-                                                                        __half* __restrict__ xout2, // rows from r_first on go here, as rows 0.. of a (b, r - r_first) matrix
+                                                                        E* __restrict__ xout2, // rows from r_first on go here, as rows 0.. of a (b, r - r_first) matrix
                                                                         uint32_t r_first, // rows [0, r_first) go to xout, a (b, r_first) matrix; == r: one output
                                                                         TileOrder ord )
 {
@@ -153,9 +152,9 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
   const uint32_t x_cols = min( (uint32_t)TN2, b - tile_col0 );
   const uint32_t k0 = blockIdx.y * k_len; // this split's k range starts here; the descriptors start there too and end with the tile's last row
   const __amdgpu_buffer_rsrc_t w_rsrc
-    = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
+    = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
   const __amdgpu_buffer_rsrc_t x_rsrc
-    = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
+    = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
   // A load-to-LDS writes lane l of a wave to (wave's base) + 16 l: thread t fills slot t % 8 of row
   // t / 8 (+ 64 i), so it fetches the chunk that the swizzle keeps in that slot.
   const uint32_t voff = ( threadIdx.x >> 3 ) * ld_bytes + ( ( threadIdx.x & 7 ) ^ ( ( threadIdx.x >> 4 ) & 7 ) ) * 16;
@@ -202,17 +201,17 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
   };
   struct Frags
   {
-    f16x8 a[NA], bb[4];
+    typename Mfma<E>::x8 a[NA], bb[4];
   };
   auto read_k16 = [&]( Frags& f, const uint4* wt, const uint4* xt, int kk ) {
     const uint32_t ch = 2 * kk + g2;
 #pragma unroll
     for ( int rt = 0; rt < NA; rt++ ) {
-      f.a[rt] = __builtin_bit_cast( f16x8, wt[swz( 32 * NA * wr + 32 * rt + fr, ch )] );
+      f.a[rt] = __builtin_bit_cast( typename Mfma<E>::x8, wt[swz( 32 * NA * wr + 32 * rt + fr, ch )] );
     }
 #pragma unroll
     for ( int t = 0; t < 4; t++ ) {
-      f.bb[t] = __builtin_bit_cast( f16x8, xt[swz( 128 * wc + 32 * t + fr, ch )] );
+      f.bb[t] = __builtin_bit_cast( typename Mfma<E>::x8, xt[swz( 128 * wc + 32 * t + fr, ch )] );
     }
   };
   auto mfma_k16 = [&]( const Frags& f ) {
@@ -220,7 +219,7 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
     for ( int t = 0; t < 4; t++ ) {
 #pragma unroll
       for ( int rt = 0; rt < NA; rt++ ) {
-        acc[rt][t] = __builtin_amdgcn_mfma_f32_32x32x16_f16( f.a[rt], f.bb[t], acc[rt][t], 0, 0, 0 );
+        acc[rt][t] = Mfma<E>::k16( f.a[rt], f.bb[t], acc[rt][t] );
       }
     }
   };
@@ -302,11 +301,11 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
           union
           {
             uint2 raw;
-            __half h[4];
+            E h[4];
           } o;
 #pragma unroll
           for ( int e = 0; e < 4; e++ ) {
-            o.h[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+            o.h[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
           }
           const uint32_t chunk = 4 * NA * wr + 4 * rt + q4;
           out[( token * CHUNKS + ( chunk ^ ( token & SWZ_MASK ) ) ) * 2 + g2] = o.raw;
@@ -324,14 +323,14 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
         union
         {
           uint4 raw;
-          __half h[8];
+          E h[8];
         } y, old;
         y.raw = region[j];
         if ( EPI == EPI_ACCUM ) { // the op that follows the product, on the rounded product
           old.raw = *dst;
 #pragma unroll
           for ( int e = 0; e < 8; e++ ) {
-            y.h[e] = __float2half_rn( __half2float( old.h[e] ) + __half2float( y.h[e] ) );
+            y.h[e] = from_f32<E>( to_f32<E>( old.h[e] ) + to_f32<E>( y.h[e] ) );
           }
         }
         *dst = y.raw;
@@ -393,22 +392,22 @@ __global__ __launch_bounds__( T256_THREADS, 1 ) void gemm_tile256_kernel( __half
             }
           }
         } else {
-          __half* dst = xout + (uint64_t)col * r + row; // (one output only: the launch refuses two with r % 8 != 0)
+          E* dst = xout + (uint64_t)col * r + row; // (one output only: the launch refuses two with r % 8 != 0)
           if ( whole ) {
             union
             {
               uint2 raw;
-              __half h[4];
+              E h[4];
             } o;
 #pragma unroll
             for ( int e = 0; e < 4; e++ ) {
-              o.h[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+              o.h[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
             }
             *reinterpret_cast<uint2*>( dst ) = o.raw;
           } else {
             for ( int e = 0; e < 4; e++ ) {
               if ( row + e < r ) {
-                dst[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+                dst[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
               }
             }
           }
@@ -453,6 +452,7 @@ struct W4Stages
 };
 
 // acc = w[tile rows] . x[tile tokens]^T over n_steps (even) steps of 64 k, both descriptors starting at the range's first k.
+template<typename E>
 __device__ __forceinline__ void w4_multiply( f32x16 ( &acc )[4][4], const __amdgpu_buffer_rsrc_t w_rsrc, const __amdgpu_buffer_rsrc_t x_rsrc, uint32_t ld_bytes,
                                              uint32_t n_steps, const W4Stages& st )
 {
@@ -475,7 +475,7 @@ __device__ __forceinline__ void w4_multiply( f32x16 ( &acc )[4][4], const __amdg
   }
   struct Frags
   {
-    f16x8 a[4], bb[4];
+    typename Mfma<E>::x8 a[4], bb[4];
   };
   Frags f0, f1;
   uint4 ra[16], rq[16]; // W0 X0 W1 X1 ... W7 X7 of a step (32 rows of the tile each), two steps in turn
@@ -483,8 +483,8 @@ __device__ __forceinline__ void w4_multiply( f32x16 ( &acc )[4][4], const __amdg
     const uint32_t ch = 2 * kk + g2;
 #pragma unroll
     for ( int i = 0; i < 4; i++ ) {
-      f.a[i] = __builtin_bit_cast( f16x8, wt[swz( 128 * wr + 32 * i + fr, ch )] );
-      f.bb[i] = __builtin_bit_cast( f16x8, xt[swz( 128 * wc + 32 * i + fr, ch )] );
+      f.a[i] = __builtin_bit_cast( typename Mfma<E>::x8, wt[swz( 128 * wr + 32 * i + fr, ch )] );
+      f.bb[i] = __builtin_bit_cast( typename Mfma<E>::x8, xt[swz( 128 * wc + 32 * i + fr, ch )] );
     }
   };
   auto mfma_k16 = [&]( const Frags& f ) __attribute__( ( always_inline ) ) {
@@ -492,7 +492,7 @@ __device__ __forceinline__ void w4_multiply( f32x16 ( &acc )[4][4], const __amdg
     for ( int t = 0; t < 4; t++ ) {
 #pragma unroll
       for ( int rt = 0; rt < 4; rt++ ) {
-        acc[rt][t] = __builtin_amdgcn_mfma_f32_32x32x16_f16( f.a[rt], f.bb[t], acc[rt][t], 0, 0, 0 );
+        acc[rt][t] = Mfma<E>::k16( f.a[rt], f.bb[t], acc[rt][t] );
       }
     }
   };
@@ -575,16 +575,17 @@ __device__ __forceinline__ void w4_multiply( f32x16 ( &acc )[4][4], const __amdg
 // acc[rt][t][v]: row = tile_row0 + 128*wr + 32*rt + 8*(v/4) + 4*(lane/32) + v%4, token = tile_col0 + 128*wc + 32*t + lane%32.
 // Output of a whole tile: through LDS (token-major, the four stage arrays as four regions of 64 tokens x 256 rows) as whole row
 // segments where r % 8 == 0, else (and for the fp32 sums of a K split) from the registers.
+template<typename E>
 struct W4Out
 {
-  __half* xout;
-  __half* xout2;    // rows from r_first on go here, as rows 0.. of a (b, r - r_first) matrix
+  E* xout;
+  E* xout2;    // rows from r_first on go here, as rows 0.. of a (b, r - r_first) matrix
   float* partial;   // EPI_PARTIAL: (splits, b, r)
   uint32_t r, b, r_first, split;
 };
 
-template<int EPI>
-__device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Out& o, uint32_t tile_row0, uint32_t tile_col0, const W4Stages& st )
+template<typename E, int EPI>
+__device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Out<E>& o, uint32_t tile_row0, uint32_t tile_col0, const W4Stages& st )
 {
   const uint32_t wave = __builtin_amdgcn_readfirstlane( threadIdx.x >> 6 );
   const uint32_t lane = threadIdx.x & 63;
@@ -606,11 +607,11 @@ __device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Ou
           union
           {
             uint2 raw;
-            __half h[4];
+            E h[4];
           } v;
 #pragma unroll
           for ( int e = 0; e < 4; e++ ) {
-            v.h[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+            v.h[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
           }
           const uint32_t chunk = 16 * wr + 4 * rt + q4;
           out[( token * CHUNKS + ( chunk ^ ( token & SWZ_MASK ) ) ) * 2 + g2] = v.raw;
@@ -631,14 +632,14 @@ __device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Ou
         union
         {
           uint4 raw;
-          __half h[8];
+          E h[8];
         } y, old;
         y.raw = region[j];
         if ( EPI == EPI_ACCUM ) { // the op that follows the product, on the rounded product
           old.raw = *dst;
 #pragma unroll
           for ( int e = 0; e < 8; e++ ) {
-            y.h[e] = __float2half_rn( __half2float( old.h[e] ) + __half2float( y.h[e] ) );
+            y.h[e] = from_f32<E>( to_f32<E>( old.h[e] ) + to_f32<E>( y.h[e] ) );
           }
         }
         *dst = y.raw;
@@ -670,22 +671,22 @@ __device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Ou
             }
           }
         } else {
-          __half* dst = o.xout + (uint64_t)col * o.r + row; // (one output only: the launch refuses two with r % 8 != 0)
+          E* dst = o.xout + (uint64_t)col * o.r + row; // (one output only: the launch refuses two with r % 8 != 0)
           if ( whole ) {
             union
             {
               uint2 raw;
-              __half h[4];
+              E h[4];
             } v;
 #pragma unroll
             for ( int e = 0; e < 4; e++ ) {
-              v.h[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+              v.h[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
             }
             *reinterpret_cast<uint2*>( dst ) = v.raw;
           } else {
             for ( int e = 0; e < 4; e++ ) {
               if ( row + e < o.r ) {
-                dst[e] = __float2half_rn( acc[rt][t][4 * q4 + e] );
+                dst[e] = from_f32<E>( acc[rt][t][4 * q4 + e] );
               }
             }
           }
@@ -696,16 +697,16 @@ __device__ __forceinline__ void w4_store_tile( f32x16 ( &acc )[4][4], const W4Ou
 }
 
 // grid as gemm_tile256_kernel: 8 x (padded tiles of one XCD) by K splits; k_len % 128 == 0, s % 128 == 0
-template<int EPI>
-__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_tile256w4_kernel( __half* __restrict__ xout,
+template<typename E, int EPI>
+__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_tile256w4_kernel( E* __restrict__ xout,
                                                                         float* __restrict__ partial,
-                                                                        const __half* __restrict__ x,
-                                                                        const __half* __restrict__ w,
+                                                                        const E* __restrict__ x,
+                                                                        const E* __restrict__ w,
                                                                         uint32_t s,
                                                                         uint32_t r,
                                                                         uint32_t b,
                                                                         uint32_t k_len,
-                                                                        __half* __restrict__ xout2,
+                                                                        E* __restrict__ xout2,
                                                                         uint32_t r_first,
                                                                         TileOrder ord )
 {
@@ -720,14 +721,14 @@ __global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_tile256w4_kernel( __half
   const uint32_t w_rows = min( (uint32_t)TM2, r - tile_row0 ), x_cols = min( (uint32_t)TN2, b - tile_col0 );
   const uint32_t k0 = blockIdx.y * k_len; // this split's k range starts here; the descriptors start there too and end with the tile's last row
   const __amdgpu_buffer_rsrc_t w_rsrc
-    = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
+    = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
   const __amdgpu_buffer_rsrc_t x_rsrc
-    = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
+    = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
   const W4Stages st { s_w0, s_x0, s_w1, s_x1 };
   f32x16 acc[4][4];
-  w4_multiply( acc, w_rsrc, x_rsrc, ld_bytes, min( k_len, s - k0 ) / TKS, st );
-  const W4Out o { xout, xout2, partial, r, b, r_first, blockIdx.y };
-  w4_store_tile<EPI>( acc, o, tile_row0, tile_col0, st );
+  w4_multiply<E>( acc, w_rsrc, x_rsrc, ld_bytes, min( k_len, s - k0 ) / TKS, st );
+  const W4Out<E> o { xout, xout2, partial, r, b, r_first, blockIdx.y };
+  w4_store_tile<E, EPI>( acc, o, tile_row0, tile_col0, st );
 }
 
 // Equal shares of all the 64-k steps of a product.  Tile t (token fastest: t = row tile x token tiles + token tile) owns the steps
@@ -748,14 +749,14 @@ __device__ __forceinline__ uint32_t streamk_share_of_workgroup( const StreamK& s
 }
 
 // grid: 8 * ceil(shares / 8) work-groups, one per CU
-template<int EPI>
-__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_streamk_kernel( __half* __restrict__ xout,
-                                                                         const __half* __restrict__ x,
-                                                                         const __half* __restrict__ w,
+template<typename E, int EPI>
+__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_streamk_kernel( E* __restrict__ xout,
+                                                                         const E* __restrict__ x,
+                                                                         const E* __restrict__ w,
                                                                          uint32_t s,
                                                                          uint32_t r,
                                                                          uint32_t b,
-                                                                         __half* __restrict__ xout2,
+                                                                         E* __restrict__ xout2,
                                                                          uint32_t r_first,
                                                                          StreamK sk )
 {
@@ -780,14 +781,14 @@ __global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_streamk_kernel( __hal
     const uint32_t w_rows = min( (uint32_t)TM2, r - tile_row0 ), x_cols = min( (uint32_t)TN2, b - tile_col0 );
     const uint32_t k0 = step0 * TKS;
     const __amdgpu_buffer_rsrc_t w_rsrc
-      = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
+      = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( w + (uint64_t)tile_row0 * s + k0 ), 0, (int)( w_rows * ld_bytes - k0 * 2 ), 0x00020000 );
     const __amdgpu_buffer_rsrc_t x_rsrc
-      = __builtin_amdgcn_make_buffer_rsrc( const_cast<__half*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
+      = __builtin_amdgcn_make_buffer_rsrc( const_cast<E*>( x + (uint64_t)tile_col0 * s + k0 ), 0, (int)( x_cols * ld_bytes - k0 * 2 ), 0x00020000 );
     f32x16 acc[4][4];
-    w4_multiply( acc, w_rsrc, x_rsrc, ld_bytes, n_steps, st );
+    w4_multiply<E>( acc, w_rsrc, x_rsrc, ld_bytes, n_steps, st );
     if ( n_steps == sk.steps ) { // a whole tile: finished here
-      const W4Out o { xout, xout2, nullptr, r, b, r_first, 0 };
-      w4_store_tile<EPI>( acc, o, tile_row0, tile_col0, st );
+      const W4Out<E> o { xout, xout2, nullptr, r, b, r_first, 0 };
+      w4_store_tile<E, EPI>( acc, o, tile_row0, tile_col0, st );
     } else { // a piece: its sums as they lie in the registers, 1 KiB per wave and store
       float* piece = sk.pieces + ( (uint64_t)g * 2 + ( tile == first_tile ? 0 : 1 ) ) * PIECE_FLOATS + (uint64_t)wave * ( PIECE_FLOATS / 4 );
 #pragma unroll
@@ -809,8 +810,8 @@ __global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_streamk_kernel( __hal
 
 // One work-group per tile: nothing to do for a tile that one share covered whole; else the pieces of the tile added in ascending
 // order of the share, then the same output path as a tile finished in the multiply kernel.
-template<int EPI>
-__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_fixup_kernel( __half* __restrict__ xout, uint32_t r, uint32_t b, __half* __restrict__ xout2, uint32_t r_first,
+template<typename E, int EPI>
+__global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_fixup_kernel( E* __restrict__ xout, uint32_t r, uint32_t b, E* __restrict__ xout2, uint32_t r_first,
                                                                        StreamK sk )
 {
   __shared__ uint4 s_x0[TN2 * 8], s_x1[TN2 * 8];
@@ -852,8 +853,8 @@ __global__ __launch_bounds__( T4_THREADS, 1 ) void gemm_w4_fixup_kernel( __half*
     }
   }
   const W4Stages st { s_w0, s_x0, s_w1, s_x1 };
-  const W4Out o { xout, xout2, nullptr, r, b, r_first, 0 };
-  w4_store_tile<EPI>( acc, o, ( tile / sk.token_tiles ) * TM2, ( tile % sk.token_tiles ) * TN2, st );
+  const W4Out<E> o { xout, xout2, nullptr, r, b, r_first, 0 };
+  w4_store_tile<E, EPI>( acc, o, ( tile / sk.token_tiles ) * TM2, ( tile % sk.token_tiles ) * TN2, st );
 }
 
 // GLINT_TILE_ROWS in the environment sets the start value (for the command-line profilers, which have no other way in)
@@ -999,8 +1000,9 @@ void gemm_tile256_split_plan( uint64_t s, uint64_t r, uint64_t b, const void* x,
 
 // `partial` != nullptr: fp32 sums (splits, b, r) instead of xout; else `epilogue` 0 stores, 1 accumulates into xout (needs r % 8 == 0).
 // splits > 1 (from gemm_tile256_split_plan, with its k_len) needs `partial`.
-int gemm_tile256_launch( __half* xout, float* partial, const __half* x, const __half* w, uint64_t s, uint64_t r, uint64_t b, int epilogue, hipStream_t st,
-                         uint32_t splits, uint32_t k_len, __half* xout2 = nullptr, uint64_t r_first = 0 )
+template<typename E>
+int gemm_tile256_launch( E* xout, float* partial, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, int epilogue, hipStream_t st, uint32_t splits,
+                         uint32_t k_len, E* xout2, uint64_t r_first )
 {
   if ( xout2 == nullptr ) {
     r_first = r;
@@ -1037,11 +1039,11 @@ int gemm_tile256_launch( __half* xout, float* partial, const __half* x, const __
       sk.pieces = static_cast<float*>( pieces );
       const unsigned wgs = 8 * ( ( sk.shares + 7 ) / 8 );
       if ( epi_sk == EPI_STORE ) {
-        gemm_w4_streamk_kernel<EPI_STORE><<<wgs, T4_THREADS, 0, st>>>( xout, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
-        gemm_w4_fixup_kernel<EPI_STORE><<<sk.tiles, T4_THREADS, 0, st>>>( xout, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
+        gemm_w4_streamk_kernel<E, EPI_STORE><<<wgs, T4_THREADS, 0, st>>>( xout, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
+        gemm_w4_fixup_kernel<E, EPI_STORE><<<sk.tiles, T4_THREADS, 0, st>>>( xout, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
       } else {
-        gemm_w4_streamk_kernel<EPI_ACCUM><<<wgs, T4_THREADS, 0, st>>>( xout, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
-        gemm_w4_fixup_kernel<EPI_ACCUM><<<sk.tiles, T4_THREADS, 0, st>>>( xout, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
+        gemm_w4_streamk_kernel<E, EPI_ACCUM><<<wgs, T4_THREADS, 0, st>>>( xout, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
+        gemm_w4_fixup_kernel<E, EPI_ACCUM><<<sk.tiles, T4_THREADS, 0, st>>>( xout, (uint32_t)r, (uint32_t)b, xout2, (uint32_t)r_first, sk );
       }
       GH_LAUNCH_CHECK();
       return GH_OK;
@@ -1067,9 +1069,9 @@ int gemm_tile256_launch( __half* xout, float* partial, const __half* x, const __
   const int epi = partial != nullptr ? EPI_PARTIAL : epilogue;
   GH_REQUIRE( epi == EPI_STORE || epi == EPI_ACCUM || epi == EPI_PARTIAL, "gh_matmul: unknown tile epilogue %d", epi );
   GH_REQUIRE( epi != EPI_ACCUM || r % 8 == 0, "gh_matmul: the accumulating tile epilogue needs r %% 8 == 0" );
-#define GH_TILE256_LAUNCH( E, N ) gemm_tile256_kernel<E, N><<<grid, block, 0, st>>>( xout, partial, x, w, s32, r32, b32, k_len, xout2, (uint32_t)r_first, ord )
-#define GH_TILE256_W4( E ) gemm_tile256w4_kernel<E><<<grid, block, 0, st>>>( xout, partial, x, w, s32, r32, b32, k_len, xout2, (uint32_t)r_first, ord )
-#define GH_TILE256_ROWS( E ) ( four_waves ? GH_TILE256_W4( E ) : tile_rows == 384 ? GH_TILE256_LAUNCH( E, 3 ) : GH_TILE256_LAUNCH( E, 2 ) )
+#define GH_TILE256_LAUNCH( EP, N ) gemm_tile256_kernel<E, EP, N><<<grid, block, 0, st>>>( xout, partial, x, w, s32, r32, b32, k_len, xout2, (uint32_t)r_first, ord )
+#define GH_TILE256_W4( EP ) gemm_tile256w4_kernel<E, EP><<<grid, block, 0, st>>>( xout, partial, x, w, s32, r32, b32, k_len, xout2, (uint32_t)r_first, ord )
+#define GH_TILE256_ROWS( EP ) ( four_waves ? GH_TILE256_W4( EP ) : tile_rows == 384 ? GH_TILE256_LAUNCH( EP, 3 ) : GH_TILE256_LAUNCH( EP, 2 ) )
   switch ( epi ) {
     case EPI_STORE: GH_TILE256_ROWS( EPI_STORE ); break;
     case EPI_ACCUM: GH_TILE256_ROWS( EPI_ACCUM ); break;
@@ -1081,5 +1083,10 @@ int gemm_tile256_launch( __half* xout, float* partial, const __half* x, const __
   GH_LAUNCH_CHECK();
   return GH_OK;
 }
+
+template int gemm_tile256_launch<__half>( __half*, float*, const __half*, const __half*, uint64_t, uint64_t, uint64_t, int, hipStream_t, uint32_t, uint32_t,
+                                          __half*, uint64_t );
+template int gemm_tile256_launch<__bf16>( __bf16*, float*, const __bf16*, const __bf16*, uint64_t, uint64_t, uint64_t, int, hipStream_t, uint32_t, uint32_t,
+                                          __bf16*, uint64_t );
 
 } // namespace gh
