@@ -101,6 +101,15 @@ OTHER_WORKLOADS = {
     "llama2-70b-churn-256": "Llama2-70B GQA shape, one stage of 10 layers, fp16: 256 context slots with lengths U[16,4096]; every "
                             "step decodes all slots, then 10 % of them finish and are refilled in place with 128-token prefills",
 }
+# run-time sized designs at layer sizes of a real model (--design), each beside the Llama2 shape of the same width, heads and hidden size
+DESIGNS = {
+    "famidra-w4096": dict(
+        llama=("llama2-7b", 8, 4), batch=32, context=1024, prefill=(8, 1024),
+        config=dict(width=4096, ff=11008, heads=32, kv_heads=32, dim=128, window=1024, mlstm=dict(heads=8, dim=256, vdim=512))),
+    "famidra-w8192": dict(
+        llama=("llama2-70b-4k", 10, 4), batch=64, context=2048, prefill=(4, 2048),
+        config=dict(width=8192, ff=28672, heads=64, kv_heads=8, dim=128, window=2048, mlstm=dict(heads=16, dim=256, vdim=512))),
+}
 LAYER_TENSORS = ("rms_att_weight", "wq", "wkv", "wo", "rms_ffn_weight", "w1", "w2", "w3")
 
 
@@ -617,6 +626,94 @@ def churn_bench(steps, warmup, cpu=True):
     }
 
 
+def famidra_config(c, positions):
+    """config.json of a Famidra model of these layer sizes: two mLSTM and two attention layers, the middle two passed twice."""
+    mlstm = {"type": "mlstm", "mixer": dict(gate_cap=15.0, **c["mlstm"]), "mlp": None}
+    attention = {"type": "attention", "mlp": {"kind": "dense", "ff": c["ff"]},
+                 "mixer": {"heads": c["heads"], "kv_heads": c["kv_heads"], "dim": c["dim"], "vdim": c["dim"], "scale": c["dim"] ** -0.5, "bias_max": 512,
+                           "mask": {"size": c["window"], "keep_first": 4}}}
+    return {"architecture": "Famidra", "width": c["width"], "vocab": 32000, "max_positions": positions, "norm": {"eps": 1e-5}, "logit_scale": 1.0,
+            "layers": [mlstm, attention, mlstm, attention], "loop": {"start": 1, "stop": 3, "times": 2}}
+
+
+def design_bench(name, steps, warmup):
+    """Prefill and decode of a run-time sized design (random weights) and of the closest Llama2 stage of equal layer sizes: decode of
+    `batch` contexts at `context` keys, prefill of `prefill` prompts x tokens, both through the drivers' own entry points."""
+    import tempfile
+
+    import numpy as np
+
+    from glinthawk_amd import ops, stage as S
+
+    d = DESIGNS[name]
+    ops.init(0)
+    (n_prompts, T), batch, context = d["prefill"], d["batch"], d["context"]
+    positions = max(context + 2 * (steps + warmup) + 8, T)
+    rng = np.random.default_rng(9)
+
+    def timed(run, n):
+        for _ in range(warmup):
+            run()
+        ops.sync()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            run()
+        ops.sync()
+        return (time.perf_counter() - t0) * 1e3 / n
+
+    with tempfile.TemporaryDirectory() as tmp:
+        cfg = famidra_config(d["config"], positions)
+        with open(os.path.join(tmp, "config.json"), "w") as f:
+            json.dump(cfg, f)
+        st = S.DesignStage(tmp, "bf16", batch, batch, random_weights=True)
+    ids = list(range(batch))
+    prompts = rng.integers(0, cfg["vocab"], (n_prompts, T))
+
+    def design_prefill():
+        st.prefill_logits(ids[:n_prompts], [0] * n_prompts, prompts, want_next_tokens=True)
+
+    prefill_ms = timed(design_prefill, max(1, steps // 4))
+    for i in range(0, batch, n_prompts):        # every context at the decode length
+        part = ids[i:i + n_prompts]
+        st.prefill_logits(part, [0] * len(part), rng.integers(0, cfg["vocab"], (len(part), context)))
+    st.new_state(batch)
+    st.set_prompts(ids, [1] * batch, [context] * batch, prompt_length=1, max_completion_length=positions)
+    st.time_device_spans(True)
+    decode_ms = timed(lambda: st.forward(), steps)
+    span_ms, spans = st.device_spans()
+    runs = st.layer_runs
+    st.close()
+
+    cfg_name, first, hosted = d["llama"]
+    shape = SHAPES[cfg_name]
+    ll = S.Stage(cfg_name, "f16", first, hosted, batch, batch)
+    x = ops.pinned_empty((n_prompts * T, shape["dim"]), np.float16)
+    x[:] = rng.standard_normal(x.shape).astype(np.float16)
+    y = ops.pinned_empty(x.shape, np.float16)
+    llama_prefill_ms = timed(lambda: ll.prefill(ids[:n_prompts], [0] * n_prompts, T, first, activations=x, want_activations=False), max(1, steps // 4))
+
+    def llama_decode():
+        ll.new_state(batch, next_layer=first)
+        ll.set_prompts(ids, [1] * batch, [context] * batch)
+        ll.activations(allocate=True)
+        ll.forward()
+
+    ll.time_device_spans(True)
+    llama_ms = timed(llama_decode, steps)
+    llama_span_ms, llama_spans = ll.device_spans()
+    ll.close()
+    del y
+    return {"design": name, "metric": "prefill and decode tokens/s beside the closest Llama2 stage of equal layer sizes", "n_gpus": 1, "steps": steps,
+            "warmup": warmup, "data": "synthetic", "dtype": "bf16", "config": {**d["config"], "layer_runs": runs, "vocab": cfg["vocab"]},
+            "decode": {"batch": batch, "context": context, "ms_per_step": round(decode_ms, 4), "device_ms_per_step": round(span_ms / spans, 4),
+                       "tokens_per_s": round(batch / decode_ms * 1e3, 1), "device_ms_per_layer_run": round(span_ms / spans / runs, 4)},
+            "prefill": {"prompts": n_prompts, "tokens": T, "ms_per_step": round(prefill_ms, 3), "tokens_per_s": round(n_prompts * T / prefill_ms * 1e3, 1),
+                        "ms_per_layer_run": round(prefill_ms / runs, 3)},
+            "llama": {"stage": cfg_name, "layers": hosted, "dtype": "f16",
+                      "decode": {"ms_per_step": round(llama_ms, 4), "device_ms_per_layer": round(llama_span_ms / llama_spans / hosted, 4)},
+                      "prefill": {"ms_per_step": round(llama_prefill_ms, 3), "ms_per_layer": round(llama_prefill_ms / hosted, 3)}}}
+
+
 def with_own_kernels(others):
     """When a run was asked to send products to the vendor's GEMM library, the same prefill and churn steps once more on
     the kernels of this library, so that the line carries both (`ms_per_step_own_kernels`)."""
@@ -689,6 +786,8 @@ def main():
     ap.add_argument("--full-configs", action="store_true",
                     help="the other configurations at their stated run lengths instead of the headline line: 128 decode steps at 1024..1151 keys "
                          "(7B shape), the 8 x 2048 prefill with its 64 decode steps (13B shape), 512 churn steps (70B shape); takes some minutes")
+    ap.add_argument("--design", default=None, choices=sorted(DESIGNS),
+                    help="instead of the headline line: prefill and decode of a run-time sized design beside the closest Llama2 stage of equal layer sizes")
     args = ap.parse_args()
 
     if args.gpus != 1:
@@ -696,6 +795,9 @@ def main():
               "(the path shards by context, slot -> GPU, with no collective; only the one-GPU share is built)", file=sys.stderr)
         sys.exit(2)
 
+    if args.design:
+        print(json.dumps(design_bench(args.design, args.steps, args.warmup)))
+        return
     cpu = not args.no_cpu_baseline
     if args.calibration_copy_mib > 0:
         from glinthawk_amd import ops

@@ -53,11 +53,28 @@ class Shape:
                        self.n_heads, self.n_kv_heads, self.gqa_size, self.vocab_size, self.seq_len)
 
 
+GH_ACT_SILU, GH_ACT_GELU_TANH = 0, 1
+
+
+class GhStreamStep(C.Structure):
+    _fields_ = [("bias", C.c_void_p), ("post_norm", C.c_void_p), ("add", C.c_void_p), ("next_norm", C.c_void_p), ("out", C.c_void_p),
+                ("out_stride", C.c_uint64), ("eps", C.c_float), ("accumulate", C.c_int)]
+
+
+class GhWindowAttn(C.Structure):
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "kv_heads", "dim", "vdim", "window", "keep_first", "n_dist")] + [("scale", C.c_float)]
+
+
+class GhMlstm(C.Structure):
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "dim", "vdim")] + [("gate_cap", C.c_float), ("eps", C.c_float)]
+
+
 _lib: Optional[C.CDLL] = None
 
 # name -> (restype, argtypes); every symbol declared in include/glint_hip.h
 _u64, _u32, _vp, _i, _f = C.c_uint64, C.c_uint32, C.c_void_p, C.c_int, C.c_float
 _shp = C.POINTER(GhShape)
+_step, _win, _mls = C.POINTER(GhStreamStep), C.POINTER(GhWindowAttn), C.POINTER(GhMlstm)
 SIGNATURES = {
     "gh_init": (_i, [_i]),
     "gh_last_error": (C.c_char_p, []),
@@ -134,6 +151,19 @@ SIGNATURES = {
     "gh_attn_set_prefill_tiles": (_i, [_i]),
     "gh_attn_prefill_workspace": (_u64, [_u64, _u32, _shp]),
     "gh_attn_prefill": (_i, [_vp, _vp, _vp, _vp, _u64, _u32, _u32, _shp, _i, _vp, _u64, _i, _vp]),
+    "gh_embed_positions": (_i, [_vp, _vp, _vp, _u64, _u32, _vp, _vp, _u64, _u64, _u64, _vp, _u64, _i, _vp]),
+    "gh_matmul_stream": (_i, [_vp, _vp, _vp, _u64, _u64, _u64, _step, _i, _vp]),
+    "gh_stream_out": (_i, [_vp, _u64, _u64, _step, _i, _vp]),
+    "gh_matmul_gate": (_i, [_vp, _vp, _vp, _vp, _u64, _u64, _u64, _i, _i, _vp]),
+    "gh_matmul_scaled": (_i, [_vp, _vp, _vp, _u64, _u64, _u64, _f, _i, _vp]),
+    "gh_gather_rows": (_i, [_vp, _vp, _vp, _u64, _u64, _u64, _vp]),
+    "gh_window_row_bytes": (_u64, [_win, _i]),
+    "gh_window_query_elements": (_u64, [_win]),
+    "gh_matmul_window_append": (_i, [_vp, _vp, _vp, _vp, _u64, _win, _vp, _vp, _f, _vp, _u64, _vp, _u64, _u32, _i, _vp]),
+    "gh_attn_window": (_i, [_vp, _vp, _win, _vp, _vp, _u64, _vp, _u64, _u32, _u32, _i, _vp]),
+    "gh_mlstm_state_bytes": (_u64, [_mls]),
+    "gh_mlstm_weight_rows": (_u64, [_mls, C.POINTER(_u64)]),
+    "gh_mlstm_forward": (_i, [_vp, _vp, _vp, _u64, _mls, _vp, _vp, _vp, _vp, _u64, _vp, _u64, _u32, _i, _vp]),
     "gh_attn_timing_enable": (_i, [_i]),
     "gh_attn_timing_reset": (_i, []),
     "gh_attn_timing_read": (_i, [C.POINTER(C.c_double), C.POINTER(C.c_double), C.POINTER(_u64)]),

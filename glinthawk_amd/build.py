@@ -4,7 +4,9 @@ Usage: ``python -m glinthawk_amd.build``.  hipcc cross-compiles for gfx950 witho
 """
 from __future__ import annotations
 
+import fcntl
 import glob
+import hashlib
 import os
 import subprocess
 import sys
@@ -76,6 +78,8 @@ def build_tools() -> list[str]:
     """profile-stage-hip and profile-gemm-hip: the reference's profiling front ends for this target."""
     built = []
     for src in sorted(glob.glob(os.path.join(HOST, "bin", "*.cc"))):
+        if os.path.basename(src) == "trace_run.cc":     # links its kernels into itself, see trace_run_program()
+            continue
         name = os.path.splitext(os.path.basename(src))[0].replace("_", "-") + "-hip"
         exe = os.path.join(LIB_DIR, name)
         _run([HIPCC, *COMMON_FLAGS, "-std=c++20", "-x", "c++", "-I" + HOST, "-o", exe, src,
@@ -84,10 +88,52 @@ def build_tools() -> list[str]:
     return built
 
 
+# kernels of the run-time sized designs and what they stand on: all that the trace runner needs
+TRACE_KERNELS = ("gh_runtime", "gh_elementwise", "gh_gemm", "gh_gemm_lib", "gh_gemm_stream", "gh_gemm_tile", "gh_gemm_tile256",
+                 "gh_stream_rows", "gh_attn_window", "gh_mlstm")
+
+
+def _trace_run_path() -> str:
+    """The program's path, named by a digest of everything it is built from: a program of other sources is not taken for it."""
+    digest = hashlib.sha256(" ".join([*DEVICE_FLAGS, *COMMON_FLAGS[:4]]).encode())
+    sources = [os.path.join(CSRC, k + ".hip") for k in TRACE_KERNELS] + [os.path.join(HOST, "bin", "trace_run.cc")]
+    for pattern in (os.path.join(CSRC, "*.h"), os.path.join(ROOT, "include", "*.h"), os.path.join(HOST, "glint", "**", "*.hh")):
+        sources += glob.glob(pattern, recursive=True)
+    for path in sorted(sources):
+        with open(path, "rb") as f:
+            digest.update(os.path.relpath(path, ROOT).encode() + b"\0" + f.read())
+    return os.path.join(LIB_DIR, f"trace-run-{digest.hexdigest()[:16]}-hip")
+
+
+def trace_run_program() -> str:
+    """Path of the trace runner, compiled first where it is not there yet."""
+    exe = _trace_run_path()
+    if os.path.exists(exe):
+        return exe
+    os.makedirs(LIB_DIR, exist_ok=True)
+    work = os.path.join(PKG, "build", "trace")
+    os.makedirs(work, exist_ok=True)
+    with open(os.path.join(work, "lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)        # calls that start together compile once
+        if not os.path.exists(exe):
+            jobs = [[HIPCC, *DEVICE_FLAGS, *COMMON_FLAGS, "-std=c++17", "-c", os.path.join(CSRC, k + ".hip"), "-o", os.path.join(work, k + ".o")]
+                    for k in TRACE_KERNELS]
+            jobs.append([HIPCC, *COMMON_FLAGS, "-std=c++20", "-x", "c++", "-I" + HOST, "-c", os.path.join(HOST, "bin", "trace_run.cc"),
+                         "-o", os.path.join(work, "trace_run.o")])
+            with ThreadPoolExecutor(max_workers=min(len(jobs), os.cpu_count() or 1, 16)) as pool:
+                list(pool.map(_run, jobs))
+            for old in glob.glob(os.path.join(LIB_DIR, "trace-run-*-hip")):
+                os.unlink(old)
+            _run([HIPCC, "--offload-arch=gfx950", "-o", exe + ".part", *[j[-1] for j in jobs], "-pthread"])
+            os.replace(exe + ".part", exe)
+    return exe
+
+
 def build_all() -> None:
     build_kernels()
     build_host()
     build_tools()
+    trace_run_program()
 
 
 if __name__ == "__main__":

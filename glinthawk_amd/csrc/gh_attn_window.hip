@@ -1,0 +1,474 @@
+// Attention over a sliding window with kept first tokens and a bias by distance (storage type bf16 or fp32, sizes at run time).
+//
+//   position i sees j <= i with i - j < window or j < keep_first;  score = (q . k) * scale + bias[h][min(i - j, n_dist - 1)]
+//
+// cache row   [K of every kv head | V of every kv head], each head padded with zeros to a multiple of 8 elements, so that any head size
+//             is read in 16-byte (bf16) or 32-byte (fp32) pieces
+// keys        a query's visible keys are numbered 0 .. count - 1: first the kept ones in front of the window, then the window
+// rows kernel work-group = 4 waves on one (token, kv head, block of query heads, split of the keys); 16 lanes hold one key, eight
+//             elements a lane, so a wave takes four keys at a time; every 16-lane group keeps its own running maximum and sum for
+//             each of its query heads and they meet once, at the end.  Scores, weights and sums are fp32.
+#include "gh_product.h"
+
+#include <algorithm>
+
+namespace gh {
+namespace {
+
+struct WindowShape
+{
+  uint32_t heads, kv_heads, group; // query heads, kv heads, query heads per kv head
+  uint32_t dim, vdim, dpad, vpad;  // padded head sizes of the cache
+  uint32_t window, keep_first, n_dist;
+  float scale;
+  __host__ __device__ uint32_t k_elems() const { return kv_heads * dpad; }
+  __host__ __device__ uint32_t row_elems() const { return kv_heads * ( dpad + vpad ); }
+};
+
+struct WindowRows
+{
+  void* const* rows; // context regions; NULL: no context
+  uint64_t offset;   // bytes from there to this layer's rows
+  const uint32_t* start_pos;
+  uint32_t n_tokens;
+};
+
+// ---- q / k norm over the whole projection, cache append ------------------------------------------
+template<typename E, typename View>
+__global__ __launch_bounds__( 256 ) void window_append_kernel( E* __restrict__ q_out,
+                                                               View y,
+                                                               const E* __restrict__ bias,
+                                                               const E* __restrict__ q_norm,
+                                                               const E* __restrict__ k_norm,
+                                                               WindowRows wr,
+                                                               WindowShape s,
+                                                               float eps )
+{
+  extern __shared__ float vals[]; // q and k of the row
+  __shared__ float s_red[2][4];
+  const uint64_t row = blockIdx.x;
+  const uint32_t ctx = (uint32_t)( row / wr.n_tokens ), tok = (uint32_t)( row % wr.n_tokens );
+  uint8_t* base = static_cast<uint8_t*>( wr.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  E* cache = reinterpret_cast<E*>( base + wr.offset ) + (uint64_t)( wr.start_pos[ctx] + tok ) * s.row_elems();
+  const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim, nv = s.kv_heads * s.vdim;
+  float ssq = 0.0f, ssk = 0.0f;
+  for ( uint32_t c = threadIdx.x; c < nq + nk; c += blockDim.x ) {
+    const float v = y.at( row, c ) + ( bias != nullptr ? to_f32( bias[c] ) : 0.0f );
+    vals[c] = v;
+    if ( c < nq ) {
+      ssq += v * v;
+    } else {
+      ssk += v * v;
+    }
+  }
+  ssq = wave_sum( ssq );
+  ssk = wave_sum( ssk );
+  if ( ( threadIdx.x & 63 ) == 0 ) {
+    s_red[0][threadIdx.x >> 6] = ssq;
+    s_red[1][threadIdx.x >> 6] = ssk;
+  }
+  __syncthreads();
+  ssq = ( s_red[0][0] + s_red[0][1] ) + ( s_red[0][2] + s_red[0][3] );
+  ssk = ( s_red[1][0] + s_red[1][1] ) + ( s_red[1][2] + s_red[1][3] );
+  const float iq = q_norm != nullptr ? 1.0f / sqrtf( ssq / (float)nq + eps ) : 1.0f;
+  const float ik = k_norm != nullptr ? 1.0f / sqrtf( ssk / (float)nk + eps ) : 1.0f;
+  E* q = q_out + row * s.heads * s.dpad;
+  for ( uint32_t c = threadIdx.x; c < s.heads * s.dpad; c += blockDim.x ) {
+    const uint32_t h = c / s.dpad, e = c % s.dpad, src = h * s.dim + e;
+    q[c] = from_f32<E>( e < s.dim ? vals[src] * iq * ( q_norm != nullptr ? to_f32( q_norm[src] ) : 1.0f ) : 0.0f );
+  }
+  for ( uint32_t c = threadIdx.x; c < s.k_elems(); c += blockDim.x ) {
+    const uint32_t h = c / s.dpad, e = c % s.dpad, src = h * s.dim + e;
+    cache[c] = from_f32<E>( e < s.dim ? vals[nq + src] * ik * ( k_norm != nullptr ? to_f32( k_norm[src] ) : 1.0f ) : 0.0f );
+  }
+  for ( uint32_t c = threadIdx.x; c < s.kv_heads * s.vpad; c += blockDim.x ) {
+    const uint32_t h = c / s.vpad, e = c % s.vpad, src = nq + nk + h * s.vdim + e;
+    cache[s.k_elems() + c] = from_f32<E>( e < s.vdim ? y.at( row, src ) + ( bias != nullptr ? to_f32( bias[src] ) : 0.0f ) : 0.0f );
+  }
+  (void)nv;
+}
+
+// ---- visible keys ------------------------------------------------------------------------------
+struct Visible
+{
+  uint32_t kept, first, count; // kept keys in front of the window, first key of the window, all of them
+  __device__ __forceinline__ uint32_t key( uint32_t idx ) const { return idx < kept ? idx : first + ( idx - kept ); }
+};
+__device__ __forceinline__ Visible visible_keys( uint32_t pos, const WindowShape& s )
+{
+  Visible v;
+  v.first = pos + 1 > s.window ? pos + 1 - s.window : 0;
+  v.kept = min( s.keep_first, v.first );
+  v.count = v.kept + ( pos + 1 - v.first );
+  return v;
+}
+
+template<typename E>
+__device__ __forceinline__ void load8( float out[8], const E* p )
+{
+  if constexpr ( sizeof( E ) == 2 ) {
+    union
+    {
+      uint4 raw;
+      E e[8];
+    } u;
+    u.raw = *reinterpret_cast<const uint4*>( p );
+#pragma unroll
+    for ( int i = 0; i < 8; i++ ) {
+      out[i] = to_f32( u.e[i] );
+    }
+  } else {
+    const float4 a = *reinterpret_cast<const float4*>( p ), b = *reinterpret_cast<const float4*>( p + 4 );
+    out[0] = a.x, out[1] = a.y, out[2] = a.z, out[3] = a.w, out[4] = b.x, out[5] = b.y, out[6] = b.z, out[7] = b.w;
+  }
+}
+
+constexpr float NO_KEY = -1e30f; // running maximum before the first key: exp(NO_KEY - anything real) is 0
+
+// partial result of one split of one (row, head): vpad weighted sums, then the sum of the weights and the maximum
+__host__ __device__ inline uint64_t partial_stride( const WindowShape& s ) { return s.vpad + 2; }
+
+// HQ query heads at a time; NC pieces of 128 elements per head (a lane holds 8 of each)
+template<typename E, int HQ, int NC>
+__global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out,
+                                                             float* __restrict__ partial,
+                                                             const E* __restrict__ q,
+                                                             const float* __restrict__ bias,
+                                                             WindowRows wr,
+                                                             WindowShape s,
+                                                             uint32_t keys_per_split,
+                                                             uint32_t splits )
+{
+  extern __shared__ float lds[]; // 4 waves x HQ x (vpad + 2)
+  const uint32_t head_blocks = ( s.group + HQ - 1 ) / HQ;
+  const uint32_t g = blockIdx.y / head_blocks, hb = blockIdx.y % head_blocks;
+  const uint64_t row = blockIdx.x;
+  const uint32_t split = blockIdx.z;
+  const uint32_t ctx = (uint32_t)( row / wr.n_tokens ), tok = (uint32_t)( row % wr.n_tokens );
+  const uint8_t* base = static_cast<const uint8_t*>( wr.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  const uint32_t pos = wr.start_pos[ctx] + tok;
+  const Visible vis = visible_keys( pos, s );
+  const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, l16 = lane & 15, g4 = lane >> 4;
+  const uint32_t h0 = g * s.group + hb * HQ;
+  const uint32_t nh = min( (uint32_t)HQ, s.group - hb * HQ );
+  const E* cache = reinterpret_cast<const E*>( base + wr.offset );
+  const uint32_t k_begin = split * keys_per_split, k_end = min( vis.count, k_begin + keys_per_split );
+
+  float qv[HQ][NC][8], acc[HQ][NC][8], mx[HQ], sum[HQ];
+#pragma unroll
+  for ( int h = 0; h < HQ; h++ ) {
+    mx[h] = NO_KEY;
+    sum[h] = 0.0f;
+#pragma unroll
+    for ( int c = 0; c < NC; c++ ) {
+#pragma unroll
+      for ( int e = 0; e < 8; e++ ) {
+        qv[h][c][e] = 0.0f;
+        acc[h][c][e] = 0.0f;
+      }
+      const uint32_t at = c * 128 + l16 * 8;
+      if ( (uint32_t)h < nh && at < s.dpad ) {
+        load8( qv[h][c], q + ( row * s.heads + h0 + h ) * s.dpad + at );
+      }
+    }
+  }
+  for ( uint32_t i0 = k_begin + wave * 4; i0 < k_end; i0 += 16 ) {
+    const uint32_t idx = i0 + g4;
+    const bool live = idx < k_end;
+    const uint32_t j = vis.key( live ? idx : i0 );
+    const E* kr = cache + (uint64_t)j * s.row_elems() + g * s.dpad;
+    const E* vr = cache + (uint64_t)j * s.row_elems() + s.k_elems() + g * s.vpad;
+    float kv[NC][8], vv[NC][8];
+#pragma unroll
+    for ( int c = 0; c < NC; c++ ) {
+      const uint32_t at = c * 128 + l16 * 8;
+#pragma unroll
+      for ( int e = 0; e < 8; e++ ) {
+        kv[c][e] = 0.0f;
+        vv[c][e] = 0.0f;
+      }
+      if ( at < s.dpad ) {
+        load8( kv[c], kr + at );
+      }
+      if ( at < s.vpad ) {
+        load8( vv[c], vr + at );
+      }
+    }
+    const uint32_t dist = min( pos - j, s.n_dist - 1 );
+#pragma unroll
+    for ( int h = 0; h < HQ; h++ ) {
+      float dot = 0.0f;
+#pragma unroll
+      for ( int c = 0; c < NC; c++ ) {
+#pragma unroll
+        for ( int e = 0; e < 8; e++ ) {
+          dot += qv[h][c][e] * kv[c][e];
+        }
+      }
+      dot = row16_sum( dot );
+      const float b = bias != nullptr && (uint32_t)h < nh ? bias[(uint64_t)( h0 + h ) * s.n_dist + dist] : 0.0f;
+      const float score = live ? dot * s.scale + b : NO_KEY;
+      const float m_new = fmaxf( mx[h], score );
+      const float old = __expf( mx[h] - m_new );
+      const float p = live ? __expf( score - m_new ) : 0.0f;
+      mx[h] = m_new;
+      sum[h] = sum[h] * old + p;
+#pragma unroll
+      for ( int c = 0; c < NC; c++ ) {
+#pragma unroll
+        for ( int e = 0; e < 8; e++ ) {
+          acc[h][c][e] = acc[h][c][e] * old + p * vv[c][e];
+        }
+      }
+    }
+  }
+  // the four 16-lane groups of the wave, then the four waves
+  const uint32_t stride = s.vpad + 2;
+#pragma unroll
+  for ( int h = 0; h < HQ; h++ ) {
+    float m = fmaxf( mx[h], __shfl_xor( mx[h], 16 ) );
+    m = fmaxf( m, __shfl_xor( m, 32 ) );
+    const float f = __expf( mx[h] - m );
+    float sm = sum[h] * f;
+    sm += __shfl_xor( sm, 16 );
+    sm += __shfl_xor( sm, 32 );
+    float* mine = lds + ( wave * HQ + h ) * stride;
+#pragma unroll
+    for ( int c = 0; c < NC; c++ ) {
+      const uint32_t at = c * 128 + l16 * 8;
+#pragma unroll
+      for ( int e = 0; e < 8; e++ ) {
+        float a = acc[h][c][e] * f;
+        a += __shfl_xor( a, 16 );
+        a += __shfl_xor( a, 32 );
+        if ( g4 == 0 && at + e < s.vpad ) {
+          mine[at + e] = a;
+        }
+      }
+    }
+    if ( lane == 0 ) {
+      mine[s.vpad] = sm;
+      mine[s.vpad + 1] = m;
+    }
+  }
+  __syncthreads();
+  for ( uint32_t i = threadIdx.x; i < nh * s.vpad; i += 256 ) {
+    const uint32_t h = i / s.vpad, e = i % s.vpad;
+    float m = NO_KEY;
+#pragma unroll
+    for ( int w = 0; w < 4; w++ ) {
+      m = fmaxf( m, lds[( w * HQ + h ) * stride + s.vpad + 1] );
+    }
+    float a = 0.0f, sm = 0.0f;
+#pragma unroll
+    for ( int w = 0; w < 4; w++ ) {
+      const float* src = lds + ( w * HQ + h ) * stride;
+      const float f = __expf( src[s.vpad + 1] - m );
+      a += src[e] * f;
+      sm += src[s.vpad] * f;
+    }
+    if ( splits == 1 ) {
+      if ( e < s.vdim ) {
+        out[( row * s.heads + h0 + h ) * s.vdim + e] = from_f32<E>( a / sm );
+      }
+    } else {
+      float* dst = partial + ( ( row * s.heads + h0 + h ) * splits + split ) * stride;
+      dst[e] = a;
+      if ( e == 0 ) {
+        dst[s.vpad] = sm;
+        dst[s.vpad + 1] = m;
+      }
+    }
+  }
+}
+
+// one wave per (row, head)
+template<typename E>
+__global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ out, const float* __restrict__ partial, WindowRows wr, WindowShape s, uint32_t splits,
+                                                              uint64_t pairs )
+{
+  const uint64_t pair = (uint64_t)blockIdx.x * 4 + ( threadIdx.x >> 6 );
+  if ( pair >= pairs || wr.rows[pair / s.heads / wr.n_tokens] == nullptr ) {
+    return;
+  }
+  const uint32_t lane = threadIdx.x & 63, stride = s.vpad + 2;
+  const float* src = partial + pair * splits * stride;
+  float m = NO_KEY;
+  for ( uint32_t k = 0; k < splits; k++ ) {
+    m = fmaxf( m, src[k * stride + s.vpad + 1] );
+  }
+  float sm = 0.0f;
+  for ( uint32_t k = 0; k < splits; k++ ) {
+    sm += src[k * stride + s.vpad] * __expf( src[k * stride + s.vpad + 1] - m );
+  }
+  for ( uint32_t e = lane; e < s.vdim; e += 64 ) {
+    float a = 0.0f;
+    for ( uint32_t k = 0; k < splits; k++ ) {
+      a += src[k * stride + e] * __expf( src[k * stride + s.vpad + 1] - m );
+    }
+    out[pair * s.vdim + e] = from_f32<E>( a / sm );
+  }
+}
+
+WindowShape shape_of( const gh_window_attn* a )
+{
+  WindowShape s;
+  s.heads = a->heads;
+  s.kv_heads = a->kv_heads;
+  s.group = a->kv_heads ? a->heads / a->kv_heads : 0;
+  s.dim = a->dim;
+  s.vdim = a->vdim;
+  s.dpad = ( a->dim + 7 ) / 8 * 8;
+  s.vpad = ( a->vdim + 7 ) / 8 * 8;
+  s.window = a->window ? a->window : 0xffffffffu;
+  s.keep_first = a->keep_first;
+  s.n_dist = a->n_dist ? a->n_dist : 1;
+  s.scale = a->scale;
+  return s;
+}
+
+bool shape_ok( const gh_window_attn* a )
+{
+  return a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0 && a->dim <= 512 && a->vdim <= 512 && a->heads <= 4096;
+}
+
+template<typename E, int NC>
+void launch_rows( int hq, dim3 grid, hipStream_t st, E* out, float* partial, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s,
+                  uint32_t keys_per_split, uint32_t splits )
+{
+  const size_t lds = 4ull * hq * ( s.vpad + 2 ) * sizeof( float );
+  if constexpr ( NC <= 1 ) {
+    if ( hq == 8 ) {
+      window_rows_kernel<E, 8, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      return;
+    }
+  }
+  if constexpr ( NC <= 2 ) {
+    if ( hq == 4 ) {
+      window_rows_kernel<E, 4, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      return;
+    }
+    if ( hq == 2 ) {
+      window_rows_kernel<E, 2, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      return;
+    }
+  }
+  window_rows_kernel<E, 1, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+}
+
+template<typename E>
+int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
+{
+  const uint32_t widest = std::max( s.dpad, s.vpad );
+  const int max_hq = widest <= 128 ? 8 : widest <= 256 ? 4 : 1;
+  int hq = 1;
+  while ( hq < max_hq && hq < (int)s.group ) {
+    hq *= 2;
+  }
+  const uint32_t head_blocks = s.kv_heads * ( ( s.group + hq - 1 ) / hq );
+  GH_REQUIRE( head_blocks <= 65535, "gh_attn_window: too many heads" );
+  // the most keys any row of the call sees, and as many splits as give every CU a few work-groups of at least 64 keys
+  const uint64_t most = std::min<uint64_t>( (uint64_t)max_pos + 1, (uint64_t)s.window + s.keep_first );
+  const uint64_t groups = rows * head_blocks;
+  uint64_t splits = std::max<uint64_t>( 1, 2ull * cu_count() / std::max<uint64_t>( 1, groups ) );
+  splits = std::min( { splits, std::max<uint64_t>( 1, most / 64 ), (uint64_t)64 } );
+  const uint32_t per = (uint32_t)( ( ( most + splits - 1 ) / splits + 15 ) / 16 * 16 );
+  splits = ( most + per - 1 ) / per;
+  float* partial = nullptr;
+  if ( splits > 1 ) {
+    void* p = nullptr;
+    if ( int rc = stream_scratch( st, SCRATCH_MIXER, rows * s.heads * splits * partial_stride( s ) * sizeof( float ), 1ull << 20, &p ) ) {
+      return rc;
+    }
+    partial = static_cast<float*>( p );
+  }
+  const dim3 grid( (unsigned)rows, head_blocks, (unsigned)splits );
+  if ( widest <= 128 ) {
+    launch_rows<E, 1>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+  } else if ( widest <= 256 ) {
+    launch_rows<E, 2>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+  } else {
+    launch_rows<E, 4>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+  }
+  GH_LAUNCH_CHECK();
+  if ( splits > 1 ) {
+    const uint64_t pairs = rows * s.heads;
+    window_merge_kernel<E><<<(unsigned)( ( pairs + 3 ) / 4 ), 256, 0, st>>>( out, partial, wr, s, (uint32_t)splits, pairs );
+    GH_LAUNCH_CHECK();
+  }
+  return GH_OK;
+}
+
+} // namespace
+} // namespace gh
+
+using namespace gh;
+
+extern "C" {
+
+uint64_t gh_window_row_bytes( const gh_window_attn* a, gh_dtype dt ) { return (uint64_t)shape_of( a ).row_elems() * dtype_size( dt ); }
+
+uint64_t gh_window_query_elements( const gh_window_attn* a ) { return (uint64_t)a->heads * shape_of( a ).dpad; }
+
+int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const void* bias, uint64_t width, const gh_window_attn* a, const void* q_norm,
+                             const void* k_norm, float eps, void* const* context_rows_dev, uint64_t cache_offset, const uint32_t* start_pos_dev, uint64_t batch,
+                             uint32_t n_tokens, gh_dtype dt, gh_stream stream )
+{
+  if ( int rc = ensure_init() ) {
+    return rc;
+  }
+  const uint64_t rows = batch * n_tokens;
+  if ( rows == 0 ) {
+    return GH_OK;
+  }
+  GH_REQUIRE( q && x && wqkv && a && context_rows_dev && start_pos_dev, "gh_matmul_window_append: NULL pointer" );
+  GH_REQUIRE( dt == GH_BF16 || dt == GH_F32, "gh_matmul_window_append: unsupported dtype %d", (int)dt );
+  GH_REQUIRE( shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_matmul_window_append: bad shape" );
+  const WindowShape s = shape_of( a );
+  const uint64_t r = (uint64_t)s.heads * s.dim + (uint64_t)s.kv_heads * ( s.dim + s.vdim );
+  const size_t lds = ( (uint64_t)s.heads + s.kv_heads ) * s.dim * sizeof( float );
+  GH_REQUIRE( lds <= 63 * 1024, "gh_matmul_window_append: query and key of a token do not fit in LDS" );
+  hipStream_t st = as_stream( stream );
+  Product y;
+  if ( int rc = make_product( x, wqkv, width, r, rows, dt, false, st, &y ) ) {
+    return rc;
+  }
+  const WindowRows wr { context_rows_dev, cache_offset, start_pos_dev, n_tokens };
+  return with_product( dt, y, [&]( auto tag, auto view ) -> int {
+    using E = decltype( tag );
+    window_append_kernel<E><<<(unsigned)rows, 256, lds, st>>>( static_cast<E*>( q ), view, static_cast<const E*>( bias ), static_cast<const E*>( q_norm ),
+                                                              static_cast<const E*>( k_norm ), wr, s, eps );
+    GH_LAUNCH_CHECK();
+    return GH_OK;
+  } );
+}
+
+int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const float* distance_bias_dev, void* const* context_rows_dev, uint64_t cache_offset,
+                    const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, uint32_t max_start_pos, gh_dtype dt, gh_stream stream )
+{
+  if ( int rc = ensure_init() ) {
+    return rc;
+  }
+  const uint64_t rows = batch * n_tokens;
+  if ( rows == 0 ) {
+    return GH_OK;
+  }
+  GH_REQUIRE( out && q && a && context_rows_dev && start_pos_dev, "gh_attn_window: NULL pointer" );
+  GH_REQUIRE( dt == GH_BF16 || dt == GH_F32, "gh_attn_window: unsupported dtype %d", (int)dt );
+  GH_REQUIRE( shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_attn_window: bad shape" );
+  const WindowShape s = shape_of( a );
+  const WindowRows wr { context_rows_dev, cache_offset, start_pos_dev, n_tokens };
+  const uint32_t max_pos = max_start_pos + n_tokens - 1;
+  if ( dt == GH_F32 ) {
+    return attend_rows<float>( static_cast<float*>( out ), static_cast<const float*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+  }
+  return attend_rows<__bf16>( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+}
+
+} // extern "C"

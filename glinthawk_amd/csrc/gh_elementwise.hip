@@ -319,6 +319,17 @@ using namespace gh;
     }                                                                                                                  \
   } while ( 0 )
 
+// fills also serve the bf16 buffers of the run-time sized designs
+#define GH_DISPATCH_FILL( dt, ... )                                                                                    \
+  do {                                                                                                                 \
+    if ( ( dt ) == GH_BF16 ) {                                                                                         \
+      using T = __bf16;                                                                                                \
+      __VA_ARGS__;                                                                                                     \
+    } else {                                                                                                           \
+      GH_DISPATCH_DT( dt, __VA_ARGS__ );                                                                               \
+    }                                                                                                                  \
+  } while ( 0 )
+
 extern "C" {
 
 int gh_accum( void* a, const void* b, uint64_t size, uint64_t batch, gh_dtype dt, gh_stream stream )
@@ -429,7 +440,7 @@ int gh_fill_uniform( void* dst, uint64_t n, float lo, float hi, uint64_t seed, g
     return GH_OK;
   }
   GH_REQUIRE( dst, "gh_fill_uniform: NULL pointer" );
-  GH_DISPATCH_DT( dt, fill_uniform_kernel<T><<<blocks_for( n / 4 + 1, EW_THREADS, 16384 ), EW_THREADS, 0, as_stream( stream )>>>(
+  GH_DISPATCH_FILL( dt, fill_uniform_kernel<T><<<blocks_for( n / 4 + 1, EW_THREADS, 16384 ), EW_THREADS, 0, as_stream( stream )>>>(
                         static_cast<T*>( dst ), n, lo, hi, seed ) );
   GH_LAUNCH_CHECK();
   return GH_OK;
@@ -444,7 +455,7 @@ int gh_fill_normal( void* dst, uint64_t n, float mean, float std, uint64_t seed,
     return GH_OK;
   }
   GH_REQUIRE( dst, "gh_fill_normal: NULL pointer" );
-  GH_DISPATCH_DT( dt, fill_normal_kernel<T><<<blocks_for( n / 4 + 1, EW_THREADS, 16384 ), EW_THREADS, 0, as_stream( stream )>>>(
+  GH_DISPATCH_FILL( dt, fill_normal_kernel<T><<<blocks_for( n / 4 + 1, EW_THREADS, 16384 ), EW_THREADS, 0, as_stream( stream )>>>(
                         static_cast<T*>( dst ), n, mean, std, seed ) );
   GH_LAUNCH_CHECK();
   return GH_OK;

@@ -128,8 +128,10 @@ static int init_locked( int device )
   if ( int rc = check_buffer_bounds() ) {
     return rc;
   }
-  if ( int rc = attn_static_scratch_init( device ) ) {
-    return rc;
+  if ( attn_static_scratch_init != nullptr ) {
+    if ( int rc = attn_static_scratch_init( device ) ) {
+      return rc;
+    }
   }
   for ( int i = 0; i < STAGE_SLOTS; i++ ) {
     GH_HIP( hipHostMalloc( reinterpret_cast<void**>( &g_slots[i].pinned ), STAGE_SLOT_BYTES, hipHostMallocDefault ) );

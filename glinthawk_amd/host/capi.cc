@@ -10,84 +10,29 @@
 #include <vector>
 
 #include "glint/contextman.hh"
+#include "glint/designs.hh"
 #include "glint/kernel.hh"
 #include "glint/loader.hh"
 #include "glint/model.hh"
+#include "glint/stage.hh"
 
 using namespace glint;
 
 namespace {
 
 // ---------------------------------------------------------------------------------------------
-// type-erased stage harness
+// stage harness of the Llama2 shapes
 // ---------------------------------------------------------------------------------------------
-struct StageBase
-{
-  virtual ~StageBase() = default;
-  virtual void set_layer_tensor( size_t layer, size_t k, const void* host, uint64_t n ) = 0;
-  virtual void set_base_tensor( size_t k, const void* host, uint64_t n ) = 0;
-  virtual const void* layer_tensor_ptr( size_t layer, size_t k, uint64_t* n ) = 0;
-  virtual const void* base_tensor_ptr( size_t k, uint64_t* n ) = 0;
-  virtual std::string load_dir( const char* model_dir ) = 0;
-  virtual std::string set_state_bytes( const void* bytes, uint64_t len ) = 0;
-  virtual std::string get_state_bytes() = 0;
-  virtual void new_state( uint32_t batch, uint32_t next_layer, int next_stage ) = 0;
-  virtual void set_prompt( size_t i, uint32_t context_id, uint32_t token, uint32_t pos, float temp, uint32_t plen, uint32_t mcl ) = 0;
-  virtual void discard( size_t i ) = 0;
-  virtual void set_next( uint32_t layer, int stage ) = 0;
-  virtual int acquire_contexts() = 0;
-  virtual int forward( int which ) = 0;
-  virtual void* buffer( int which, uint64_t* bytes, bool allocate ) = 0;
-  virtual void row_info( size_t i, uint32_t out[6] ) = 0;
-  virtual void state_info( uint32_t out[4] ) = 0;
-  virtual void* context_layer_ptr( size_t row, size_t layer ) = 0;
-  virtual int32_t context_slot( size_t row ) = 0;
-  virtual void slot_counts( uint64_t out[3] ) = 0;
-  virtual void* scratch( int which ) = 0;
-  virtual int release_context( uint32_t id ) = 0;
-  virtual void paging_info( size_t row, size_t layer, uint64_t out[3] ) = 0;
-  virtual void sync() = 0;
-  virtual void copy_bytes( void* dst, const void* src, uint64_t bytes, int kind ) = 0;
-  virtual void time_device_spans( bool on ) = 0;
-  virtual void device_spans( double* ms, uint64_t* spans ) = 0;
-  virtual int prefill( uint32_t batch, const uint32_t* context_ids, const uint32_t* start_pos, uint32_t n_tokens, uint32_t first_layer,
-                       const uint32_t* token_ids, const void* acts_in, void* acts_out, uint32_t* next_tokens ) = 0;
-};
-
 template<typename Config, typename DType, typename Ctx>
-struct StageImpl : StageBase
+struct StageImpl : StageOf<Llama2<Config, DType, hip::LlamaOperations<Config, DType, Ctx>, Ctx>>
 {
-  using Model = Llama2<Config, DType, hip::LlamaOperations<Config, DType, Ctx>, Ctx>;
-  using State = typename Model::StateType;
+  using Base = StageOf<Llama2<Config, DType, hip::LlamaOperations<Config, DType, Ctx>, Ctx>>;
+  using Base::Base;
+  using Base::held;
+  using Base::model;
+  using Base::state;
 
-  Model model;
-  PreallocatingContextManager<Model> contexts;
-  State state {};
-  typename Model::ContextVector held {};
-
-  StageImpl( const StageSettings<Config>& s, const ModelOptions& o )
-    : model( s, o )
-    , contexts( s )
-  {
-  }
   std::string load_dir( const char* model_dir ) override { return load_model_dir( model, model_dir ); }
-  // a state as it arrives from / leaves for the neighbouring stage (models/common/state.hh:512-594)
-  std::string set_state_bytes( const void* bytes, uint64_t len ) override
-  {
-    std::string why;
-    State parsed;
-    if ( !State::parse( std::string_view( static_cast<const char*>( bytes ), len ), parsed, &why ) ) {
-      return why;
-    }
-    if ( parsed.dtype() != dtype_of<DType>() && parsed.next_stage() != InferenceStage::Attention ) {
-      return "state data type does not match the stage";
-    }
-    state = std::move( parsed );
-    held.clear();
-    return {};
-  }
-  std::string get_state_bytes() override { return state.serialize(); }
-
   void set_layer_tensor( size_t layer, size_t k, const void* host, uint64_t n ) override
   {
     model.set_layer_tensor( layer, k, static_cast<const DType*>( host ), n );
@@ -115,44 +60,11 @@ struct StageImpl : StageBase
     return t[k];
   }
 
-  void new_state( uint32_t batch, uint32_t next_layer, int next_stage ) override
-  {
-    state = State( batch, dtype_of<DType>() );
-    state.set_next_layer( next_layer );
-    state.set_next_stage( static_cast<InferenceStage>( next_stage ) );
-    held.clear();
-  }
-  void set_prompt( size_t i, uint32_t context_id, uint32_t token, uint32_t pos, float temp, uint32_t plen, uint32_t mcl ) override
-  {
-    GLINT_CHECK( i < state.batch_size() );
-    state.set_prompt( i, context_id, token, pos, temp, plen, mcl );
-  }
-  void discard( size_t i ) override
-  {
-    GLINT_CHECK( i < state.batch_size() );
-    state.discard( i );
-  }
-  void set_next( uint32_t layer, int stage ) override
-  {
-    state.set_next_layer( layer );
-    state.set_next_stage( static_cast<InferenceStage>( stage ) );
-  }
-
-  int acquire_contexts() override
-  {
-    auto got = contexts.get_contexts( state );
-    if ( !got.has_value() ) {
-      return -1; // not enough free slots: nothing was allocated
-    }
-    held = std::move( *got );
-    return 0;
-  }
-
   // which: 0 forward (all hosted stages), 1 pre-attention, 2 attention, 3 post-attention, 4 classify
   int forward( int which ) override
   {
     if ( which == 0 || which == 2 ) {
-      if ( acquire_contexts() != 0 ) {
+      if ( this->acquire_contexts() != 0 ) {
         return -1;
       }
     }
@@ -184,33 +96,7 @@ struct StageImpl : StageBase
     return b->data();
   }
 
-  void row_info( size_t i, uint32_t out[6] ) override
-  {
-    out[0] = state.active( i );
-    out[1] = state.context_id( i );
-    out[2] = state.token( i );
-    out[3] = state.token_pos( i );
-    out[4] = state.finished( i );
-    out[5] = static_cast<uint32_t>( state.temperature( i ) * 255.0f + 0.5f );
-  }
-  void state_info( uint32_t out[4] ) override
-  {
-    out[0] = state.batch_size();
-    out[1] = state.next_layer();
-    out[2] = static_cast<uint32_t>( state.next_stage() );
-    out[3] = ( state.has_activations() ? 1u : 0u ) | ( state.has_queries() ? 2u : 0u ) | ( state.has_kvs() ? 4u : 0u );
-  }
-
   void* context_layer_ptr( size_t row, size_t layer ) override { return row < held.size() ? held[row]->layer( layer ).data() : nullptr; }
-  int32_t context_slot( size_t row ) override { return row < held.size() ? contexts.slot_index( held[row] ) : -2; }
-  void slot_counts( uint64_t out[3] ) override
-  {
-    out[0] = contexts.free();
-    out[1] = contexts.allocated();
-    out[2] = contexts.total();
-  }
-  int release_context( uint32_t id ) override { return contexts.release_context( id ) ? 1 : 0; }
-
   void paging_info( size_t row, size_t layer, uint64_t out[3] ) override
   {
     out[0] = out[1] = out[2] = 0;
@@ -234,32 +120,17 @@ struct StageImpl : StageBase
       default: return model.scratch_logits();
     }
   }
-  void sync() override { model.ops().synchronize(); }
   // the instantiation the reference's concept names: convert_and_copy<void, void>, a copy of `bytes` bytes
   void copy_bytes( void* dst, const void* src, uint64_t bytes, int kind ) override
   {
     model.ops().template convert_and_copy<void, void>( dst, src, bytes, static_cast<CopyType>( kind ) );
   }
-  void time_device_spans( bool on ) override { model.time_device_spans( on ); }
-  void device_spans( double* ms, uint64_t* spans ) override
-  {
-    const auto [total, n] = model.device_spans();
-    *ms = total;
-    *spans = n;
-  }
-
   int prefill( uint32_t batch, const uint32_t* context_ids, const uint32_t* start_pos, uint32_t n_tokens, uint32_t first_layer, const uint32_t* token_ids,
                const void* acts_in, void* acts_out, uint32_t* next_tokens ) override
   {
-    State tmp( batch, dtype_of<DType>() );
-    for ( uint32_t i = 0; i < batch; i++ ) {
-      tmp.set_prompt( i, context_ids[i], 0, start_pos[i], 0.0f, n_tokens, 0 );
-    }
-    auto got = contexts.get_contexts( tmp );
-    if ( !got.has_value() ) {
+    if ( this->hold( batch, context_ids, start_pos, n_tokens ) != 0 ) {
       return -1;
     }
-    held = std::move( *got );
     model.prefill( held, start_pos, n_tokens, first_layer, token_ids, static_cast<const DType*>( acts_in ), static_cast<DType*>( acts_out ), next_tokens );
     return 0;
   }
@@ -351,6 +222,19 @@ struct BookManager
 
 using PagedBookContext = glint::DynamicContext<BookConfig, float16_t, CountingRegion>;
 
+DesignOptions design_options( int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+{
+  DesignOptions o;
+  o.dtype = dtype == 1 ? DataType::Float32 : dtype == 2 ? DataType::BFloat16 : DataType::Float16;
+  o.paged = flags & 4u;
+  o.concurrency_limit = concurrency;
+  o.max_context_count = max_contexts;
+  o.model.seed = seed;
+  o.model.weight_std = weight_std;
+  o.model.randomize = flags & 64u;
+  return o;
+}
+
 thread_local std::string g_last_error;
 thread_local std::string g_bytes; // result of the last call that returns bytes
 
@@ -413,6 +297,8 @@ struct KernelImpl : KernelBase
   {
     if constexpr ( requires( Model& m ) { m.base_weights(); } ) {
       return load_model_dir( kernel.model(), dir );
+    } else if constexpr ( requires( Model& m ) { m.load( dir ); } ) {
+      return kernel.model().load( dir );
     } else {
       return KernelBase::load_dir( dir );
     }
@@ -484,6 +370,29 @@ void* glint_stage_create( const char* config, int dtype, uint32_t first_layer, u
 #undef GLINT_CASE
   return nullptr;
 }
+
+// A stage over the model in a directory: a run-time sized design named by config.json, weights loaded (flags & 64: drawn, only
+// config.json is read).  dtype 1 f32, 2 bf16; flags & 4 paged contexts.  NULL on failure, see glint_last_error().
+void* glint_stage_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+{
+  return open_design_stage( model_dir, design_options( dtype, concurrency, max_contexts, flags, seed, weight_std ), g_last_error ).release();
+}
+// what: 0 vocabulary, 1 positions, 2 layer runs of one step (0 for models that do not say)
+uint64_t glint_stage_size( void* h, int what )
+{
+  auto* s = static_cast<StageBase*>( h );
+  return what == 0 ? s->vocab_size() : what == 1 ? s->max_positions() : s->layer_runs();
+}
+// prefill with the logits (n_want, vocab) of the rows in `want`; next_tokens (batch) and residuals_out (layer runs, rows, width) may be
+// NULL.  0, or -1 no context space, -2 not offered by this model, -3 positions the contexts cannot take
+int glint_stage_prefill_logits( void* h, uint32_t batch, const uint32_t* context_ids, const uint32_t* start_pos, uint32_t n_tokens, const uint32_t* token_ids,
+                                const uint32_t* want, uint32_t n_want, float* logits_out, uint32_t* next_tokens, float* residuals_out )
+{
+  return static_cast<StageBase*>( h )->prefill_logits( batch, context_ids, start_pos, n_tokens, token_ids, std::vector<uint32_t>( want, want + n_want ), logits_out,
+                                                       next_tokens, residuals_out );
+}
+// logits (rows, vocab) of the last forward
+int glint_stage_logits( void* h, float* out, uint32_t rows ) { return static_cast<StageBase*>( h )->copy_logits( out, rows ); }
 
 void glint_stage_destroy( void* h ) { delete static_cast<StageBase*>( h ); }
 
@@ -791,6 +700,24 @@ void* glint_kernel_create( const char* config, int dtype, uint32_t first_layer, 
   GLINT_CASE( "test-tiny", Test_Tiny )
 #undef GLINT_CASE
   return nullptr;
+}
+// the compute kernel around the design in a model directory, arguments as glint_stage_open
+void* glint_kernel_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+{
+  KernelBase* kernel = nullptr;
+  const DesignOptions o = design_options( dtype, concurrency, max_contexts, flags, seed, weight_std );
+  g_last_error = with_design( model_dir, o, [&]( auto tag, const auto& config, const auto& settings, const ModelOptions& options ) -> std::string {
+    using Model = typename decltype( tag )::type;
+    auto made = std::make_unique<KernelImpl<Model>>( config, settings, options );
+    if ( !settings.randomize_parameters ) {
+      if ( auto err = made->kernel.model().load( model_dir ); !err.empty() ) {
+        return err;
+      }
+    }
+    kernel = made.release();
+    return {};
+  } );
+  return kernel;
 }
 // host-only kernel around a model that just advances tokens (shape of "test-tiny")
 void* glint_kernel_create_echo( uint32_t concurrency, uint32_t max_contexts )

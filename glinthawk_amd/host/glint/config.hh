@@ -43,6 +43,27 @@ concept ModelConfig = requires {
   requires T::head_size == T::dim / T::n_heads;
 };
 
+// A design whose sizes come from a model directory instead of a type: a tag with `sized_at_run_time`.  Such a model is hosted whole, so
+// its batched states carry prompts only, and where a sequence ends for lack of positions is the model driver's business.
+template<class T>
+concept RunTimeModelConfig = requires { requires T::sized_at_run_time; };
+
+// what a batched state needs to know of its model: the row widths of its buffers, and when a token ends a text
+template<class T>
+struct StateTraits;
+template<ModelConfig T>
+struct StateTraits<T>
+{
+  constexpr static uint64_t dim = T::dim, kv_dim = T::kv_dim, seq_len = T::seq_len;
+  static bool ends_text( const uint32_t token ) { return token == T::token_eos || token == T::token_eot; }
+};
+template<RunTimeModelConfig T>
+struct StateTraits<T>
+{
+  constexpr static uint64_t dim = 0, kv_dim = 0, seq_len = UINT64_MAX;
+  static bool ends_text( uint32_t ) { return false; }
+};
+
 namespace configs {
 
 struct Llama2Family

@@ -12,6 +12,7 @@
 
 #include "glint/config.hh"
 #include "glint/context.hh"
+#include "glint/layered_context.hh"
 #include "glint/state.hh"
 #include "glint/types.hh"
 #include "glint_hip.h"
@@ -28,7 +29,7 @@ namespace glint::hip {
 template<typename DType>
 constexpr gh_dtype gh_type()
 {
-  return sizeof( DType ) == 2 ? GH_F16 : GH_F32;
+  return std::is_same_v<DType, bfloat16_t> ? GH_BF16 : sizeof( DType ) == 2 ? GH_F16 : GH_F32;
 }
 
 inline gh_copy_kind gh_kind( const CopyType t )
@@ -243,6 +244,25 @@ public:
 
 template<typename Config, typename DType>
 using DynamicContext = glint::DynamicContext<Config, DType, VirtualMemoryRegion>;
+
+// contexts of the run-time sized designs: one allocation per context, or the paged form of it
+class LayeredContext : public glint::LayeredContext
+{
+  typename Operations<uint8_t>::DeviceUniquePtr storage_ {};
+
+public:
+  explicit LayeredContext( const DesignSettings& settings, const bool make_empty = false )
+  {
+    if ( !make_empty ) {
+      void* p = nullptr;
+      GLINT_GH( gh_malloc( &p, settings.plan->bytes ) );
+      storage_.reset( static_cast<uint8_t*>( p ) );
+      set_base( p );
+    }
+  }
+};
+
+using DynamicLayeredContext = glint::DynamicLayeredContext<VirtualMemoryRegion>;
 
 template<typename Config, typename DType, typename Ctx = Context<Config, DType>>
 requires ModelConfig<Config> && ContextConcept<Ctx, DType>

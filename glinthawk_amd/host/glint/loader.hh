@@ -17,11 +17,6 @@
 // keep just its own slice on disk.  A directory that works for the reference works here.
 #pragma once
 
-#include <fcntl.h>
-#include <sys/mman.h>
-#include <sys/stat.h>
-#include <unistd.h>
-
 #include <array>
 #include <cstdint>
 #include <cstdlib>
@@ -31,6 +26,7 @@
 #include <string>
 
 #include "glint/config.hh"
+#include "glint/mapped_file.hh"
 #include "glint/model.hh"
 #include "glint/types.hh"
 
@@ -101,67 +97,6 @@ constexpr const char* dtype_suffix()
 {
   return sizeof( DType ) == 2 ? "FP16" : "FP32"; // models/types.hh dtype_str
 }
-
-// read-only private mapping of a whole file (util/file_descriptor.hh + MMap_Region in the reference)
-class MappedFile
-{
-public:
-  MappedFile() = default;
-  MappedFile( const MappedFile& ) = delete;
-  MappedFile& operator=( const MappedFile& ) = delete;
-  ~MappedFile() { close(); }
-
-  // empty string on success
-  std::string open( const std::filesystem::path& path, uint64_t expected_bytes )
-  {
-    close();
-    std::error_code ec;
-    const auto size = std::filesystem::file_size( path, ec );
-    if ( ec ) {
-      return "cannot stat " + path.string() + ": " + ec.message();
-    }
-    if ( size != expected_bytes ) {
-      return "file " + path.string() + " is not the expected size (" + std::to_string( size ) + " bytes, " + std::to_string( expected_bytes ) + " expected)";
-    }
-    fd_ = ::open( path.c_str(), O_RDONLY );
-    if ( fd_ < 0 ) {
-      return "cannot open " + path.string() + ": " + std::strerror( errno );
-    }
-    if ( size == 0 ) {
-      return {};
-    }
-    void* p = ::mmap( nullptr, size, PROT_READ, MAP_PRIVATE, fd_, 0 );
-    if ( p == MAP_FAILED ) {
-      const std::string msg = "cannot map " + path.string() + ": " + std::strerror( errno );
-      close();
-      return msg;
-    }
-    addr_ = static_cast<const uint8_t*>( p );
-    len_ = size;
-    return {};
-  }
-
-  void close()
-  {
-    if ( addr_ != nullptr ) {
-      ::munmap( const_cast<uint8_t*>( addr_ ), len_ );
-      addr_ = nullptr;
-      len_ = 0;
-    }
-    if ( fd_ >= 0 ) {
-      ::close( fd_ );
-      fd_ = -1;
-    }
-  }
-
-  [[nodiscard]] const uint8_t* addr() const { return addr_; }
-  [[nodiscard]] uint64_t len() const { return len_; }
-
-private:
-  int fd_ { -1 };
-  const uint8_t* addr_ { nullptr };
-  uint64_t len_ { 0 };
-};
 
 // element offsets of the tensors inside their file (prefix sums of the on-disk sizes, base.hh:385-400,511-530)
 template<size_t N>

@@ -23,11 +23,11 @@
 #include "glint/config.hh"
 #include "glint/context.hh"
 #include "glint/hip/ops.hh"
+#include "glint/model_options.hh"
+#include "glint/span_timer.hh"
 #include "glint/state.hh"
 
 namespace glint {
-
-constexpr size_t MAX_BATCH_SIZE = 1024; // models/llama2/base.hh:26
 
 // element counts of the weight files, in file order (models/llama2/base.hh:357-373,477-499)
 template<typename Config>
@@ -111,17 +111,6 @@ struct LayerWeights
   }
 };
 
-struct ModelOptions
-{
-  bool fused_attention { true };  // false: the reference's three unfused ops + score buffer
-  bool fused_projections { true }; // with fused_attention: projections fused with the ops that follow them
-  int balanced_attention { 0 };   // fused decode attention over equal runs of keys: 0 where the step's lengths call for it, 1 always (shapes that have it), -1 never
-  bool allocate_logits { true };  // only needed when the classifier is hosted
-  uint64_t seed { 1 };            // random initialisation of weights
-  float weight_std { 0.02f };     // N(0, std) for every tensor, as the benchmark configurations say
-  bool randomize { true };        // false: leave the weights for load() / set_*_tensor()
-};
-
 template<typename Config, typename DType, typename LlamaOperations = hip::LlamaOperations<Config, DType>, typename Context = hip::Context<Config, DType>>
 requires ModelConfig<Config>
 class Llama2
@@ -175,25 +164,9 @@ public:
 
   const SettingsType& settings() const { return settings_; }
   LlamaOperations& ops() { return ops_; }
-  // device time of forward() (see SpanTimer): switch it on or off, read the accumulated milliseconds and steps, which a read resets
-  void time_device_spans( const bool on )
-  {
-    if ( on && !span_timer_ ) {
-      span_timer_ = std::make_unique<SpanTimer>();
-    } else if ( !on ) {
-      span_timer_.reset();
-    }
-  }
-  std::pair<double, uint64_t> device_spans()
-  {
-    std::pair<double, uint64_t> out { 0.0, 0 };
-    if ( span_timer_ ) {
-      out = { span_timer_->total_ms, span_timer_->spans };
-      span_timer_->total_ms = 0;
-      span_timer_->spans = 0;
-    }
-    return out;
-  }
+  // device time of forward() (see DeviceSpans): switch it on or off, read the accumulated milliseconds and steps, which a read resets
+  void time_device_spans( const bool on ) { spans_.enable( on ); }
+  std::pair<double, uint64_t> device_spans() { return spans_.take(); }
   const BaseWeights<DType>& base_weights() const { return base_; }
   const LayerWeights<DType>& layer_weights( size_t l ) const { return layers_[l]; }
 
@@ -248,7 +221,7 @@ public:
       upload_tables( contexts, run );
     }
 
-    mark_device_span( 0 ); // the activations and the tables are queued: from here to the copy back it is kernels only
+    spans_.mark( 0, ops_.stream() ); // the activations and the tables are queued: from here to the copy back it is kernels only
     const bool fused_layers = options_.fused_attention && options_.fused_projections;
     if ( fused_layers && !run.empty() ) {
       // the first attention norm stands alone; every later one rides on the epilogue of the previous w2
@@ -275,13 +248,13 @@ public:
 
     if ( last == Config::n_layers - 1 && settings_.hosts( last, InferenceStage::Classification ) ) {
       classify_ops();
-      mark_device_span( 1 );
+      spans_.mark( 1, ops_.stream() );
       postlude( states, last, true );
     } else {
-      mark_device_span( 1 );
+      spans_.mark( 1, ops_.stream() );
       postlude( states, last, false );
     }
-    close_device_span();
+    spans_.close();
   }
 
   // ------------------------------------------------------------------------------------------
@@ -1023,44 +996,6 @@ private:
     CopyLane( const CopyLane& ) = delete;
     CopyLane& operator=( const CopyLane& ) = delete;
   };
-  // Device time of forward(): the span on the stream from the first kernel of a step to its last, without the copies of the
-  // state over the host boundary on either side.  Off by default; two event records per step when on.
-  struct SpanTimer
-  {
-    gh_event mark[2] {};
-    double total_ms { 0 };
-    uint64_t spans { 0 };
-    bool open { false };
-    SpanTimer()
-    {
-      GLINT_GH( gh_event_create_timed( &mark[0] ) );
-      GLINT_GH( gh_event_create_timed( &mark[1] ) );
-    }
-    ~SpanTimer()
-    {
-      (void)gh_event_destroy( mark[0] );
-      (void)gh_event_destroy( mark[1] );
-    }
-    SpanTimer( const SpanTimer& ) = delete;
-    SpanTimer& operator=( const SpanTimer& ) = delete;
-  };
-  void mark_device_span( const int which )
-  {
-    if ( span_timer_ ) {
-      GLINT_GH( gh_event_record( span_timer_->mark[which], ops_.stream() ) );
-      span_timer_->open = which == 1;
-    }
-  }
-  void close_device_span()
-  {
-    if ( span_timer_ && span_timer_->open ) {
-      float ms = 0;
-      GLINT_GH( gh_event_elapsed_ms( span_timer_->mark[0], span_timer_->mark[1], &ms ) );
-      span_timer_->total_ms += ms;
-      span_timer_->spans++;
-      span_timer_->open = false;
-    }
-  }
   void ensure_copy_stream()
   {
     if ( !copy_lane_ ) {
@@ -1074,7 +1009,7 @@ private:
   DevicePtr pf_x_ {}, pf_xb_ {}, pf_q_ {}, pf_hb_ {}, pf_hb2_ {}, pf_xb2_ {}, pf_kv_ {}, pf_tables_ {}, pf_attn_ws_ {};
   uint64_t pf_capacity_ { 0 }, pf_attn_ws_bytes_ { 0 };
   std::unique_ptr<CopyLane> copy_lane_ {};
-  std::unique_ptr<SpanTimer> span_timer_ {};
+  DeviceSpans spans_ {};
   uint64_t attn_ws_bytes_ { 0 };
   DevicePtr attn_bal_ws_ {};
   uint64_t attn_bal_ws_bytes_ { 0 };

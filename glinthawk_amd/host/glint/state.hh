@@ -220,16 +220,18 @@ public:
 };
 
 template<typename Config>
-requires ModelConfig<Config>
+requires ModelConfig<Config> || RunTimeModelConfig<Config>
 class BatchedInferenceState
 {
+  using Traits = StateTraits<Config>;
+
   StateMetadata metadata_ {};
   std::vector<PromptData> prompts_ {};
   DataBuffer activations_ {}, queries_ {}, kvs_ {};
 
-  size_t activation_len() const { return Config::dim * DataTypeSize( metadata_.dtype ); }
-  size_t q_len() const { return Config::dim * DataTypeSize( metadata_.dtype ); }
-  size_t kv_len() const { return 2 * Config::kv_dim * DataTypeSize( metadata_.dtype ); }
+  size_t activation_len() const { return Traits::dim * DataTypeSize( metadata_.dtype ); }
+  size_t q_len() const { return Traits::dim * DataTypeSize( metadata_.dtype ); }
+  size_t kv_len() const { return 2 * Traits::kv_dim * DataTypeSize( metadata_.dtype ); }
 
   // rows [first, first + n) of `from` become rows [at, at + n) of this state's buffers
   void copy_rows( size_t at, const BatchedInferenceState& from, size_t first, size_t n )
@@ -306,8 +308,8 @@ public:
   static size_t wire_size( const StateMetadata& m )
   {
     const size_t elem = DataTypeSize( m.dtype );
-    return sizeof( StateMetadata ) + sizeof( PromptData ) * (size_t)m.batch_size + ( m.has_activations ? (size_t)m.batch_size * Config::dim * elem : 0 )
-           + ( m.has_queries ? (size_t)m.batch_size * Config::dim * elem : 0 ) + ( m.has_kvs ? (size_t)m.batch_size * 2 * Config::kv_dim * elem : 0 );
+    return sizeof( StateMetadata ) + sizeof( PromptData ) * (size_t)m.batch_size + ( m.has_activations ? (size_t)m.batch_size * Traits::dim * elem : 0 )
+           + ( m.has_queries ? (size_t)m.batch_size * Traits::dim * elem : 0 ) + ( m.has_kvs ? (size_t)m.batch_size * 2 * Traits::kv_dim * elem : 0 );
   }
 
   // false (and the reason in *why) unless `bytes` is exactly one serialized state of this model
@@ -490,8 +492,8 @@ public:
   bool check_finished( size_t i ) const
   {
     const PromptData p = prompts_[i];
-    const bool saw_end = p.max_completion_length == 0 && ( p.token == Config::token_eos || p.token == Config::token_eot );
-    const bool out_of_seq = p.token_pos >= Config::seq_len;
+    const bool saw_end = p.max_completion_length == 0 && Traits::ends_text( p.token );
+    const bool out_of_seq = p.token_pos >= Traits::seq_len;
     const bool end_of_gen = p.max_completion_length > 0 && p.token_pos >= p.max_completion_length + p.prompt_length;
     return saw_end || out_of_seq || end_of_gen;
   }

@@ -6,6 +6,7 @@
 #include <cstdint>
 #include <cstdio>
 #include <cstdlib>
+#include <type_traits>
 
 namespace glint {
 
@@ -43,12 +44,13 @@ enum class CopyType
 
 using float16_t = _Float16;
 using float32_t = float;
+using bfloat16_t = __bf16;
 
 template<typename DType>
 constexpr DataType dtype_of()
 {
   static_assert( sizeof( DType ) == 2 || sizeof( DType ) == 4 );
-  return sizeof( DType ) == 2 ? DataType::Float16 : DataType::Float32;
+  return std::is_same_v<DType, bfloat16_t> ? DataType::BFloat16 : sizeof( DType ) == 2 ? DataType::Float16 : DataType::Float32;
 }
 
 // The reference aborts on every failed check on the op path (glog CHECK / LOG(FATAL),

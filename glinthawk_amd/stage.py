@@ -18,6 +18,8 @@ _HOST_LIB_PATH = os.environ.get("GLINT_HOST_LIB") or os.path.join(_PKG, "lib", "
 STAGE_PRE, STAGE_ATT, STAGE_POST, STAGE_CLS = 0, 1, 2, 3
 FWD_ALL, FWD_PRE, FWD_ATT, FWD_POST, FWD_CLS = 0, 1, 2, 3, 4
 FLAG_FUSED, FLAG_CLS, FLAG_PAGED, FLAG_UNFUSED_PROJ, FLAG_BALANCED, FLAG_NOT_BALANCED = 1, 2, 4, 8, 16, 32
+FLAG_RANDOM_WEIGHTS = 64
+DESIGN_DTYPES = {"f32": 1, "bf16": 2}
 
 # layer tensors in file order (rms_att_weight, wq, wkv, wo, rms_ffn_weight, w1, w2, w3)
 LAYER_TENSORS = ("rms_att_weight", "wq", "wkv", "wo", "rms_ffn_weight", "w1", "w2", "w3")
@@ -39,6 +41,10 @@ def host_lib() -> C.CDLL:
         vp, u32, u64, i32 = C.c_void_p, C.c_uint32, C.c_uint64, C.c_int32
         sig = {
             "glint_stage_create": (vp, [C.c_char_p, C.c_int, u32, u32, u32, u32, u32, u64, C.c_float]),
+            "glint_stage_open": (vp, [C.c_char_p, C.c_int, u32, u32, u32, u64, C.c_float]),
+            "glint_stage_size": (u64, [vp, C.c_int]),
+            "glint_stage_prefill_logits": (C.c_int, [vp, u32, vp, vp, u32, vp, vp, u32, vp, vp, vp]),
+            "glint_stage_logits": (C.c_int, [vp, vp, u32]),
             "glint_stage_destroy": (None, [vp]),
             "glint_stage_set_layer_tensor": (None, [vp, u32, u32, vp, u64]),
             "glint_stage_set_base_tensor": (None, [vp, u32, vp, u64]),
@@ -300,6 +306,58 @@ class Stage:
         if rc != 0:
             return None
         return out, nxt
+
+
+class DesignStage(Stage):
+    """A whole model of a run-time sized design, opened from its model directory (config.json names the architecture,
+    model.safetensors holds the weights; random_weights: only config.json is read).  The batched state, the context slots and
+    forward() are Stage's; prefill returns logits."""
+
+    def __init__(self, model_dir: str, dtype: str = "bf16", concurrency: int = 1, max_contexts: int = 1, paged: bool = False,
+                 random_weights: bool = False, seed: int = 1, weight_std: float = 0.02):
+        self.np_dtype = np.float32
+        flags = (FLAG_PAGED if paged else 0) | (FLAG_RANDOM_WEIGHTS if random_weights else 0)
+        self._h = host_lib().glint_stage_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, flags, seed, weight_std)
+        if not self._h:
+            raise GlintError(host_lib().glint_last_error().decode(errors="replace"))
+        self.vocab_size, self.max_positions, self.layer_runs = (int(host_lib().glint_stage_size(self._h, k)) for k in range(3))
+
+    def prefill_logits(self, context_ids, start_pos, token_ids, want=(), want_next_tokens: bool = False, residual_width: int = 0):
+        """token_ids (batch, n_tokens).  Returns (logits (len(want), vocab), next tokens or None, residual stream (layer runs, rows,
+        residual_width) or None); None overall when there is no context space.  `want`: ascending rows, context * n_tokens + token."""
+        toks = np.ascontiguousarray(np.asarray(token_ids, dtype=np.uint32))
+        batch, n_tokens = toks.shape
+        ids = np.ascontiguousarray(np.asarray(context_ids, dtype=np.uint32))
+        start = np.ascontiguousarray(np.asarray(start_pos, dtype=np.uint32))
+        rows = np.ascontiguousarray(np.asarray(want, dtype=np.uint32).reshape(-1))
+        if ids.size != batch or start.size != batch:
+            raise ValueError("prefill_logits: a context id and a start position per row of tokens")
+        logits = np.empty((rows.size, self.vocab_size), dtype=np.float32)
+        nxt = np.zeros(batch, dtype=np.uint32) if want_next_tokens else None
+        res = np.empty((self.layer_runs, batch * n_tokens, residual_width), dtype=np.float32) if residual_width else None
+        rc = host_lib().glint_stage_prefill_logits(self._h, batch, ids.ctypes.data, start.ctypes.data, n_tokens, toks.ctypes.data, rows.ctypes.data,
+                                                   rows.size, logits.ctypes.data, None if nxt is None else nxt.ctypes.data,
+                                                   None if res is None else res.ctypes.data)
+        if rc == -1:
+            return None
+        if rc != 0:
+            raise GlintError("tokens at positions their contexts cannot take")
+        return logits, nxt, res
+
+    def forward(self, which: int = FWD_ALL) -> bool:
+        rc = host_lib().glint_stage_forward(self._h, which)
+        if rc == -3:
+            raise GlintError("tokens at positions their contexts cannot take")
+        if rc == -2:
+            raise GlintError("bad forward selector")
+        return rc == 0
+
+    def logits(self, rows: int) -> np.ndarray:
+        """Logits of the first `rows` rows of the last forward()."""
+        out = np.empty((rows, self.vocab_size), dtype=np.float32)
+        if host_lib().glint_stage_logits(self._h, out.ctypes.data, rows) != 0:
+            raise GlintError("no logits of that many rows")
+        return out
 
 
 class BookManager:

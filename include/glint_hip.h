@@ -41,7 +41,7 @@ typedef enum gh_dtype
 {
   GH_F16 = 0,
   GH_F32 = 1,
-  GH_BF16 = 2 /* declared for wire compatibility; no kernel accepts it (the reference's amd64 bf16 is an alias of fp16, arch/float.hh:13) */
+  GH_BF16 = 2 /* the dense products and the ops of the run-time sized designs below; the Llama2 ops refuse it (the reference's amd64 bf16 is an alias of fp16, arch/float.hh:13) */
 } gh_dtype;
 
 /* values equal glinthawk::CopyType (models/types.hh:127-133) */
@@ -319,6 +319,92 @@ uint64_t gh_attn_prefill_workspace( uint64_t batch, uint32_t n_tokens, const gh_
 int gh_attn_set_prefill_tiles( int column_tiles_per_wave );
 int gh_attn_prefill( const void* q, const void* const* layer_rows_dev, const uint32_t* start_pos_dev, void* xb, uint64_t batch, uint32_t n_tokens,
                      uint32_t max_start_pos, const gh_shape* shape, gh_dtype dt, void* workspace, uint64_t workspace_bytes, int variant, gh_stream stream );
+
+/* ---- designs whose sizes come at run time ---------------------------------------------------------
+ * Ops of decoder-only designs beyond Llama2 (no counterpart in the reference): storage type GH_BF16 or GH_F32, the residual stream x,
+ * norms, scores, weights, gates and recurrent state fp32.  Rows are (context, token): row = context * n_tokens + token, n_tokens
+ * consecutive tokens per context from position start_pos_dev[context] on; one entry point serves decode (n_tokens 1) and prefill.
+ * `context_rows_dev[context]` is the start of a context's memory (NULL: an empty context, whose rows are skipped) and every layer
+ * finds its cache rows or state at a byte offset from there. */
+typedef enum gh_activation
+{
+  GH_ACT_SILU = 0,
+  GH_ACT_GELU_TANH = 1 /* 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
+} gh_activation;
+
+/* x(row) = embed[token] + pos_table[position] (pos_table may be NULL); `copy` (optional) receives DType(x), rows copy_stride elements apart */
+int gh_embed_positions( float* x, const uint32_t* tokens_dev, const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, const void* embed,
+                        const void* pos_table, uint64_t width, uint64_t vocab, uint64_t max_pos, void* copy, uint64_t copy_stride, gh_dtype dt, gh_stream stream );
+
+/* What happens to the fp32 residual stream behind a projection y:
+ *   y += bias;  y = rms(y) * post_norm;  x = accumulate ? x + y : y;  x += add;  out = DType( next_norm ? rms(x) * next_norm : x )
+ * with rms(z) = z / sqrt(mean(z^2) + eps); any of the pointers may be NULL, its part is then left out. */
+typedef struct gh_stream_step
+{
+  const void* bias;
+  const void* post_norm;
+  const void* add;
+  const void* next_norm;
+  void* out;
+  uint64_t out_stride; /* elements from row to row of `out` */
+  float eps;
+  int accumulate;
+} gh_stream_step;
+/* y = in (rows, s) . w (width, s)^T */
+int gh_matmul_stream( float* x, const void* in, const void* w, uint64_t s, uint64_t width, uint64_t rows, const gh_stream_step* step, gh_dtype dt,
+                      gh_stream stream );
+/* the last part alone: out from x */
+int gh_stream_out( float* x, uint64_t width, uint64_t rows, const gh_stream_step* step, gh_dtype dt, gh_stream stream );
+/* hb = DType( act(x . gate^T + bias) * (x . up^T + bias) ); w_gate_up = rows of gate then rows of up, bias (may be NULL) alike */
+int gh_matmul_gate( void* hb, const void* x, const void* w_gate_up, const void* bias, uint64_t s, uint64_t hidden, uint64_t rows, int activation, gh_dtype dt,
+                    gh_stream stream );
+/* out (fp32) = (x . w^T) * scale */
+int gh_matmul_scaled( float* out, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t rows, float scale, gh_dtype dt, gh_stream stream );
+/* out(i) = x(rows_dev[i]), n rows out of n_rows */
+int gh_gather_rows( float* out, const float* x, const uint32_t* rows_dev, uint64_t n, uint64_t n_rows, uint64_t width, gh_stream stream );
+
+/* Attention over a sliding window with kept first tokens and a bias by distance: position i sees j <= i with i - j < window or
+ * j < keep_first, score = (q . k) * scale + distance_bias[h][min(i - j, n_dist - 1)], ordinary softmax.  window 0: no window.
+ * Query head h uses kv head h / (heads / kv_heads).  Head sizes up to 512. */
+typedef struct gh_window_attn
+{
+  uint32_t heads;
+  uint32_t kv_heads;
+  uint32_t dim;
+  uint32_t vdim;
+  uint32_t window;
+  uint32_t keep_first;
+  uint32_t n_dist;
+  float scale;
+} gh_window_attn;
+uint64_t gh_window_row_bytes( const gh_window_attn* a, gh_dtype dt );  /* one token's cache row (heads padded to 8 elements) */
+uint64_t gh_window_query_elements( const gh_window_attn* a );          /* one row of q as the ops below exchange it */
+/* wqkv = rows of q, k, v; bias (may be NULL) alike.  q and k are normed over their whole projection (NULL: not), then q goes to `q`
+ * and [k | v] to the context's cache row at the token's position. */
+int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const void* bias, uint64_t width, const gh_window_attn* a, const void* q_norm,
+                             const void* k_norm, float eps, void* const* context_rows_dev, uint64_t cache_offset, const uint32_t* start_pos_dev, uint64_t batch,
+                             uint32_t n_tokens, gh_dtype dt, gh_stream stream );
+/* out (rows, heads * vdim); the rows of this call are in the cache already.  distance_bias_dev (heads, n_dist) fp32 or NULL;
+ * max_start_pos: host-side upper bound of the start positions */
+int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const float* distance_bias_dev, void* const* context_rows_dev, uint64_t cache_offset,
+                    const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, uint32_t max_start_pos, gh_dtype dt, gh_stream stream );
+
+/* Matrix-memory LSTM mixer up to its output projection: projections, log gates, recurrence, norm of each head, output gate.
+ *   w: rows of q, k (heads * dim each), v, g (heads * vdim each), zeros up to gate_row, rows of i, f (heads each), zeros up to the end
+ *   (gh_mlstm_weight_rows gives the row count and gate_row).  State: gh_mlstm_state_bytes per context, zero before position 0. */
+typedef struct gh_mlstm
+{
+  uint32_t heads;
+  uint32_t dim;
+  uint32_t vdim;
+  float gate_cap;
+  float eps;
+} gh_mlstm;
+uint64_t gh_mlstm_state_bytes( const gh_mlstm* m );
+uint64_t gh_mlstm_weight_rows( const gh_mlstm* m, uint64_t* gate_row );
+int gh_mlstm_forward( void* out, const void* x, const void* w, uint64_t width, const gh_mlstm* m, const void* bias_i, const void* bias_f, const void* norm,
+                      void* const* context_rows_dev, uint64_t state_offset, const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, gh_dtype dt,
+                      gh_stream stream );
 
 /* Timing hooks for the benchmark: HIP events recorded on `stream` around the two kernels of
  * gh_attn_decode.  gh_attn_timing_read() synchronises and returns, accumulated since
