@@ -9,7 +9,7 @@ import select
 from typing import Optional
 
 from ._lib import GlintError
-from .stage import FLAG_CLS, FLAG_FUSED, FLAG_UNFUSED_PROJ, host_lib
+from .stage import DESIGN_DTYPES, FLAG_CLS, FLAG_FUSED, FLAG_PAGED, FLAG_UNFUSED_PROJ, host_lib
 
 _signed = False
 
@@ -21,6 +21,7 @@ def _lib():
         vp, u32, u64, i = C.c_void_p, C.c_uint32, C.c_uint64, C.c_int
         sig = {
             "glint_kernel_create": (vp, [C.c_char_p, i, u32, u32, u32, u32, u32, u64, C.c_float]),
+            "glint_kernel_open": (vp, [C.c_char_p, i, u32, u32, u32, u64, C.c_float]),
             "glint_kernel_create_echo": (vp, [u32, u32]),
             "glint_kernel_destroy": (None, [vp]),
             "glint_kernel_load": (i, [vp, C.c_char_p]),
@@ -41,9 +42,16 @@ def _lib():
 class ComputeKernel:
     def __init__(self, config: Optional[str] = None, dtype: str = "f16", first_layer: int = 0, n_hosted: int = 1,
                  concurrency: int = 1, max_contexts: int = 1, with_cls: bool = False, fused: bool = True,
-                 fused_projections: bool = True, seed: int = 1, weight_std: float = 0.02, echo: bool = False):
-        """`echo=True`: a host-only kernel (no GPU) whose model advances every active row by one token."""
-        if echo:
+                 fused_projections: bool = True, seed: int = 1, weight_std: float = 0.02, echo: bool = False, model_dir: Optional[str] = None,
+                 paged: bool = False):
+        """`echo=True`: a host-only kernel (no GPU) whose model advances every active row by one token.  `model_dir`: the run-time sized
+        design in that directory (dtype bf16 or f32), weights loaded; its states carry prompts only."""
+        if model_dir is not None:
+            self._h = _lib().glint_kernel_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, FLAG_PAGED if paged else 0, seed,
+                                               weight_std)
+            if not self._h:
+                raise GlintError(_lib().glint_last_error().decode(errors="replace"))
+        elif echo:
             self._h = _lib().glint_kernel_create_echo(concurrency, max_contexts)
         else:
             flags = (FLAG_FUSED if fused else 0) | (FLAG_CLS if with_cls else 0) | (0 if fused_projections else FLAG_UNFUSED_PROJ)

@@ -12,7 +12,7 @@ from typing import Optional, Sequence
 import torch
 
 from . import _lib
-from ._lib import GH_ATTN_AUTO, GH_F16, GH_F32, Shape, check, lib
+from ._lib import GH_ACT_GELU_TANH, GH_ATTN_AUTO, GH_BF16, GH_F16, GH_F32, GhMlstm, GhStreamStep, GhWindowAttn, Shape, check, lib
 
 
 def _dt(t: torch.Tensor) -> int:
@@ -20,6 +20,8 @@ def _dt(t: torch.Tensor) -> int:
         return GH_F16
     if t.dtype == torch.float32:
         return GH_F32
+    if t.dtype == torch.bfloat16:
+        return GH_BF16
     raise TypeError(f"unsupported dtype {t.dtype}")
 
 
@@ -342,6 +344,89 @@ def convert_and_copy(dst, src, n: int, kind: int) -> None:
 
 def convert(dst: torch.Tensor, src: torch.Tensor, n: int) -> None:
     check(lib().gh_convert(_p(dst), _dt(dst), _p(src), _dt(src), n, _stream()), "gh_convert")
+
+
+# ---- run-time sized designs -----------------------------------------------------------------------
+# `ctx_rows` is a device table of context regions (row_table), `offset` the byte offset of the layer's part in them.
+def embed_positions(tokens, start_pos, n_tokens: int, embed, pos_table=None, copy=None):
+    rows, width = tokens.numel(), embed.shape[1]
+    x = torch.empty((rows, width), dtype=torch.float32, device=embed.device)
+    check(lib().gh_embed_positions(_p(x), _p(tokens), _p(start_pos), start_pos.numel(), n_tokens, _p(embed), _p(pos_table), width, embed.shape[0],
+                                   1 if pos_table is None else pos_table.shape[0], None if copy is None else copy.data_ptr(),
+                                   0 if copy is None else copy.stride(0), _dt(embed), _stream()), "gh_embed_positions")
+    return x
+
+
+def _stream_step(eps, bias=None, post_norm=None, accumulate=True, add=None, next_norm=None, out=None):
+    return GhStreamStep(_p(bias), _p(post_norm), _p(add), _p(next_norm), None if out is None else out.data_ptr(), 0 if out is None else out.stride(0), eps,
+                        int(accumulate))
+
+
+def matmul_stream(x, inp, w, eps: float = 1e-5, **step) -> None:
+    """x (fp32 residual stream) updated behind inp . w^T; see gh_stream_step for the parts of the step."""
+    s = _stream_step(eps, **step)
+    check(lib().gh_matmul_stream(_p(x), _p(inp), _p(w), w.shape[1], w.shape[0], x.shape[0], C.byref(s), _dt(w), _stream()), "gh_matmul_stream")
+
+
+def stream_out(x, out, next_norm=None, eps: float = 1e-5) -> None:
+    s = _stream_step(eps, next_norm=next_norm, out=out)
+    check(lib().gh_stream_out(_p(x), x.shape[1], x.shape[0], C.byref(s), _dt(out), _stream()), "gh_stream_out")
+
+
+def matmul_gate(x, w_gate_up, bias=None, activation: int = GH_ACT_GELU_TANH):
+    hidden = w_gate_up.shape[0] // 2
+    hb = torch.empty((x.shape[0], hidden), dtype=x.dtype, device=x.device)
+    check(lib().gh_matmul_gate(_p(hb), _p(x), _p(w_gate_up), _p(bias), x.shape[1], hidden, x.shape[0], activation, _dt(x), _stream()), "gh_matmul_gate")
+    return hb
+
+
+def matmul_scaled(x, w, scale: float):
+    out = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32, device=x.device)
+    check(lib().gh_matmul_scaled(_p(out), _p(x), _p(w), x.shape[1], w.shape[0], x.shape[0], scale, _dt(x), _stream()), "gh_matmul_scaled")
+    return out
+
+
+def window_attn(heads, kv_heads, dim, vdim, scale, window=0, keep_first=0, n_dist=0) -> GhWindowAttn:
+    return GhWindowAttn(heads, kv_heads, dim, vdim, window, keep_first, n_dist, scale)
+
+
+def window_row_bytes(a: GhWindowAttn, dtype) -> int:
+    return int(lib().gh_window_row_bytes(C.byref(a), GH_BF16 if dtype == torch.bfloat16 else GH_F32))
+
+
+def window_query_elements(a: GhWindowAttn) -> int:
+    return int(lib().gh_window_query_elements(C.byref(a)))
+
+
+def matmul_window_append(x, wqkv, a: GhWindowAttn, ctx_rows, start_pos, n_tokens: int, bias=None, q_norm=None, k_norm=None, eps: float = 1e-5, offset: int = 0):
+    q = torch.zeros((x.shape[0], window_query_elements(a)), dtype=x.dtype, device=x.device)
+    check(lib().gh_matmul_window_append(_p(q), _p(x), _p(wqkv), _p(bias), x.shape[1], C.byref(a), _p(q_norm), _p(k_norm), eps, _p(ctx_rows), offset,
+                                        _p(start_pos), start_pos.numel(), n_tokens, _dt(x), _stream()), "gh_matmul_window_append")
+    return q
+
+
+def attn_window(q, a: GhWindowAttn, ctx_rows, start_pos, n_tokens: int, max_start_pos: int, distance_bias=None, offset: int = 0):
+    out = torch.zeros((q.shape[0], a.heads * a.vdim), dtype=q.dtype, device=q.device)
+    check(lib().gh_attn_window(_p(out), _p(q), C.byref(a), _p(distance_bias), _p(ctx_rows), offset, _p(start_pos), start_pos.numel(), n_tokens,
+                               max_start_pos, _dt(q), _stream()), "gh_attn_window")
+    return out
+
+
+def mlstm_state_bytes(m: GhMlstm) -> int:
+    return int(lib().gh_mlstm_state_bytes(C.byref(m)))
+
+
+def mlstm_weight_rows(m: GhMlstm):
+    """(rows of the projection matrix, first row of the gates)"""
+    gate = C.c_uint64(0)
+    return int(lib().gh_mlstm_weight_rows(C.byref(m), C.byref(gate))), int(gate.value)
+
+
+def mlstm_forward(x, w, m: GhMlstm, bias_i, bias_f, norm, ctx_rows, start_pos, n_tokens: int, offset: int = 0):
+    out = torch.zeros((x.shape[0], m.heads * m.vdim), dtype=x.dtype, device=x.device)
+    check(lib().gh_mlstm_forward(_p(out), _p(x), _p(w), x.shape[1], C.byref(m), _p(bias_i), _p(bias_f), _p(norm), _p(ctx_rows), offset, _p(start_pos),
+                                 start_pos.numel(), n_tokens, _dt(x), _stream()), "gh_mlstm_forward")
+    return out
 
 
 def sync() -> None:
