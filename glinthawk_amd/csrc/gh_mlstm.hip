@@ -13,11 +13,13 @@
 #include "gh_product.h"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace gh {
 namespace {
 
-constexpr uint32_t SLICE = 64; // columns of v per work-group of the walk
+constexpr uint32_t SLICE = 64;          // columns of v per work-group
+constexpr uint32_t CHUNKED_TOKENS = 24; // from this many tokens per context on, bf16 runs in chunks on the matrix cores
 
 struct MlstmShape
 {
@@ -193,6 +195,402 @@ __global__ __launch_bounds__( 256 ) void mlstm_walk_kernel( float* __restrict__ 
   }
 }
 
+// ---- many tokens: chunks of 64 on the matrix cores (bf16 products) -------------------------------------------------------------
+//
+// With b_t the sum of the log forget gates of the chunk up to token t, c_s = i_s - b_s and M_t = max(m0, c_1 .. c_t) (m0: the running
+// maximum in front of the chunk), the recurrence unrolls to m_t = b_t + M_t and
+//
+//   S_t = e^(m0 - M_t) S_0 + sum_(s <= t) e^(c_s - M_t) k_s v_s^T                      (n_t likewise)
+//   o_t = (e^(m0 - M_t) S_0^T q_t + sum_(s <= t) e^(c_s - M_t) (k_s . q_t) v_s) / (max(|n_t . q_t|, e^(-m_t)) + 1e-6)
+//
+// work-group  2 waves on one (context, head, 64 columns of v) walk the chunks; a wave owns 32 columns, its part of S (dim x 32, fp32) stays in
+//             accumulator registers from the first chunk to the last.  Two work-groups per CU cover each other's loads.
+// exactness   q, k, v are bf16 already; everything fp32 that meets them in a product (S, the weights of the keys, the weighted values) goes
+//             in as three bf16 terms, 24 bits, so that the sums are those of fp32 operands at the rate of bf16 matrix instructions.
+// operands    an accumulator tile of v_mfma_f32_32x32x16_bf16 (lane = column, registers = rows 8 (v / 4) + 4 (lane / 32) + v % 4) is, as it
+//             lies, an operand of the next product over those rows when the other operand takes its sixteen k in the same order:
+//               scores^T = K Q^T        lane = query, registers = keys   -> left operand of   P V     (V out of LDS transposed)
+//               S                       lane = column of v, registers = dim -> right operand of Q S   (Q out of LDS in pieces of 4)
+//             S += K^T (w V): both operands out of LDS with transposing reads (ds_read_b64_tr_b16).
+// LDS         64 rows each of q, k (16-byte chunks XORed with bits of the row, so that row reads and transposing reads both spread over
+//             the banks) and of v, straight from memory (buffer_load ... lds; rows past the sequence and padding read as zero).
+constexpr int CHUNK = 64;
+typedef __attribute__( ( address_space( 3 ) ) ) void* lds_ptr;
+typedef __attribute__( ( address_space( 3 ) ) ) char lds_char;
+typedef short v4s __attribute__( ( ext_vector_type( 4 ) ) );
+typedef __attribute__( ( address_space( 3 ) ) ) v4s* lds_v4s;
+typedef Mfma<__bf16>::x8 bf16x8;
+
+// slot of 16-byte chunk `chunk` of row `row` in a tile of DT * 4 chunks a row
+template<int DT>
+__device__ __forceinline__ uint32_t swizzle( uint32_t row, uint32_t chunk )
+{
+  return DT == 2 ? chunk ^ ( ( ( ( row >> 1 ) & 1 ) << 2 ) | ( ( row >> 2 ) & 3 ) ) : chunk ^ ( ( ( row & 3 ) << 2 ) | ( ( row >> 2 ) & 3 ) );
+}
+__device__ __forceinline__ uint32_t swizzle_v( uint32_t row, uint32_t chunk ) { return chunk ^ ( 4 * ( ( row >> 1 ) & 1 ) ); }
+
+// x = hi + mid + lo, 8 bits each
+struct Split3
+{
+  bf16x8 t[3];
+};
+__device__ __forceinline__ void split3( Split3& s, int e, float x )
+{
+  const __bf16 hi = (__bf16)x;
+  const float r = x - (float)hi;
+  const __bf16 mid = (__bf16)r;
+  s.t[0][e] = hi;
+  s.t[1][e] = mid;
+  s.t[2][e] = (__bf16)( r - (float)mid );
+}
+__device__ __forceinline__ mfma_f32x16 mma3( const bf16x8 a, const Split3& b, mfma_f32x16 c )
+{
+  c = Mfma<__bf16>::k16( a, b.t[2], c );
+  c = Mfma<__bf16>::k16( a, b.t[1], c );
+  return Mfma<__bf16>::k16( a, b.t[0], c );
+}
+__device__ __forceinline__ mfma_f32x16 mma3( const Split3& a, const bf16x8 b, mfma_f32x16 c )
+{
+  c = Mfma<__bf16>::k16( a.t[2], b, c );
+  c = Mfma<__bf16>::k16( a.t[1], b, c );
+  return Mfma<__bf16>::k16( a.t[0], b, c );
+}
+__device__ __forceinline__ double shfl_up_f64( double v, int by )
+{
+  const uint64_t bits = __builtin_bit_cast( uint64_t, v );
+  const uint32_t lo = __shfl_up( (uint32_t)bits, by ), hi = __shfl_up( (uint32_t)( bits >> 32 ), by );
+  return __builtin_bit_cast( double, ( (uint64_t)hi << 32 ) | lo );
+}
+__device__ __forceinline__ double last_lane_f64( double v )
+{
+  const uint64_t bits = __builtin_bit_cast( uint64_t, v );
+  const uint32_t lo = __builtin_amdgcn_readlane( (uint32_t)bits, 63 ), hi = __builtin_amdgcn_readlane( (uint32_t)( bits >> 32 ), 63 );
+  return __builtin_bit_cast( double, ( (uint64_t)hi << 32 ) | lo );
+}
+
+// DT: 32-row tiles of S, dim <= 32 DT.  dim % 8 == 0, vdim % 8 == 0, 16-byte aligned product rows.
+template<int DT>
+__global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restrict__ o_out, float* __restrict__ nm_out, MlstmIn<__bf16, ProductView<__bf16>> in, MlstmState st,
+                                                                MlstmShape s )
+{
+  constexpr uint32_t RB = DT * 64; // bytes of a q or k row in LDS
+  __shared__ uint4 s_k[CHUNK * RB / 16], s_q[CHUNK * RB / 16];
+  __shared__ uint4 s_v[CHUNK * 8];
+  __shared__ float s_n[2][32 * DT];                                   // each wave its own copy of everything below
+  __shared__ __attribute__( ( aligned( 16 ) ) ) float s_c[2][CHUNK]; // c_s - M of the chunk's last token, s_w: e to the power of it
+  __shared__ __attribute__( ( aligned( 16 ) ) ) float s_w[2][CHUNK];
+  __shared__ __attribute__( ( aligned( 16 ) ) ) float s_a[2][CHUNK];   // factor of the state in front of the chunk, per token
+  __shared__ __attribute__( ( aligned( 16 ) ) ) float s_inv[2][CHUNK]; // one over the denominator
+
+  const uint32_t slice = blockIdx.x, h = blockIdx.y, ctx = blockIdx.z;
+  uint8_t* base = static_cast<uint8_t*>( st.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  float* S_mem = reinterpret_cast<float*>( base + st.offset );
+  const float* n_in = S_mem + s.n_off() + (uint64_t)h * s.dim;
+  const float m_mem = S_mem[s.m_off() + h];
+  S_mem += (uint64_t)h * s.dim * s.vpad;
+  const bool fresh = st.start_pos[ctx] == 0;
+  const uint32_t wave = __builtin_amdgcn_readfirstlane( threadIdx.x >> 6 );
+  const uint32_t lane = threadIdx.x & 63, r = lane & 31, g2 = lane >> 5;
+  const uint32_t col = slice * 64 + wave * 32 + r; // this lane's column of v
+
+  constexpr uint32_t PAST_THE_END = 0x80000000u; // an offset beyond any descriptor: reads zero, stores nothing
+  const __amdgpu_buffer_rsrc_t S_rsrc = __builtin_amdgcn_make_buffer_rsrc( S_mem, 0, (int)( s.dim * s.vpad * 4 ), 0x00020000 );
+  const uint32_t S_off = col < s.vpad ? ( 4 * g2 * s.vpad + col ) * 4 : PAST_THE_END;
+  mfma_f32x16 S[DT];
+#pragma unroll
+  for ( int dt = 0; dt < DT; dt++ ) {
+#pragma unroll
+    for ( int v = 0; v < 16; v++ ) {
+      S[dt][v] = __builtin_bit_cast( float, __builtin_amdgcn_raw_buffer_load_b32( S_rsrc, fresh ? PAST_THE_END : S_off, ( 32 * dt + 8 * ( v / 4 ) + v % 4 ) * s.vpad * 4, 0 ) );
+    }
+  }
+  for ( uint32_t d = lane; d < 32 * DT; d += 64 ) {
+    s_n[wave][d] = !fresh && d < s.dim ? n_in[d] : 0.0f;
+  }
+  double m0 = fresh ? 0.0 : (double)m_mem;
+  const float bi = in.bias_i != nullptr ? to_f32( in.bias_i[h] ) : 0.0f, bf = in.bias_f != nullptr ? to_f32( in.bias_f[h] ) : 0.0f;
+  const uint64_t row_first = (uint64_t)ctx * st.n_tokens;
+  const uint32_t ld_bytes = (uint32_t)( in.main.stride * 2 );
+
+  // LDS byte addresses: a part that depends on the lane, a constant, and a constant XORed with a lane value (the swizzle acts on the
+  // sixteen slots of 256 bytes, or eight of 128).  Computed where they are used: kept in registers over the loop there are too many of them.
+  constexpr uint32_t PERIOD = DT == 2 ? 128 : 256;
+  auto slot_at = [&]( uint32_t constant, uint32_t lane_xor ) __attribute__( ( always_inline ) ) {
+    return constant / PERIOD * PERIOD + ( ( constant % PERIOD ) ^ lane_xor );
+  };
+  auto opaque = []( uint32_t v ) __attribute__( ( always_inline ) ) {
+    asm volatile( "" : "+v"( v ) );
+    return v;
+  };
+  const uint32_t row_swz = swizzle<DT>( r, 0 ) * 16; // of rows r and r + 32
+
+  // rows [0, rows) x `chunks` 16-byte chunks of the product at `p`, LDS rows of 64 DT (or, for v, 128) bytes; the rest reads as zero
+  auto fetch = [&]( uint4* tile, const __bf16* p, uint32_t rows, uint32_t chunks, auto slot_of, auto row_bytes_tag ) {
+    constexpr uint32_t BYTES = decltype( row_bytes_tag )::value;
+    const __amdgpu_buffer_rsrc_t rsrc
+      = __builtin_amdgcn_make_buffer_rsrc( const_cast<__bf16*>( p ), 0, (int)( rows > 0 ? ( rows - 1 ) * ld_bytes + chunks * 16 : 0 ), 0x00020000 );
+    constexpr uint32_t ROWS = 1024 / BYTES; // rows of one instruction of one wave
+    const uint32_t ln = opaque( lane );
+#pragma unroll
+    for ( uint32_t i = 0; i < CHUNK / ( 2 * ROWS ); i++ ) {
+      const uint32_t row0 = ( 2 * i + wave ) * ROWS;
+      const uint32_t row = row0 + ln / ( BYTES / 16 );
+      const uint32_t chunk = slot_of( row, ln % ( BYTES / 16 ) ); // the swizzle is its own inverse
+      const uint32_t off = chunk < chunks ? row * ld_bytes + chunk * 16 : PAST_THE_END;
+      __builtin_amdgcn_raw_ptr_buffer_load_lds( rsrc, (lds_ptr)( tile + row0 * ( BYTES / 16 ) ), 16, off, 0, 0, 0 );
+    }
+  };
+
+  // transposing reads: lane j = 4 e + q of a 16-lane group points at row e (0..3) of its half-wave's four, dims 16 grp + 4 q .. + 3
+  const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
+  const uint32_t trk_row = ( 4 * g2 + tr_e ) * RB + ( tr_q & 1 ) * 8, trk_swz = ( swizzle<DT>( 4 * g2 + tr_e, 2 * tr_grp + ( tr_q >> 1 ) ) ) * 16;
+  auto tr_k = [&]( int kk, int dt, uint32_t row, uint32_t swz ) __attribute__( ( always_inline ) ) {
+    union
+    {
+      v4s half[2];
+      bf16x8 x;
+    } u;
+#pragma unroll
+    for ( int hf = 0; hf < 2; hf++ ) { // rows 8 further on: bit 1 of the swizzle's low part
+      u.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_k + row + ( 16 * kk + 8 * hf ) * RB + slot_at( ( 64 * dt ) ^ ( 32 * hf ), swz ) ) );
+    }
+    return u.x;
+  };
+  auto tr_v = [&]( int kk ) __attribute__( ( always_inline ) ) {
+    union
+    {
+      v4s half[2];
+      bf16x8 x;
+    } u;
+#pragma unroll
+    for ( int hf = 0; hf < 2; hf++ ) {
+      const uint32_t row = 16 * kk + 8 * hf + 4 * g2 + tr_e;
+      u.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+        (lds_v4s)( (lds_char*)s_v + row * 128 + swizzle_v( row, 4 * wave + 2 * tr_grp + ( tr_q >> 1 ) ) * 16 + ( tr_q & 1 ) * 8 ) );
+    }
+    return u.x;
+  };
+
+  for ( uint32_t t0 = 0; t0 < st.n_tokens; t0 += CHUNK ) {
+    const uint32_t rows = min( (uint32_t)CHUNK, st.n_tokens - t0 );
+    const __bf16* first = in.main.data + ( row_first + t0 ) * in.main.stride;
+    __syncthreads(); // the last chunk's readers are done
+    fetch( s_k, first + in.col.k + h * s.dim, rows, s.dim / 8, []( uint32_t row, uint32_t c ) { return swizzle<DT>( row, c ); }, std::integral_constant<uint32_t, RB> {} );
+    fetch( s_q, first + in.col.q + h * s.dim, rows, s.dim / 8, []( uint32_t row, uint32_t c ) { return swizzle<DT>( row, c ); }, std::integral_constant<uint32_t, RB> {} );
+    fetch( s_v, first + in.col.v + h * s.vdim + slice * 64, rows, min( 8u, ( s.vdim - slice * 64 ) / 8 ), swizzle_v, std::integral_constant<uint32_t, 128> {} );
+
+    // gates: lane = token
+    const bool live = lane < rows;
+    const uint64_t grow = row_first + t0 + ( live ? lane : 0 );
+    const float gi = soft_cap( in.gates.at( grow, in.col.i + h ) + bi, s.cap );
+    const float gf = log_sigmoid( soft_cap( in.gates.at( grow, in.col.f + h ) + bf, s.cap ) );
+    double b = live ? (double)gf : 0.0;
+#pragma unroll
+    for ( int by = 1; by < 64; by *= 2 ) {
+      const double up = shfl_up_f64( b, by );
+      b += (int)lane >= by ? up : 0.0;
+    }
+    const double c = live ? (double)gi - b : -1e300;
+    double M = c > m0 ? c : m0;
+#pragma unroll
+    for ( int by = 1; by < 64; by *= 2 ) {
+      const double up = shfl_up_f64( M, by );
+      M = (int)lane >= by && up > M ? up : M;
+    }
+    const double M_end = last_lane_f64( M ), b_end = last_lane_f64( b );
+    const float c_rel = live ? (float)( c - M_end ) : -INFINITY;
+    const float state_decay = expf( (float)( m0 - M_end ) );
+    s_c[wave][lane] = c_rel;
+    s_w[wave][lane] = expf( c_rel );
+    s_a[wave][lane] = expf( (float)( m0 - M ) );
+    const float M_rel = (float)( M - M_end ), floor_den = expf( -(float)( b + M ) ); // of token `lane`
+    m0 = b_end + M_end;
+
+    __builtin_amdgcn_s_waitcnt( 0x0F70 ); // vmcnt(0): this wave's part of the tiles has landed
+    __syncthreads();
+
+    // ---- scores^T and the weights P: query tile tt, key tiles up to it
+    Split3 P[2][4]; // [query tile][16 keys]
+    float den[2];
+#pragma unroll
+    for ( int tt = 0; tt < 2; tt++ ) {
+      const float Mq = __shfl( M_rel, 32 * tt + r ); // of this lane's query
+      den[tt] = 0.0f;
+#pragma unroll
+      for ( int kt = 0; kt <= tt; kt++ ) {
+        __builtin_amdgcn_sched_barrier( 0 );
+        const uint32_t rb = opaque( r * RB ), swz = opaque( row_swz ^ ( 16 * g2 ) );
+        mfma_f32x16 sc = { 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0 };
+#pragma unroll
+        for ( int k16 = 0; k16 < 2 * DT; k16++ ) {
+          const uint32_t at = slot_at( 32 * k16, swz );
+          const bf16x8 a = *reinterpret_cast<const bf16x8*>( reinterpret_cast<const char*>( s_k ) + 32 * kt * RB + rb + at );
+          const bf16x8 bq = *reinterpret_cast<const bf16x8*>( reinterpret_cast<const char*>( s_q ) + 32 * tt * RB + rb + at );
+          sc = Mfma<__bf16>::k16( a, bq, sc );
+        }
+#pragma unroll
+        for ( int q4 = 0; q4 < 4; q4++ ) {
+          const uint32_t key0 = opaque( 32 * kt + 8 * q4 + 4 * g2 );
+          const float4 ck = *reinterpret_cast<const float4*>( &s_c[wave][key0] );
+          const float cks[4] = { ck.x, ck.y, ck.z, ck.w };
+#pragma unroll
+          for ( int e = 0; e < 4; e++ ) {
+            const bool seen = kt < tt || key0 + e <= 32 * tt + r;
+            const float p = seen ? sc[4 * q4 + e] * s.q_scale * __expf( cks[e] - Mq ) : 0.0f;
+            den[tt] += p;
+            split3( P[tt][2 * kt + ( q4 >> 1 )], 4 * ( q4 & 1 ) + e, p );
+          }
+        }
+      }
+    }
+    // ---- Q S (state in front of the chunk), n . q beside it
+    mfma_f32x16 O[2];
+    float nq[2] = { 0.0f, 0.0f };
+#pragma unroll
+    for ( int tt = 0; tt < 2; tt++ ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        O[tt][v] = 0.0f;
+      }
+    }
+    __builtin_amdgcn_sched_barrier( 0 ); // (without these fences the scheduler asks for all operands of a phase at once and spills)
+#pragma unroll
+    for ( int dt = 0; dt < DT; dt++ ) {
+#pragma unroll
+      for ( int half = 0; half < 2; half++ ) {
+        __builtin_amdgcn_sched_barrier( 0 );
+        const uint32_t rb = opaque( r * RB + 8 * g2 ), swz = opaque( row_swz );
+        Split3 sp;
+#pragma unroll
+        for ( int e = 0; e < 8; e++ ) {
+          split3( sp, e, S[dt][8 * half + e] );
+        }
+        const float4 n0 = *reinterpret_cast<const float4*>( &s_n[wave][32 * dt + 16 * half + 4 * g2] );
+        const float4 n1 = *reinterpret_cast<const float4*>( &s_n[wave][32 * dt + 16 * half + 8 + 4 * g2] );
+#pragma unroll
+        for ( int tt = 0; tt < 2; tt++ ) {
+          union
+          {
+            uint2 p[2];
+            bf16x8 x;
+          } a;
+          a.p[0] = *reinterpret_cast<const uint2*>( reinterpret_cast<const char*>( s_q ) + 32 * tt * RB + rb + slot_at( 64 * dt + 32 * half, swz ) );
+          a.p[1] = *reinterpret_cast<const uint2*>( reinterpret_cast<const char*>( s_q ) + 32 * tt * RB + rb + slot_at( 64 * dt + 32 * half + 16, swz ) );
+          O[tt] = mma3( a.x, sp, O[tt] );
+          nq[tt] += (float)a.x[0] * n0.x + (float)a.x[1] * n0.y + (float)a.x[2] * n0.z + (float)a.x[3] * n0.w + (float)a.x[4] * n1.x + (float)a.x[5] * n1.y
+                    + (float)a.x[6] * n1.z + (float)a.x[7] * n1.w;
+        }
+      }
+    }
+#pragma unroll
+    for ( int tt = 0; tt < 2; tt++ ) {
+      // the lane 32 further on holds the other half of this query's dims and keys
+      const float a_q = s_a[wave][32 * tt + r];
+      float d = nq[tt] * s.q_scale * a_q + den[tt];
+      d += __shfl_xor( d, 32 );
+      const float lo = __shfl( floor_den, 32 * tt + r );
+      if ( g2 == 0 ) {
+        s_inv[wave][32 * tt + r] = 1.0f / ( fmaxf( fabsf( d ), lo ) + 1e-6f );
+      }
+    }
+    __builtin_amdgcn_sched_barrier( 0 );
+    // ---- O = a Q S + P V, then out
+    const uint32_t hv = s.heads * s.vdim;
+    const __amdgpu_buffer_rsrc_t o_rsrc
+      = __builtin_amdgcn_make_buffer_rsrc( o_out + ( row_first + t0 ) * hv + h * s.vdim, 0, (int)( ( ( rows - 1 ) * hv + s.vdim ) * 4 ), 0x00020000 );
+    const uint32_t o_off = col < s.vdim ? ( 4 * g2 * hv + col ) * 4 : PAST_THE_END;
+    bf16x8 V[4];
+#pragma unroll
+    for ( int kk = 0; kk < 4; kk++ ) {
+      V[kk] = tr_v( kk );
+    }
+#pragma unroll
+    for ( int tt = 0; tt < 2; tt++ ) {
+#pragma unroll
+      for ( int q4 = 0; q4 < 4; q4++ ) {
+        const float4 f = *reinterpret_cast<const float4*>( &s_a[wave][32 * tt + 8 * q4 + 4 * g2] );
+        O[tt][4 * q4] *= f.x * s.q_scale;
+        O[tt][4 * q4 + 1] *= f.y * s.q_scale;
+        O[tt][4 * q4 + 2] *= f.z * s.q_scale;
+        O[tt][4 * q4 + 3] *= f.w * s.q_scale;
+      }
+#pragma unroll
+      for ( int kk = 0; kk < 2 * tt + 2; kk++ ) {
+        O[tt] = mma3( P[tt][kk], V[kk], O[tt] );
+      }
+#pragma unroll
+      for ( int q4 = 0; q4 < 4; q4++ ) {
+        const uint32_t tok = 32 * tt + 8 * q4 + 4 * g2;
+        const float4 f = *reinterpret_cast<const float4*>( &s_inv[wave][tok] );
+        const float inv[4] = { f.x, f.y, f.z, f.w };
+#pragma unroll
+        for ( int e = 0; e < 4; e++ ) {
+          __builtin_amdgcn_raw_buffer_store_b32( __builtin_bit_cast( unsigned, O[tt][4 * q4 + e] * inv[e] ), o_rsrc, o_off, ( 32 * tt + 8 * q4 + e ) * hv * 4, 0 );
+        }
+      }
+    }
+    __builtin_amdgcn_sched_barrier( 0 );
+    // ---- S and n behind the chunk
+    Split3 wv[4];
+#pragma unroll
+    for ( int kk = 0; kk < 4; kk++ ) {
+#pragma unroll
+      for ( int hf = 0; hf < 2; hf++ ) {
+        const float4 w = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 8 * hf + 4 * g2] );
+        split3( wv[kk], 4 * hf, (float)V[kk][4 * hf] * w.x );
+        split3( wv[kk], 4 * hf + 1, (float)V[kk][4 * hf + 1] * w.y );
+        split3( wv[kk], 4 * hf + 2, (float)V[kk][4 * hf + 2] * w.z );
+        split3( wv[kk], 4 * hf + 3, (float)V[kk][4 * hf + 3] * w.w );
+      }
+    }
+#pragma unroll
+    for ( int dt = 0; dt < DT; dt++ ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        S[dt][v] *= state_decay;
+      }
+      float nd = 0.0f;
+      __builtin_amdgcn_sched_barrier( 0 );
+      const uint32_t k_row = opaque( trk_row ), k_swz = opaque( trk_swz );
+#pragma unroll
+      for ( int kk = 0; kk < 4; kk++ ) {
+        const bf16x8 a = tr_k( kk, dt, k_row, k_swz );
+        S[dt] = mma3( a, wv[kk], S[dt] );
+        const float4 w0 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 4 * g2] );
+        const float4 w1 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 8 + 4 * g2] );
+        nd += (float)a[0] * w0.x + (float)a[1] * w0.y + (float)a[2] * w0.z + (float)a[3] * w0.w + (float)a[4] * w1.x + (float)a[5] * w1.y + (float)a[6] * w1.z
+              + (float)a[7] * w1.w;
+      }
+      nd += __shfl_xor( nd, 32 );
+      if ( g2 == 0 ) {
+        s_n[wave][32 * dt + r] = s_n[wave][32 * dt + r] * state_decay + nd;
+      }
+    }
+  }
+
+  uint32_t vpad = s.vpad; // (the row offsets anew: kept from the loads above they would occupy the scalar registers all along)
+  asm volatile( "" : "+s"( vpad ) );
+#pragma unroll
+  for ( int dt = 0; dt < DT; dt++ ) {
+#pragma unroll
+    for ( int v = 0; v < 16; v++ ) {
+      __builtin_amdgcn_raw_buffer_store_b32( __builtin_bit_cast( unsigned, (float)S[dt][v] ), S_rsrc, S_off, ( 32 * dt + 8 * ( v / 4 ) + v % 4 ) * vpad * 4, 0 );
+    }
+  }
+  if ( slice == 0 && wave == 0 ) {
+    float* dst = nm_out + ( (uint64_t)ctx * s.heads + h ) * ( s.dim + 1 );
+    for ( uint32_t d = lane; d < s.dim; d += 64 ) {
+      dst[d] = s_n[0][d];
+    }
+    if ( lane == 0 ) {
+      dst[s.dim] = (float)m0;
+    }
+  }
+}
+
 // one work-group per token, one wave per head in turn
 template<typename E, typename View>
 __global__ __launch_bounds__( 256 ) void mlstm_finish_kernel( E* __restrict__ out,
@@ -292,8 +690,9 @@ int gh_mlstm_forward( void* out, const void* x, const void* w, uint64_t width, c
   const uint32_t hd = s.heads * s.dim, hv = s.heads * s.vdim;
   MlstmCols col { 0, hd, 2 * hd, 2 * hd + hv, (uint32_t)gate_row, (uint32_t)gate_row + s.heads };
   Product y, gates;
-  if ( dt == GH_BF16 && rows >= PRODUCT_ROUNDED_ROWS ) { // the gates stay fp32 sums
-    if ( int rc = make_product( x, w, width, gate_row, rows, dt, false, st, &y ) ) {
+  const bool chunked = dt == GH_BF16 && n_tokens >= CHUNKED_TOKENS && s.dim <= 256 && s.dim % 8 == 0 && s.vdim % 8 == 0;
+  if ( dt == GH_BF16 && ( chunked || rows >= PRODUCT_ROUNDED_ROWS ) ) { // the gates stay fp32 sums
+    if ( int rc = make_product( x, w, width, gate_row, rows, dt, false, st, &y, 1 ) ) {
       return rc;
     }
     if ( int rc = make_product( x, static_cast<const char*>( w ) + gate_row * width * dtype_size( dt ), width, r - gate_row, rows, dt, true, st, &gates ) ) {
@@ -320,8 +719,23 @@ int gh_mlstm_forward( void* out, const void* x, const void* w, uint64_t width, c
     using View = decltype( view );
     const MlstmIn<E, View> in { view, ProductView<float>( gates ), col, static_cast<const E*>( bias_i ), static_cast<const E*>( bias_f ) };
     const dim3 grid( ( s.vpad + SLICE - 1 ) / SLICE, s.heads, (unsigned)batch );
+    bool walked = false;
+    if constexpr ( std::is_same_v<View, ProductView<__bf16>> ) {
+      if ( chunked ) {
+        if ( s.dim <= 64 ) {
+          mlstm_chunk_kernel<2><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+        } else if ( s.dim <= 128 ) {
+          mlstm_chunk_kernel<4><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+        } else {
+          mlstm_chunk_kernel<8><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+        }
+        walked = true;
+      }
+    }
     const size_t lds = ( 3 * ( ( s.dim + 3 ) / 4 * 4 ) + SLICE + 16 + 16 * SLICE ) * sizeof( float );
-    if ( s.dim <= 64 ) {
+    if ( walked ) {
+      // the chunk kernel has done it
+    } else if ( s.dim <= 64 ) {
       mlstm_walk_kernel<E, View, 4><<<grid, 256, lds, st>>>( o, nm, in, state, s );
     } else if ( s.dim <= 128 ) {
       mlstm_walk_kernel<E, View, 8><<<grid, 256, lds, st>>>( o, nm, in, state, s );

@@ -21,12 +21,13 @@ struct Product
 
 constexpr uint64_t PRODUCT_ROUNDED_ROWS = 192; // from this many rows on (16-bit storage) the output is rounded to DType
 
-// x (b, s) . w (r, s)^T.  `exact`: fp32 sums whatever the row count.  The result lives in the stream's scratch until the next product.
-inline int make_product( const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, bool exact, hipStream_t st, Product* out )
+// x (b, s) . w (r, s)^T.  `exact`: fp32 sums whatever the row count; `rounded_from`: rows from which on the output is rounded.  The result lives in the stream's scratch until the next product.
+inline int make_product( const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, bool exact, hipStream_t st, Product* out,
+                         uint64_t rounded_from = PRODUCT_ROUNDED_ROWS )
 {
   out->stride = r;
   out->plane = b * r;
-  if ( !exact && dt != GH_F32 && b >= PRODUCT_ROUNDED_ROWS ) {
+  if ( !exact && dt != GH_F32 && b >= rounded_from ) {
     void* p = nullptr;
     if ( int rc = stream_scratch( st, SCRATCH_PRODUCT, b * r * dtype_size( dt ), 0, &p ) ) {
       return rc;

@@ -409,9 +409,17 @@ def models(tmp_path_factory):
             weights = M.random_weights(cfg, seed=sum(map(ord, name)))
             path = M.write_model(tmp_path_factory.mktemp(name), cfg, weights)
             rng = np.random.default_rng(11)
-            seqs = [rng.integers(0, cfg["vocab"], T) for _ in range(4)]
-            residuals = []
-            want = [P.forward(cfg, weights, s, residuals=residuals if i == 0 else None) for i, s in enumerate(seqs)]
+            # At a first token a head's normed output is v times the sign of k . q: where that product almost vanishes, rounding decides.
+            # Sequences that rounding errors of weights in bf16 throw off like that say nothing about the code and are drawn again.
+            noisy = {k: a * (1 + 2.0 ** -9 * rng.standard_normal(a.shape)) for k, a in weights.items()}
+            seqs, want, residuals = [], [], []
+            while len(seqs) < 4:
+                s, res = rng.integers(0, cfg["vocab"], T), []
+                w = P.forward(cfg, weights, s, residuals=res)
+                if np.sort(logit_error(P.forward(cfg, noisy, s), w))[-2:].mean() < 0.06:
+                    seqs.append(s)
+                    want.append(w)
+                    residuals = residuals or res
             made[name] = (path, cfg, weights, seqs, want, residuals)
         return made[name]
 
