@@ -338,8 +338,7 @@ __global__ __launch_bounds__( 256, NQT == 1 ? 2 : 1 ) void attn_prefill_mfma_ker
         }
       }
       float mx = fmaxf( fmaxf( m4[0], m4[1] ), fmaxf( m4[2], m4[3] ) );
-      const auto halves = __builtin_amdgcn_permlane32_swap( __builtin_bit_cast( unsigned, mx ), __builtin_bit_cast( unsigned, mx ), false, false );
-      mx = fmaxf( __builtin_bit_cast( float, halves[0] ), __builtin_bit_cast( float, halves[1] ) ) * scale_log2e; // log2 domain from here on
+      mx = half_wave_max( mx ) * scale_log2e; // log2 domain from here on
       // The reference point of the exponentials only moves when the maximum has grown by more than 2^LAZY since it was set:
       // weights stay below 2^LAZY (fine for fp32 sums and fp16 operands) and the 64 accumulators are rescaled rarely.  The
       // result does not depend on the reference point.  -inf: a column that has seen no key yet (padding, or hidden so far).

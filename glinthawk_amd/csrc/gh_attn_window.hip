@@ -316,6 +316,282 @@ __global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ ou
   }
 }
 
+// ---- many tokens: key tiles on the matrix cores (bf16, head sizes up to 128) -----------------------------------------------------
+//
+// work-group  4 waves on one (context, kv head), 32 query columns a wave; a column is (token, query head) with the query heads of a group side
+//             by side where their number is a power of two, else one query head per work-group
+// keys        64 at a time: the tiles of the kept first tokens in front of the window, then those of the window of the work-group's
+//             tokens.  A tile that every column sees whole takes no mask, one farther away than the bias table is long a constant bias.
+// scores^T    K Q^T by v_mfma_f32_32x32x16_bf16 (K out of LDS, Q in registers): a lane holds 32 of the tile's 64 scores of ITS column, the
+//             lane 32 further on the others, so maximum and sum stay in the lane but for one exchange
+// values      O^T += V^T P^T: the weights are, as they lie, the right operand; V^T comes out of LDS by transposing reads.  The weights
+//             are fp32: they enter as two bf16 terms (16 bits of mantissa), their sum is taken in fp32.
+// LDS         rows of 256 bytes whatever the head size (the rest is zero), 16-byte chunks XORed with bits of the row; the next tile's
+//             rows are in registers while this one is multiplied, and two work-groups share a CU.
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr float LAZY = 8.0f; // the reference point of a column's exponentials moves when its maximum has grown by 2^LAZY
+constexpr uint32_t TILE_KEYS = 64;
+constexpr uint32_t BIAS_LDS = 4096; // floats of bias table a work-group can hold
+typedef __attribute__( ( address_space( 3 ) ) ) char lds_char;
+typedef short v4s __attribute__( ( ext_vector_type( 4 ) ) );
+typedef __attribute__( ( address_space( 3 ) ) ) v4s* lds_v4s;
+typedef uint32_t u32x4_t __attribute__( ( ext_vector_type( 4 ) ) );
+typedef const u32x4_t __attribute__( ( address_space( 1 ) ) ) global_u32x4_t;
+typedef Mfma<__bf16>::x8 bf16x8;
+
+// KS: steps of 16 of the query/key size; VB: blocks of 32 of the value size
+template<int KS, int VB>
+__global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restrict__ out,
+                                                                 const __bf16* __restrict__ q,
+                                                                 const float* __restrict__ bias,
+                                                                 WindowRows wr,
+                                                                 WindowShape s,
+                                                                 uint32_t head_cols,  // query heads side by side in the columns
+                                                                 uint32_t col_blocks, // work-groups along the tokens of a pair
+                                                                 uint32_t n_pairs,    // contexts x kv heads x (query heads of a group / head_cols)
+                                                                 uint32_t bias_floats )
+{
+  extern __shared__ uint4 lds16[];
+  uint4* s_k = lds16;
+  uint4* s_v = s_k + TILE_KEYS * 16;
+  float* s_bias = reinterpret_cast<float*>( s_v + TILE_KEYS * 16 ); // (head_cols, n_dist), times log2(e)
+
+  // all column blocks of a pair on one XCD, next to each other in time: its keys come into one L2 once; the longest first
+  const uint32_t xcd = blockIdx.x & 7, slot = blockIdx.x >> 3;
+  const uint32_t cb = col_blocks - 1 - slot % col_blocks;
+  const uint32_t pair = ( slot / col_blocks ) * 8 + xcd;
+  if ( pair >= n_pairs ) {
+    return;
+  }
+  const uint32_t per_group = s.group / head_cols;
+  const uint32_t ctx = pair / ( s.kv_heads * per_group );
+  const uint32_t g = pair / per_group % s.kv_heads;
+  const uint32_t h0 = g * s.group + pair % per_group * head_cols;
+  const uint8_t* base = static_cast<const uint8_t*>( wr.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  const __bf16* cache = reinterpret_cast<const __bf16*>( base + wr.offset );
+  const uint32_t start = wr.start_pos[ctx];
+  const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 31, g2 = lane >> 5;
+  const uint32_t tok_wg = cb * ( 128 / head_cols );
+  const uint32_t tok_last = min( wr.n_tokens, tok_wg + 128 / head_cols ) - 1;
+  const uint32_t colnum = wave * 32 + r;
+  const uint32_t tok = tok_wg + colnum / head_cols, hc = colnum % head_cols;
+  const bool col_ok = tok < wr.n_tokens;
+  const uint32_t pos = start + ( col_ok ? tok : tok_last ); // a column without a query does as the last one and is not stored
+  const uint32_t pos_first = start + tok_wg, pos_last = start + tok_last;
+
+  for ( uint32_t i = threadIdx.x; i < bias_floats; i += 256 ) {
+    s_bias[i] = bias[(uint64_t)h0 * s.n_dist + i] * LOG2E;
+  }
+
+  bf16x8 qb[KS];
+  {
+    const __bf16* qp = q + ( ( (uint64_t)ctx * wr.n_tokens + ( col_ok ? tok : tok_last ) ) * s.heads + h0 + hc ) * s.dpad;
+#pragma unroll
+    for ( int k = 0; k < KS; k++ ) {
+      const uint32_t ch = 2 * k + g2;
+      u32x4_t v = { 0, 0, 0, 0 };
+      if ( ch * 8 < s.dpad ) {
+        v = *(global_u32x4_t*)( qp + ch * 8 );
+      }
+      qb[k] = __builtin_bit_cast( bf16x8, v );
+    }
+  }
+
+  // tiles: kept keys [0, kept), then [first, pos_last]
+  const uint32_t first = pos_first + 1 > s.window ? pos_first + 1 - s.window : 0;
+  const uint32_t kept = min( s.keep_first, first );
+  const uint32_t kept_tiles = ( kept + TILE_KEYS - 1 ) / TILE_KEYS;
+  const uint32_t tiles = kept_tiles + ( pos_last + 1 - first + TILE_KEYS - 1 ) / TILE_KEYS;
+  auto tile_at = [&]( uint32_t i ) { return i < kept_tiles ? i * TILE_KEYS : first + ( i - kept_tiles ) * TILE_KEYS; };
+
+  // a thread's four 16-byte pieces of a tile of K and of V: row threadIdx / 16 + 16 i, chunk threadIdx % 16
+  const uint32_t ld_chunk = threadIdx.x & 15, ld_row = threadIdx.x >> 4;
+  u32x4_t rk[4], rv[4];
+  auto load = [&]( uint32_t i ) {
+    const uint32_t t0 = tile_at( i ), end = i < kept_tiles ? kept : pos_last + 1;
+#pragma unroll
+    for ( int k = 0; k < 4; k++ ) {
+      const uint32_t key = t0 + ld_row + 16 * k;
+      rk[k] = u32x4_t { 0, 0, 0, 0 };
+      rv[k] = u32x4_t { 0, 0, 0, 0 };
+      const __bf16* row = cache + (uint64_t)min( key, end - 1 ) * s.row_elems();
+      if ( key < end && ld_chunk * 8 < s.dpad && ld_chunk < 2 * KS ) {
+        rk[k] = *(global_u32x4_t*)( row + g * s.dpad + ld_chunk * 8 );
+      }
+      if ( key < end && ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB ) {
+        rv[k] = *(global_u32x4_t*)( row + s.k_elems() + g * s.vpad + ld_chunk * 8 );
+      }
+    }
+  };
+  auto store = [&] {
+#pragma unroll
+    for ( int k = 0; k < 4; k++ ) {
+      const uint32_t row = ld_row + 16 * k;
+      s_k[row * 16 + ( ld_chunk ^ ( row & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
+      s_v[row * 16 + ( ld_chunk ^ ( 4 * ( row & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+    }
+  };
+  const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
+  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ) * 16 ) + ( tr_q & 1 ) * 8;
+
+  mfma_f32x16 acc[VB];
+#pragma unroll
+  for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+    for ( int v = 0; v < 16; v++ ) {
+      acc[vb][v] = 0.0f;
+    }
+  }
+  float m = NO_KEY, l = 0.0f;
+  const float scale_log2e = s.scale * LOG2E;
+  const float* my_bias = s_bias + hc * s.n_dist;
+
+  load( 0 );
+  for ( uint32_t i = 0; i < tiles; i++ ) {
+    __syncthreads(); // the last tile's readers are done (and the bias table is written)
+    store();
+    __syncthreads();
+    if ( i + 1 < tiles ) {
+      load( i + 1 );
+    }
+    const uint32_t t0 = tile_at( i );
+    mfma_f32x16 st[2];
+#pragma unroll
+    for ( int sub = 0; sub < 2; sub++ ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        st[sub][v] = 0.0f;
+      }
+#pragma unroll
+      for ( int k = 0; k < KS; k++ ) {
+        const uint32_t row = 32 * sub + r;
+        const bf16x8 a = __builtin_bit_cast( bf16x8, s_k[row * 16 + ( ( 2 * k + g2 ) ^ ( row & 15 ) )] );
+        st[sub] = Mfma<__bf16>::k16( a, qb[k], st[sub] );
+      }
+    }
+    // ---- scale, bias by distance, mask (log2 domain)
+    const uint32_t key_l = t0 + 4 * g2; // key of register v: key_l + 32 sub + 8 (v / 4) + v % 4
+    const uint32_t last_key = t0 + TILE_KEYS - 1;
+    if ( bias_floats == 0 || ( last_key <= pos_first && pos_first - last_key >= s.n_dist - 1 ) ) { // every distance in the table's last row
+      const float b = bias_floats == 0 ? 0.0f : my_bias[s.n_dist - 1];
+#pragma unroll
+      for ( int sub = 0; sub < 2; sub++ ) {
+#pragma unroll
+        for ( int v = 0; v < 16; v++ ) {
+          st[sub][v] = st[sub][v] * scale_log2e + b;
+        }
+      }
+    } else {
+#pragma unroll
+      for ( int sub = 0; sub < 2; sub++ ) {
+#pragma unroll
+        for ( int v = 0; v < 16; v++ ) {
+          const uint32_t key = key_l + 32 * sub + 8 * ( v / 4 ) + v % 4;
+          st[sub][v] = st[sub][v] * scale_log2e + my_bias[min( pos - min( key, pos ), s.n_dist - 1 )];
+        }
+      }
+    }
+    const bool in_window = i >= kept_tiles;
+    const bool whole = in_window ? last_key <= pos_first && ( pos_last - t0 < s.window || last_key < s.keep_first ) : last_key < kept;
+    if ( !whole ) {
+      const uint32_t end = in_window ? 0xffffffffu : kept;
+#pragma unroll
+      for ( int sub = 0; sub < 2; sub++ ) {
+#pragma unroll
+        for ( int v = 0; v < 16; v++ ) {
+          const uint32_t key = key_l + 32 * sub + 8 * ( v / 4 ) + v % 4;
+          const bool seen = key <= pos && key < end && ( pos - key < s.window || key < s.keep_first );
+          st[sub][v] = seen ? st[sub][v] : -INFINITY;
+        }
+      }
+    }
+    // ---- online softmax
+    float mx4[4];
+#pragma unroll
+    for ( int c = 0; c < 4; c++ ) {
+      mx4[c] = st[c >> 1][8 * ( c & 1 )];
+#pragma unroll
+      for ( int e = 1; e < 8; e++ ) {
+        mx4[c] = fmaxf( mx4[c], st[c >> 1][8 * ( c & 1 ) + e] );
+      }
+    }
+    const float mx = half_wave_max( fmaxf( fmaxf( mx4[0], mx4[1] ), fmaxf( mx4[2], mx4[3] ) ) );
+    if ( __builtin_amdgcn_ballot_w64( mx > m + LAZY ) != 0 ) {
+      const float m_new = fmaxf( m, mx );
+      const float alpha = __builtin_amdgcn_exp2f( m - m_new );
+      m = m_new;
+      l *= alpha;
+#pragma unroll
+      for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+        for ( int v = 0; v < 16; v++ ) {
+          acc[vb][v] *= alpha;
+        }
+      }
+    }
+#pragma unroll
+    for ( int kk = 0; kk < 4; kk++ ) { // 16 keys
+      bf16x8 hi, lo;
+#pragma unroll
+      for ( int e = 0; e < 8; e++ ) {
+        const float p = __builtin_amdgcn_exp2f( st[kk >> 1][8 * ( kk & 1 ) + e] - m );
+        l += p;
+        hi[e] = (__bf16)p;
+        lo[e] = (__bf16)( p - (float)hi[e] );
+      }
+#pragma unroll
+      for ( int vb = 0; vb < VB; vb++ ) {
+        union
+        {
+          v4s half[2];
+          bf16x8 x;
+        } a;
+#pragma unroll
+        for ( int hf = 0; hf < 2; hf++ ) {
+          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
+        }
+        acc[vb] = Mfma<__bf16>::k16( a.x, lo, acc[vb] );
+        acc[vb] = Mfma<__bf16>::k16( a.x, hi, acc[vb] );
+      }
+    }
+  }
+  l += __shfl_xor( l, 32 );
+  if ( !col_ok ) {
+    return;
+  }
+  const float inv = 1.0f / l;
+  __bf16* o = out + ( ( (uint64_t)ctx * wr.n_tokens + tok ) * s.heads + h0 + hc ) * s.vdim;
+  const bool wide = s.vdim % 4 == 0;
+#pragma unroll
+  for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+    for ( int q4 = 0; q4 < 4; q4++ ) {
+      const uint32_t d = 32 * vb + 8 * q4 + 4 * g2;
+      union
+      {
+        __bf16 e[4];
+        uint2 raw;
+      } y;
+#pragma unroll
+      for ( int e = 0; e < 4; e++ ) {
+        y.e[e] = (__bf16)( acc[vb][4 * q4 + e] * inv );
+      }
+      if ( wide && d < s.vdim ) {
+        *reinterpret_cast<uint2*>( o + d ) = y.raw;
+      } else if ( !wide ) {
+        for ( int e = 0; e < 4; e++ ) {
+          if ( d + e < s.vdim ) {
+            o[d + e] = y.e[e];
+          }
+        }
+      }
+    }
+  }
+}
+
 WindowShape shape_of( const gh_window_attn* a )
 {
   WindowShape s;
@@ -405,6 +681,35 @@ int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, co
   return GH_OK;
 }
 
+// Whether the tile kernel serves a call; its launch.
+uint32_t tile_head_cols( const WindowShape& s ) { return s.group <= 32 && ( s.group & ( s.group - 1 ) ) == 0 ? s.group : 1; }
+bool tiles_applicable( const WindowShape& s, const float* bias, uint32_t n_tokens )
+{
+  return n_tokens >= 16 && s.dpad <= 128 && s.vpad <= 128 && ( bias == nullptr || (uint64_t)tile_head_cols( s ) * s.n_dist <= BIAS_LDS );
+}
+int attend_tiles( __bf16* out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t batch, hipStream_t st )
+{
+  const uint32_t head_cols = tile_head_cols( s );
+  const uint32_t col_blocks = ( wr.n_tokens + 128 / head_cols - 1 ) / ( 128 / head_cols );
+  const uint64_t n_pairs = batch * s.kv_heads * ( s.group / head_cols );
+  const uint64_t grid = ( n_pairs + 7 ) / 8 * 8 * col_blocks;
+  GH_REQUIRE( grid < ( 1ull << 31 ), "gh_attn_window: grid too large" );
+  const uint32_t bias_floats = bias == nullptr ? 0 : head_cols * s.n_dist;
+  const size_t lds = 2 * TILE_KEYS * 256 + bias_floats * sizeof( float );
+#define GH_WINDOW_TILES( KS, VB ) \
+  window_tiles_kernel<KS, VB><<<(unsigned)grid, 256, lds, st>>>( out, q, bias, wr, s, head_cols, col_blocks, (uint32_t)n_pairs, bias_floats )
+  if ( s.dpad <= 64 && s.vpad <= 64 ) {
+    GH_WINDOW_TILES( 4, 2 );
+  } else if ( s.vpad <= 64 ) {
+    GH_WINDOW_TILES( 8, 2 );
+  } else {
+    GH_WINDOW_TILES( 8, 4 );
+  }
+#undef GH_WINDOW_TILES
+  GH_LAUNCH_CHECK();
+  return GH_OK;
+}
+
 } // namespace
 } // namespace gh
 
@@ -467,6 +772,9 @@ int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const flo
   const uint32_t max_pos = max_start_pos + n_tokens - 1;
   if ( dt == GH_F32 ) {
     return attend_rows<float>( static_cast<float*>( out ), static_cast<const float*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+  }
+  if ( tiles_applicable( s, distance_bias_dev, n_tokens ) ) {
+    return attend_tiles( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, batch, as_stream( stream ) );
   }
   return attend_rows<__bf16>( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
 }

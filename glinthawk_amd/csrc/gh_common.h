@@ -161,6 +161,16 @@ __device__ __forceinline__ float wave_max( float v )
   return fmaxf( fmaxf( lane_value( v, 0 ), lane_value( v, 16 ) ), fmaxf( lane_value( v, 32 ), lane_value( v, 48 ) ) );
 }
 
+// Maximum of a lane's value and that of the lane 32 further on, in both lanes, without a trip through LDS.  (The two results are
+// copied to variables first: a bit cast straight from an element of the builtin's vector result reads element 0 whichever is named.)
+__device__ __forceinline__ float half_wave_max( float v )
+{
+  const unsigned bits = __builtin_bit_cast( unsigned, v );
+  const auto halves = __builtin_amdgcn_permlane32_swap( bits, bits, false, false );
+  const unsigned low = halves[0], high = halves[1];
+  return fmaxf( __builtin_bit_cast( float, low ), __builtin_bit_cast( float, high ) );
+}
+
 template<typename T>
 __device__ __forceinline__ float to_f32( T v );
 template<>

@@ -295,3 +295,28 @@ def test_stage_prefill_copies_overlapped_with_compute_equal_plain_call():
             np.testing.assert_allclose(ka.astype(np.float32), kb.astype(np.float32), rtol=4e-3, atol=4e-3)
     a.close()
     b.close()
+
+
+@pytest.mark.parametrize("shape", [MHA, GQA4], ids=["mha", "gqa4"])
+def test_prefill_one_key_stands_out(shape):
+    """A key whose score lies far above all others, at each place of a 16-key group in turn: whichever lane of the wave holds it, the
+    softmax has to take its reference point from it."""
+    T = 80
+    rng = np.random.default_rng(3)
+    hs, group = shape.head_size, shape.n_heads // shape.n_kv_heads
+    for j in (0, 3, 4, 7, 12, 15, 36, 63, 70):
+        arena = Arena(shape, 1, torch.float16, seed=9, std=0.05)
+        q = np.tile(rng.standard_normal((1, shape.dim)), (T, 1)).astype(np.float16)
+        for h in range(shape.n_kv_heads):
+            arena.host[0, j, h * hs:(h + 1) * hs] = 4 * q[0, h * group * hs:(h * group + 1) * hs]
+        arena.dev.copy_(torch.from_numpy(arena.host))
+        xb = torch.zeros((T, shape.dim), dtype=torch.float16, device="cuda")
+        ops.attn_prefill(torch.from_numpy(q).cuda(), ops.row_table([arena.layer_ptr(0)]), torch.tensor([0], dtype=torch.int32, device="cuda"), xb, T, 0, shape)
+        cfg, rows, pos = oracle_cfg(shape), [arena.host_layers_f32([True])[0]] * T, list(range(T))
+        att, want = np.zeros((T, shape.n_heads, shape.seq_len), np.float32), np.zeros((T, shape.dim), np.float32)
+        O.attention_0_gemm(cfg, q.astype(np.float32), rows, att, pos)
+        O.attention_softmax(cfg, att, pos)
+        O.attention_2_gemm(cfg, att, rows, want, pos)
+        got = xb.float().cpu().numpy()
+        assert np.isfinite(got).all(), f"key {j}"
+        assert_close(got, want, mean_rel=4e-3, what=f"key {j}")
