@@ -15,6 +15,10 @@
 namespace gh {
 namespace {
 
+// cache rows are reached through pointers out of a table: the cast names the address space, so that no flat loads are used
+typedef uint32_t u32x4_t __attribute__( ( ext_vector_type( 4 ) ) );
+typedef const u32x4_t __attribute__( ( address_space( 1 ) ) ) global_u32x4_t;
+
 struct WindowShape
 {
   uint32_t heads, kv_heads, group; // query heads, kv heads, query heads per kv head
@@ -34,61 +38,157 @@ struct WindowRows
 };
 
 // ---- q / k norm over the whole projection, cache append ------------------------------------------
-template<typename E, typename View>
-__global__ __launch_bounds__( 256 ) void window_append_kernel( E* __restrict__ q_out,
-                                                               View y,
-                                                               const E* __restrict__ bias,
-                                                               const E* __restrict__ q_norm,
-                                                               const E* __restrict__ k_norm,
-                                                               WindowRows wr,
-                                                               WindowShape s,
-                                                               float eps )
+// work-group = one token's q, its k or its v (blockIdx.y): columns of the product, normed where there is a norm, to padded heads
+struct AppendPart
 {
-  extern __shared__ float vals[]; // q and k of the row
-  __shared__ float s_red[2][4];
-  const uint64_t row = blockIdx.x;
+  uint32_t first, cols, dim, pad; // columns of the product; head size and its padded form
+  const void* norm;               // (cols) or NULL
+};
+
+template<typename E>
+__device__ __forceinline__ E* append_target( E* q_out, const WindowRows& wr, const WindowShape& s, uint64_t row )
+{
   const uint32_t ctx = (uint32_t)( row / wr.n_tokens ), tok = (uint32_t)( row % wr.n_tokens );
   uint8_t* base = static_cast<uint8_t*>( wr.rows[ctx] );
   if ( base == nullptr ) {
-    return;
+    return nullptr;
+  }
+  if ( blockIdx.y == 0 ) {
+    return q_out + row * s.heads * s.dpad;
   }
   E* cache = reinterpret_cast<E*>( base + wr.offset ) + (uint64_t)( wr.start_pos[ctx] + tok ) * s.row_elems();
-  const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim, nv = s.kv_heads * s.vdim;
-  float ssq = 0.0f, ssk = 0.0f;
-  for ( uint32_t c = threadIdx.x; c < nq + nk; c += blockDim.x ) {
-    const float v = y.at( row, c ) + ( bias != nullptr ? to_f32( bias[c] ) : 0.0f );
-    vals[c] = v;
-    if ( c < nq ) {
-      ssq += v * v;
-    } else {
-      ssk += v * v;
-    }
-  }
-  ssq = wave_sum( ssq );
-  ssk = wave_sum( ssk );
+  return cache + ( blockIdx.y == 1 ? 0 : s.k_elems() );
+}
+
+__device__ __forceinline__ float append_row_sum( float v, float* smem )
+{
+  v = wave_sum( v );
   if ( ( threadIdx.x & 63 ) == 0 ) {
-    s_red[0][threadIdx.x >> 6] = ssq;
-    s_red[1][threadIdx.x >> 6] = ssk;
+    smem[threadIdx.x >> 6] = v;
   }
   __syncthreads();
-  ssq = ( s_red[0][0] + s_red[0][1] ) + ( s_red[0][2] + s_red[0][3] );
-  ssk = ( s_red[1][0] + s_red[1][1] ) + ( s_red[1][2] + s_red[1][3] );
-  const float iq = q_norm != nullptr ? 1.0f / sqrtf( ssq / (float)nq + eps ) : 1.0f;
-  const float ik = k_norm != nullptr ? 1.0f / sqrtf( ssk / (float)nk + eps ) : 1.0f;
-  E* q = q_out + row * s.heads * s.dpad;
-  for ( uint32_t c = threadIdx.x; c < s.heads * s.dpad; c += blockDim.x ) {
-    const uint32_t h = c / s.dpad, e = c % s.dpad, src = h * s.dim + e;
-    q[c] = from_f32<E>( e < s.dim ? vals[src] * iq * ( q_norm != nullptr ? to_f32( q_norm[src] ) : 1.0f ) : 0.0f );
+  float total = 0.0f;
+  for ( uint32_t w = 0; w < blockDim.x / WAVE; w++ ) {
+    total += smem[w];
   }
-  for ( uint32_t c = threadIdx.x; c < s.k_elems(); c += blockDim.x ) {
-    const uint32_t h = c / s.dpad, e = c % s.dpad, src = h * s.dim + e;
-    cache[c] = from_f32<E>( e < s.dim ? vals[nq + src] * ik * ( k_norm != nullptr ? to_f32( k_norm[src] ) : 1.0f ) : 0.0f );
+  return total;
+}
+
+// head size, product columns and tables in groups of four; a thread owns NV groups, kept in registers across the norm
+template<typename E, typename View, int NV>
+__global__ __launch_bounds__( 1024 ) void window_append4_kernel( E* __restrict__ q_out, View y, const E* __restrict__ bias, AppendPart pq, AppendPart pk, AppendPart pv,
+                                                                 WindowRows wr, WindowShape s, float eps )
+{
+  __shared__ float smem[16];
+  const uint64_t row = blockIdx.x;
+  E* dst = append_target( q_out, wr, s, row );
+  if ( dst == nullptr ) {
+    return;
   }
-  for ( uint32_t c = threadIdx.x; c < s.kv_heads * s.vpad; c += blockDim.x ) {
-    const uint32_t h = c / s.vpad, e = c % s.vpad, src = nq + nk + h * s.vdim + e;
-    cache[s.k_elems() + c] = from_f32<E>( e < s.vdim ? y.at( row, src ) + ( bias != nullptr ? to_f32( bias[src] ) : 0.0f ) : 0.0f );
+  const AppendPart p = blockIdx.y == 0 ? pq : blockIdx.y == 1 ? pk : pv;
+  const E* norm = static_cast<const E*>( p.norm );
+  float4 v[NV], w[NV];
+  float ss = 0.0f;
+#pragma unroll
+  for ( int g = 0; g < NV; g++ ) {
+    const uint32_t c = ( g * blockDim.x + threadIdx.x ) * 4, at = c < p.cols ? c : 0;
+    v[g] = y.at4( row, p.first + at );
+    w[g] = norm != nullptr ? ProductView<E>::load4( norm + at ) : make_float4( 1.0f, 1.0f, 1.0f, 1.0f );
+    if ( bias != nullptr ) {
+      const float4 b = ProductView<E>::load4( bias + p.first + at );
+      v[g] = make_float4( v[g].x + b.x, v[g].y + b.y, v[g].z + b.z, v[g].w + b.w );
+    }
+    ss += c < p.cols ? v[g].x * v[g].x + v[g].y * v[g].y + v[g].z * v[g].z + v[g].w * v[g].w : 0.0f;
   }
-  (void)nv;
+  const float inv = norm != nullptr ? 1.0f / sqrtf( append_row_sum( ss, smem ) / (float)p.cols + eps ) : 1.0f;
+#pragma unroll
+  for ( int g = 0; g < NV; g++ ) {
+    const uint32_t c = ( g * blockDim.x + threadIdx.x ) * 4;
+    if ( c >= p.cols ) {
+      continue;
+    }
+    const uint32_t h = c / p.dim, e = c % p.dim;
+    union
+    {
+      E e[4];
+      uint2 half;
+      uint4 full;
+    } o;
+    o.e[0] = from_f32<E>( v[g].x * inv * w[g].x );
+    o.e[1] = from_f32<E>( v[g].y * inv * w[g].y );
+    o.e[2] = from_f32<E>( v[g].z * inv * w[g].z );
+    o.e[3] = from_f32<E>( v[g].w * inv * w[g].w );
+    E* at = dst + (uint64_t)h * p.pad + e;
+    if constexpr ( sizeof( E ) == 2 ) {
+      *reinterpret_cast<uint2*>( at ) = o.half;
+    } else {
+      *reinterpret_cast<uint4*>( at ) = o.full;
+    }
+    if ( e + 4 == p.dim ) {
+      for ( uint32_t z = p.dim; z < p.pad; z++ ) {
+        dst[(uint64_t)h * p.pad + z] = from_f32<E>( 0.0f );
+      }
+    }
+  }
+}
+
+// any sizes: the columns of the part pass through LDS
+template<typename E, typename View>
+__global__ __launch_bounds__( 256 ) void window_append_any_kernel( E* __restrict__ q_out, View y, const E* __restrict__ bias, AppendPart pq, AppendPart pk, AppendPart pv,
+                                                                   WindowRows wr, WindowShape s, float eps )
+{
+  extern __shared__ float vals[];
+  __shared__ float smem[4];
+  const uint64_t row = blockIdx.x;
+  E* dst = append_target( q_out, wr, s, row );
+  if ( dst == nullptr ) {
+    return;
+  }
+  const AppendPart p = blockIdx.y == 0 ? pq : blockIdx.y == 1 ? pk : pv;
+  const E* norm = static_cast<const E*>( p.norm );
+  float ss = 0.0f;
+  for ( uint32_t c = threadIdx.x; c < p.cols; c += blockDim.x ) {
+    const float v = y.at( row, p.first + c ) + ( bias != nullptr ? to_f32( bias[p.first + c] ) : 0.0f );
+    vals[c] = v;
+    ss += v * v;
+  }
+  const float total = append_row_sum( ss, smem ); // (also the barrier in front of the reads below)
+  const float inv = norm != nullptr ? 1.0f / sqrtf( total / (float)p.cols + eps ) : 1.0f;
+  for ( uint32_t c = threadIdx.x; c < p.cols / p.dim * p.pad; c += blockDim.x ) {
+    const uint32_t h = c / p.pad, e = c % p.pad, src = h * p.dim + e;
+    dst[c] = from_f32<E>( e < p.dim ? vals[src] * inv * ( norm != nullptr ? to_f32( norm[src] ) : 1.0f ) : 0.0f );
+  }
+}
+
+template<typename E, typename View>
+int launch_append( E* q, const View& y, const E* bias, const void* q_norm, const void* k_norm, float eps, const WindowRows& wr, const WindowShape& s, uint64_t rows,
+                   hipStream_t st )
+{
+  const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim, nv = s.kv_heads * s.vdim;
+  const AppendPart pq { 0, nq, s.dim, s.dpad, q_norm }, pk { nq, nk, s.dim, s.dpad, k_norm }, pv { nq + nk, nv, s.vdim, s.vpad, nullptr };
+  const uint32_t most = std::max( { nq, nk, nv } );
+  const dim3 grid( (unsigned)rows, 3 );
+  const uintptr_t tables = reinterpret_cast<uintptr_t>( bias ) | reinterpret_cast<uintptr_t>( q_norm ) | reinterpret_cast<uintptr_t>( k_norm );
+  if ( s.dim % 4 == 0 && s.vdim % 4 == 0 && y.stride % 4 == 0 && ( tables & 15u ) == 0 && most <= 32768 ) {
+    const uint32_t groups = most / 4;
+    const uint32_t want = rows >= 1024 ? ( groups + 3 ) / 4 : groups;
+    const uint32_t threads = std::min<uint32_t>( 1024, std::max<uint32_t>( 64, ( want + 63 ) / 64 * 64 ) );
+    const uint32_t per = ( groups + threads - 1 ) / threads;
+    if ( per <= 1 ) {
+      window_append4_kernel<E, View, 1><<<grid, threads, 0, st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+    } else if ( per <= 2 ) {
+      window_append4_kernel<E, View, 2><<<grid, threads, 0, st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+    } else if ( per <= 4 ) {
+      window_append4_kernel<E, View, 4><<<grid, threads, 0, st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+    } else {
+      window_append4_kernel<E, View, 8><<<grid, threads, 0, st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+    }
+  } else {
+    GH_REQUIRE( most <= 15 * 1024, "gh_matmul_window_append: the heads of a token do not fit in LDS" );
+    window_append_any_kernel<E, View><<<grid, 256, most * sizeof( float ), st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+  }
+  GH_LAUNCH_CHECK();
+  return GH_OK;
 }
 
 // ---- visible keys ------------------------------------------------------------------------------
@@ -115,13 +215,13 @@ __device__ __forceinline__ void load8( float out[8], const E* p )
       uint4 raw;
       E e[8];
     } u;
-    u.raw = *reinterpret_cast<const uint4*>( p );
+    u.raw = __builtin_bit_cast( uint4, *(global_u32x4_t*)( p ) );
 #pragma unroll
     for ( int i = 0; i < 8; i++ ) {
       out[i] = to_f32( u.e[i] );
     }
   } else {
-    const float4 a = *reinterpret_cast<const float4*>( p ), b = *reinterpret_cast<const float4*>( p + 4 );
+    const float4 a = __builtin_bit_cast( float4, *(global_u32x4_t*)( p ) ), b = __builtin_bit_cast( float4, *(global_u32x4_t*)( p + 4 ) );
     out[0] = a.x, out[1] = a.y, out[2] = a.z, out[3] = a.w, out[4] = b.x, out[5] = b.y, out[6] = b.z, out[7] = b.w;
   }
 }
@@ -178,52 +278,74 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
       }
     }
   }
-  for ( uint32_t i0 = k_begin + wave * 4; i0 < k_end; i0 += 16 ) {
-    const uint32_t idx = i0 + g4;
-    const bool live = idx < k_end;
-    const uint32_t j = vis.key( live ? idx : i0 );
-    const E* kr = cache + (uint64_t)j * s.row_elems() + g * s.dpad;
-    const E* vr = cache + (uint64_t)j * s.row_elems() + s.k_elems() + g * s.vpad;
-    float kv[NC][8], vv[NC][8];
+  // U keys per 16-lane group and step: all their loads go out before the first is used.  A key past the end reads the step's first again
+  // and gets no weight.
+  constexpr uint32_t U = HQ * NC >= 4 ? 2 : 4;
+  const uint32_t at_k = g * s.dpad, at_v = s.k_elems() + g * s.vpad;
+  for ( uint32_t i0 = k_begin + wave * 4 * U; i0 < k_end; i0 += 16 * U ) {
+    float kv[U][NC][8], vv[U][NC][8];
+    uint32_t dist[U];
+    bool live[U];
 #pragma unroll
-    for ( int c = 0; c < NC; c++ ) {
-      const uint32_t at = c * 128 + l16 * 8;
-#pragma unroll
-      for ( int e = 0; e < 8; e++ ) {
-        kv[c][e] = 0.0f;
-        vv[c][e] = 0.0f;
-      }
-      if ( at < s.dpad ) {
-        load8( kv[c], kr + at );
-      }
-      if ( at < s.vpad ) {
-        load8( vv[c], vr + at );
-      }
-    }
-    const uint32_t dist = min( pos - j, s.n_dist - 1 );
-#pragma unroll
-    for ( int h = 0; h < HQ; h++ ) {
-      float dot = 0.0f;
+    for ( uint32_t u = 0; u < U; u++ ) {
+      const uint32_t idx = i0 + 4 * u + g4;
+      live[u] = idx < k_end;
+      const uint32_t j = vis.key( live[u] ? idx : i0 );
+      dist[u] = min( pos - j, s.n_dist - 1 );
+      const E* row_j = cache + (uint64_t)j * s.row_elems();
 #pragma unroll
       for ( int c = 0; c < NC; c++ ) {
+        const uint32_t at = c * 128 + l16 * 8;
 #pragma unroll
         for ( int e = 0; e < 8; e++ ) {
-          dot += qv[h][c][e] * kv[c][e];
+          kv[u][c][e] = 0.0f;
+          vv[u][c][e] = 0.0f;
+        }
+        if ( at < s.dpad ) {
+          load8( kv[u][c], row_j + at_k + at );
+        }
+        if ( at < s.vpad ) {
+          load8( vv[u][c], row_j + at_v + at );
         }
       }
-      dot = row16_sum( dot );
-      const float b = bias != nullptr && (uint32_t)h < nh ? bias[(uint64_t)( h0 + h ) * s.n_dist + dist] : 0.0f;
-      const float score = live ? dot * s.scale + b : NO_KEY;
-      const float m_new = fmaxf( mx[h], score );
+    }
+#pragma unroll
+    for ( int h = 0; h < HQ; h++ ) {
+      float score[U];
+      float m_new = mx[h];
+#pragma unroll
+      for ( uint32_t u = 0; u < U; u++ ) {
+        float dot = 0.0f;
+#pragma unroll
+        for ( int c = 0; c < NC; c++ ) {
+#pragma unroll
+          for ( int e = 0; e < 8; e++ ) {
+            dot += qv[h][c][e] * kv[u][c][e];
+          }
+        }
+        const float b = bias != nullptr && (uint32_t)h < nh ? bias[(uint64_t)( h0 + h ) * s.n_dist + dist[u]] : 0.0f;
+        score[u] = live[u] ? row16_sum( dot ) * s.scale + b : NO_KEY;
+        m_new = fmaxf( m_new, score[u] );
+      }
       const float old = __expf( mx[h] - m_new );
-      const float p = live ? __expf( score - m_new ) : 0.0f;
       mx[h] = m_new;
-      sum[h] = sum[h] * old + p;
+      float p[U], p_sum = 0.0f;
+#pragma unroll
+      for ( uint32_t u = 0; u < U; u++ ) {
+        p[u] = live[u] ? __expf( score[u] - m_new ) : 0.0f;
+        p_sum += p[u];
+      }
+      sum[h] = sum[h] * old + p_sum;
 #pragma unroll
       for ( int c = 0; c < NC; c++ ) {
 #pragma unroll
         for ( int e = 0; e < 8; e++ ) {
-          acc[h][c][e] = acc[h][c][e] * old + p * vv[c][e];
+          float a = acc[h][c][e] * old;
+#pragma unroll
+          for ( uint32_t u = 0; u < U; u++ ) {
+            a += p[u] * vv[u][c][e];
+          }
+          acc[h][c][e] = a;
         }
       }
     }
@@ -331,12 +453,10 @@ __global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ ou
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr float LAZY = 8.0f; // the reference point of a column's exponentials moves when its maximum has grown by 2^LAZY
 constexpr uint32_t TILE_KEYS = 64;
-constexpr uint32_t BIAS_LDS = 4096; // floats of bias table a work-group can hold
+constexpr uint32_t BIAS_LDS = 8192; // floats of bias table a work-group can hold
 typedef __attribute__( ( address_space( 3 ) ) ) char lds_char;
 typedef short v4s __attribute__( ( ext_vector_type( 4 ) ) );
 typedef __attribute__( ( address_space( 3 ) ) ) v4s* lds_v4s;
-typedef uint32_t u32x4_t __attribute__( ( ext_vector_type( 4 ) ) );
-typedef const u32x4_t __attribute__( ( address_space( 1 ) ) ) global_u32x4_t;
 typedef Mfma<__bf16>::x8 bf16x8;
 
 // KS: steps of 16 of the query/key size; VB: blocks of 32 of the value size
@@ -682,7 +802,14 @@ int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, co
 }
 
 // Whether the tile kernel serves a call; its launch.
-uint32_t tile_head_cols( const WindowShape& s ) { return s.group <= 32 && ( s.group & ( s.group - 1 ) ) == 0 ? s.group : 1; }
+uint32_t tile_head_cols( const WindowShape& s )
+{
+  uint32_t cols = s.group <= 32 && ( s.group & ( s.group - 1 ) ) == 0 ? s.group : 1;
+  while ( cols > 1 && (uint64_t)cols * s.n_dist > BIAS_LDS ) { // as many as have their bias tables fit
+    cols /= 2;
+  }
+  return cols;
+}
 bool tiles_applicable( const WindowShape& s, const float* bias, uint32_t n_tokens )
 {
   return n_tokens >= 16 && s.dpad <= 128 && s.vpad <= 128 && ( bias == nullptr || (uint64_t)tile_head_cols( s ) * s.n_dist <= BIAS_LDS );
@@ -737,8 +864,6 @@ int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const voi
   GH_REQUIRE( shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_matmul_window_append: bad shape" );
   const WindowShape s = shape_of( a );
   const uint64_t r = (uint64_t)s.heads * s.dim + (uint64_t)s.kv_heads * ( s.dim + s.vdim );
-  const size_t lds = ( (uint64_t)s.heads + s.kv_heads ) * s.dim * sizeof( float );
-  GH_REQUIRE( lds <= 63 * 1024, "gh_matmul_window_append: query and key of a token do not fit in LDS" );
   hipStream_t st = as_stream( stream );
   Product y;
   if ( int rc = make_product( x, wqkv, width, r, rows, dt, false, st, &y ) ) {
@@ -747,10 +872,7 @@ int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const voi
   const WindowRows wr { context_rows_dev, cache_offset, start_pos_dev, n_tokens };
   return with_product( dt, y, [&]( auto tag, auto view ) -> int {
     using E = decltype( tag );
-    window_append_kernel<E><<<(unsigned)rows, 256, lds, st>>>( static_cast<E*>( q ), view, static_cast<const E*>( bias ), static_cast<const E*>( q_norm ),
-                                                              static_cast<const E*>( k_norm ), wr, s, eps );
-    GH_LAUNCH_CHECK();
-    return GH_OK;
+    return launch_append<E>( static_cast<E*>( q ), view, static_cast<const E*>( bias ), q_norm, k_norm, eps, wr, s, rows, st );
   } );
 }
 

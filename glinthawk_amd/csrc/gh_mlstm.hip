@@ -41,14 +41,34 @@ struct MlstmCols
   uint32_t q, k, v, g, i, f;
 };
 
+// `gates`: (rows, 2 heads) fp32, the log input gates of a token's heads, then its log forget gates (mlstm_gates_kernel)
 template<typename E, typename View>
 struct MlstmIn
 {
   View main;
-  ProductView<float> gates;
+  const float* gates;
   MlstmCols col;
-  const E *bias_i, *bias_f;
 };
+
+template<typename E>
+__global__ __launch_bounds__( 256 ) void mlstm_gates_kernel( float* __restrict__ out,
+                                                             ProductView<float> y,
+                                                             MlstmCols col,
+                                                             const E* __restrict__ bias_i,
+                                                             const E* __restrict__ bias_f,
+                                                             uint32_t heads,
+                                                             uint64_t rows,
+                                                             float cap )
+{
+  const uint64_t total = rows * 2 * heads, stride = (uint64_t)gridDim.x * blockDim.x;
+  for ( uint64_t i = (uint64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += stride ) {
+    const uint64_t row = i / ( 2 * heads );
+    const uint32_t g = (uint32_t)( i % ( 2 * heads ) ), h = g < heads ? g : g - heads;
+    const E* bias = g < heads ? bias_i : bias_f;
+    const float z = soft_cap( y.at( row, ( g < heads ? col.i : col.f ) + h ) + ( bias != nullptr ? to_f32( bias[h] ) : 0.0f ), cap );
+    out[i] = g < heads ? z : log_sigmoid( z );
+  }
+}
 
 struct MlstmState
 {
@@ -104,7 +124,6 @@ __global__ __launch_bounds__( 256 ) void mlstm_walk_kernel( float* __restrict__ 
     n_s[d] = fresh ? 0.0f : n_in[d];
   }
   float m = fresh ? 0.0f : *m_in;
-  const float bi = in.bias_i != nullptr ? to_f32( in.bias_i[h] ) : 0.0f, bf = in.bias_f != nullptr ? to_f32( in.bias_f[h] ) : 0.0f;
 
   for ( uint32_t tok = 0; tok < st.n_tokens; tok++ ) {
     const uint64_t row_in = (uint64_t)ctx * st.n_tokens + tok;
@@ -117,8 +136,7 @@ __global__ __launch_bounds__( 256 ) void mlstm_walk_kernel( float* __restrict__ 
       const uint32_t c = slice * SLICE + t;
       v_s[t] = c < s.vdim ? in.main.at( row_in, in.col.v + h * s.vdim + c ) : 0.0f;
     }
-    const float gi = soft_cap( in.gates.at( row_in, in.col.i + h ) + bi, s.cap );
-    const float gf = log_sigmoid( soft_cap( in.gates.at( row_in, in.col.f + h ) + bf, s.cap ) );
+    const float gi = in.gates[row_in * 2 * s.heads + h], gf = in.gates[( row_in * 2 + 1 ) * s.heads + h];
     const float m_new = fmaxf( gf + m, gi );
     const float decay = expf( gf + m - m_new ), inp = expf( gi - m_new );
     m = m_new;
@@ -271,7 +289,7 @@ __device__ __forceinline__ double last_lane_f64( double v )
 // DT: 32-row tiles of S, dim <= 32 DT.  dim % 8 == 0, vdim % 8 == 0, 16-byte aligned product rows.
 template<int DT>
 __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restrict__ o_out, float* __restrict__ nm_out, MlstmIn<__bf16, ProductView<__bf16>> in, MlstmState st,
-                                                                MlstmShape s )
+                                                                MlstmShape s, uint32_t slices, uint32_t n_pairs )
 {
   constexpr uint32_t RB = DT * 64; // bytes of a q or k row in LDS
   __shared__ uint4 s_k[CHUNK * RB / 16], s_q[CHUNK * RB / 16];
@@ -282,7 +300,12 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
   __shared__ __attribute__( ( aligned( 16 ) ) ) float s_a[2][CHUNK];   // factor of the state in front of the chunk, per token
   __shared__ __attribute__( ( aligned( 16 ) ) ) float s_inv[2][CHUNK]; // one over the denominator
 
-  const uint32_t slice = blockIdx.x, h = blockIdx.y, ctx = blockIdx.z;
+  // the slices of a (context, head) read the same q and k: all on one XCD, next to each other in time
+  const uint32_t pair = ( blockIdx.x >> 3 ) / slices * 8 + ( blockIdx.x & 7 ), slice = ( blockIdx.x >> 3 ) % slices;
+  if ( pair >= n_pairs ) {
+    return;
+  }
+  const uint32_t h = pair % s.heads, ctx = pair / s.heads;
   uint8_t* base = static_cast<uint8_t*>( st.rows[ctx] );
   if ( base == nullptr ) {
     return;
@@ -311,7 +334,6 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
     s_n[wave][d] = !fresh && d < s.dim ? n_in[d] : 0.0f;
   }
   double m0 = fresh ? 0.0 : (double)m_mem;
-  const float bi = in.bias_i != nullptr ? to_f32( in.bias_i[h] ) : 0.0f, bf = in.bias_f != nullptr ? to_f32( in.bias_f[h] ) : 0.0f;
   const uint64_t row_first = (uint64_t)ctx * st.n_tokens;
   const uint32_t ld_bytes = (uint32_t)( in.main.stride * 2 );
 
@@ -385,8 +407,7 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
     // gates: lane = token
     const bool live = lane < rows;
     const uint64_t grow = row_first + t0 + ( live ? lane : 0 );
-    const float gi = soft_cap( in.gates.at( grow, in.col.i + h ) + bi, s.cap );
-    const float gf = log_sigmoid( soft_cap( in.gates.at( grow, in.col.f + h ) + bf, s.cap ) );
+    const float gi = in.gates[grow * 2 * s.heads + h], gf = in.gates[( grow * 2 + 1 ) * s.heads + h];
     double b = live ? (double)gf : 0.0;
 #pragma unroll
     for ( int by = 1; by < 64; by *= 2 ) {
@@ -591,8 +612,8 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
   }
 }
 
-// one work-group per token, one wave per head in turn
-template<typename E, typename View>
+// one wave per (token, head); V: columns at a time
+template<typename E, typename View, int V>
 __global__ __launch_bounds__( 256 ) void mlstm_finish_kernel( E* __restrict__ out,
                                                               const float* __restrict__ o,
                                                               const float* __restrict__ nm,
@@ -602,36 +623,66 @@ __global__ __launch_bounds__( 256 ) void mlstm_finish_kernel( E* __restrict__ ou
                                                               MlstmShape s )
 {
   const uint64_t row = blockIdx.x;
+  const uint32_t h = blockIdx.y * 4 + ( threadIdx.x >> 6 ), lane = threadIdx.x & 63;
   const uint32_t ctx = (uint32_t)( row / st.n_tokens ), tok = (uint32_t)( row % st.n_tokens );
   uint8_t* base = static_cast<uint8_t*>( st.rows[ctx] );
-  if ( base == nullptr ) {
+  if ( base == nullptr || h >= s.heads ) {
     return;
   }
-  const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  for ( uint32_t h = wave; h < s.heads; h += 4 ) {
-    const float* oh = o + row * s.heads * s.vdim + (uint64_t)h * s.vdim;
+  const float* oh = o + row * s.heads * s.vdim + (uint64_t)h * s.vdim;
+  E* dst = out + row * s.heads * s.vdim + (uint64_t)h * s.vdim;
+  if constexpr ( V == 4 ) { // vdim <= 1024, everything in groups of four
+    float4 v[4], g[4], w[4];
+    float ss = 0.0f;
+#pragma unroll
+    for ( int k = 0; k < 4; k++ ) {
+      const uint32_t c = ( k * 64 + lane ) * 4, at = c < s.vdim ? c : 0;
+      v[k] = *reinterpret_cast<const float4*>( oh + at );
+      g[k] = in.main.at4( row, in.col.g + h * s.vdim + at );
+      w[k] = ProductView<E>::load4( norm + h * s.vdim + at );
+      ss += c < s.vdim ? v[k].x * v[k].x + v[k].y * v[k].y + v[k].z * v[k].z + v[k].w * v[k].w : 0.0f;
+    }
+    const float inv = 1.0f / sqrtf( wave_sum( ss ) / (float)s.vdim + s.eps );
+#pragma unroll
+    for ( int k = 0; k < 4; k++ ) {
+      const uint32_t c = ( k * 64 + lane ) * 4;
+      union
+      {
+        E e[4];
+        uint2 half;
+        uint4 full;
+      } y;
+      y.e[0] = from_f32<E>( v[k].x * inv * w[k].x / ( 1.0f + expf( -g[k].x ) ) );
+      y.e[1] = from_f32<E>( v[k].y * inv * w[k].y / ( 1.0f + expf( -g[k].y ) ) );
+      y.e[2] = from_f32<E>( v[k].z * inv * w[k].z / ( 1.0f + expf( -g[k].z ) ) );
+      y.e[3] = from_f32<E>( v[k].w * inv * w[k].w / ( 1.0f + expf( -g[k].w ) ) );
+      if ( c < s.vdim ) {
+        if constexpr ( sizeof( E ) == 2 ) {
+          *reinterpret_cast<uint2*>( dst + c ) = y.half;
+        } else {
+          *reinterpret_cast<uint4*>( dst + c ) = y.full;
+        }
+      }
+    }
+  } else {
     float ss = 0.0f;
     for ( uint32_t c = lane; c < s.vdim; c += 64 ) {
       ss += oh[c] * oh[c];
     }
     const float inv = 1.0f / sqrtf( wave_sum( ss ) / (float)s.vdim + s.eps );
     for ( uint32_t c = lane; c < s.vdim; c += 64 ) {
-      const uint32_t hc = h * s.vdim + c;
-      const float g = in.main.at( row, in.col.g + hc );
-      out[row * s.heads * s.vdim + hc] = from_f32<E>( oh[c] * inv * to_f32( norm[hc] ) / ( 1.0f + expf( -g ) ) );
+      const float g = in.main.at( row, in.col.g + h * s.vdim + c );
+      dst[c] = from_f32<E>( oh[c] * inv * to_f32( norm[h * s.vdim + c] ) / ( 1.0f + expf( -g ) ) );
     }
   }
   if ( tok + 1 == st.n_tokens ) {
     float* S = reinterpret_cast<float*>( base + st.offset );
-    for ( uint32_t h = 0; h < s.heads; h++ ) {
-      const float* src = nm + ( (uint64_t)ctx * s.heads + h ) * ( s.dim + 1 );
-      for ( uint32_t d = threadIdx.x; d <= s.dim; d += blockDim.x ) {
-        if ( d < s.dim ) {
-          S[s.n_off() + (uint64_t)h * s.dim + d] = src[d];
-        } else {
-          S[s.m_off() + h] = src[d];
-        }
-      }
+    const float* src = nm + ( (uint64_t)ctx * s.heads + h ) * ( s.dim + 1 );
+    for ( uint32_t d = lane; d < s.dim; d += 64 ) {
+      S[s.n_off() + (uint64_t)h * s.dim + d] = src[d];
+    }
+    if ( lane == 0 ) {
+      S[s.m_off() + h] = src[s.dim];
     }
   }
 }
@@ -708,26 +759,33 @@ int gh_mlstm_forward( void* out, const void* x, const void* w, uint64_t width, c
   }
   void* scratch = nullptr;
   const uint64_t o_bytes = ( rows * hv * sizeof( float ) + 255 ) / 256 * 256;
-  if ( int rc = stream_scratch( st, SCRATCH_MIXER, o_bytes + batch * s.heads * ( s.dim + 1ull ) * sizeof( float ), 1ull << 20, &scratch ) ) {
+  const uint64_t nm_bytes = ( batch * s.heads * ( s.dim + 1ull ) * sizeof( float ) + 255 ) / 256 * 256;
+  if ( int rc = stream_scratch( st, SCRATCH_MIXER, o_bytes + nm_bytes + rows * 2 * s.heads * sizeof( float ), 1ull << 20, &scratch ) ) {
     return rc;
   }
   float* o = static_cast<float*>( scratch );
   float* nm = reinterpret_cast<float*>( static_cast<char*>( scratch ) + o_bytes );
+  float* log_gates = reinterpret_cast<float*>( static_cast<char*>( scratch ) + o_bytes + nm_bytes );
   const MlstmState state { context_rows_dev, state_offset, start_pos_dev, n_tokens };
   return with_product( dt, y, [&]( auto tag, auto view ) -> int {
     using E = decltype( tag );
     using View = decltype( view );
-    const MlstmIn<E, View> in { view, ProductView<float>( gates ), col, static_cast<const E*>( bias_i ), static_cast<const E*>( bias_f ) };
+    mlstm_gates_kernel<E><<<(unsigned)std::min<uint64_t>( ( rows * 2 * s.heads + 255 ) / 256, 4096 ), 256, 0, st>>>(
+      log_gates, ProductView<float>( gates ), col, static_cast<const E*>( bias_i ), static_cast<const E*>( bias_f ), s.heads, rows, s.cap );
+    GH_LAUNCH_CHECK();
+    const MlstmIn<E, View> in { view, log_gates, col };
     const dim3 grid( ( s.vpad + SLICE - 1 ) / SLICE, s.heads, (unsigned)batch );
     bool walked = false;
     if constexpr ( std::is_same_v<View, ProductView<__bf16>> ) {
       if ( chunked ) {
+        const uint32_t n_pairs = (uint32_t)batch * s.heads;
+        const unsigned groups = ( n_pairs + 7 ) / 8 * 8 * grid.x;
         if ( s.dim <= 64 ) {
-          mlstm_chunk_kernel<2><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+          mlstm_chunk_kernel<2><<<groups, 128, 0, st>>>( o, nm, in, state, s, grid.x, n_pairs );
         } else if ( s.dim <= 128 ) {
-          mlstm_chunk_kernel<4><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+          mlstm_chunk_kernel<4><<<groups, 128, 0, st>>>( o, nm, in, state, s, grid.x, n_pairs );
         } else {
-          mlstm_chunk_kernel<8><<<grid, 128, 0, st>>>( o, nm, in, state, s );
+          mlstm_chunk_kernel<8><<<groups, 128, 0, st>>>( o, nm, in, state, s, grid.x, n_pairs );
         }
         walked = true;
       }
@@ -745,7 +803,13 @@ int gh_mlstm_forward( void* out, const void* x, const void* w, uint64_t width, c
       mlstm_walk_kernel<E, View, 0><<<grid, 256, lds, st>>>( o, nm, in, state, s );
     }
     GH_LAUNCH_CHECK();
-    mlstm_finish_kernel<E, View><<<(unsigned)rows, 256, 0, st>>>( static_cast<E*>( out ), o, nm, in, static_cast<const E*>( norm ), state, s );
+    const dim3 finish( (unsigned)rows, ( s.heads + 3 ) / 4 );
+    if ( s.vdim % 4 == 0 && s.vdim <= 1024 && view.stride % 4 == 0 && col.g % 4 == 0 && ( reinterpret_cast<uintptr_t>( norm ) & 15u ) == 0
+         && ( reinterpret_cast<uintptr_t>( out ) & 15u ) == 0 ) {
+      mlstm_finish_kernel<E, View, 4><<<finish, 256, 0, st>>>( static_cast<E*>( out ), o, nm, in, static_cast<const E*>( norm ), state, s );
+    } else {
+      mlstm_finish_kernel<E, View, 1><<<finish, 256, 0, st>>>( static_cast<E*>( out ), o, nm, in, static_cast<const E*>( norm ), state, s );
+    }
     GH_LAUNCH_CHECK();
     return GH_OK;
   } );

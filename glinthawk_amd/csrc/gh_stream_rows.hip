@@ -5,6 +5,7 @@
 #include "gh_product.h"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace gh {
 namespace {
@@ -259,43 +260,55 @@ __device__ __forceinline__ float activate( float z, int act )
   return z / ( 1.0f + ( sizeof( E ) == 4 ? expf( -z ) : __expf( -z ) ) );
 }
 
+// grid: (column groups of a row / 256, rows); V columns a thread: 8 (rounded products), 4 or 1
 template<typename E, typename View, int V>
-__global__ __launch_bounds__( 256 ) void gate_rows_kernel( E* __restrict__ hb, View y, const E* __restrict__ bias, uint32_t hidden, uint64_t rows, int act )
+__global__ __launch_bounds__( 256 ) void gate_rows_kernel( E* __restrict__ hb, View y, const E* __restrict__ bias, uint32_t hidden, int act )
 {
-  const uint32_t per_row = hidden / V;
-  const uint64_t total = rows * per_row, stride = (uint64_t)gridDim.x * blockDim.x;
-  for ( uint64_t i = (uint64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += stride ) {
-    const uint64_t row = i / per_row;
-    const uint32_t c = (uint32_t)( i % per_row ) * V;
-    if constexpr ( V == 4 ) {
-      float4 g = y.at4( row, c ), u = y.at4( row, hidden + c );
-      if ( bias != nullptr ) {
-        const float4 bg = load4_e<E>( bias, c ), bu = load4_e<E>( bias, hidden + c );
-        g = make_float4( g.x + bg.x, g.y + bg.y, g.z + bg.z, g.w + bg.w );
-        u = make_float4( u.x + bu.x, u.y + bu.y, u.z + bu.z, u.w + bu.w );
+  const uint64_t row = blockIdx.y;
+  const uint32_t c = ( blockIdx.x * 256 + threadIdx.x ) * V;
+  if ( c >= hidden ) {
+    return;
+  }
+  if constexpr ( V == 1 ) {
+    float g = y.at( row, c ), u = y.at( row, hidden + c );
+    if ( bias != nullptr ) {
+      g += to_f32( bias[c] );
+      u += to_f32( bias[hidden + c] );
+    }
+    hb[row * hidden + c] = from_f32<E>( activate<E>( g, act ) * u );
+  } else {
+    float g[V], u[V];
+#pragma unroll
+    for ( int k = 0; k < V; k += 4 ) {
+      const float4 a = y.at4( row, c + k ), b = y.at4( row, hidden + c + k );
+      g[k] = a.x, g[k + 1] = a.y, g[k + 2] = a.z, g[k + 3] = a.w;
+      u[k] = b.x, u[k + 1] = b.y, u[k + 2] = b.z, u[k + 3] = b.w;
+    }
+    if ( bias != nullptr ) {
+#pragma unroll
+      for ( int k = 0; k < V; k += 4 ) {
+        const float4 a = load4_e<E>( bias, c + k ), b = load4_e<E>( bias, hidden + c + k );
+        g[k] += a.x, g[k + 1] += a.y, g[k + 2] += a.z, g[k + 3] += a.w;
+        u[k] += b.x, u[k + 1] += b.y, u[k + 2] += b.z, u[k + 3] += b.w;
       }
-      union
-      {
-        E e[4];
-        uint2 half;
-        uint4 full;
-      } o;
-      o.e[0] = from_f32<E>( activate<E>( g.x, act ) * u.x );
-      o.e[1] = from_f32<E>( activate<E>( g.y, act ) * u.y );
-      o.e[2] = from_f32<E>( activate<E>( g.z, act ) * u.z );
-      o.e[3] = from_f32<E>( activate<E>( g.w, act ) * u.w );
-      if constexpr ( sizeof( E ) == 2 ) {
-        *reinterpret_cast<uint2*>( hb + row * hidden + c ) = o.half;
-      } else {
-        *reinterpret_cast<uint4*>( hb + row * hidden + c ) = o.full;
-      }
+    }
+    union
+    {
+      E e[V];
+      uint2 half[V * sizeof( E ) / 8];
+      uint4 full[( V * sizeof( E ) + 15 ) / 16];
+    } o;
+#pragma unroll
+    for ( int k = 0; k < V; k++ ) {
+      o.e[k] = from_f32<E>( activate<E>( g[k], act ) * u[k] );
+    }
+    if constexpr ( V * sizeof( E ) == 8 ) {
+      *reinterpret_cast<uint2*>( hb + row * hidden + c ) = o.half[0];
     } else {
-      float g = y.at( row, c ), u = y.at( row, hidden + c );
-      if ( bias != nullptr ) {
-        g += to_f32( bias[c] );
-        u += to_f32( bias[hidden + c] );
+#pragma unroll
+      for ( uint32_t k = 0; k < V * sizeof( E ) / 16; k++ ) {
+        reinterpret_cast<uint4*>( hb + row * hidden + c )[k] = o.full[k];
       }
-      hb[row * hidden + c] = from_f32<E>( activate<E>( g, act ) * u );
     }
   }
 }
@@ -415,10 +428,22 @@ int gh_matmul_gate( void* hb, const void* x, const void* w_gate_up, const void* 
     using E = decltype( tag );
     using View = decltype( view );
     const E* b = static_cast<const E*>( bias );
-    if ( hidden % 4 == 0 && aligned16( hb ) && aligned16( bias ) ) {
-      gate_rows_kernel<E, View, 4><<<grid_for( rows * hidden / 4 ), 256, 0, st>>>( static_cast<E*>( hb ), view, b, (uint32_t)hidden, rows, activation );
+    const bool vec = aligned16( hb ) && aligned16( bias );
+    auto launch = [&]( auto v_tag ) {
+      constexpr int V = decltype( v_tag )::value;
+      for ( uint64_t r0 = 0; r0 < rows; r0 += 65535 ) { // a grid's second dimension ends there
+        View part = view;
+        part.data += r0 * view.stride;
+        const dim3 grid( (unsigned)( ( hidden + 256 * V - 1 ) / ( 256 * V ) ), (unsigned)std::min<uint64_t>( 65535, rows - r0 ) );
+        gate_rows_kernel<E, View, V><<<grid, 256, 0, st>>>( static_cast<E*>( hb ) + r0 * hidden, part, b, (uint32_t)hidden, activation );
+      }
+    };
+    if ( vec && hidden % 8 == 0 && std::is_same_v<View, ProductView<__bf16>> ) {
+      launch( std::integral_constant<int, 8> {} );
+    } else if ( vec && hidden % 4 == 0 ) {
+      launch( std::integral_constant<int, 4> {} );
     } else {
-      gate_rows_kernel<E, View, 1><<<grid_for( rows * hidden ), 256, 0, st>>>( static_cast<E*>( hb ), view, b, (uint32_t)hidden, rows, activation );
+      launch( std::integral_constant<int, 1> {} );
     }
     GH_LAUNCH_CHECK();
     return GH_OK;
