@@ -231,6 +231,43 @@ constexpr float NO_KEY = -1e30f; // running maximum before the first key: exp(NO
 // partial result of one split of one (row, head): vpad weighted sums, then the sum of the weights and the maximum
 __host__ __device__ inline uint64_t partial_stride( const WindowShape& s ) { return s.vpad + 2; }
 
+// The results of a work-group's four waves for the query heads h0 .. h0 + nh - 1 of a row, wave w's for head h at
+// lds[(w * hq + h) * (vpad + 2)]: added up and stored, as the output or as the partial result of a split.
+template<typename E>
+__device__ __forceinline__ void finish_split( E* out, float* partial, const float* lds, uint32_t hq, uint32_t nh, uint64_t row, uint32_t h0, uint32_t split,
+                                              uint32_t splits, const WindowShape& s )
+{
+  const uint32_t stride = s.vpad + 2;
+  for ( uint32_t i = threadIdx.x; i < nh * s.vpad; i += 256 ) {
+    const uint32_t h = i / s.vpad, e = i % s.vpad;
+    float m = NO_KEY;
+#pragma unroll
+    for ( int w = 0; w < 4; w++ ) {
+      m = fmaxf( m, lds[( w * hq + h ) * stride + s.vpad + 1] );
+    }
+    float a = 0.0f, sm = 0.0f;
+#pragma unroll
+    for ( int w = 0; w < 4; w++ ) {
+      const float* src = lds + ( w * hq + h ) * stride;
+      const float f = __expf( src[s.vpad + 1] - m );
+      a += src[e] * f;
+      sm += src[s.vpad] * f;
+    }
+    if ( splits == 1 ) {
+      if ( e < s.vdim ) {
+        out[( row * s.heads + h0 + h ) * s.vdim + e] = from_f32<E>( a / sm );
+      }
+    } else {
+      float* dst = partial + ( ( row * s.heads + h0 + h ) * splits + split ) * stride;
+      dst[e] = a;
+      if ( e == 0 ) {
+        dst[s.vpad] = sm;
+        dst[s.vpad + 1] = m;
+      }
+    }
+  }
+}
+
 // HQ query heads at a time; NC pieces of 128 elements per head (a lane holds 8 of each)
 template<typename E, int HQ, int NC>
 __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out,
@@ -380,34 +417,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
     }
   }
   __syncthreads();
-  for ( uint32_t i = threadIdx.x; i < nh * s.vpad; i += 256 ) {
-    const uint32_t h = i / s.vpad, e = i % s.vpad;
-    float m = NO_KEY;
-#pragma unroll
-    for ( int w = 0; w < 4; w++ ) {
-      m = fmaxf( m, lds[( w * HQ + h ) * stride + s.vpad + 1] );
-    }
-    float a = 0.0f, sm = 0.0f;
-#pragma unroll
-    for ( int w = 0; w < 4; w++ ) {
-      const float* src = lds + ( w * HQ + h ) * stride;
-      const float f = __expf( src[s.vpad + 1] - m );
-      a += src[e] * f;
-      sm += src[s.vpad] * f;
-    }
-    if ( splits == 1 ) {
-      if ( e < s.vdim ) {
-        out[( row * s.heads + h0 + h ) * s.vdim + e] = from_f32<E>( a / sm );
-      }
-    } else {
-      float* dst = partial + ( ( row * s.heads + h0 + h ) * splits + split ) * stride;
-      dst[e] = a;
-      if ( e == 0 ) {
-        dst[s.vpad] = sm;
-        dst[s.vpad + 1] = m;
-      }
-    }
-  }
+  finish_split<E>( out, partial, lds, HQ, nh, row, h0, split, splits, s );
 }
 
 // one wave per (row, head)
@@ -712,6 +722,208 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
   }
 }
 
+// ---- few tokens: one query row at a time on the matrix cores (bf16, head sizes up to 128) ---------------------------------------
+//
+// The products of the tile kernel with the query heads of a group as the columns (most of the 32 stay empty: the kernel streams keys, and
+// the matrix cores keep up with that many times over).  A wave takes every fourth tile of 32 of the row's visible keys, numbered as
+// in the rows kernel, so nothing needs a mask but the end; its tiles pass through LDS of its own, the next one's rows on their way
+// into registers meanwhile, without a barrier.  Adjacent work-groups read adjacent heads of the same cache rows.
+constexpr uint32_t STEP_KEYS = 32;
+constexpr uint32_t STEP_COLS = 16; // query heads of a work-group
+
+template<int KS, int VB>
+__global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __restrict__ out,
+                                                                  float* __restrict__ partial,
+                                                                  const __bf16* __restrict__ q,
+                                                                  const float* __restrict__ bias,
+                                                                  WindowRows wr,
+                                                                  WindowShape s,
+                                                                  uint32_t head_cols,
+                                                                  uint32_t keys_per_split,
+                                                                  uint32_t splits )
+{
+  __shared__ uint4 tiles[4][2][STEP_KEYS * 16]; // K and V of each wave, 256 bytes a key
+  const uint32_t head_blocks = s.heads / head_cols;
+  const uint32_t hb = blockIdx.x % head_blocks, split = blockIdx.x / head_blocks % splits;
+  const uint64_t row = blockIdx.x / head_blocks / splits;
+  const uint32_t ctx = (uint32_t)( row / wr.n_tokens ), tok = (uint32_t)( row % wr.n_tokens );
+  const uint8_t* base = static_cast<const uint8_t*>( wr.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  const __bf16* cache = reinterpret_cast<const __bf16*>( base + wr.offset );
+  const uint32_t h0 = hb * head_cols, g = h0 / s.group;
+  const uint32_t pos = wr.start_pos[ctx] + tok;
+  const Visible vis = visible_keys( pos, s );
+  const uint32_t k_begin = split * keys_per_split, k_end = min( vis.count, k_begin + keys_per_split );
+  const uint32_t wave = __builtin_amdgcn_readfirstlane( threadIdx.x >> 6 );
+  const uint32_t lane = threadIdx.x & 63, r = lane & 31, g2 = lane >> 5;
+  const uint32_t hc = min( r, head_cols - 1 ); // columns beyond do as the last one and are not stored
+  uint4* s_k = tiles[wave][0];
+  uint4* s_v = tiles[wave][1];
+
+  bf16x8 qb[KS];
+#pragma unroll
+  for ( int k = 0; k < KS; k++ ) {
+    const uint32_t ch = 2 * k + g2;
+    u32x4_t v = { 0, 0, 0, 0 };
+    if ( ch * 8 < s.dpad ) {
+      v = *(global_u32x4_t*)( q + ( row * s.heads + h0 + hc ) * s.dpad + ch * 8 );
+    }
+    qb[k] = __builtin_bit_cast( bf16x8, v );
+  }
+  const uint32_t ld_chunk = lane & 15, ld_row = lane >> 4;
+  const bool k_chunk = ld_chunk * 8 < s.dpad && ld_chunk < 2 * KS, v_chunk = ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB;
+  const uint32_t at_k = g * s.dpad + ld_chunk * 8, at_v = s.k_elems() + g * s.vpad + ld_chunk * 8;
+  u32x4_t rk[8], rv[8];
+  auto load = [&]( uint32_t i0 ) {
+#pragma unroll
+    for ( int k = 0; k < 8; k++ ) {
+      const uint32_t j = vis.key( min( i0 + ld_row + 4 * k, k_end - 1 ) ); // past the end: the last key again, without weight
+      const __bf16* p = cache + (uint64_t)j * s.row_elems();
+      rk[k] = u32x4_t { 0, 0, 0, 0 };
+      rv[k] = u32x4_t { 0, 0, 0, 0 };
+      if ( k_chunk ) {
+        rk[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_k ) );
+      }
+      if ( v_chunk ) {
+        rv[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_v ) );
+      }
+    }
+  };
+  const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
+  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ) * 16 ) + ( tr_q & 1 ) * 8;
+  const float scale_log2e = s.scale * LOG2E;
+  const float* my_bias = bias != nullptr ? bias + (uint64_t)( h0 + hc ) * s.n_dist : nullptr;
+  const float far_bias = bias != nullptr ? my_bias[s.n_dist - 1] * LOG2E : 0.0f;
+
+  mfma_f32x16 acc[VB];
+#pragma unroll
+  for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+    for ( int v = 0; v < 16; v++ ) {
+      acc[vb][v] = 0.0f;
+    }
+  }
+  float m = NO_KEY, l = 0.0f;
+  uint32_t i0 = k_begin + wave * STEP_KEYS;
+  if ( i0 < k_end ) {
+    load( i0 );
+  }
+  for ( ; i0 < k_end; i0 += 4 * STEP_KEYS ) {
+#pragma unroll
+    for ( int k = 0; k < 8; k++ ) {
+      const uint32_t krow = ld_row + 4 * k;
+      s_k[krow * 16 + ( ld_chunk ^ ( krow & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
+      s_v[krow * 16 + ( ld_chunk ^ ( 4 * ( krow & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+    }
+    if ( i0 + 4 * STEP_KEYS < k_end ) {
+      load( i0 + 4 * STEP_KEYS );
+    }
+    __builtin_amdgcn_fence( __ATOMIC_RELEASE, "wavefront" );
+    mfma_f32x16 st;
+#pragma unroll
+    for ( int v = 0; v < 16; v++ ) {
+      st[v] = 0.0f;
+    }
+#pragma unroll
+    for ( int k = 0; k < KS; k++ ) {
+      st = Mfma<__bf16>::k16( __builtin_bit_cast( bf16x8, s_k[r * 16 + ( ( 2 * k + g2 ) ^ ( r & 15 ) )] ), qb[k], st );
+    }
+    // every distance of the tile in the bias table's last row?
+    const uint32_t nearest = vis.key( min( i0 + STEP_KEYS, k_end ) - 1 );
+    if ( bias == nullptr || pos - nearest >= s.n_dist - 1 ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        st[v] = st[v] * scale_log2e + far_bias;
+      }
+    } else {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        const uint32_t j = vis.key( min( i0 + 8 * ( v / 4 ) + 4 * g2 + v % 4, k_end - 1 ) );
+        st[v] = st[v] * scale_log2e + my_bias[min( pos - j, s.n_dist - 1 )] * LOG2E;
+      }
+    }
+    if ( i0 + STEP_KEYS > k_end ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        st[v] = i0 + 8 * ( v / 4 ) + 4 * g2 + v % 4 < k_end ? st[v] : -INFINITY;
+      }
+    }
+    float mx2[2];
+#pragma unroll
+    for ( int c = 0; c < 2; c++ ) {
+      mx2[c] = st[8 * c];
+#pragma unroll
+      for ( int e = 1; e < 8; e++ ) {
+        mx2[c] = fmaxf( mx2[c], st[8 * c + e] );
+      }
+    }
+    const float mx = half_wave_max( fmaxf( mx2[0], mx2[1] ) );
+    if ( __builtin_amdgcn_ballot_w64( mx > m + LAZY ) != 0 ) {
+      const float m_new = fmaxf( m, mx );
+      const float alpha = __builtin_amdgcn_exp2f( m - m_new );
+      m = m_new;
+      l *= alpha;
+#pragma unroll
+      for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+        for ( int v = 0; v < 16; v++ ) {
+          acc[vb][v] *= alpha;
+        }
+      }
+    }
+#pragma unroll
+    for ( int kk = 0; kk < 2; kk++ ) {
+      bf16x8 hi, lo;
+#pragma unroll
+      for ( int e = 0; e < 8; e++ ) {
+        const float p = __builtin_amdgcn_exp2f( st[8 * kk + e] - m );
+        l += p;
+        hi[e] = (__bf16)p;
+        lo[e] = (__bf16)( p - (float)hi[e] );
+      }
+#pragma unroll
+      for ( int vb = 0; vb < VB; vb++ ) {
+        union
+        {
+          v4s half[2];
+          bf16x8 x;
+        } a;
+#pragma unroll
+        for ( int hf = 0; hf < 2; hf++ ) {
+          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
+        }
+        acc[vb] = Mfma<__bf16>::k16( a.x, lo, acc[vb] );
+        acc[vb] = Mfma<__bf16>::k16( a.x, hi, acc[vb] );
+      }
+    }
+    __builtin_amdgcn_fence( __ATOMIC_ACQUIRE, "wavefront" );
+  }
+  l += __shfl_xor( l, 32 );
+  __syncthreads(); // the tiles' LDS takes the waves' results
+  float* results = reinterpret_cast<float*>( &tiles[0][0][0] );
+  if ( r < head_cols ) {
+    float* mine = results + ( wave * head_cols + r ) * ( s.vpad + 2 );
+#pragma unroll
+    for ( int vb = 0; vb < VB; vb++ ) {
+#pragma unroll
+      for ( int v = 0; v < 16; v++ ) {
+        const uint32_t d = 32 * vb + 8 * ( v / 4 ) + 4 * g2 + v % 4;
+        if ( d < s.vpad ) {
+          mine[d] = acc[vb][v];
+        }
+      }
+    }
+    if ( g2 == 0 ) {
+      mine[s.vpad] = l;
+      mine[s.vpad + 1] = m * ( 1.0f / LOG2E ); // the sums are joined in natural units
+    }
+  }
+  __syncthreads();
+  finish_split<__bf16>( out, partial, results, head_cols, head_cols, row, h0, split, splits, s );
+}
+
 WindowShape shape_of( const gh_window_attn* a )
 {
   WindowShape s;
@@ -758,6 +970,66 @@ void launch_rows( int hq, dim3 grid, hipStream_t st, E* out, float* partial, con
   window_rows_kernel<E, 1, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
 }
 
+// Splits of the visible keys of a call's rows, and room for their partial results: as many as give every CU two work-groups, of at
+// least `least` keys each.
+struct SplitPlan
+{
+  uint32_t keys { 0 }, splits { 1 };
+  float* partial { nullptr };
+};
+int plan_splits( const WindowShape& s, uint64_t rows, uint64_t head_blocks, uint32_t max_pos, uint64_t least, hipStream_t st, SplitPlan* plan )
+{
+  const uint64_t most = std::min<uint64_t>( (uint64_t)max_pos + 1, (uint64_t)s.window + s.keep_first );
+  uint64_t splits = std::max<uint64_t>( 1, 2ull * cu_count() / std::max<uint64_t>( 1, rows * head_blocks ) );
+  splits = std::min( { splits, std::max<uint64_t>( 1, most / least ), (uint64_t)64 } );
+  plan->keys = (uint32_t)( ( ( most + splits - 1 ) / splits + 31 ) / 32 * 32 );
+  plan->splits = (uint32_t)( ( most + plan->keys - 1 ) / plan->keys );
+  if ( plan->splits > 1 ) {
+    void* p = nullptr;
+    if ( int rc = stream_scratch( st, SCRATCH_MIXER, rows * s.heads * plan->splits * partial_stride( s ) * sizeof( float ), 1ull << 20, &p ) ) {
+      return rc;
+    }
+    plan->partial = static_cast<float*>( p );
+  }
+  return GH_OK;
+}
+template<typename E>
+int merge_splits( E* out, const SplitPlan& plan, const WindowRows& wr, const WindowShape& s, uint64_t rows, hipStream_t st )
+{
+  if ( plan.splits > 1 ) {
+    const uint64_t pairs = rows * s.heads;
+    window_merge_kernel<E><<<(unsigned)( ( pairs + 3 ) / 4 ), 256, 0, st>>>( out, plan.partial, wr, s, plan.splits, pairs );
+    GH_LAUNCH_CHECK();
+  }
+  return GH_OK;
+}
+
+// few rows of bf16 with heads of up to 128
+int attend_decode( __bf16* out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
+{
+  uint32_t head_cols = s.group; // the largest divisor of the group that fits
+  while ( head_cols > STEP_COLS || s.group % head_cols != 0 ) {
+    head_cols--;
+  }
+  const uint64_t head_blocks = s.heads / head_cols;
+  SplitPlan plan;
+  if ( int rc = plan_splits( s, rows, head_blocks, max_pos, 4 * STEP_KEYS, st, &plan ) ) {
+    return rc;
+  }
+  const uint64_t grid = rows * head_blocks * plan.splits;
+  GH_REQUIRE( grid < ( 1ull << 31 ), "gh_attn_window: grid too large" );
+#define GH_WINDOW_DECODE( KS, VB ) \
+  window_decode_kernel<KS, VB><<<(unsigned)grid, 256, 0, st>>>( out, plan.partial, q, bias, wr, s, head_cols, plan.keys, plan.splits )
+  if ( s.dpad <= 64 && s.vpad <= 64 ) {
+    GH_WINDOW_DECODE( 4, 2 );
+  } else {
+    GH_WINDOW_DECODE( 8, 4 );
+  }
+#undef GH_WINDOW_DECODE
+  GH_LAUNCH_CHECK();
+  return merge_splits( out, plan, wr, s, rows, st );
+}
+
 template<typename E>
 int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
 {
@@ -769,21 +1041,13 @@ int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, co
   }
   const uint32_t head_blocks = s.kv_heads * ( ( s.group + hq - 1 ) / hq );
   GH_REQUIRE( head_blocks <= 65535, "gh_attn_window: too many heads" );
-  // the most keys any row of the call sees, and as many splits as give every CU a few work-groups of at least 64 keys
-  const uint64_t most = std::min<uint64_t>( (uint64_t)max_pos + 1, (uint64_t)s.window + s.keep_first );
-  const uint64_t groups = rows * head_blocks;
-  uint64_t splits = std::max<uint64_t>( 1, 2ull * cu_count() / std::max<uint64_t>( 1, groups ) );
-  splits = std::min( { splits, std::max<uint64_t>( 1, most / 64 ), (uint64_t)64 } );
-  const uint32_t per = (uint32_t)( ( ( most + splits - 1 ) / splits + 15 ) / 16 * 16 );
-  splits = ( most + per - 1 ) / per;
-  float* partial = nullptr;
-  if ( splits > 1 ) {
-    void* p = nullptr;
-    if ( int rc = stream_scratch( st, SCRATCH_MIXER, rows * s.heads * splits * partial_stride( s ) * sizeof( float ), 1ull << 20, &p ) ) {
-      return rc;
-    }
-    partial = static_cast<float*>( p );
+  SplitPlan plan;
+  if ( int rc = plan_splits( s, rows, head_blocks, max_pos, 64, st, &plan ) ) {
+    return rc;
   }
+  const uint32_t per = plan.keys;
+  const uint32_t splits = plan.splits;
+  float* partial = plan.partial;
   const dim3 grid( (unsigned)rows, head_blocks, (unsigned)splits );
   if ( widest <= 128 ) {
     launch_rows<E, 1>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
@@ -793,12 +1057,7 @@ int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, co
     launch_rows<E, 4>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
   }
   GH_LAUNCH_CHECK();
-  if ( splits > 1 ) {
-    const uint64_t pairs = rows * s.heads;
-    window_merge_kernel<E><<<(unsigned)( ( pairs + 3 ) / 4 ), 256, 0, st>>>( out, partial, wr, s, (uint32_t)splits, pairs );
-    GH_LAUNCH_CHECK();
-  }
-  return GH_OK;
+  return merge_splits( out, plan, wr, s, rows, st );
 }
 
 // Whether the tile kernel serves a call; its launch.
@@ -897,6 +1156,9 @@ int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const flo
   }
   if ( tiles_applicable( s, distance_bias_dev, n_tokens ) ) {
     return attend_tiles( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, batch, as_stream( stream ) );
+  }
+  if ( s.dpad <= 128 && s.vpad <= 128 ) {
+    return attend_decode( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
   }
   return attend_rows<__bf16>( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
 }
