@@ -5,10 +5,13 @@
 //
 // Weights are random, as in the reference's profiler (profile/profiler.hh:68); <model_root> is
 // only consulted for its CONFIG file, which must describe <model_name> when it exists ("-" skips it).
+// A run-time sized design takes its sizes from <model_root>/config.json: <model_name> is then the architecture named there, and <stage>
+// is all.
 #include <cstdlib>
 #include <fstream>
 #include <iostream>
 
+#include "glint/designs.hh"
 #include "glint/loader.hh"
 #include "glint/profiler.hh"
 
@@ -58,6 +61,42 @@ int run( const std::string& model_root, const std::string& model_name, Inference
   return EXIT_SUCCESS;
 }
 
+int run_design( const std::string& model_root, const std::string& model_name, const bool paged, const InferenceStage stage, const uint32_t batch, const uint64_t token_pos,
+                const uint64_t duration_s, const std::string& log_path )
+{
+  if ( stage != InferenceStage::__ALL__ ) {
+    std::cerr << model_name << " is hosted whole: the stage is all\n";
+    return EXIT_FAILURE;
+  }
+  if ( batch == 0 || batch > MAX_BATCH_SIZE ) {
+    std::cerr << "Batch size out of range (1.." << MAX_BATCH_SIZE << ")\n";
+    return EXIT_FAILURE;
+  }
+  DesignOptions options;
+  options.paged = paged;
+  options.concurrency_limit = options.max_context_count = batch;
+  options.model.seed = 7;
+  options.model.randomize = true;
+  const std::string err = with_design( model_root, options, [&]( auto tag, const auto& config, const auto& settings, const ModelOptions& o ) -> std::string {
+    if ( token_pos >= config.max_positions ) {
+      return "Token position out of range";
+    }
+    std::ofstream out( log_path, std::ios::out | std::ios::trunc );
+    if ( !out ) {
+      return "cannot open " + log_path;
+    }
+    typename decltype( tag )::type model( config, settings, o );
+    DesignProfiler profiler( model, model_name, batch, (uint32_t)token_pos, duration_s );
+    const uint64_t calls = profiler.run( out );
+    std::cerr << "profile-stage-hip: " << profiler.header() << ": " << calls << " calls\n";
+    return {};
+  } );
+  if ( !err.empty() ) {
+    std::cerr << "Error: " << err << '\n';
+  }
+  return err.empty() ? EXIT_SUCCESS : EXIT_FAILURE;
+}
+
 } // namespace
 
 int main( int argc, char* argv[] )
@@ -79,6 +118,9 @@ int main( int argc, char* argv[] )
     return EXIT_FAILURE;
   }
   const bool paged = context_name == "paged";
+  if ( is_known_design( model_name ) ) {
+    return run_design( model_root, model_name, paged, stage, batch, token_pos, duration_s, log_path );
+  }
 #define GLINT_MODEL( NAME, CFG )                                                                                                      \
   if ( model_name == NAME ) {                                                                                                       \
     return paged ? run<configs::CFG, hip::DynamicContext<configs::CFG, float16_t>>( model_root, model_name, stage, batch, token_pos, duration_s, log_path ) \

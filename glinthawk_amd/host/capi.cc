@@ -235,6 +235,8 @@ DesignOptions design_options( int dtype, uint32_t concurrency, uint32_t max_cont
   return o;
 }
 
+using LayeredBookContext = glint::DynamicLayeredContext<CountingRegion>;
+
 thread_local std::string g_last_error;
 thread_local std::string g_bytes; // result of the last call that returns bytes
 
@@ -535,6 +537,52 @@ uint64_t glint_book_paged_prepare( void* c, uint32_t layer, uint32_t token_pos, 
   out[0] = ctx->blocks_committed();
   out[1] = ctx->clears();
   return ctx->allocated_bytes( layer );
+}
+
+// paged context of a run-time sized design over a counting region: parts in order, row_bytes[i] > 0: cache rows, else a state of state_bytes[i]
+void* glint_book_layered_new( uint32_t max_positions, uint32_t n_parts, const uint64_t* row_bytes, const uint64_t* state_bytes )
+{
+  auto plan = std::make_shared<ContextPlan>( max_positions );
+  for ( uint32_t i = 0; i < n_parts; i++ ) {
+    if ( row_bytes[i] > 0 ) {
+      plan->add_rows( row_bytes[i] );
+    } else {
+      plan->add_state( state_bytes[i] );
+    }
+  }
+  DesignSettings settings;
+  settings.plan = std::move( plan );
+  return new LayeredBookContext( settings );
+}
+void glint_book_layered_delete( void* c ) { delete static_cast<LayeredBookContext*>( c ); }
+// 1 and the blocks committed now and the clears so far, or 0 when the context does not take tokens at `pos` (nothing is then changed)
+int glint_book_layered_append( void* c, uint32_t pos, uint32_t n_tokens, uint64_t out[2] )
+{
+  auto* ctx = static_cast<LayeredBookContext*>( c );
+  if ( !ctx->takes( pos ) ) {
+    return 0;
+  }
+  GLINT_CHECK( ctx->prepare( pos, n_tokens ) );
+  ctx->set_length( pos + n_tokens );
+  out[0] = ctx->blocks_committed();
+  out[1] = ctx->clears();
+  return 1;
+}
+uint32_t glint_book_distance_bucket( uint64_t distance, uint32_t rows, double bias_max ) { return distance_bucket( distance, rows, bias_max ); }
+// what a config.json's layers run as: (layer, pass + 1) of each run, up to cap runs; the number of runs, or -1 (see glint_last_error())
+int64_t glint_book_famidra_runs( const char* config_json, uint32_t* out, uint64_t cap )
+{
+  FamidraConfig config;
+  g_last_error = FamidraConfig::parse( config_json, config );
+  if ( !g_last_error.empty() ) {
+    return -1;
+  }
+  const auto runs = config.runs();
+  for ( size_t i = 0; i < runs.size() && i < cap; i++ ) {
+    out[2 * i] = runs[i].layer;
+    out[2 * i + 1] = static_cast<uint32_t>( runs[i].pass + 1 );
+  }
+  return static_cast<int64_t>( runs.size() );
 }
 
 // KV addressing of the host layer, in elements from the context base (UINT64_MAX: layer not hosted)

@@ -225,6 +225,83 @@ private:
   std::vector<State> states_ {};
 };
 
+// The same log for a run-time sized design, which is hosted whole: one call = one forward() of the model.  The contexts are brought to
+// `token_pos` by a prefill of random tokens; a recurrent state cannot be rewound, so every call decodes the next position, and the
+// contexts start again from the prefill when the model's positions run out.
+template<typename Model>
+class DesignProfiler
+{
+public:
+  DesignProfiler( Model& model, const std::string& model_name, const uint32_t batch_size, const uint32_t token_pos, const size_t duration_s )
+    : model_( model )
+    , batch_size_( batch_size )
+    , token_pos_( token_pos )
+    , duration_( duration_s )
+    , state_( batch_size, dtype_of<typename Model::DataTypeT>() )
+  {
+    header_ = "model='" + model_name + "', stage=" + stage_text( InferenceStage::__ALL__ ) + ", batch_size=" + std::to_string( batch_size )
+              + ", token_pos=" + std::to_string( token_pos ) + ", duration_s=" + std::to_string( duration_s );
+    for ( uint32_t i = 0; i < batch_size; i++ ) {
+      contexts_.push_back( std::make_shared<typename Model::ContextType>( model.settings() ) );
+    }
+    restart();
+  }
+
+  const std::string& header() const { return header_; }
+
+  ProfileRow step( const uint64_t repeat )
+  {
+    if ( state_.token_pos( 0 ) >= model_.max_positions() ) {
+      restart();
+    }
+    const auto wall = std::chrono::system_clock::now();
+    const auto start = std::chrono::steady_clock::now();
+    model_.forward( state_, contexts_ );
+    const auto end = std::chrono::steady_clock::now();
+    return { repeat, (uint64_t)std::chrono::duration_cast<std::chrono::milliseconds>( wall.time_since_epoch() ).count(),
+             (uint64_t)std::chrono::duration_cast<std::chrono::microseconds>( end - start ).count() };
+  }
+
+  uint64_t run( std::ostream& out )
+  {
+    write_profile_header( out, header_ );
+    const auto end_time = std::chrono::steady_clock::now() + duration_;
+    uint64_t r = 0;
+    for ( ;; r++ ) {
+      write_profile_row( out, step( r ) );
+      if ( std::chrono::steady_clock::now() >= end_time ) {
+        break;
+      }
+    }
+    return r + 1;
+  }
+
+private:
+  void restart()
+  {
+    std::mt19937_64 rng( 12345 );
+    std::uniform_int_distribution<uint32_t> token( 0, model_.vocab_size() - 1 );
+    const std::vector<uint32_t> start( batch_size_, 0 );
+    if ( token_pos_ > 0 ) {
+      std::vector<uint32_t> tokens( (uint64_t)batch_size_ * token_pos_ );
+      for ( auto& t : tokens ) {
+        t = token( rng );
+      }
+      model_.prefill( contexts_, start.data(), token_pos_, tokens.data(), {}, nullptr, nullptr );
+    }
+    for ( uint32_t i = 0; i < batch_size_; i++ ) {
+      state_.set_prompt( i, PromptID {}, ContextID { i + 1 }, token( rng ), token_pos_, 0.5f, 1, model_.max_positions(), 0, 0 );
+    }
+  }
+
+  Model& model_;
+  const uint32_t batch_size_, token_pos_;
+  const std::chrono::seconds duration_;
+  std::string header_ {};
+  typename Model::ContextVector contexts_ {};
+  typename Model::StateType state_;
+};
+
 // untemplated_matmul( out(dim1, dim3), in(dim1, dim2), w(dim3, dim2) ) over 128 rotating input/output
 // buffers (profile/gemm_profiler.hh); every call is bracketed by a device synchronisation
 template<typename DType>

@@ -86,6 +86,11 @@ def host_lib() -> C.CDLL:
             "glint_book_paged_new": (vp, [u32]),
             "glint_book_paged_delete": (None, [vp]),
             "glint_book_paged_prepare": (u64, [vp, u32, u32, C.c_int, C.POINTER(u64)]),
+            "glint_book_layered_new": (vp, [u32, u32, vp, vp]),
+            "glint_book_layered_delete": (None, [vp]),
+            "glint_book_layered_append": (C.c_int, [vp, u32, u32, C.POINTER(u64)]),
+            "glint_book_distance_bucket": (u32, [u64, u32, C.c_double]),
+            "glint_book_famidra_runs": (C.c_int64, [C.c_char_p, vp, u64]),
             "glint_book_key_head_offset": (u64, [vp, u32, u32, u32, C.c_int]),
         }
         for name, (res, args) in sig.items():
@@ -408,6 +413,36 @@ class BookPagedContext:
         out = (C.c_uint64 * 2)()
         allocated = host_lib().glint_book_paged_prepare(self._c, layer, token_pos, int(can_release), out)
         return int(allocated), int(out[0]), int(out[1])
+
+
+class BookLayeredContext:
+    """Host-only paged context of a run-time sized design over a region that only records commits; `parts`: ("rows", bytes a token) or
+    ("state", bytes)."""
+
+    def __init__(self, max_positions: int, parts):
+        rows = np.array([n if kind == "rows" else 0 for kind, n in parts], dtype=np.uint64)
+        states = np.array([0 if kind == "rows" else n for kind, n in parts], dtype=np.uint64)
+        self._c = host_lib().glint_book_layered_new(max_positions, len(parts), rows.ctypes.data, states.ctypes.data)
+
+    def __del__(self):
+        if getattr(self, "_c", None):
+            host_lib().glint_book_layered_delete(self._c)
+            self._c = None
+
+    def append(self, pos: int, n_tokens: int):
+        """(2 MiB blocks committed, clears so far), or None when the context does not take tokens at `pos`."""
+        out = (C.c_uint64 * 2)()
+        return (int(out[0]), int(out[1])) if host_lib().glint_book_layered_append(self._c, pos, n_tokens, out) else None
+
+
+def famidra_runs(config_json: str):
+    """Host-only: (layer, pass or None) of every layer run of a Famidra config.json, in order.  Raises GlintError for a bad one."""
+    cap = 4096
+    out = np.zeros((cap, 2), dtype=np.uint32)
+    n = host_lib().glint_book_famidra_runs(config_json.encode(), out.ctypes.data, cap)
+    if n < 0:
+        raise GlintError(host_lib().glint_last_error().decode(errors="replace"))
+    return [(int(a), int(b) - 1 if b else None) for a, b in out[:n]]
 
 
 def model_dir_walk(config: str, dtype: str, first_layer: int, n_hosted: int, with_cls: bool, model_dir: str):

@@ -29,6 +29,10 @@ def test_command_line_refusals(tmp_path):
     assert r.returncode != 0 and "Unknown model name" in r.stderr
     r = run([STAGE, "-", "test-gqa4", "static", "att", "4", "320", "0", log])          # seq_len is 320
     assert r.returncode != 0 and "Token position out of range" in r.stderr
+    r = run([STAGE, str(tmp_path), "Famidra", "static", "all", "4", "10", "0", log])
+    assert r.returncode != 0 and "config.json" in r.stderr
+    r = run([STAGE, str(tmp_path), "Famidra", "static", "att", "4", "10", "0", log])
+    assert r.returncode != 0 and "hosted whole" in r.stderr
     r = run([GEMM, "64", "512"])
     assert r.returncode != 0 and "Usage:" in r.stderr
     r = run([GEMM, "64", "0", "512", "0", log])
@@ -54,6 +58,20 @@ def test_profile_stage_log(tmp_path, ctx, stage, text):
     assert (df["duration_us"] > 0).all() and (df["timestamp_ms"] > 1.6e12).all()
     # the consumer splits the file name into six fields after protecting "all_no_cls"
     assert len(log.name[:-4].replace("all_no_cls", "all-no-cls").split("_")) == 6
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("ctx", ["static", "paged"])
+def test_profile_of_a_design(tmp_path, ctx):
+    import famidra_models as M
+    M.write_model(tmp_path, M.CONFIGS["odd"], {})            # sizes only: the weights are drawn
+    log = tmp_path / f"famidra_all_{ctx}_297_0_3.csv"
+    r = run([STAGE, str(tmp_path), "Famidra", ctx, "all", "3", "297", "0", str(log)])
+    assert r.returncode == 0, r.stderr
+    assert open(log).readline().strip() == "# model='Famidra', stage=Pre+Att+Post+Cls, batch_size=3, token_pos=297, duration_s=0"
+    assert (pd.read_csv(log, skiprows=1)["duration_us"] > 0).all()
+    r = run([STAGE, str(tmp_path), "Famidra", ctx, "all", "3", "300", "0", str(log)])
+    assert r.returncode != 0 and "out of range" in r.stderr
 
 
 @pytest.mark.gpu
