@@ -223,8 +223,10 @@ __global__ __launch_bounds__( 256 ) void mlstm_walk_kernel( float* __restrict__ 
 //
 // work-group  2 waves on one (context, head, 64 columns of v) walk the chunks; a wave owns 32 columns, its part of S (dim x 32, fp32) stays in
 //             accumulator registers from the first chunk to the last.  Two work-groups per CU cover each other's loads.
-// exactness   q, k, v are bf16 already; everything fp32 that meets them in a product (S, the weights of the keys, the weighted values) goes
-//             in as three bf16 terms, 24 bits, so that the sums are those of fp32 operands at the rate of bf16 matrix instructions.
+// exactness   q, k, v are bf16 already.  What enters the state (the weighted values) meets k as three bf16 terms, 24 bits: the state's sums are
+//             those of fp32 operands at the rate of bf16 matrix instructions.  What is read out of it for the output (S, the weights of
+//             the keys) meets q and v as two terms, 16 bits.  n is carried in fp32, each wave half of it.
+// loads       k of a chunk is requested at its head, q and v of the next one as soon as both waves have read this one's.
 // operands    an accumulator tile of v_mfma_f32_32x32x16_bf16 (lane = column, registers = rows 8 (v / 4) + 4 (lane / 32) + v % 4) is, as it
 //             lies, an operand of the next product over those rows when the other operand takes its sixteen k in the same order:
 //               scores^T = K Q^T        lane = query, registers = keys   -> left operand of   P V     (V out of LDS transposed)
@@ -247,31 +249,45 @@ __device__ __forceinline__ uint32_t swizzle( uint32_t row, uint32_t chunk )
 }
 __device__ __forceinline__ uint32_t swizzle_v( uint32_t row, uint32_t chunk ) { return chunk ^ ( 4 * ( ( row >> 1 ) & 1 ) ); }
 
-// x = hi + mid + lo, 8 bits each
-struct Split3
+// Eight fp32 values as N bf16 terms each, 8 bits of mantissa a term; taken two at a time, as the conversion instruction does.
+typedef float f32x2 __attribute__( ( ext_vector_type( 2 ) ) );
+typedef __bf16 bf16x2 __attribute__( ( ext_vector_type( 2 ) ) );
+template<int N>
+struct Split
 {
-  bf16x8 t[3];
+  union
+  {
+    bf16x2 pair[4];
+    bf16x8 x;
+  } t[N];
+  __device__ __forceinline__ void set( int k, float x0, float x1 ) // elements 2 k, 2 k + 1
+  {
+#pragma unroll
+    for ( int n = 0; n < N; n++ ) {
+      const bf16x2 b = __builtin_convertvector( ( f32x2 { x0, x1 } ), bf16x2 );
+      t[n].pair[k] = b;
+      x0 -= (float)b[0];
+      x1 -= (float)b[1];
+    }
+  }
 };
-__device__ __forceinline__ void split3( Split3& s, int e, float x )
+template<int N>
+__device__ __forceinline__ mfma_f32x16 mma( const bf16x8 a, const Split<N>& b, mfma_f32x16 c )
 {
-  const __bf16 hi = (__bf16)x;
-  const float r = x - (float)hi;
-  const __bf16 mid = (__bf16)r;
-  s.t[0][e] = hi;
-  s.t[1][e] = mid;
-  s.t[2][e] = (__bf16)( r - (float)mid );
+#pragma unroll
+  for ( int n = N - 1; n >= 0; n-- ) {
+    c = Mfma<__bf16>::k16( a, b.t[n].x, c );
+  }
+  return c;
 }
-__device__ __forceinline__ mfma_f32x16 mma3( const bf16x8 a, const Split3& b, mfma_f32x16 c )
+template<int N>
+__device__ __forceinline__ mfma_f32x16 mma( const Split<N>& a, const bf16x8 b, mfma_f32x16 c )
 {
-  c = Mfma<__bf16>::k16( a, b.t[2], c );
-  c = Mfma<__bf16>::k16( a, b.t[1], c );
-  return Mfma<__bf16>::k16( a, b.t[0], c );
-}
-__device__ __forceinline__ mfma_f32x16 mma3( const Split3& a, const bf16x8 b, mfma_f32x16 c )
-{
-  c = Mfma<__bf16>::k16( a.t[2], b, c );
-  c = Mfma<__bf16>::k16( a.t[1], b, c );
-  return Mfma<__bf16>::k16( a.t[0], b, c );
+#pragma unroll
+  for ( int n = N - 1; n >= 0; n-- ) {
+    c = Mfma<__bf16>::k16( a.t[n].x, b, c );
+  }
+  return c;
 }
 __device__ __forceinline__ double shfl_up_f64( double v, int by )
 {
@@ -294,7 +310,8 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
   constexpr uint32_t RB = DT * 64; // bytes of a q or k row in LDS
   __shared__ uint4 s_k[CHUNK * RB / 16], s_q[CHUNK * RB / 16];
   __shared__ uint4 s_v[CHUNK * 8];
-  __shared__ float s_n[2][32 * DT];                                   // each wave its own copy of everything below
+  __shared__ float s_n[32 * DT];                                      // a wave reads and writes its half only
+  __shared__ __attribute__( ( aligned( 16 ) ) ) float s_nq[2][CHUNK]; // n . q over each wave's half; everything below: each wave its own copy
   __shared__ __attribute__( ( aligned( 16 ) ) ) float s_c[2][CHUNK]; // c_s - M of the chunk's last token, s_w: e to the power of it
   __shared__ __attribute__( ( aligned( 16 ) ) ) float s_w[2][CHUNK];
   __shared__ __attribute__( ( aligned( 16 ) ) ) float s_a[2][CHUNK];   // factor of the state in front of the chunk, per token
@@ -330,8 +347,8 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
       S[dt][v] = __builtin_bit_cast( float, __builtin_amdgcn_raw_buffer_load_b32( S_rsrc, fresh ? PAST_THE_END : S_off, ( 32 * dt + 8 * ( v / 4 ) + v % 4 ) * s.vpad * 4, 0 ) );
     }
   }
-  for ( uint32_t d = lane; d < 32 * DT; d += 64 ) {
-    s_n[wave][d] = !fresh && d < s.dim ? n_in[d] : 0.0f;
+  for ( uint32_t d = threadIdx.x; d < 32 * DT; d += 128 ) {
+    s_n[d] = !fresh && d < s.dim ? n_in[d] : 0.0f;
   }
   double m0 = fresh ? 0.0 : (double)m_mem;
   const uint64_t row_first = (uint64_t)ctx * st.n_tokens;
@@ -364,6 +381,14 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
       const uint32_t off = chunk < chunks ? row * ld_bytes + chunk * 16 : PAST_THE_END;
       __builtin_amdgcn_raw_ptr_buffer_load_lds( rsrc, (lds_ptr)( tile + row0 * ( BYTES / 16 ) ), 16, off, 0, 0, 0 );
     }
+  };
+
+  auto swizzle_row = []( uint32_t row, uint32_t c ) { return swizzle<DT>( row, c ); };
+  auto fetch_qv = [&]( uint32_t t0 ) {
+    const uint32_t rows = min( (uint32_t)CHUNK, st.n_tokens - t0 );
+    const __bf16* first = in.main.data + ( row_first + t0 ) * in.main.stride;
+    fetch( s_q, first + in.col.q + h * s.dim, rows, s.dim / 8, swizzle_row, std::integral_constant<uint32_t, RB> {} );
+    fetch( s_v, first + in.col.v + h * s.vdim + slice * 64, rows, min( 8u, ( s.vdim - slice * 64 ) / 8 ), swizzle_v, std::integral_constant<uint32_t, 128> {} );
   };
 
   // transposing reads: lane j = 4 e + q of a 16-lane group points at row e (0..3) of its half-wave's four, dims 16 grp + 4 q .. + 3
@@ -399,10 +424,10 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
   for ( uint32_t t0 = 0; t0 < st.n_tokens; t0 += CHUNK ) {
     const uint32_t rows = min( (uint32_t)CHUNK, st.n_tokens - t0 );
     const __bf16* first = in.main.data + ( row_first + t0 ) * in.main.stride;
-    __syncthreads(); // the last chunk's readers are done
-    fetch( s_k, first + in.col.k + h * s.dim, rows, s.dim / 8, []( uint32_t row, uint32_t c ) { return swizzle<DT>( row, c ); }, std::integral_constant<uint32_t, RB> {} );
-    fetch( s_q, first + in.col.q + h * s.dim, rows, s.dim / 8, []( uint32_t row, uint32_t c ) { return swizzle<DT>( row, c ); }, std::integral_constant<uint32_t, RB> {} );
-    fetch( s_v, first + in.col.v + h * s.vdim + slice * 64, rows, min( 8u, ( s.vdim - slice * 64 ) / 8 ), swizzle_v, std::integral_constant<uint32_t, 128> {} );
+    fetch( s_k, first + in.col.k + h * s.dim, rows, s.dim / 8, swizzle_row, std::integral_constant<uint32_t, RB> {} );
+    if ( t0 == 0 ) {
+      fetch_qv( 0 );
+    }
 
     // gates: lane = token
     const bool live = lane < rows;
@@ -434,7 +459,7 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
     __syncthreads();
 
     // ---- scores^T and the weights P: query tile tt, key tiles up to it
-    Split3 P[2][4]; // [query tile][16 keys]
+    Split<2> P[2][4]; // [query tile][16 keys]
     float den[2];
 #pragma unroll
     for ( int tt = 0; tt < 2; tt++ ) {
@@ -457,13 +482,15 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
           const uint32_t key0 = opaque( 32 * kt + 8 * q4 + 4 * g2 );
           const float4 ck = *reinterpret_cast<const float4*>( &s_c[wave][key0] );
           const float cks[4] = { ck.x, ck.y, ck.z, ck.w };
+          float p[4];
 #pragma unroll
           for ( int e = 0; e < 4; e++ ) {
             const bool seen = kt < tt || key0 + e <= 32 * tt + r;
-            const float p = seen ? sc[4 * q4 + e] * s.q_scale * __expf( cks[e] - Mq ) : 0.0f;
-            den[tt] += p;
-            split3( P[tt][2 * kt + ( q4 >> 1 )], 4 * ( q4 & 1 ) + e, p );
+            p[e] = seen ? sc[4 * q4 + e] * s.q_scale * __expf( cks[e] - Mq ) : 0.0f;
+            den[tt] += p[e];
           }
+          P[tt][2 * kt + ( q4 >> 1 )].set( 2 * ( q4 & 1 ), p[0], p[1] );
+          P[tt][2 * kt + ( q4 >> 1 )].set( 2 * ( q4 & 1 ) + 1, p[2], p[3] );
         }
       }
     }
@@ -484,13 +511,11 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
       for ( int half = 0; half < 2; half++ ) {
         __builtin_amdgcn_sched_barrier( 0 );
         const uint32_t rb = opaque( r * RB + 8 * g2 ), swz = opaque( row_swz );
-        Split3 sp;
+        Split<2> sp;
 #pragma unroll
-        for ( int e = 0; e < 8; e++ ) {
-          split3( sp, e, S[dt][8 * half + e] );
+        for ( int k = 0; k < 4; k++ ) {
+          sp.set( k, S[dt][8 * half + 2 * k], S[dt][8 * half + 2 * k + 1] );
         }
-        const float4 n0 = *reinterpret_cast<const float4*>( &s_n[wave][32 * dt + 16 * half + 4 * g2] );
-        const float4 n1 = *reinterpret_cast<const float4*>( &s_n[wave][32 * dt + 16 * half + 8 + 4 * g2] );
 #pragma unroll
         for ( int tt = 0; tt < 2; tt++ ) {
           union
@@ -500,21 +525,40 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
           } a;
           a.p[0] = *reinterpret_cast<const uint2*>( reinterpret_cast<const char*>( s_q ) + 32 * tt * RB + rb + slot_at( 64 * dt + 32 * half, swz ) );
           a.p[1] = *reinterpret_cast<const uint2*>( reinterpret_cast<const char*>( s_q ) + 32 * tt * RB + rb + slot_at( 64 * dt + 32 * half + 16, swz ) );
-          O[tt] = mma3( a.x, sp, O[tt] );
-          nq[tt] += (float)a.x[0] * n0.x + (float)a.x[1] * n0.y + (float)a.x[2] * n0.z + (float)a.x[3] * n0.w + (float)a.x[4] * n1.x + (float)a.x[5] * n1.y
-                    + (float)a.x[6] * n1.z + (float)a.x[7] * n1.w;
+          O[tt] = mma( a.x, sp, O[tt] );
+          if ( (uint32_t)( dt / ( DT / 2 ) ) == wave ) { // uniform
+            const float4 n0 = *reinterpret_cast<const float4*>( &s_n[32 * dt + 16 * half + 4 * g2] );
+            const float4 n1 = *reinterpret_cast<const float4*>( &s_n[32 * dt + 16 * half + 8 + 4 * g2] );
+            nq[tt] += (float)a.x[0] * n0.x + (float)a.x[1] * n0.y + (float)a.x[2] * n0.z + (float)a.x[3] * n0.w + (float)a.x[4] * n1.x + (float)a.x[5] * n1.y
+                      + (float)a.x[6] * n1.z + (float)a.x[7] * n1.w;
+          }
         }
       }
     }
+    bf16x8 V[4];
+#pragma unroll
+    for ( int kk = 0; kk < 4; kk++ ) {
+      V[kk] = tr_v( kk );
+    }
+#pragma unroll
+    for ( int tt = 0; tt < 2; tt++ ) { // the lane 32 further on holds the other half of this query's dims and keys
+      nq[tt] += __shfl_xor( nq[tt], 32 );
+      den[tt] += __shfl_xor( den[tt], 32 );
+      if ( g2 == 0 ) {
+        s_nq[wave][32 * tt + r] = nq[tt];
+      }
+    }
+    __syncthreads(); // both waves have read q and v, and their parts of n . q are there
+    if ( t0 + CHUNK < st.n_tokens ) {
+      fetch_qv( t0 + CHUNK );
+    }
 #pragma unroll
     for ( int tt = 0; tt < 2; tt++ ) {
-      // the lane 32 further on holds the other half of this query's dims and keys
-      const float a_q = s_a[wave][32 * tt + r];
-      float d = nq[tt] * s.q_scale * a_q + den[tt];
-      d += __shfl_xor( d, 32 );
-      const float lo = __shfl( floor_den, 32 * tt + r );
+      const uint32_t t = 32 * tt + r;
+      const float d = ( s_nq[0][t] + s_nq[1][t] ) * s.q_scale * s_a[wave][t] + den[tt];
+      const float lo = __shfl( floor_den, t );
       if ( g2 == 0 ) {
-        s_inv[wave][32 * tt + r] = 1.0f / ( fmaxf( fabsf( d ), lo ) + 1e-6f );
+        s_inv[wave][t] = 1.0f / ( fmaxf( fabsf( d ), lo ) + 1e-6f );
       }
     }
     __builtin_amdgcn_sched_barrier( 0 );
@@ -523,11 +567,6 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
     const __amdgpu_buffer_rsrc_t o_rsrc
       = __builtin_amdgcn_make_buffer_rsrc( o_out + ( row_first + t0 ) * hv + h * s.vdim, 0, (int)( ( ( rows - 1 ) * hv + s.vdim ) * 4 ), 0x00020000 );
     const uint32_t o_off = col < s.vdim ? ( 4 * g2 * hv + col ) * 4 : PAST_THE_END;
-    bf16x8 V[4];
-#pragma unroll
-    for ( int kk = 0; kk < 4; kk++ ) {
-      V[kk] = tr_v( kk );
-    }
 #pragma unroll
     for ( int tt = 0; tt < 2; tt++ ) {
 #pragma unroll
@@ -540,7 +579,7 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
       }
 #pragma unroll
       for ( int kk = 0; kk < 2 * tt + 2; kk++ ) {
-        O[tt] = mma3( P[tt][kk], V[kk], O[tt] );
+        O[tt] = mma( P[tt][kk], V[kk], O[tt] );
       }
 #pragma unroll
       for ( int q4 = 0; q4 < 4; q4++ ) {
@@ -555,16 +594,14 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
     }
     __builtin_amdgcn_sched_barrier( 0 );
     // ---- S and n behind the chunk
-    Split3 wv[4];
+    Split<3> wv[4];
 #pragma unroll
     for ( int kk = 0; kk < 4; kk++ ) {
 #pragma unroll
       for ( int hf = 0; hf < 2; hf++ ) {
         const float4 w = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 8 * hf + 4 * g2] );
-        split3( wv[kk], 4 * hf, (float)V[kk][4 * hf] * w.x );
-        split3( wv[kk], 4 * hf + 1, (float)V[kk][4 * hf + 1] * w.y );
-        split3( wv[kk], 4 * hf + 2, (float)V[kk][4 * hf + 2] * w.z );
-        split3( wv[kk], 4 * hf + 3, (float)V[kk][4 * hf + 3] * w.w );
+        wv[kk].set( 2 * hf, (float)V[kk][4 * hf] * w.x, (float)V[kk][4 * hf + 1] * w.y );
+        wv[kk].set( 2 * hf + 1, (float)V[kk][4 * hf + 2] * w.z, (float)V[kk][4 * hf + 3] * w.w );
       }
     }
 #pragma unroll
@@ -579,15 +616,19 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
 #pragma unroll
       for ( int kk = 0; kk < 4; kk++ ) {
         const bf16x8 a = tr_k( kk, dt, k_row, k_swz );
-        S[dt] = mma3( a, wv[kk], S[dt] );
-        const float4 w0 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 4 * g2] );
-        const float4 w1 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 8 + 4 * g2] );
-        nd += (float)a[0] * w0.x + (float)a[1] * w0.y + (float)a[2] * w0.z + (float)a[3] * w0.w + (float)a[4] * w1.x + (float)a[5] * w1.y + (float)a[6] * w1.z
-              + (float)a[7] * w1.w;
+        S[dt] = mma( a, wv[kk], S[dt] );
+        if ( (uint32_t)( dt / ( DT / 2 ) ) == wave ) {
+          const float4 w0 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 4 * g2] );
+          const float4 w1 = *reinterpret_cast<const float4*>( &s_w[wave][16 * kk + 8 + 4 * g2] );
+          nd += (float)a[0] * w0.x + (float)a[1] * w0.y + (float)a[2] * w0.z + (float)a[3] * w0.w + (float)a[4] * w1.x + (float)a[5] * w1.y + (float)a[6] * w1.z
+                + (float)a[7] * w1.w;
+        }
       }
-      nd += __shfl_xor( nd, 32 );
-      if ( g2 == 0 ) {
-        s_n[wave][32 * dt + r] = s_n[wave][32 * dt + r] * state_decay + nd;
+      if ( (uint32_t)( dt / ( DT / 2 ) ) == wave ) {
+        nd += __shfl_xor( nd, 32 );
+        if ( g2 == 0 ) {
+          s_n[32 * dt + r] = s_n[32 * dt + r] * state_decay + nd;
+        }
       }
     }
   }
@@ -601,12 +642,13 @@ __global__ __launch_bounds__( 128, 1 ) void mlstm_chunk_kernel( float* __restric
       __builtin_amdgcn_raw_buffer_store_b32( __builtin_bit_cast( unsigned, (float)S[dt][v] ), S_rsrc, S_off, ( 32 * dt + 8 * ( v / 4 ) + v % 4 ) * vpad * 4, 0 );
     }
   }
-  if ( slice == 0 && wave == 0 ) {
+  if ( slice == 0 ) {
     float* dst = nm_out + ( (uint64_t)ctx * s.heads + h ) * ( s.dim + 1 );
-    for ( uint32_t d = lane; d < s.dim; d += 64 ) {
-      dst[d] = s_n[0][d];
+    __syncthreads();
+    for ( uint32_t d = threadIdx.x; d < s.dim; d += 128 ) {
+      dst[d] = s_n[d];
     }
-    if ( lane == 0 ) {
+    if ( threadIdx.x == 0 ) {
       dst[s.dim] = (float)m0;
     }
   }
