@@ -107,7 +107,6 @@ __global__ __launch_bounds__( 1024 ) void window_append4_kernel( E* __restrict__
     if ( c >= p.cols ) {
       continue;
     }
-    const uint32_t h = c / p.dim, e = c % p.dim;
     union
     {
       E e[4];
@@ -118,13 +117,16 @@ __global__ __launch_bounds__( 1024 ) void window_append4_kernel( E* __restrict__
     o.e[1] = from_f32<E>( v[g].y * inv * w[g].y );
     o.e[2] = from_f32<E>( v[g].z * inv * w[g].z );
     o.e[3] = from_f32<E>( v[g].w * inv * w[g].w );
+    // (without padding the columns are where they belong already, and the divisions can be saved)
+    const bool padded = p.pad != p.dim;
+    const uint32_t h = padded ? c / p.dim : 0, e = c - h * p.dim;
     E* at = dst + (uint64_t)h * p.pad + e;
     if constexpr ( sizeof( E ) == 2 ) {
       *reinterpret_cast<uint2*>( at ) = o.half;
     } else {
       *reinterpret_cast<uint4*>( at ) = o.full;
     }
-    if ( e + 4 == p.dim ) {
+    if ( padded && e + 4 == p.dim ) {
       for ( uint32_t z = p.dim; z < p.pad; z++ ) {
         dst[(uint64_t)h * p.pad + z] = from_f32<E>( 0.0f );
       }

@@ -231,6 +231,49 @@ __global__ __launch_bounds__( 256 ) void gemm_reduce_kernel( E* __restrict__ xou
   }
 }
 
+// Few weight rows (r <= 32: the gates of a recurrent mixer) under many activation rows: bound by the activations, which the tile kernels
+// would read with most of their matrix work wasted on rows that are not there.  A work-group takes 32 activation rows, its four waves every
+// fourth 64 of the K range, straight from memory in operand order (eight lanes' pieces make whole 128-byte lines); their sums meet in LDS.
+// fp32 output (b, r).  s % 256 == 0, 16-byte aligned operands.
+constexpr uint32_t SKINNY_ROWS = 32;
+template<typename E>
+__global__ __launch_bounds__( 256 ) void gemm_skinny_kernel( float* __restrict__ out, const E* __restrict__ x, const E* __restrict__ w, uint32_t s, uint32_t r, uint32_t b )
+{
+  __shared__ float sums[4][16][64];
+  const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63, fr = lane & 31, g2 = lane >> 5;
+  const uint32_t token = blockIdx.x * 32 + fr;
+  const E* xp = x + (uint64_t)min( token, b - 1 ) * s + 8 * g2;
+  const E* wp = w + (uint64_t)min( fr, r - 1 ) * s + 8 * g2; // rows past the last repeat it and are not stored
+  mfma_f32x16 acc;
+#pragma unroll
+  for ( int v = 0; v < 16; v++ ) {
+    acc[v] = 0.0f;
+  }
+  for ( uint32_t k = wave * 64; k < s; k += 256 ) {
+#pragma unroll
+    for ( int i = 0; i < 4; i++ ) {
+      const auto a = *reinterpret_cast<const typename Mfma<E>::x8*>( wp + k + 16 * i );
+      const auto bb = *reinterpret_cast<const typename Mfma<E>::x8*>( xp + k + 16 * i );
+      acc = Mfma<E>::k16( a, bb, acc );
+    }
+  }
+  // acc[v]: weight row 8 * (v / 4) + 4 * g2 + v % 4, token fr
+#pragma unroll
+  for ( int v = 0; v < 16; v++ ) {
+    sums[wave][v][lane] = acc[v];
+  }
+  __syncthreads();
+#pragma unroll
+  for ( uint32_t i = 0; i < 4; i++ ) {
+    const uint32_t v = wave * 4 + i;
+    const uint32_t row = 8 * ( v / 4 ) + 4 * g2 + v % 4;
+    const float y = ( sums[0][v][lane] + sums[1][v][lane] ) + ( sums[2][v][lane] + sums[3][v][lane] );
+    if ( row < r && token < b ) {
+      out[(uint64_t)token * r + row] = y;
+    }
+  }
+}
+
 // f32: one wave per weight row, batch columns looped
 __global__ __launch_bounds__( 256 ) void gemm_f32_kernel( float* __restrict__ xout, const float* __restrict__ x, const float* __restrict__ w, uint32_t s, uint32_t r, uint32_t b )
 {
@@ -311,6 +354,18 @@ template<typename E>
 int gemm_half_partials( E* xout, const E* x, const E* w, uint64_t s, uint64_t r, uint64_t b, hipStream_t st, bool want_partials, float** partial_out,
                         uint32_t* splits_out )
 {
+  if ( want_partials && g_force_kernel == 0 && r <= SKINNY_ROWS && b >= 192 && b < ( 1ull << 31 ) && s % 256 == 0
+       && ( ( reinterpret_cast<uintptr_t>( x ) | reinterpret_cast<uintptr_t>( w ) ) & 15u ) == 0 ) {
+    float* ws = nullptr;
+    if ( int rc = ensure_workspace( b * r * sizeof( float ), &ws, st ) ) {
+      return rc;
+    }
+    *partial_out = ws;
+    *splits_out = 1;
+    gemm_skinny_kernel<E><<<(unsigned)( ( b + 31 ) / 32 ), 256, 0, st>>>( ws, x, w, (uint32_t)s, (uint32_t)r, (uint32_t)b );
+    GH_LAUNCH_CHECK();
+    return GH_OK;
+  }
   // many tokens at once (prefill): the MFMA-bound tile kernel; few (decode): the weight-streaming one
   if ( ( g_force_kernel == 0 || g_force_kernel == 4 ) && gemm_tile256_applicable( s, r, b, x, w, xout ? xout : x ) ) {
     float* ws = nullptr;

@@ -60,7 +60,7 @@ def assert_logits(got, want, dtype, what=""):
 
 
 # ---- mechanisms alone ----------------------------------------------------------------------------
-@pytest.mark.parametrize("b,s,r", [(1, 64, 40), (3, 52, 17), (7, 256, 512), (70, 136, 200), (200, 256, 384), (300, 512, 2048), (2048, 1024, 8192)])
+@pytest.mark.parametrize("b,s,r", [(1, 64, 40), (3, 52, 17), (7, 256, 512), (70, 136, 200), (200, 256, 384), (300, 512, 2048), (200, 512, 8), (333, 1024, 24), (1030, 2048, 32), (2048, 1024, 8192)])
 def test_bf16_products(b, s, r):
     import torch
     from glinthawk_amd import ops
