@@ -134,6 +134,87 @@ __global__ __launch_bounds__( 1024 ) void window_append4_kernel( E* __restrict__
   }
 }
 
+// prompts (bias and both norms present): work-group = a token's q, k and v together, the columns of the product in one run; all loads go out
+// together and both sums meet at one barrier
+template<typename E, typename View, int NV>
+__global__ __launch_bounds__( 1024 ) void window_append_row_kernel( E* __restrict__ q_out, View y, const E* __restrict__ bias, AppendPart pq, AppendPart pk, AppendPart pv,
+                                                                    WindowRows wr, WindowShape s, float eps )
+{
+  __shared__ float q_sums[16], k_sums[16];
+  const uint64_t row = blockIdx.x;
+  const uint32_t ctx = (uint32_t)( row / wr.n_tokens ), tok = (uint32_t)( row % wr.n_tokens );
+  uint8_t* base = static_cast<uint8_t*>( wr.rows[ctx] );
+  if ( base == nullptr ) {
+    return;
+  }
+  const uint32_t cols = pv.first + pv.cols;
+  const E *q_norm = static_cast<const E*>( pq.norm ), *k_norm = static_cast<const E*>( pk.norm );
+  float4 v[NV], w[NV];
+  float qq = 0.0f, kk = 0.0f;
+#pragma unroll
+  for ( int g = 0; g < NV; g++ ) {
+    const uint32_t c = ( g * blockDim.x + threadIdx.x ) * 4, at = c < cols ? c : 0;
+    v[g] = y.at4( row, at );
+    const bool is_q = at < pk.first;
+    w[g] = ProductView<E>::load4( is_q ? q_norm + at : k_norm + ( at < pv.first ? at - pk.first : 0 ) ); // (v: not used)
+    const float4 b = ProductView<E>::load4( bias + at );
+    v[g] = make_float4( v[g].x + b.x, v[g].y + b.y, v[g].z + b.z, v[g].w + b.w );
+    const float sum = c < pv.first ? v[g].x * v[g].x + v[g].y * v[g].y + v[g].z * v[g].z + v[g].w * v[g].w : 0.0f;
+    qq += is_q ? sum : 0.0f;
+    kk += is_q ? 0.0f : sum;
+  }
+  qq = wave_sum( qq );
+  kk = wave_sum( kk );
+  if ( ( threadIdx.x & 63 ) == 0 ) {
+    q_sums[threadIdx.x >> 6] = qq;
+    k_sums[threadIdx.x >> 6] = kk;
+  }
+  __syncthreads();
+  qq = kk = 0.0f;
+  for ( uint32_t i = 0; i < blockDim.x / WAVE; i++ ) {
+    qq += q_sums[i];
+    kk += k_sums[i];
+  }
+  const float q_inv = 1.0f / sqrtf( qq / (float)pq.cols + eps );
+  const float k_inv = 1.0f / sqrtf( kk / (float)pk.cols + eps );
+  E* q_dst = q_out + row * s.heads * s.dpad;
+  E* k_dst = reinterpret_cast<E*>( base + wr.offset ) + (uint64_t)( wr.start_pos[ctx] + tok ) * s.row_elems();
+  E* v_dst = k_dst + s.k_elems();
+#pragma unroll
+  for ( int g = 0; g < NV; g++ ) {
+    const uint32_t c = ( g * blockDim.x + threadIdx.x ) * 4;
+    if ( c >= cols ) {
+      continue;
+    }
+    const bool is_q = c < pk.first, is_v = c >= pv.first;
+    const float inv = is_q ? q_inv : k_inv;
+    const uint32_t local = c - ( is_q ? 0 : is_v ? pv.first : pk.first );
+    const uint32_t dim = is_v ? pv.dim : pq.dim, pad = is_v ? pv.pad : pq.pad;
+    union
+    {
+      E e[4];
+      uint2 half;
+      uint4 full;
+    } o;
+    o.e[0] = from_f32<E>( is_v ? v[g].x : v[g].x * inv * w[g].x );
+    o.e[1] = from_f32<E>( is_v ? v[g].y : v[g].y * inv * w[g].y );
+    o.e[2] = from_f32<E>( is_v ? v[g].z : v[g].z * inv * w[g].z );
+    o.e[3] = from_f32<E>( is_v ? v[g].w : v[g].w * inv * w[g].w );
+    const uint32_t h = pad != dim ? local / dim : 0, e = local - h * dim;
+    E* at = ( is_q ? q_dst : is_v ? v_dst : k_dst ) + (uint64_t)h * pad + e;
+    if constexpr ( sizeof( E ) == 2 ) {
+      *reinterpret_cast<uint2*>( at ) = o.half;
+    } else {
+      *reinterpret_cast<uint4*>( at ) = o.full;
+    }
+    if ( pad != dim && e + 4 == dim ) {
+      for ( uint32_t z = dim; z < pad; z++ ) {
+        at[z - e] = from_f32<E>( 0.0f );
+      }
+    }
+  }
+}
+
 // any sizes: the columns of the part pass through LDS
 template<typename E, typename View>
 __global__ __launch_bounds__( 256 ) void window_append_any_kernel( E* __restrict__ q_out, View y, const E* __restrict__ bias, AppendPart pq, AppendPart pk, AppendPart pv,
@@ -172,6 +253,12 @@ int launch_append( E* q, const View& y, const E* bias, const void* q_norm, const
   const dim3 grid( (unsigned)rows, 3 );
   const uintptr_t tables = reinterpret_cast<uintptr_t>( bias ) | reinterpret_cast<uintptr_t>( q_norm ) | reinterpret_cast<uintptr_t>( k_norm );
   if ( s.dim % 4 == 0 && s.vdim % 4 == 0 && y.stride % 4 == 0 && ( tables & 15u ) == 0 && most <= 32768 ) {
+    if ( const uint32_t all = ( nq + nk + nv ) / 4; rows >= 1024 && all <= 4096 && bias != nullptr && q_norm != nullptr && k_norm != nullptr ) {
+      const uint32_t threads = std::max<uint32_t>( 64, ( ( all + 3 ) / 4 + 63 ) / 64 * 64 );
+      window_append_row_kernel<E, View, 4><<<(unsigned)rows, threads, 0, st>>>( q, y, bias, pq, pk, pv, wr, s, eps );
+      GH_LAUNCH_CHECK();
+      return GH_OK;
+    }
     const uint32_t groups = most / 4;
     const uint32_t want = rows >= 1024 ? ( groups + 3 ) / 4 : groups;
     const uint32_t threads = std::min<uint32_t>( 1024, std::max<uint32_t>( 64, ( want + 63 ) / 64 * 64 ) );

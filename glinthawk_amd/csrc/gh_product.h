@@ -62,11 +62,13 @@ struct ProductView
     , splits( p.splits )
   {
   }
+  // a rounded output has one plane: no loop over splits, so that the loads of neighbouring groups go out together
+  __device__ __forceinline__ uint32_t planes() const { return sizeof( S ) == 2 ? 1 : splits; }
   __device__ __forceinline__ float at( uint64_t row, uint64_t col ) const
   {
     const uint64_t i = row * stride + col;
     float sum = to_f32( data[i] );
-    for ( uint32_t k = 1; k < splits; k++ ) {
+    for ( uint32_t k = 1; k < planes(); k++ ) {
       sum += to_f32( data[(uint64_t)k * plane + i] );
     }
     return sum;
@@ -77,7 +79,7 @@ struct ProductView
     const uint64_t i = row * stride + col;
     float4 sum = load4( data + i );
     // four splits in flight at a time; a split past the last reads the last again and is not added
-    for ( uint32_t k0 = 1; k0 < splits; k0 += 4 ) {
+    for ( uint32_t k0 = 1; k0 < planes(); k0 += 4 ) {
       float4 p[4];
 #pragma unroll
       for ( uint32_t u = 0; u < 4; u++ ) {

@@ -258,7 +258,7 @@ def test_bias_by_distance_in_every_row_of_the_table(dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("n_tokens", [1, 4, 250])
+@pytest.mark.parametrize("n_tokens", [1, 4, 250, 600])
 def test_query_key_norm_and_append(dtype, n_tokens):
     import torch
     from glinthawk_amd import ops
