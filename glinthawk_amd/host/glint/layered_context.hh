@@ -1,6 +1,6 @@
 // Context memory of designs whose layers keep different things per sequence: cache rows that grow with the sequence (attention) or a
 // recurrent state of fixed size.  A ContextPlan lays the parts of all layer runs out in one region; a context is one such region plus
-// the length of the sequence in it.  Recurrent state makes the order of tokens part of the contract: a context takes the token at its
+// the length of the sequence in it.  Recurrent state fixes the order of tokens: a context takes the token at its
 // length next, or starts again at position 0.  Static and paged contexts as for Llama2 (Context / DynamicContext): one allocation, or
 // 2 MiB blocks committed as the rows grow and dropped when the slot restarts.
 #pragma once
