@@ -58,11 +58,15 @@ GH_ACT_SILU, GH_ACT_GELU_TANH = 0, 1
 
 class GhStreamStep(C.Structure):
     _fields_ = [("bias", C.c_void_p), ("post_norm", C.c_void_p), ("add", C.c_void_p), ("next_norm", C.c_void_p), ("out", C.c_void_p),
-                ("out_stride", C.c_uint64), ("eps", C.c_float), ("accumulate", C.c_int)]
+                ("out_stride", C.c_uint64), ("eps", C.c_float), ("accumulate", C.c_int), ("norm_base", C.c_float)]
 
 
 class GhWindowAttn(C.Structure):
-    _fields_ = [(n, C.c_uint32) for n in ("heads", "kv_heads", "dim", "vdim", "window", "keep_first", "n_dist")] + [("scale", C.c_float)]
+    _fields_ = [(n, C.c_uint32) for n in ("heads", "kv_heads", "dim", "vdim", "window", "keep_first", "n_dist")] + [("scale", C.c_float), ("values_are_keys", C.c_uint32)]
+
+
+class GhUnitHeads(C.Structure):
+    _fields_ = [("eps", C.c_float), ("temp_coef", C.c_float), ("temp_every", C.c_uint32)]
 
 
 class GhMlstm(C.Structure):
@@ -94,6 +98,7 @@ SIGNATURES = {
     "gh_host_malloc": (_i, [C.POINTER(_vp), _u64]),
     "gh_host_free": (_i, [_vp]),
     "gh_memcpy": (_i, [_vp, _vp, _u64, _i, _i, _vp]),
+    "gh_memcpy_rows": (_i, [_vp, _u64, _vp, _u64, _u64, _u64, _i, _vp]),
     "gh_memset_zero": (_i, [_vp, _u64, _vp]),
     "gh_fill_uniform": (_i, [_vp, _u64, _f, _f, _u64, _i, _vp]),
     "gh_fill_normal": (_i, [_vp, _u64, _f, _f, _u64, _i, _vp]),
@@ -158,9 +163,12 @@ SIGNATURES = {
     "gh_matmul_scaled": (_i, [_vp, _vp, _vp, _u64, _u64, _u64, _f, _i, _vp]),
     "gh_gather_rows": (_i, [_vp, _vp, _vp, _u64, _u64, _u64, _vp]),
     "gh_window_row_bytes": (_u64, [_win, _i]),
+    "gh_window_factor_bytes": (_u64, [_win]),
     "gh_window_query_elements": (_u64, [_win]),
     "gh_matmul_window_append": (_i, [_vp, _vp, _vp, _vp, _u64, _win, _vp, _vp, _f, _vp, _u64, _vp, _u64, _u32, _i, _vp]),
-    "gh_attn_window": (_i, [_vp, _vp, _win, _vp, _vp, _u64, _vp, _u64, _u32, _u32, _i, _vp]),
+    "gh_attn_window": (_i, [_vp, _u64, _vp, _vp, _win, _vp, _vp, _u64, _u64, _vp, _u64, _u32, _u32, _i, _vp]),
+    "gh_parallel_weight_rows": (_u64, [_win, _i, _u64, C.POINTER(_u64)]),
+    "gh_matmul_parallel": (_i, [_vp, _vp, _vp, _u64, _vp, _vp, _u64, _win, C.POINTER(GhUnitHeads), _u64, _i, _vp, _u64, _u64, _vp, _u64, _u32, _i, _vp]),
     "gh_mlstm_state_bytes": (_u64, [_mls]),
     "gh_mlstm_weight_rows": (_u64, [_mls, C.POINTER(_u64)]),
     "gh_mlstm_forward": (_i, [_vp, _vp, _vp, _u64, _mls, _vp, _vp, _vp, _vp, _u64, _vp, _u64, _u32, _i, _vp]),

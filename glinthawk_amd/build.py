@@ -90,7 +90,7 @@ def build_tools() -> list[str]:
 
 # kernels of the run-time sized designs and what they stand on: all that the trace runner needs
 TRACE_KERNELS = ("gh_runtime", "gh_elementwise", "gh_gemm", "gh_gemm_lib", "gh_gemm_stream", "gh_gemm_tile", "gh_gemm_tile256",
-                 "gh_stream_rows", "gh_attn_window", "gh_mlstm")
+                 "gh_stream_rows", "gh_attn_window", "gh_parallel", "gh_mlstm")
 
 
 def _trace_run_path() -> str:

@@ -3,12 +3,14 @@
 //   position i sees j <= i with i - j < window or j < keep_first;  score = (q . k) * scale + bias[h][min(i - j, n_dist - 1)]
 //
 // cache row   [K of every kv head | V of every kv head], each head padded with zeros to a multiple of 8 elements, so that any head size
-//             is read in 16-byte (bf16) or 32-byte (fp32) pieces
+//             is read in 16-byte (bf16) or 32-byte (fp32) pieces.  Where values are keys (SHARED) a head is there once, as projected: it
+//             is read once, is the value, and its score takes 1 / rms of the key as a factor, so no second form of a key exists anywhere.
 // keys        a query's visible keys are numbered 0 .. count - 1: first the kept ones in front of the window, then the window
 // rows kernel work-group = 4 waves on one (token, kv head, block of query heads, split of the keys); 16 lanes hold one key, eight
 //             elements a lane, so a wave takes four keys at a time; every 16-lane group keeps its own running maximum and sum for
 //             each of its query heads and they meet once, at the end.  Scores, weights and sums are fp32.
 #include "gh_product.h"
+#include "gh_window.h"
 
 #include <algorithm>
 
@@ -19,22 +21,15 @@ namespace {
 typedef uint32_t u32x4_t __attribute__( ( ext_vector_type( 4 ) ) );
 typedef const u32x4_t __attribute__( ( address_space( 1 ) ) ) global_u32x4_t;
 
-struct WindowShape
+// where a row's heads go: heads * vdim columns, rows `stride` elements apart; a factor for each head's output, or NULL
+template<typename E>
+struct WindowOut
 {
-  uint32_t heads, kv_heads, group; // query heads, kv heads, query heads per kv head
-  uint32_t dim, vdim, dpad, vpad;  // padded head sizes of the cache
-  uint32_t window, keep_first, n_dist;
-  float scale;
-  __host__ __device__ uint32_t k_elems() const { return kv_heads * dpad; }
-  __host__ __device__ uint32_t row_elems() const { return kv_heads * ( dpad + vpad ); }
-};
-
-struct WindowRows
-{
-  void* const* rows; // context regions; NULL: no context
-  uint64_t offset;   // bytes from there to this layer's rows
-  const uint32_t* start_pos;
-  uint32_t n_tokens;
+  E* out;
+  uint64_t stride;
+  const float* gates;
+  uint32_t heads;
+  __device__ __forceinline__ float gate( uint64_t row, uint32_t head ) const { return gates != nullptr ? gates[row * heads + head] : 1.0f; }
 };
 
 // ---- q / k norm over the whole projection, cache append ------------------------------------------
@@ -323,7 +318,7 @@ __host__ __device__ inline uint64_t partial_stride( const WindowShape& s ) { ret
 // The results of a work-group's four waves for the query heads h0 .. h0 + nh - 1 of a row, wave w's for head h at
 // lds[(w * hq + h) * (vpad + 2)]: added up and stored, as the output or as the partial result of a split.
 template<typename E>
-__device__ __forceinline__ void finish_split( E* out, float* partial, const float* lds, uint32_t hq, uint32_t nh, uint64_t row, uint32_t h0, uint32_t split,
+__device__ __forceinline__ void finish_split( const WindowOut<E>& out, float* partial, const float* lds, uint32_t hq, uint32_t nh, uint64_t row, uint32_t h0, uint32_t split,
                                               uint32_t splits, const WindowShape& s )
 {
   const uint32_t stride = s.vpad + 2;
@@ -344,7 +339,7 @@ __device__ __forceinline__ void finish_split( E* out, float* partial, const floa
     }
     if ( splits == 1 ) {
       if ( e < s.vdim ) {
-        out[( row * s.heads + h0 + h ) * s.vdim + e] = from_f32<E>( a / sm );
+        out.out[row * out.stride + ( h0 + h ) * s.vdim + e] = from_f32<E>( a / sm * out.gate( row, h0 + h ) );
       }
     } else {
       float* dst = partial + ( ( row * s.heads + h0 + h ) * splits + split ) * stride;
@@ -358,8 +353,8 @@ __device__ __forceinline__ void finish_split( E* out, float* partial, const floa
 }
 
 // HQ query heads at a time; NC pieces of 128 elements per head (a lane holds 8 of each)
-template<typename E, int HQ, int NC>
-__global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out,
+template<typename E, int HQ, int NC, bool SHARED>
+__global__ __launch_bounds__( 256 ) void window_rows_kernel( WindowOut<E> out,
                                                              float* __restrict__ partial,
                                                              const E* __restrict__ q,
                                                              const float* __restrict__ bias,
@@ -408,8 +403,9 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
   // and gets no weight.
   constexpr uint32_t U = HQ * NC >= 4 ? 2 : 4;
   const uint32_t at_k = g * s.dpad, at_v = s.k_elems() + g * s.vpad;
+  const float* factors = reinterpret_cast<const float*>( base + wr.factors );
   for ( uint32_t i0 = k_begin + wave * 4 * U; i0 < k_end; i0 += 16 * U ) {
-    float kv[U][NC][8], vv[U][NC][8];
+    float kv[U][NC][8], vv[SHARED ? 1 : U][NC][8], factor[U];
     uint32_t dist[U];
     bool live[U];
 #pragma unroll
@@ -418,6 +414,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
       live[u] = idx < k_end;
       const uint32_t j = vis.key( live[u] ? idx : i0 );
       dist[u] = min( pos - j, s.n_dist - 1 );
+      factor[u] = SHARED ? s.scale * factors[factor_index( j, g, s.kv_heads )] : s.scale;
       const E* row_j = cache + (uint64_t)j * s.row_elems();
 #pragma unroll
       for ( int c = 0; c < NC; c++ ) {
@@ -425,13 +422,18 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
 #pragma unroll
         for ( int e = 0; e < 8; e++ ) {
           kv[u][c][e] = 0.0f;
-          vv[u][c][e] = 0.0f;
         }
         if ( at < s.dpad ) {
           load8( kv[u][c], row_j + at_k + at );
         }
-        if ( at < s.vpad ) {
-          load8( vv[u][c], row_j + at_v + at );
+        if constexpr ( !SHARED ) {
+#pragma unroll
+          for ( int e = 0; e < 8; e++ ) {
+            vv[u][c][e] = 0.0f;
+          }
+          if ( at < s.vpad ) {
+            load8( vv[u][c], row_j + at_v + at );
+          }
         }
       }
     }
@@ -450,7 +452,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
           }
         }
         const float b = bias != nullptr && (uint32_t)h < nh ? bias[(uint64_t)( h0 + h ) * s.n_dist + dist[u]] : 0.0f;
-        score[u] = live[u] ? row16_sum( dot ) * s.scale + b : NO_KEY;
+        score[u] = live[u] ? row16_sum( dot ) * factor[u] + b : NO_KEY;
         m_new = fmaxf( m_new, score[u] );
       }
       const float old = __expf( mx[h] - m_new );
@@ -469,7 +471,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
           float a = acc[h][c][e] * old;
 #pragma unroll
           for ( uint32_t u = 0; u < U; u++ ) {
-            a += p[u] * vv[u][c][e];
+            a += p[u] * ( SHARED ? kv[u][c][e] : vv[SHARED ? 0 : u][c][e] );
           }
           acc[h][c][e] = a;
         }
@@ -511,7 +513,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( E* __restrict__ out
 
 // one wave per (row, head)
 template<typename E>
-__global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ out, const float* __restrict__ partial, WindowRows wr, WindowShape s, uint32_t splits,
+__global__ __launch_bounds__( 256 ) void window_merge_kernel( WindowOut<E> out, const float* __restrict__ partial, WindowRows wr, WindowShape s, uint32_t splits,
                                                               uint64_t pairs )
 {
   const uint64_t pair = (uint64_t)blockIdx.x * 4 + ( threadIdx.x >> 6 );
@@ -524,6 +526,9 @@ __global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ ou
   for ( uint32_t k = 0; k < splits; k++ ) {
     m = fmaxf( m, src[k * stride + s.vpad + 1] );
   }
+  const uint64_t row = pair / s.heads;
+  const uint32_t head = (uint32_t)( pair % s.heads );
+  const float gate = out.gate( row, head );
   float sm = 0.0f;
   for ( uint32_t k = 0; k < splits; k++ ) {
     sm += src[k * stride + s.vpad] * __expf( src[k * stride + s.vpad + 1] - m );
@@ -533,7 +538,7 @@ __global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ ou
     for ( uint32_t k = 0; k < splits; k++ ) {
       a += src[k * stride + e] * __expf( src[k * stride + s.vpad + 1] - m );
     }
-    out[pair * s.vdim + e] = from_f32<E>( a / sm );
+    out.out[row * out.stride + head * s.vdim + e] = from_f32<E>( a / sm * gate );
   }
 }
 
@@ -548,7 +553,9 @@ __global__ __launch_bounds__( 256 ) void window_merge_kernel( E* __restrict__ ou
 // values      O^T += V^T P^T: the weights are, as they lie, the right operand; V^T comes out of LDS by transposing reads.  The weights
 //             are fp32: they enter as two bf16 terms (16 bits of mantissa), their sum is taken in fp32.
 // LDS         rows of 256 bytes whatever the head size (the rest is zero), 16-byte chunks XORed with bits of the row; the next tile's
-//             rows are in registers while this one is multiplied, and two work-groups share a CU.
+//             rows are in registers while this one is multiplied, and two work-groups share a CU.  Where values are keys both products
+//             read one tile: the low four bits of the row, pairs exchanged, keep the plain reads (16 rows, one chunk) and the
+//             transposing ones (4 rows, 4 chunks) apart.
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr float LAZY = 8.0f; // the reference point of a column's exponentials moves when its maximum has grown by 2^LAZY
 constexpr uint32_t TILE_KEYS = 64;
@@ -558,9 +565,11 @@ typedef short v4s __attribute__( ( ext_vector_type( 4 ) ) );
 typedef __attribute__( ( address_space( 3 ) ) ) v4s* lds_v4s;
 typedef Mfma<__bf16>::x8 bf16x8;
 
+__device__ __forceinline__ uint32_t shared_swizzle( uint32_t row ) { return ( ( row & 3 ) << 2 ) | ( ( row >> 2 ) & 3 ); }
+
 // KS: steps of 16 of the query/key size; VB: blocks of 32 of the value size
-template<int KS, int VB>
-__global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restrict__ out,
+template<int KS, int VB, bool SHARED>
+__global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( WindowOut<__bf16> out,
                                                                  const __bf16* __restrict__ q,
                                                                  const float* __restrict__ bias,
                                                                  WindowRows wr,
@@ -572,8 +581,9 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
 {
   extern __shared__ uint4 lds16[];
   uint4* s_k = lds16;
-  uint4* s_v = s_k + TILE_KEYS * 16;
-  float* s_bias = reinterpret_cast<float*>( s_v + TILE_KEYS * 16 ); // (head_cols, n_dist), times log2(e)
+  uint4* s_v = SHARED ? s_k : s_k + TILE_KEYS * 16;
+  float* s_factor = reinterpret_cast<float*>( s_v + TILE_KEYS * 16 );  // SHARED: of the tile's keys, times scale and log2(e)
+  float* s_bias = s_factor + ( SHARED ? TILE_KEYS : 0 );               // (head_cols, n_dist), times log2(e)
 
   // all column blocks of a pair on one XCD, next to each other in time: its keys come into one L2 once; the longest first
   const uint32_t xcd = blockIdx.x & 7, slot = blockIdx.x >> 3;
@@ -628,33 +638,46 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
 
   // a thread's four 16-byte pieces of a tile of K and of V: row threadIdx / 16 + 16 i, chunk threadIdx % 16
   const uint32_t ld_chunk = threadIdx.x & 15, ld_row = threadIdx.x >> 4;
-  u32x4_t rk[4], rv[4];
+  u32x4_t rk[4], rv[SHARED ? 1 : 4];
+  const float* factors = reinterpret_cast<const float*>( base + wr.factors );
+  float rf = 0.0f;
   auto load = [&]( uint32_t i ) {
     const uint32_t t0 = tile_at( i ), end = i < kept_tiles ? kept : pos_last + 1;
+    if ( SHARED && threadIdx.x < TILE_KEYS ) {
+      rf = factors[factor_index( min( t0 + threadIdx.x, end - 1 ), g, s.kv_heads )];
+    }
 #pragma unroll
     for ( int k = 0; k < 4; k++ ) {
       const uint32_t key = t0 + ld_row + 16 * k;
       rk[k] = u32x4_t { 0, 0, 0, 0 };
-      rv[k] = u32x4_t { 0, 0, 0, 0 };
       const __bf16* row = cache + (uint64_t)min( key, end - 1 ) * s.row_elems();
       if ( key < end && ld_chunk * 8 < s.dpad && ld_chunk < 2 * KS ) {
         rk[k] = *(global_u32x4_t*)( row + g * s.dpad + ld_chunk * 8 );
       }
-      if ( key < end && ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB ) {
-        rv[k] = *(global_u32x4_t*)( row + s.k_elems() + g * s.vpad + ld_chunk * 8 );
+      if constexpr ( !SHARED ) {
+        rv[k] = u32x4_t { 0, 0, 0, 0 };
+        if ( key < end && ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB ) {
+          rv[k] = *(global_u32x4_t*)( row + s.k_elems() + g * s.vpad + ld_chunk * 8 );
+        }
       }
     }
   };
+  const float scale_log2e = s.scale * LOG2E;
   auto store = [&] {
 #pragma unroll
     for ( int k = 0; k < 4; k++ ) {
       const uint32_t row = ld_row + 16 * k;
-      s_k[row * 16 + ( ld_chunk ^ ( row & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
-      s_v[row * 16 + ( ld_chunk ^ ( 4 * ( row & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+      s_k[row * 16 + ( ld_chunk ^ ( SHARED ? shared_swizzle( row ) : row & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
+      if constexpr ( !SHARED ) {
+        s_v[row * 16 + ( ld_chunk ^ ( 4 * ( row & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+      }
+    }
+    if ( SHARED && threadIdx.x < TILE_KEYS ) {
+      s_factor[threadIdx.x] = rf * scale_log2e;
     }
   };
   const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
-  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ) * 16 ) + ( tr_q & 1 ) * 8;
+  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ^ ( SHARED ? g2 : 0 ) ) * 16 ) + ( tr_q & 1 ) * 8;
 
   mfma_f32x16 acc[VB];
 #pragma unroll
@@ -665,7 +688,6 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
     }
   }
   float m = NO_KEY, l = 0.0f;
-  const float scale_log2e = s.scale * LOG2E;
   const float* my_bias = s_bias + hc * s.n_dist;
 
   load( 0 );
@@ -687,8 +709,21 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
 #pragma unroll
       for ( int k = 0; k < KS; k++ ) {
         const uint32_t row = 32 * sub + r;
-        const bf16x8 a = __builtin_bit_cast( bf16x8, s_k[row * 16 + ( ( 2 * k + g2 ) ^ ( row & 15 ) )] );
+        const bf16x8 a = __builtin_bit_cast( bf16x8, s_k[row * 16 + ( ( 2 * k + g2 ) ^ ( SHARED ? shared_swizzle( row ) : row & 15 ) )] );
         st[sub] = Mfma<__bf16>::k16( a, qb[k], st[sub] );
+      }
+    }
+    // what a score is multiplied with: one number, or that of its key
+    float factor[2][16];
+#pragma unroll
+    for ( int sub = 0; sub < 2; sub++ ) {
+#pragma unroll
+      for ( int q4 = 0; q4 < 4; q4++ ) {
+        float4 f = make_float4( scale_log2e, scale_log2e, scale_log2e, scale_log2e );
+        if constexpr ( SHARED ) {
+          f = *reinterpret_cast<const float4*>( s_factor + 32 * sub + 8 * q4 + 4 * g2 );
+        }
+        factor[sub][4 * q4] = f.x, factor[sub][4 * q4 + 1] = f.y, factor[sub][4 * q4 + 2] = f.z, factor[sub][4 * q4 + 3] = f.w;
       }
     }
     // ---- scale, bias by distance, mask (log2 domain)
@@ -700,7 +735,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
       for ( int sub = 0; sub < 2; sub++ ) {
 #pragma unroll
         for ( int v = 0; v < 16; v++ ) {
-          st[sub][v] = st[sub][v] * scale_log2e + b;
+          st[sub][v] = st[sub][v] * factor[sub][v] + b;
         }
       }
     } else {
@@ -709,7 +744,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
 #pragma unroll
         for ( int v = 0; v < 16; v++ ) {
           const uint32_t key = key_l + 32 * sub + 8 * ( v / 4 ) + v % 4;
-          st[sub][v] = st[sub][v] * scale_log2e + my_bias[min( pos - min( key, pos ), s.n_dist - 1 )];
+          st[sub][v] = st[sub][v] * factor[sub][v] + my_bias[min( pos - min( key, pos ), s.n_dist - 1 )];
         }
       }
     }
@@ -770,7 +805,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
         } a;
 #pragma unroll
         for ( int hf = 0; hf < 2; hf++ ) {
-          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
+          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ^ ( SHARED ? 32 * hf : 0 ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
         }
         acc[vb] = Mfma<__bf16>::k16( a.x, lo, acc[vb] );
         acc[vb] = Mfma<__bf16>::k16( a.x, hi, acc[vb] );
@@ -781,9 +816,10 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
   if ( !col_ok ) {
     return;
   }
-  const float inv = 1.0f / l;
-  __bf16* o = out + ( ( (uint64_t)ctx * wr.n_tokens + tok ) * s.heads + h0 + hc ) * s.vdim;
-  const bool wide = s.vdim % 4 == 0;
+  const uint64_t row = (uint64_t)ctx * wr.n_tokens + tok;
+  const float inv = 1.0f / l * out.gate( row, h0 + hc );
+  __bf16* o = out.out + row * out.stride + ( h0 + hc ) * s.vdim;
+  const bool wide = s.vdim % 4 == 0 && out.stride % 4 == 0;
 #pragma unroll
   for ( int vb = 0; vb < VB; vb++ ) {
 #pragma unroll
@@ -819,9 +855,13 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( __bf16* __restr
 // into registers meanwhile, without a barrier.  Adjacent work-groups read adjacent heads of the same cache rows.
 constexpr uint32_t STEP_KEYS = 32;
 constexpr uint32_t STEP_COLS = 16; // query heads of a work-group
+// LDS of a work-group in 16-byte units: the waves' tiles, and the factors of their keys behind them; the results of the waves take its place
+// at the end
+constexpr uint32_t step_lds( bool shared ) { return 4 * STEP_KEYS * ( shared ? 16 : 32 ) + ( shared ? STEP_KEYS : 0 ); }
+static_assert( step_lds( true ) * 16 >= 4 * STEP_COLS * ( 128 + 2 ) * sizeof( float ), "results of four waves, heads of up to 128" );
 
-template<int KS, int VB>
-__global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __restrict__ out,
+template<int KS, int VB, bool SHARED>
+__global__ __launch_bounds__( 256, SHARED && VB <= 2 ? 3 : 2 ) void window_decode_kernel( WindowOut<__bf16> out,
                                                                   float* __restrict__ partial,
                                                                   const __bf16* __restrict__ q,
                                                                   const float* __restrict__ bias,
@@ -831,7 +871,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
                                                                   uint32_t keys_per_split,
                                                                   uint32_t splits )
 {
-  __shared__ uint4 tiles[4][2][STEP_KEYS * 16]; // K and V of each wave, 256 bytes a key
+  __shared__ uint4 tiles[step_lds( SHARED )]; // K and V of each wave, 256 bytes a key
   const uint32_t head_blocks = s.heads / head_cols;
   const uint32_t hb = blockIdx.x % head_blocks, split = blockIdx.x / head_blocks % splits;
   const uint64_t row = blockIdx.x / head_blocks / splits;
@@ -848,8 +888,9 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
   const uint32_t wave = __builtin_amdgcn_readfirstlane( threadIdx.x >> 6 );
   const uint32_t lane = threadIdx.x & 63, r = lane & 31, g2 = lane >> 5;
   const uint32_t hc = min( r, head_cols - 1 ); // columns beyond do as the last one and are not stored
-  uint4* s_k = tiles[wave][0];
-  uint4* s_v = tiles[wave][1];
+  uint4* s_k = tiles + wave * STEP_KEYS * ( SHARED ? 16 : 32 );
+  uint4* s_v = SHARED ? s_k : s_k + STEP_KEYS * 16;
+  float* s_factor = reinterpret_cast<float*>( tiles + 4 * STEP_KEYS * ( SHARED ? 16 : 32 ) ) + wave * STEP_KEYS; // times scale and log2(e)
 
   bf16x8 qb[KS];
 #pragma unroll
@@ -864,24 +905,31 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
   const uint32_t ld_chunk = lane & 15, ld_row = lane >> 4;
   const bool k_chunk = ld_chunk * 8 < s.dpad && ld_chunk < 2 * KS, v_chunk = ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB;
   const uint32_t at_k = g * s.dpad + ld_chunk * 8, at_v = s.k_elems() + g * s.vpad + ld_chunk * 8;
-  u32x4_t rk[8], rv[8];
+  u32x4_t rk[8], rv[SHARED ? 1 : 8];
+  const float* factors = reinterpret_cast<const float*>( base + wr.factors );
+  float rf = 0.0f;
   auto load = [&]( uint32_t i0 ) {
+    if constexpr ( SHARED ) {
+      rf = factors[factor_index( vis.key( min( i0 + r, k_end - 1 ) ), g, s.kv_heads )];
+    }
 #pragma unroll
     for ( int k = 0; k < 8; k++ ) {
       const uint32_t j = vis.key( min( i0 + ld_row + 4 * k, k_end - 1 ) ); // past the end: the last key again, without weight
       const __bf16* p = cache + (uint64_t)j * s.row_elems();
       rk[k] = u32x4_t { 0, 0, 0, 0 };
-      rv[k] = u32x4_t { 0, 0, 0, 0 };
       if ( k_chunk ) {
         rk[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_k ) );
       }
-      if ( v_chunk ) {
-        rv[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_v ) );
+      if constexpr ( !SHARED ) {
+        rv[k] = u32x4_t { 0, 0, 0, 0 };
+        if ( v_chunk ) {
+          rv[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_v ) );
+        }
       }
     }
   };
   const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
-  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ) * 16 ) + ( tr_q & 1 ) * 8;
+  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ^ ( SHARED ? g2 : 0 ) ) * 16 ) + ( tr_q & 1 ) * 8;
   const float scale_log2e = s.scale * LOG2E;
   const float* my_bias = bias != nullptr ? bias + (uint64_t)( h0 + hc ) * s.n_dist : nullptr;
   const float far_bias = bias != nullptr ? my_bias[s.n_dist - 1] * LOG2E : 0.0f;
@@ -903,8 +951,13 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
 #pragma unroll
     for ( int k = 0; k < 8; k++ ) {
       const uint32_t krow = ld_row + 4 * k;
-      s_k[krow * 16 + ( ld_chunk ^ ( krow & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
-      s_v[krow * 16 + ( ld_chunk ^ ( 4 * ( krow & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+      s_k[krow * 16 + ( ld_chunk ^ ( SHARED ? shared_swizzle( krow ) : krow & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
+      if constexpr ( !SHARED ) {
+        s_v[krow * 16 + ( ld_chunk ^ ( 4 * ( krow & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+      }
+    }
+    if ( SHARED && g2 == 0 ) {
+      s_factor[r] = rf * scale_log2e;
     }
     if ( i0 + 4 * STEP_KEYS < k_end ) {
       load( i0 + 4 * STEP_KEYS );
@@ -917,20 +970,29 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
     }
 #pragma unroll
     for ( int k = 0; k < KS; k++ ) {
-      st = Mfma<__bf16>::k16( __builtin_bit_cast( bf16x8, s_k[r * 16 + ( ( 2 * k + g2 ) ^ ( r & 15 ) )] ), qb[k], st );
+      st = Mfma<__bf16>::k16( __builtin_bit_cast( bf16x8, s_k[r * 16 + ( ( 2 * k + g2 ) ^ ( SHARED ? shared_swizzle( r ) : r & 15 ) )] ), qb[k], st );
+    }
+    float factor[16];
+#pragma unroll
+    for ( int q4 = 0; q4 < 4; q4++ ) {
+      float4 f = make_float4( scale_log2e, scale_log2e, scale_log2e, scale_log2e );
+      if constexpr ( SHARED ) {
+        f = *reinterpret_cast<const float4*>( s_factor + 8 * q4 + 4 * g2 );
+      }
+      factor[4 * q4] = f.x, factor[4 * q4 + 1] = f.y, factor[4 * q4 + 2] = f.z, factor[4 * q4 + 3] = f.w;
     }
     // every distance of the tile in the bias table's last row?
     const uint32_t nearest = vis.key( min( i0 + STEP_KEYS, k_end ) - 1 );
     if ( bias == nullptr || pos - nearest >= s.n_dist - 1 ) {
 #pragma unroll
       for ( int v = 0; v < 16; v++ ) {
-        st[v] = st[v] * scale_log2e + far_bias;
+        st[v] = st[v] * factor[v] + far_bias;
       }
     } else {
 #pragma unroll
       for ( int v = 0; v < 16; v++ ) {
         const uint32_t j = vis.key( min( i0 + 8 * ( v / 4 ) + 4 * g2 + v % 4, k_end - 1 ) );
-        st[v] = st[v] * scale_log2e + my_bias[min( pos - j, s.n_dist - 1 )] * LOG2E;
+        st[v] = st[v] * factor[v] + my_bias[min( pos - j, s.n_dist - 1 )] * LOG2E;
       }
     }
     if ( i0 + STEP_KEYS > k_end ) {
@@ -981,7 +1043,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
         } a;
 #pragma unroll
         for ( int hf = 0; hf < 2; hf++ ) {
-          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
+          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ^ ( SHARED ? 32 * hf : 0 ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
         }
         acc[vb] = Mfma<__bf16>::k16( a.x, lo, acc[vb] );
         acc[vb] = Mfma<__bf16>::k16( a.x, hi, acc[vb] );
@@ -991,7 +1053,7 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
   }
   l += __shfl_xor( l, 32 );
   __syncthreads(); // the tiles' LDS takes the waves' results
-  float* results = reinterpret_cast<float*>( &tiles[0][0][0] );
+  float* results = reinterpret_cast<float*>( tiles );
   if ( r < head_cols ) {
     float* mine = results + ( wave * head_cols + r ) * ( s.vpad + 2 );
 #pragma unroll
@@ -1013,50 +1075,28 @@ __global__ __launch_bounds__( 256, 2 ) void window_decode_kernel( __bf16* __rest
   finish_split<__bf16>( out, partial, results, head_cols, head_cols, row, h0, split, splits, s );
 }
 
-WindowShape shape_of( const gh_window_attn* a )
-{
-  WindowShape s;
-  s.heads = a->heads;
-  s.kv_heads = a->kv_heads;
-  s.group = a->kv_heads ? a->heads / a->kv_heads : 0;
-  s.dim = a->dim;
-  s.vdim = a->vdim;
-  s.dpad = ( a->dim + 7 ) / 8 * 8;
-  s.vpad = ( a->vdim + 7 ) / 8 * 8;
-  s.window = a->window ? a->window : 0xffffffffu;
-  s.keep_first = a->keep_first;
-  s.n_dist = a->n_dist ? a->n_dist : 1;
-  s.scale = a->scale;
-  return s;
-}
-
-bool shape_ok( const gh_window_attn* a )
-{
-  return a->heads > 0 && a->kv_heads > 0 && a->heads % a->kv_heads == 0 && a->dim > 0 && a->vdim > 0 && a->dim <= 512 && a->vdim <= 512 && a->heads <= 4096;
-}
-
-template<typename E, int NC>
-void launch_rows( int hq, dim3 grid, hipStream_t st, E* out, float* partial, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s,
+template<typename E, int NC, bool SHARED>
+void launch_rows( int hq, dim3 grid, hipStream_t st, const WindowOut<E>& out, float* partial, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s,
                   uint32_t keys_per_split, uint32_t splits )
 {
   const size_t lds = 4ull * hq * ( s.vpad + 2 ) * sizeof( float );
   if constexpr ( NC <= 1 ) {
     if ( hq == 8 ) {
-      window_rows_kernel<E, 8, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      window_rows_kernel<E, 8, NC, SHARED><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
       return;
     }
   }
   if constexpr ( NC <= 2 ) {
     if ( hq == 4 ) {
-      window_rows_kernel<E, 4, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      window_rows_kernel<E, 4, NC, SHARED><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
       return;
     }
     if ( hq == 2 ) {
-      window_rows_kernel<E, 2, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+      window_rows_kernel<E, 2, NC, SHARED><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
       return;
     }
   }
-  window_rows_kernel<E, 1, NC><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
+  window_rows_kernel<E, 1, NC, SHARED><<<grid, 256, lds, st>>>( out, partial, q, bias, wr, s, keys_per_split, splits );
 }
 
 // Splits of the visible keys of a call's rows, and room for their partial results: as many as give every CU two work-groups, of at
@@ -1083,7 +1123,7 @@ int plan_splits( const WindowShape& s, uint64_t rows, uint64_t head_blocks, uint
   return GH_OK;
 }
 template<typename E>
-int merge_splits( E* out, const SplitPlan& plan, const WindowRows& wr, const WindowShape& s, uint64_t rows, hipStream_t st )
+int merge_splits( const WindowOut<E>& out, const SplitPlan& plan, const WindowRows& wr, const WindowShape& s, uint64_t rows, hipStream_t st )
 {
   if ( plan.splits > 1 ) {
     const uint64_t pairs = rows * s.heads;
@@ -1094,7 +1134,7 @@ int merge_splits( E* out, const SplitPlan& plan, const WindowRows& wr, const Win
 }
 
 // few rows of bf16 with heads of up to 128
-int attend_decode( __bf16* out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
+int attend_decode( const WindowOut<__bf16>& out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
 {
   uint32_t head_cols = s.group; // the largest divisor of the group that fits
   while ( head_cols > STEP_COLS || s.group % head_cols != 0 ) {
@@ -1107,20 +1147,25 @@ int attend_decode( __bf16* out, const __bf16* q, const float* bias, const Window
   }
   const uint64_t grid = rows * head_blocks * plan.splits;
   GH_REQUIRE( grid < ( 1ull << 31 ), "gh_attn_window: grid too large" );
-#define GH_WINDOW_DECODE( KS, VB ) \
-  window_decode_kernel<KS, VB><<<(unsigned)grid, 256, 0, st>>>( out, plan.partial, q, bias, wr, s, head_cols, plan.keys, plan.splits )
-  if ( s.dpad <= 64 && s.vpad <= 64 ) {
-    GH_WINDOW_DECODE( 4, 2 );
+#define GH_WINDOW_DECODE( KS, VB, SHARED ) \
+  window_decode_kernel<KS, VB, SHARED><<<(unsigned)grid, 256, 0, st>>>( out, plan.partial, q, bias, wr, s, head_cols, plan.keys, plan.splits )
+  const bool small = s.dpad <= 64 && s.vpad <= 64;
+  if ( small && s.values_are_keys ) {
+    GH_WINDOW_DECODE( 4, 2, true );
+  } else if ( small ) {
+    GH_WINDOW_DECODE( 4, 2, false );
+  } else if ( s.values_are_keys ) {
+    GH_WINDOW_DECODE( 8, 4, true );
   } else {
-    GH_WINDOW_DECODE( 8, 4 );
+    GH_WINDOW_DECODE( 8, 4, false );
   }
 #undef GH_WINDOW_DECODE
   GH_LAUNCH_CHECK();
   return merge_splits( out, plan, wr, s, rows, st );
 }
 
-template<typename E>
-int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
+template<typename E, bool SHARED>
+int attend_rows( const WindowOut<E>& out, const E* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t rows, uint32_t max_pos, hipStream_t st )
 {
   const uint32_t widest = std::max( s.dpad, s.vpad );
   const int max_hq = widest <= 128 ? 8 : widest <= 256 ? 4 : 1;
@@ -1139,11 +1184,11 @@ int attend_rows( E* out, const E* q, const float* bias, const WindowRows& wr, co
   float* partial = plan.partial;
   const dim3 grid( (unsigned)rows, head_blocks, (unsigned)splits );
   if ( widest <= 128 ) {
-    launch_rows<E, 1>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+    launch_rows<E, 1, SHARED>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
   } else if ( widest <= 256 ) {
-    launch_rows<E, 2>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+    launch_rows<E, 2, SHARED>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
   } else {
-    launch_rows<E, 4>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
+    launch_rows<E, 4, SHARED>( hq, grid, st, out, partial, q, bias, wr, s, per, (uint32_t)splits );
   }
   GH_LAUNCH_CHECK();
   return merge_splits( out, plan, wr, s, rows, st );
@@ -1162,7 +1207,7 @@ bool tiles_applicable( const WindowShape& s, const float* bias, uint32_t n_token
 {
   return n_tokens >= 16 && s.dpad <= 128 && s.vpad <= 128 && ( bias == nullptr || (uint64_t)tile_head_cols( s ) * s.n_dist <= BIAS_LDS );
 }
-int attend_tiles( __bf16* out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t batch, hipStream_t st )
+int attend_tiles( const WindowOut<__bf16>& out, const __bf16* q, const float* bias, const WindowRows& wr, const WindowShape& s, uint64_t batch, hipStream_t st )
 {
   const uint32_t head_cols = tile_head_cols( s );
   const uint32_t col_blocks = ( wr.n_tokens + 128 / head_cols - 1 ) / ( 128 / head_cols );
@@ -1170,15 +1215,23 @@ int attend_tiles( __bf16* out, const __bf16* q, const float* bias, const WindowR
   const uint64_t grid = ( n_pairs + 7 ) / 8 * 8 * col_blocks;
   GH_REQUIRE( grid < ( 1ull << 31 ), "gh_attn_window: grid too large" );
   const uint32_t bias_floats = bias == nullptr ? 0 : head_cols * s.n_dist;
-  const size_t lds = 2 * TILE_KEYS * 256 + bias_floats * sizeof( float );
-#define GH_WINDOW_TILES( KS, VB ) \
-  window_tiles_kernel<KS, VB><<<(unsigned)grid, 256, lds, st>>>( out, q, bias, wr, s, head_cols, col_blocks, (uint32_t)n_pairs, bias_floats )
-  if ( s.dpad <= 64 && s.vpad <= 64 ) {
-    GH_WINDOW_TILES( 4, 2 );
+  const size_t lds = ( s.values_are_keys ? TILE_KEYS * ( 256 + sizeof( float ) ) : 2 * TILE_KEYS * 256 ) + bias_floats * sizeof( float );
+#define GH_WINDOW_TILES( KS, VB, SHARED ) \
+  window_tiles_kernel<KS, VB, SHARED><<<(unsigned)grid, 256, lds, st>>>( out, q, bias, wr, s, head_cols, col_blocks, (uint32_t)n_pairs, bias_floats )
+  if ( s.values_are_keys ) {
+    if ( s.dpad <= 64 ) {
+      GH_WINDOW_TILES( 4, 2, true );
+    } else if ( s.dpad <= 96 ) {
+      GH_WINDOW_TILES( 6, 3, true );
+    } else {
+      GH_WINDOW_TILES( 8, 4, true );
+    }
+  } else if ( s.dpad <= 64 && s.vpad <= 64 ) {
+    GH_WINDOW_TILES( 4, 2, false );
   } else if ( s.vpad <= 64 ) {
-    GH_WINDOW_TILES( 8, 2 );
+    GH_WINDOW_TILES( 8, 2, false );
   } else {
-    GH_WINDOW_TILES( 8, 4 );
+    GH_WINDOW_TILES( 8, 4, false );
   }
 #undef GH_WINDOW_TILES
   GH_LAUNCH_CHECK();
@@ -1192,9 +1245,11 @@ using namespace gh;
 
 extern "C" {
 
-uint64_t gh_window_row_bytes( const gh_window_attn* a, gh_dtype dt ) { return (uint64_t)shape_of( a ).row_elems() * dtype_size( dt ); }
+uint64_t gh_window_row_bytes( const gh_window_attn* a, gh_dtype dt ) { return (uint64_t)window_shape( a ).row_elems() * dtype_size( dt ); }
 
-uint64_t gh_window_query_elements( const gh_window_attn* a ) { return (uint64_t)a->heads * shape_of( a ).dpad; }
+uint64_t gh_window_factor_bytes( const gh_window_attn* a ) { return a->values_are_keys ? (uint64_t)a->kv_heads * sizeof( float ) : 0; }
+
+uint64_t gh_window_query_elements( const gh_window_attn* a ) { return (uint64_t)a->heads * window_shape( a ).dpad; }
 
 int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const void* bias, uint64_t width, const gh_window_attn* a, const void* q_norm,
                              const void* k_norm, float eps, void* const* context_rows_dev, uint64_t cache_offset, const uint32_t* start_pos_dev, uint64_t batch,
@@ -1209,23 +1264,24 @@ int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const voi
   }
   GH_REQUIRE( q && x && wqkv && a && context_rows_dev && start_pos_dev, "gh_matmul_window_append: NULL pointer" );
   GH_REQUIRE( dt == GH_BF16 || dt == GH_F32, "gh_matmul_window_append: unsupported dtype %d", (int)dt );
-  GH_REQUIRE( shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_matmul_window_append: bad shape" );
-  const WindowShape s = shape_of( a );
+  GH_REQUIRE( window_shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0 && !a->values_are_keys, "gh_matmul_window_append: bad shape" );
+  const WindowShape s = window_shape( a );
   const uint64_t r = (uint64_t)s.heads * s.dim + (uint64_t)s.kv_heads * ( s.dim + s.vdim );
   hipStream_t st = as_stream( stream );
   Product y;
   if ( int rc = make_product( x, wqkv, width, r, rows, dt, false, st, &y ) ) {
     return rc;
   }
-  const WindowRows wr { context_rows_dev, cache_offset, start_pos_dev, n_tokens };
+  const WindowRows wr { context_rows_dev, cache_offset, 0, start_pos_dev, n_tokens };
   return with_product( dt, y, [&]( auto tag, auto view ) -> int {
     using E = decltype( tag );
     return launch_append<E>( static_cast<E*>( q ), view, static_cast<const E*>( bias ), q_norm, k_norm, eps, wr, s, rows, st );
   } );
 }
 
-int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const float* distance_bias_dev, void* const* context_rows_dev, uint64_t cache_offset,
-                    const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, uint32_t max_start_pos, gh_dtype dt, gh_stream stream )
+int gh_attn_window( void* out, uint64_t out_stride, const float* head_gates, const void* q, const gh_window_attn* a, const float* distance_bias_dev,
+                    void* const* context_rows_dev, uint64_t cache_offset, uint64_t factor_offset, const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens,
+                    uint32_t max_start_pos, gh_dtype dt, gh_stream stream )
 {
   if ( int rc = ensure_init() ) {
     return rc;
@@ -1236,20 +1292,28 @@ int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const flo
   }
   GH_REQUIRE( out && q && a && context_rows_dev && start_pos_dev, "gh_attn_window: NULL pointer" );
   GH_REQUIRE( dt == GH_BF16 || dt == GH_F32, "gh_attn_window: unsupported dtype %d", (int)dt );
-  GH_REQUIRE( shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_attn_window: bad shape" );
-  const WindowShape s = shape_of( a );
-  const WindowRows wr { context_rows_dev, cache_offset, start_pos_dev, n_tokens };
+  GH_REQUIRE( window_shape_ok( a ) && rows < ( 1ull << 31 ) && cache_offset % 16 == 0, "gh_attn_window: bad shape" );
+  const WindowShape s = window_shape( a );
+  GH_REQUIRE( out_stride >= (uint64_t)s.heads * s.vdim && factor_offset % 16 == 0, "gh_attn_window: bad stride or offset" );
+  const WindowRows wr { context_rows_dev, cache_offset, factor_offset, start_pos_dev, n_tokens };
   const uint32_t max_pos = max_start_pos + n_tokens - 1;
+  hipStream_t st = as_stream( stream );
   if ( dt == GH_F32 ) {
-    return attend_rows<float>( static_cast<float*>( out ), static_cast<const float*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+    const WindowOut<float> to { static_cast<float*>( out ), out_stride, head_gates, s.heads };
+    const float* qf = static_cast<const float*>( q );
+    return s.values_are_keys ? attend_rows<float, true>( to, qf, distance_bias_dev, wr, s, rows, max_pos, st )
+                             : attend_rows<float, false>( to, qf, distance_bias_dev, wr, s, rows, max_pos, st );
   }
+  const WindowOut<__bf16> to { static_cast<__bf16*>( out ), out_stride, head_gates, s.heads };
+  const __bf16* qb = static_cast<const __bf16*>( q );
   if ( tiles_applicable( s, distance_bias_dev, n_tokens ) ) {
-    return attend_tiles( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, batch, as_stream( stream ) );
+    return attend_tiles( to, qb, distance_bias_dev, wr, s, batch, st );
   }
   if ( s.dpad <= 128 && s.vpad <= 128 ) {
-    return attend_decode( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+    return attend_decode( to, qb, distance_bias_dev, wr, s, rows, max_pos, st );
   }
-  return attend_rows<__bf16>( static_cast<__bf16*>( out ), static_cast<const __bf16*>( q ), distance_bias_dev, wr, s, rows, max_pos, as_stream( stream ) );
+  return s.values_are_keys ? attend_rows<__bf16, true>( to, qb, distance_bias_dev, wr, s, rows, max_pos, st )
+                           : attend_rows<__bf16, false>( to, qb, distance_bias_dev, wr, s, rows, max_pos, st );
 }
 
 } // extern "C"

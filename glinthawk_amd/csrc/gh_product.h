@@ -96,6 +96,25 @@ struct ProductView
     }
     return sum;
   }
+  // eight neighbouring columns; col % 8 == 0, stride % 8 == 0
+  __device__ __forceinline__ void at8( float out[8], uint64_t row, uint64_t col ) const
+  {
+    if constexpr ( sizeof( S ) == 2 ) {
+      union
+      {
+        uint4 raw;
+        S v[8];
+      } u;
+      u.raw = *reinterpret_cast<const uint4*>( data + row * stride + col );
+#pragma unroll
+      for ( int i = 0; i < 8; i++ ) {
+        out[i] = to_f32( u.v[i] );
+      }
+    } else {
+      const float4 a = at4( row, col ), b = at4( row, col + 4 );
+      out[0] = a.x, out[1] = a.y, out[2] = a.z, out[3] = a.w, out[4] = b.x, out[5] = b.y, out[6] = b.z, out[7] = b.w;
+    }
+  }
   static __device__ __forceinline__ float4 load4( const S* p )
   {
     if constexpr ( sizeof( S ) == 4 ) {
@@ -111,6 +130,18 @@ struct ProductView
     }
   }
 };
+
+// activation of a gated feed-forward, for storage type E
+template<typename E>
+__device__ __forceinline__ float activate( float z, int act )
+{
+  if ( act == GH_ACT_GELU_TANH ) {
+    const float u = 0.7978845608028654f * ( z + 0.044715f * z * z * z );
+    // 0.5 (1 + tanh u) = 1 / (1 + exp(-2u)); the fp32 build takes the library's tanh
+    return sizeof( E ) == 4 ? 0.5f * z * ( 1.0f + tanhf( u ) ) : z / ( 1.0f + __expf( -2.0f * u ) );
+  }
+  return z / ( 1.0f + ( sizeof( E ) == 4 ? expf( -z ) : __expf( -z ) ) );
+}
 
 // run( storage tag, view ): the follow-up kernel of a product, instantiated for bf16 and fp32 storage
 template<typename F>

@@ -282,6 +282,18 @@ int timer_mark( hipStream_t stream, int* slot_inout, int which )
   return GH_OK;
 }
 
+namespace {
+bool copy_kind( gh_copy_kind kind, hipMemcpyKind* out )
+{
+  switch ( kind ) {
+    case GH_HOST_TO_DEVICE: *out = hipMemcpyHostToDevice; return true;
+    case GH_DEVICE_TO_HOST: *out = hipMemcpyDeviceToHost; return true;
+    case GH_DEVICE_TO_DEVICE: *out = hipMemcpyDeviceToDevice; return true;
+    case GH_HOST_TO_HOST: *out = hipMemcpyHostToHost; return true;
+    default: return false;
+  }
+}
+} // namespace
 } // namespace gh
 
 using namespace gh;
@@ -480,17 +492,30 @@ int gh_memcpy( void* dst, const void* src, uint64_t bytes, gh_copy_kind kind, in
   }
   GH_REQUIRE( dst != nullptr && src != nullptr, "gh_memcpy: NULL pointer" );
   hipMemcpyKind k;
-  switch ( kind ) {
-    case GH_HOST_TO_DEVICE: k = hipMemcpyHostToDevice; break;
-    case GH_DEVICE_TO_HOST: k = hipMemcpyDeviceToHost; break;
-    case GH_DEVICE_TO_DEVICE: k = hipMemcpyDeviceToDevice; break;
-    case GH_HOST_TO_HOST: k = hipMemcpyHostToHost; break;
-    default: return fail( GH_ERR_INVALID, "gh_memcpy: bad copy kind %d", (int)kind );
-  }
+  GH_REQUIRE( copy_kind( kind, &k ), "gh_memcpy: bad copy kind %d", (int)kind );
   GH_HIP( hipMemcpyAsync( dst, src, bytes, k, as_stream( stream ) ) );
   if ( !async ) {
     GH_HIP( hipStreamSynchronize( as_stream( stream ) ) );
   }
+  return GH_OK;
+}
+
+int gh_memcpy_rows( void* dst, uint64_t dst_stride, const void* src, uint64_t src_stride, uint64_t bytes, uint64_t rows, gh_copy_kind kind, gh_stream stream )
+{
+  if ( dst_stride == bytes && src_stride == bytes ) {
+    return gh_memcpy( dst, src, bytes * rows, kind, 0, stream );
+  }
+  if ( int rc = ensure_init() ) {
+    return rc;
+  }
+  if ( bytes == 0 || rows == 0 ) {
+    return GH_OK;
+  }
+  GH_REQUIRE( dst != nullptr && src != nullptr && dst_stride >= bytes && src_stride >= bytes, "gh_memcpy_rows: bad argument" );
+  hipMemcpyKind k;
+  GH_REQUIRE( copy_kind( kind, &k ), "gh_memcpy_rows: bad copy kind %d", (int)kind );
+  GH_HIP( hipMemcpy2DAsync( dst, dst_stride, src, src_stride, bytes, rows, k, as_stream( stream ) ) );
+  GH_HIP( hipStreamSynchronize( as_stream( stream ) ) );
   return GH_OK;
 }
 

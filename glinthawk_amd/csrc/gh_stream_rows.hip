@@ -45,6 +45,7 @@ struct StepPtrs
   uint64_t out_stride;
   float eps;
   int accumulate;
+  float norm_base; // added to the weights of the norms
 };
 
 __device__ __forceinline__ float row_sum( float v, float* smem )
@@ -106,7 +107,8 @@ __global__ __launch_bounds__( 1024 ) void stream_step_kernel( float* __restrict_
 #pragma unroll
       for ( int g = 0; g < NV; g++ ) {
         const float4 w = load4_e<E>( p.post_norm, col[g] );
-        v[g] = make_float4( v[g].x * inv * w.x, v[g].y * inv * w.y, v[g].z * inv * w.z, v[g].w * inv * w.w );
+        v[g] = make_float4( v[g].x * inv * ( p.norm_base + w.x ), v[g].y * inv * ( p.norm_base + w.y ), v[g].z * inv * ( p.norm_base + w.z ),
+                            v[g].w * inv * ( p.norm_base + w.w ) );
       }
     }
 #pragma unroll
@@ -143,7 +145,11 @@ __global__ __launch_bounds__( 1024 ) void stream_step_kernel( float* __restrict_
   E* out = static_cast<E*>( p.out ) + row * p.out_stride;
 #pragma unroll
   for ( int g = 0; g < NV; g++ ) {
-    const float4 w = p.next_norm != nullptr ? load4_e<E>( p.next_norm, col[g] ) : make_float4( 1.0f, 1.0f, 1.0f, 1.0f );
+    float4 w = make_float4( 1.0f, 1.0f, 1.0f, 1.0f );
+    if ( p.next_norm != nullptr ) {
+      w = load4_e<E>( p.next_norm, col[g] );
+      w = make_float4( p.norm_base + w.x, p.norm_base + w.y, p.norm_base + w.z, p.norm_base + w.w );
+    }
     union
     {
       E e[4];
@@ -186,7 +192,7 @@ __global__ __launch_bounds__( 256 ) void stream_step_any_kernel( float* __restri
     for ( uint32_t c = threadIdx.x; c < width; c += blockDim.x ) {
       float v = y.at( row, c ) + ( bias != nullptr ? to_f32( bias[c] ) : 0.0f );
       if ( post != nullptr ) {
-        v = v * inv * to_f32( post[c] );
+        v = v * inv * ( p.norm_base + to_f32( post[c] ) );
       }
       v = ( p.accumulate ? xr[c] : 0.0f ) + v;
       if ( add != nullptr ) {
@@ -208,7 +214,7 @@ __global__ __launch_bounds__( 256 ) void stream_step_any_kernel( float* __restri
   }
   E* out = static_cast<E*>( p.out ) + row * p.out_stride;
   for ( uint32_t c = threadIdx.x; c < width; c += blockDim.x ) {
-    out[c] = from_f32<E>( xr[c] * inv * ( next != nullptr ? to_f32( next[c] ) : 1.0f ) );
+    out[c] = from_f32<E>( xr[c] * inv * ( next != nullptr ? p.norm_base + to_f32( next[c] ) : 1.0f ) );
   }
 }
 
@@ -245,21 +251,10 @@ int launch_step( float* x, const View& y, uint64_t width, uint64_t rows, const S
 
 StepPtrs step_ptrs( const gh_stream_step* s )
 {
-  return StepPtrs { s->bias, s->post_norm, s->add, s->next_norm, s->out, s->out_stride, s->eps, s->accumulate };
+  return StepPtrs { s->bias, s->post_norm, s->add, s->next_norm, s->out, s->out_stride, s->eps, s->accumulate, s->norm_base };
 }
 
 // ---- gate of a feed-forward --------------------------------------------------------------------
-template<typename E>
-__device__ __forceinline__ float activate( float z, int act )
-{
-  if ( act == GH_ACT_GELU_TANH ) {
-    const float u = 0.7978845608028654f * ( z + 0.044715f * z * z * z );
-    // 0.5 (1 + tanh u) = 1 / (1 + exp(-2u)); the fp32 build takes the library's tanh
-    return sizeof( E ) == 4 ? 0.5f * z * ( 1.0f + tanhf( u ) ) : z / ( 1.0f + __expf( -2.0f * u ) );
-  }
-  return z / ( 1.0f + ( sizeof( E ) == 4 ? expf( -z ) : __expf( -z ) ) );
-}
-
 // grid: (column groups of a row / 256, rows); V columns a thread: 8 (rounded products), 4 or 1
 template<typename E, typename View, int V>
 __global__ __launch_bounds__( 256 ) void gate_rows_kernel( E* __restrict__ hb, View y, const E* __restrict__ bias, uint32_t hidden, int act )

@@ -187,7 +187,9 @@ int main( int argc, char* argv[] )
       out = value;
     } else if ( arg == "--contexts" ) {
       options.max_context_count = std::strtoull( value.c_str(), nullptr, 10 );
-    } else if ( arg != "--max-tokens" ) { // contexts hold the model's positions each: nothing to size by a token count
+    } else if ( arg == "--max-tokens" ) { // a request holds no more: what a context has to where the model does not bound it
+      options.max_positions = static_cast<uint32_t>( std::min<uint64_t>( std::strtoull( value.c_str(), nullptr, 10 ), 0x3fffffff ) );
+    } else {
       quit( "unknown option " + arg );
     }
   }

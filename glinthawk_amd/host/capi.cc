@@ -222,13 +222,14 @@ struct BookManager
 
 using PagedBookContext = glint::DynamicContext<BookConfig, float16_t, CountingRegion>;
 
-DesignOptions design_options( int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+DesignOptions design_options( int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t max_positions, uint32_t flags, uint64_t seed, float weight_std )
 {
   DesignOptions o;
   o.dtype = dtype == 1 ? DataType::Float32 : dtype == 2 ? DataType::BFloat16 : DataType::Float16;
   o.paged = flags & 4u;
   o.concurrency_limit = concurrency;
   o.max_context_count = max_contexts;
+  o.max_positions = max_positions;
   o.model.seed = seed;
   o.model.weight_std = weight_std;
   o.model.randomize = flags & 64u;
@@ -374,10 +375,12 @@ void* glint_stage_create( const char* config, int dtype, uint32_t first_layer, u
 }
 
 // A stage over the model in a directory: a run-time sized design named by config.json, weights loaded (flags & 64: drawn, only
-// config.json is read).  dtype 1 f32, 2 bf16; flags & 4 paged contexts.  NULL on failure, see glint_last_error().
-void* glint_stage_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+// config.json is read).  dtype 1 f32, 2 bf16; max_positions: see DesignOptions; flags & 4 paged contexts.  NULL on failure, see
+// glint_last_error().
+void* glint_stage_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t max_positions, uint32_t flags, uint64_t seed,
+                        float weight_std )
 {
-  return open_design_stage( model_dir, design_options( dtype, concurrency, max_contexts, flags, seed, weight_std ), g_last_error ).release();
+  return open_design_stage( model_dir, design_options( dtype, concurrency, max_contexts, max_positions, flags, seed, weight_std ), g_last_error ).release();
 }
 // what: 0 vocabulary, 1 positions, 2 layer runs of one step (0 for models that do not say)
 uint64_t glint_stage_size( void* h, int what )
@@ -539,13 +542,14 @@ uint64_t glint_book_paged_prepare( void* c, uint32_t layer, uint32_t token_pos, 
   return ctx->allocated_bytes( layer );
 }
 
-// paged context of a run-time sized design over a counting region: parts in order, row_bytes[i] > 0: cache rows, else a state of state_bytes[i]
-void* glint_book_layered_new( uint32_t max_positions, uint32_t n_parts, const uint64_t* row_bytes, const uint64_t* state_bytes )
+// paged context of a run-time sized design over a counting region: parts in order, row_bytes[i] > 0: cache rows in groups of groups[i] tokens,
+// else a state of state_bytes[i]
+void* glint_book_layered_new( uint32_t max_positions, uint32_t n_parts, const uint64_t* row_bytes, const uint64_t* state_bytes, const uint32_t* groups )
 {
   auto plan = std::make_shared<ContextPlan>( max_positions );
   for ( uint32_t i = 0; i < n_parts; i++ ) {
     if ( row_bytes[i] > 0 ) {
-      plan->add_rows( row_bytes[i] );
+      plan->add_rows( row_bytes[i], groups[i] );
     } else {
       plan->add_state( state_bytes[i] );
     }
@@ -583,6 +587,28 @@ int64_t glint_book_famidra_runs( const char* config_json, uint32_t* out, uint64_
     out[2 * i + 1] = static_cast<uint32_t>( runs[i].pass + 1 );
   }
   return static_cast<int64_t>( runs.size() );
+}
+
+// sizes and constants of a Dirozen config.json: (width, vocab, layers), then (heads, kv_heads, dim, ff, temp_every) of each layer, up to cap
+// numbers, and (eps, then scale and temp_coef of each layer); the layers, or -1 (see glint_last_error())
+int64_t glint_book_dirozen_config( const char* config_json, uint32_t* sizes, uint64_t cap, float* constants )
+{
+  DirozenConfig c;
+  g_last_error = DirozenConfig::parse( config_json, c );
+  if ( !g_last_error.empty() ) {
+    return -1;
+  }
+  std::vector<uint32_t> n { c.width, c.vocab, static_cast<uint32_t>( c.layers.size() ) };
+  std::vector<float> f { c.eps };
+  for ( const auto& l : c.layers ) {
+    n.insert( n.end(), { l.heads, l.kv_heads, l.dim, l.ff, l.temp_every } );
+    f.insert( f.end(), { l.scale, l.temp_coef } );
+  }
+  if ( n.size() <= cap ) {
+    std::copy( n.begin(), n.end(), sizes );
+    std::copy( f.begin(), f.end(), constants );
+  }
+  return static_cast<int64_t>( c.layers.size() );
 }
 
 // KV addressing of the host layer, in elements from the context base (UINT64_MAX: layer not hosted)
@@ -750,10 +776,11 @@ void* glint_kernel_create( const char* config, int dtype, uint32_t first_layer, 
   return nullptr;
 }
 // the compute kernel around the design in a model directory, arguments as glint_stage_open
-void* glint_kernel_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t flags, uint64_t seed, float weight_std )
+void* glint_kernel_open( const char* model_dir, int dtype, uint32_t concurrency, uint32_t max_contexts, uint32_t max_positions, uint32_t flags, uint64_t seed,
+                         float weight_std )
 {
   KernelBase* kernel = nullptr;
-  const DesignOptions o = design_options( dtype, concurrency, max_contexts, flags, seed, weight_std );
+  const DesignOptions o = design_options( dtype, concurrency, max_contexts, max_positions, flags, seed, weight_std );
   g_last_error = with_design( model_dir, o, [&]( auto tag, const auto& config, const auto& settings, const ModelOptions& options ) -> std::string {
     using Model = typename decltype( tag )::type;
     auto made = std::make_unique<KernelImpl<Model>>( config, settings, options );

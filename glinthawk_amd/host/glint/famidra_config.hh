@@ -3,16 +3,14 @@
 // that is passed several times with the same weights.
 #pragma once
 
+#include <algorithm>
+#include <cmath>
 #include <cstdint>
-#include <filesystem>
-#include <fstream>
 #include <optional>
-#include <sstream>
 #include <string>
 #include <vector>
 
-#include "glint/json.hh"
-#include "glint/types.hh"
+#include "glint/design_config.hh"
 
 namespace glint {
 
@@ -82,32 +80,14 @@ struct FamidraConfig
   }
 
   // empty string on success
-  static std::string parse( const std::string& text, FamidraConfig& out )
-  {
-    try {
-      out = from_json( Json::parse( text ) );
-      return {};
-    } catch ( const std::exception& e ) {
-      return std::string( "config.json: " ) + e.what();
-    }
-  }
-
-private:
-  static uint32_t size_of( const Json& v, const char* what, const uint32_t least = 1 )
-  {
-    const uint64_t n = v[what].integer();
-    if ( n < least || n > 0x3fffffffull ) {
-      throw JsonError( std::string( what ) + " is out of range" );
-    }
-    return static_cast<uint32_t>( n );
-  }
+  static std::string parse( const std::string& text, FamidraConfig& out ) { return parse_config( text, out ); }
 
   static FamidraConfig from_json( const Json& j )
   {
     FamidraConfig c;
-    c.width = size_of( j, "width" );
-    c.vocab = size_of( j, "vocab" );
-    c.max_positions = size_of( j, "max_positions" );
+    c.width = json_size( j, "width" );
+    c.vocab = json_size( j, "vocab" );
+    c.max_positions = json_size( j, "max_positions" );
     c.eps = static_cast<float>( j["norm"]["eps"].number() );
     if ( const Json* s = j.find( "logit_scale" ); s != nullptr && !s->is_null() ) {
       c.logit_scale = static_cast<float>( s->number() );
@@ -117,35 +97,30 @@ private:
       const Json& m = l["mixer"];
       const std::string& type = l["type"].string();
       if ( type == "mlstm" ) {
-        layer.mlstm = MlstmConfig { size_of( m, "heads" ), size_of( m, "dim" ), size_of( m, "vdim" ), static_cast<float>( m["gate_cap"].number() ) };
+        layer.mlstm = MlstmConfig { json_size( m, "heads" ), json_size( m, "dim" ), json_size( m, "vdim" ), static_cast<float>( m["gate_cap"].number() ) };
         if ( !( layer.mlstm->gate_cap > 0 ) ) {
           throw JsonError( "gate_cap must be positive" );
         }
       } else if ( type == "attention" ) {
         WindowAttentionConfig a;
-        a.heads = size_of( m, "heads" );
-        a.kv_heads = size_of( m, "kv_heads" );
-        a.dim = size_of( m, "dim" );
-        a.vdim = size_of( m, "vdim" );
+        a.heads = json_size( m, "heads" );
+        a.kv_heads = json_size( m, "kv_heads" );
+        a.dim = json_size( m, "dim" );
+        a.vdim = json_size( m, "vdim" );
         a.scale = static_cast<float>( m["scale"].number() );
         a.bias_max = m["bias_max"].number();
         if ( a.heads % a.kv_heads != 0 || !( a.bias_max > 0 && a.bias_max < 1e8 ) ) {
           throw JsonError( "attention: heads must be a multiple of kv_heads and bias_max positive" );
         }
         if ( const Json* mask = m.find( "mask" ); mask != nullptr && !mask->is_null() ) {
-          a.window = size_of( *mask, "size" );
-          a.keep_first = mask->find( "keep_first" ) != nullptr ? size_of( *mask, "keep_first", 0 ) : 0;
+          a.window = json_size( *mask, "size" );
+          a.keep_first = mask->find( "keep_first" ) != nullptr ? json_size( *mask, "keep_first", 0 ) : 0;
         }
         layer.attention = a;
       } else {
         throw JsonError( "unknown layer type \"" + type + "\"" );
       }
-      if ( const Json* mlp = l.find( "mlp" ); mlp != nullptr && !mlp->is_null() ) {
-        if ( ( *mlp )["kind"].string() != "dense" ) {
-          throw JsonError( "unknown feed-forward kind \"" + ( *mlp )["kind"].string() + "\"" );
-        }
-        layer.ff = size_of( *mlp, "ff" );
-      }
+      layer.ff = dense_feed_forward( l );
       c.layers.push_back( layer );
     }
     if ( c.layers.empty() ) {
@@ -153,9 +128,9 @@ private:
     }
     if ( const Json* loop = j.find( "loop" ); loop != nullptr && !loop->is_null() ) {
       c.looped = true;
-      c.loop_start = size_of( *loop, "start", 0 );
-      c.loop_stop = size_of( *loop, "stop" );
-      c.loop_times = size_of( *loop, "times" );
+      c.loop_start = json_size( *loop, "start", 0 );
+      c.loop_stop = json_size( *loop, "stop" );
+      c.loop_times = json_size( *loop, "times" );
       if ( c.loop_start >= c.loop_stop || c.loop_stop > c.layers.size() || (uint64_t)c.loop_times * ( c.loop_stop - c.loop_start ) > 65536 ) {
         throw JsonError( "loop does not fit the layers" );
       }
@@ -178,33 +153,6 @@ inline uint32_t distance_bucket( const uint64_t distance, const uint32_t rows, c
   }
   const double at = std::log( static_cast<double>( distance ) / half ) / std::log( bias_max / half ) * ( rows - half );
   return !( at < rows - 1 - half ) ? rows - 1 : half + static_cast<uint32_t>( std::max( 0.0, at ) + 1e-9 );
-}
-
-// text of a file; false when it cannot be read
-inline bool read_text_file( const std::filesystem::path& path, std::string& out )
-{
-  std::ifstream in { path, std::ios::binary };
-  if ( !in ) {
-    return false;
-  }
-  std::ostringstream text;
-  text << in.rdbuf();
-  out = text.str();
-  return true;
-}
-
-// "architecture" of the config.json of a model directory; empty when there is none
-inline std::string architecture_of( const std::filesystem::path& model_dir )
-{
-  std::string text;
-  if ( !read_text_file( model_dir / "config.json", text ) ) {
-    return {};
-  }
-  try {
-    return Json::parse( text )["architecture"].string();
-  } catch ( const std::exception& ) {
-    return {};
-  }
 }
 
 } // namespace glint

@@ -23,10 +23,13 @@ struct ContextPlan
     uint64_t offset { 0 };    // from the start of the region
     uint64_t row_bytes { 0 }; // cache row of one token; 0: a state
     uint64_t bytes { 0 };
+    uint32_t group { 1 };     // tokens whose rows are laid out together
+    // of the part, for a sequence of `tokens` tokens
+    uint64_t needed( const uint64_t tokens ) const { return row_bytes == 0 ? bytes : std::min( bytes, row_bytes * ( ( tokens + group - 1 ) / group * group ) ); }
   };
   static constexpr uint64_t ALIGN = 256;
 
-  std::vector<Part> parts {}; // one per layer run
+  std::vector<Part> parts {}; // one or more per layer run, in the order a design adds them
   uint64_t bytes { 0 };
   uint32_t max_positions { 0 };
 
@@ -34,13 +37,16 @@ struct ContextPlan
     : max_positions( positions )
   {
   }
-  void add_rows( const uint64_t row_bytes ) { add( row_bytes, row_bytes * max_positions ); }
-  void add_state( const uint64_t state_bytes ) { add( 0, state_bytes ); }
+  void add_rows( const uint64_t row_bytes, const uint32_t group = 1 )
+  {
+    add( row_bytes, row_bytes * ( ( (uint64_t)max_positions + group - 1 ) / group * group ), group );
+  }
+  void add_state( const uint64_t state_bytes ) { add( 0, state_bytes, 1 ); }
 
 private:
-  void add( const uint64_t row_bytes, const uint64_t n )
+  void add( const uint64_t row_bytes, const uint64_t n, const uint32_t group )
   {
-    parts.push_back( { bytes, row_bytes, n } );
+    parts.push_back( { bytes, row_bytes, n, group } );
     bytes += ( n + ALIGN - 1 ) / ALIGN * ALIGN;
   }
 };
@@ -110,7 +116,7 @@ public:
       clears_++;
     }
     for ( const auto& part : plan_->parts ) {
-      const uint64_t need = part.row_bytes == 0 ? part.bytes : std::min( part.bytes, part.row_bytes * ( (uint64_t)pos + n_tokens ) );
+      const uint64_t need = part.needed( (uint64_t)pos + n_tokens );
       if ( need == 0 ) {
         continue;
       }

@@ -21,7 +21,7 @@ def _lib():
         vp, u32, u64, i = C.c_void_p, C.c_uint32, C.c_uint64, C.c_int
         sig = {
             "glint_kernel_create": (vp, [C.c_char_p, i, u32, u32, u32, u32, u32, u64, C.c_float]),
-            "glint_kernel_open": (vp, [C.c_char_p, i, u32, u32, u32, u64, C.c_float]),
+            "glint_kernel_open": (vp, [C.c_char_p, i, u32, u32, u32, u32, u64, C.c_float]),
             "glint_kernel_create_echo": (vp, [u32, u32]),
             "glint_kernel_destroy": (None, [vp]),
             "glint_kernel_load": (i, [vp, C.c_char_p]),
@@ -43,12 +43,13 @@ class ComputeKernel:
     def __init__(self, config: Optional[str] = None, dtype: str = "f16", first_layer: int = 0, n_hosted: int = 1,
                  concurrency: int = 1, max_contexts: int = 1, with_cls: bool = False, fused: bool = True,
                  fused_projections: bool = True, seed: int = 1, weight_std: float = 0.02, echo: bool = False, model_dir: Optional[str] = None,
-                 paged: bool = False):
+                 paged: bool = False, max_positions: int = 0):
         """`echo=True`: a host-only kernel (no GPU) whose model advances every active row by one token.  `model_dir`: the run-time sized
-        design in that directory (dtype bf16 or f32), weights loaded; its states carry prompts only."""
+        design in that directory (dtype bf16 or f32), weights loaded; its states carry prompts only.  `max_positions`: what a
+        context holds, for designs whose config.json does not bound it (0: the host layer's default)."""
         if model_dir is not None:
-            self._h = _lib().glint_kernel_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, FLAG_PAGED if paged else 0, seed,
-                                               weight_std)
+            self._h = _lib().glint_kernel_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, max_positions, FLAG_PAGED if paged else 0,
+                                               seed, weight_std)
             if not self._h:
                 raise GlintError(_lib().glint_last_error().decode(errors="replace"))
         elif echo:

@@ -12,7 +12,8 @@ from typing import Optional, Sequence
 import torch
 
 from . import _lib
-from ._lib import GH_ACT_GELU_TANH, GH_ATTN_AUTO, GH_BF16, GH_F16, GH_F32, GhMlstm, GhStreamStep, GhWindowAttn, Shape, check, lib
+from ._lib import (GH_ACT_GELU_TANH, GH_ACT_SILU, GH_ATTN_AUTO, GH_BF16, GH_F16, GH_F32, GhMlstm, GhStreamStep, GhUnitHeads, GhWindowAttn, Shape, check,
+                   lib)
 
 
 def _dt(t: torch.Tensor) -> int:
@@ -357,9 +358,9 @@ def embed_positions(tokens, start_pos, n_tokens: int, embed, pos_table=None, cop
     return x
 
 
-def _stream_step(eps, bias=None, post_norm=None, accumulate=True, add=None, next_norm=None, out=None):
+def _stream_step(eps, bias=None, post_norm=None, accumulate=True, add=None, next_norm=None, out=None, norm_base=0.0):
     return GhStreamStep(_p(bias), _p(post_norm), _p(add), _p(next_norm), None if out is None else out.data_ptr(), 0 if out is None else out.stride(0), eps,
-                        int(accumulate))
+                        int(accumulate), norm_base)
 
 
 def matmul_stream(x, inp, w, eps: float = 1e-5, **step) -> None:
@@ -368,8 +369,8 @@ def matmul_stream(x, inp, w, eps: float = 1e-5, **step) -> None:
     check(lib().gh_matmul_stream(_p(x), _p(inp), _p(w), w.shape[1], w.shape[0], x.shape[0], C.byref(s), _dt(w), _stream()), "gh_matmul_stream")
 
 
-def stream_out(x, out, next_norm=None, eps: float = 1e-5) -> None:
-    s = _stream_step(eps, next_norm=next_norm, out=out)
+def stream_out(x, out, next_norm=None, eps: float = 1e-5, norm_base: float = 0.0) -> None:
+    s = _stream_step(eps, next_norm=next_norm, out=out, norm_base=norm_base)
     check(lib().gh_stream_out(_p(x), x.shape[1], x.shape[0], C.byref(s), _dt(out), _stream()), "gh_stream_out")
 
 
@@ -386,12 +387,16 @@ def matmul_scaled(x, w, scale: float):
     return out
 
 
-def window_attn(heads, kv_heads, dim, vdim, scale, window=0, keep_first=0, n_dist=0) -> GhWindowAttn:
-    return GhWindowAttn(heads, kv_heads, dim, vdim, window, keep_first, n_dist, scale)
+def window_attn(heads, kv_heads, dim, vdim, scale, window=0, keep_first=0, n_dist=0, values_are_keys=False) -> GhWindowAttn:
+    return GhWindowAttn(heads, kv_heads, dim, vdim, window, keep_first, n_dist, scale, int(values_are_keys))
 
 
 def window_row_bytes(a: GhWindowAttn, dtype) -> int:
     return int(lib().gh_window_row_bytes(C.byref(a), GH_BF16 if dtype == torch.bfloat16 else GH_F32))
+
+
+def window_factor_bytes(a: GhWindowAttn) -> int:
+    return int(lib().gh_window_factor_bytes(C.byref(a)))
 
 
 def window_query_elements(a: GhWindowAttn) -> int:
@@ -405,11 +410,34 @@ def matmul_window_append(x, wqkv, a: GhWindowAttn, ctx_rows, start_pos, n_tokens
     return q
 
 
-def attn_window(q, a: GhWindowAttn, ctx_rows, start_pos, n_tokens: int, max_start_pos: int, distance_bias=None, offset: int = 0):
-    out = torch.zeros((q.shape[0], a.heads * a.vdim), dtype=q.dtype, device=q.device)
-    check(lib().gh_attn_window(_p(out), _p(q), C.byref(a), _p(distance_bias), _p(ctx_rows), offset, _p(start_pos), start_pos.numel(), n_tokens,
-                               max_start_pos, _dt(q), _stream()), "gh_attn_window")
+def attn_window(q, a: GhWindowAttn, ctx_rows, start_pos, n_tokens: int, max_start_pos: int, distance_bias=None, offset: int = 0, factor_offset: int = 0,
+                head_gates=None, out=None):
+    """`out`: a view whose rows may lie farther apart than they are long; a new tensor when not given."""
+    if out is None:
+        out = torch.zeros((q.shape[0], a.heads * a.vdim), dtype=q.dtype, device=q.device)
+    assert out.stride(1) == 1 and out.shape == (q.shape[0], a.heads * a.vdim)
+    check(lib().gh_attn_window(out.data_ptr(), out.stride(0), _p(head_gates), _p(q), C.byref(a), _p(distance_bias), _p(ctx_rows), offset, factor_offset,
+                               _p(start_pos), start_pos.numel(), n_tokens, max_start_pos, _dt(q), _stream()), "gh_attn_window")
     return out
+
+
+def parallel_weight_rows(a: GhWindowAttn, gated: bool, ff: int):
+    """(rows of the projection matrix, first row of the feed-forward's gate)"""
+    row = C.c_uint64(0)
+    return int(lib().gh_parallel_weight_rows(C.byref(a), int(gated), ff, C.byref(row))), int(row.value)
+
+
+def matmul_parallel(x, w, a: GhWindowAttn, ctx_rows, start_pos, n_tokens: int, eps: float, temp_coef: float = 0.0, temp_every: int = 0, gated: bool = True,
+                    hidden=None, activation: int = GH_ACT_SILU, offset: int = 0, factor_offset: int = 0):
+    """Returns (q, head gates or None); the feed-forward's part goes to `hidden`, a view of (rows, ff), when given."""
+    q = torch.zeros((x.shape[0], window_query_elements(a)), dtype=x.dtype, device=x.device)
+    gates = torch.zeros((x.shape[0], a.heads), dtype=torch.float32, device=x.device) if gated else None
+    u = GhUnitHeads(eps, temp_coef, temp_every)
+    ff = 0 if hidden is None else hidden.shape[1]
+    check(lib().gh_matmul_parallel(_p(q), _p(gates), None if hidden is None else hidden.data_ptr(), 0 if hidden is None else hidden.stride(0), _p(x), _p(w),
+                                   x.shape[1], C.byref(a), C.byref(u), ff, activation, _p(ctx_rows), offset, factor_offset, _p(start_pos), start_pos.numel(),
+                                   n_tokens, _dt(x), _stream()), "gh_matmul_parallel")
+    return q, gates
 
 
 def mlstm_state_bytes(m: GhMlstm) -> int:

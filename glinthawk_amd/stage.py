@@ -41,7 +41,7 @@ def host_lib() -> C.CDLL:
         vp, u32, u64, i32 = C.c_void_p, C.c_uint32, C.c_uint64, C.c_int32
         sig = {
             "glint_stage_create": (vp, [C.c_char_p, C.c_int, u32, u32, u32, u32, u32, u64, C.c_float]),
-            "glint_stage_open": (vp, [C.c_char_p, C.c_int, u32, u32, u32, u64, C.c_float]),
+            "glint_stage_open": (vp, [C.c_char_p, C.c_int, u32, u32, u32, u32, u64, C.c_float]),
             "glint_stage_size": (u64, [vp, C.c_int]),
             "glint_stage_prefill_logits": (C.c_int, [vp, u32, vp, vp, u32, vp, vp, u32, vp, vp, vp]),
             "glint_stage_logits": (C.c_int, [vp, vp, u32]),
@@ -86,10 +86,11 @@ def host_lib() -> C.CDLL:
             "glint_book_paged_new": (vp, [u32]),
             "glint_book_paged_delete": (None, [vp]),
             "glint_book_paged_prepare": (u64, [vp, u32, u32, C.c_int, C.POINTER(u64)]),
-            "glint_book_layered_new": (vp, [u32, u32, vp, vp]),
+            "glint_book_layered_new": (vp, [u32, u32, vp, vp, vp]),
             "glint_book_layered_delete": (None, [vp]),
             "glint_book_layered_append": (C.c_int, [vp, u32, u32, C.POINTER(u64)]),
             "glint_book_distance_bucket": (u32, [u64, u32, C.c_double]),
+            "glint_book_dirozen_config": (C.c_int64, [C.c_char_p, vp, u64, vp]),
             "glint_book_famidra_runs": (C.c_int64, [C.c_char_p, vp, u64]),
             "glint_book_key_head_offset": (u64, [vp, u32, u32, u32, C.c_int]),
         }
@@ -316,13 +317,15 @@ class Stage:
 class DesignStage(Stage):
     """A whole model of a run-time sized design, opened from its model directory (config.json names the architecture,
     model.safetensors holds the weights; random_weights: only config.json is read).  The batched state, the context slots and
-    forward() are Stage's; prefill returns logits."""
+    forward() are Stage's; prefill returns logits.  max_positions: what a context holds, for designs whose config.json does not
+    bound it (0: the host layer's default)."""
 
     def __init__(self, model_dir: str, dtype: str = "bf16", concurrency: int = 1, max_contexts: int = 1, paged: bool = False,
-                 random_weights: bool = False, seed: int = 1, weight_std: float = 0.02):
+                 random_weights: bool = False, seed: int = 1, weight_std: float = 0.02, max_positions: int = 0):
         self.np_dtype = np.float32
         flags = (FLAG_PAGED if paged else 0) | (FLAG_RANDOM_WEIGHTS if random_weights else 0)
-        self._h = host_lib().glint_stage_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, flags, seed, weight_std)
+        self._h = host_lib().glint_stage_open(os.fsencode(model_dir), DESIGN_DTYPES[dtype], concurrency, max_contexts, max_positions, flags, seed,
+                                           weight_std)
         if not self._h:
             raise GlintError(host_lib().glint_last_error().decode(errors="replace"))
         self.vocab_size, self.max_positions, self.layer_runs = (int(host_lib().glint_stage_size(self._h, k)) for k in range(3))
@@ -416,13 +419,14 @@ class BookPagedContext:
 
 
 class BookLayeredContext:
-    """Host-only paged context of a run-time sized design over a region that only records commits; `parts`: ("rows", bytes a token) or
-    ("state", bytes)."""
+    """Host-only paged context of a run-time sized design over a region that only records commits; `parts`: ("rows", bytes a token,
+    optionally how many tokens' rows are laid out together) or ("state", bytes)."""
 
     def __init__(self, max_positions: int, parts):
-        rows = np.array([n if kind == "rows" else 0 for kind, n in parts], dtype=np.uint64)
-        states = np.array([0 if kind == "rows" else n for kind, n in parts], dtype=np.uint64)
-        self._c = host_lib().glint_book_layered_new(max_positions, len(parts), rows.ctypes.data, states.ctypes.data)
+        rows = np.array([p[1] if p[0] == "rows" else 0 for p in parts], dtype=np.uint64)
+        states = np.array([0 if p[0] == "rows" else p[1] for p in parts], dtype=np.uint64)
+        groups = np.array([p[2] if len(p) > 2 else 1 for p in parts], dtype=np.uint32)
+        self._c = host_lib().glint_book_layered_new(max_positions, len(parts), rows.ctypes.data, states.ctypes.data, groups.ctypes.data)
 
     def __del__(self):
         if getattr(self, "_c", None):
@@ -443,6 +447,17 @@ def famidra_runs(config_json: str):
     if n < 0:
         raise GlintError(host_lib().glint_last_error().decode(errors="replace"))
     return [(int(a), int(b) - 1 if b else None) for a, b in out[:n]]
+
+
+def dirozen_config(config_json: str) -> dict:
+    """Host-only: what the reader takes out of a Dirozen config.json.  Raises GlintError for a bad one."""
+    sizes, constants = np.zeros(4096, dtype=np.uint32), np.zeros(4096, dtype=np.float32)
+    n = host_lib().glint_book_dirozen_config(config_json.encode(), sizes.ctypes.data, sizes.size, constants.ctypes.data)
+    if n < 0:
+        raise GlintError(host_lib().glint_last_error().decode(errors="replace"))
+    names = ("heads", "kv_heads", "dim", "ff", "temp_every")
+    layers = [dict(zip(names, map(int, sizes[3 + 5 * i:8 + 5 * i])), scale=float(constants[1 + 2 * i]), temp_coef=float(constants[2 + 2 * i])) for i in range(n)]
+    return dict(width=int(sizes[0]), vocab=int(sizes[1]), eps=float(constants[0]), layers=layers)
 
 
 def model_dir_walk(config: str, dtype: str, first_layer: int, n_hosted: int, with_cls: bool, model_dir: str):

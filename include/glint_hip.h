@@ -111,6 +111,8 @@ int gh_host_malloc( void** out, uint64_t bytes );
 int gh_host_free( void* ptr );
 /* Operations::copy (arch/cuda/common/ops.cuh:758-780): byte copy; `async` != 0 returns before completion */
 int gh_memcpy( void* dst, const void* src, uint64_t bytes, gh_copy_kind kind, int async, gh_stream stream );
+/* `rows` rows of `bytes` bytes each, dst_stride / src_stride bytes apart; synchronous */
+int gh_memcpy_rows( void* dst, uint64_t dst_stride, const void* src, uint64_t src_stride, uint64_t bytes, uint64_t rows, gh_copy_kind kind, gh_stream stream );
 int gh_memset_zero( void* dst, uint64_t bytes, gh_stream stream ); /* fill kernel, graph-capture safe */
 
 /* Operations::randomize_device_buffer (arch/cuda/common/ops.cuh:782-792): uniform [lo, hi), counter-based, seeded */
@@ -337,8 +339,10 @@ int gh_embed_positions( float* x, const uint32_t* tokens_dev, const uint32_t* st
                         const void* pos_table, uint64_t width, uint64_t vocab, uint64_t max_pos, void* copy, uint64_t copy_stride, gh_dtype dt, gh_stream stream );
 
 /* What happens to the fp32 residual stream behind a projection y:
- *   y += bias;  y = rms(y) * post_norm;  x = accumulate ? x + y : y;  x += add;  out = DType( next_norm ? rms(x) * next_norm : x )
- * with rms(z) = z / sqrt(mean(z^2) + eps); any of the pointers may be NULL, its part is then left out. */
+ *   y += bias;  y = rms(y) * (norm_base + post_norm);  x = accumulate ? x + y : y;  x += add;
+ *   out = DType( next_norm ? rms(x) * (norm_base + next_norm) : x )
+ * with rms(z) = z / sqrt(mean(z^2) + eps); any of the pointers may be NULL, its part is then left out.  norm_base: 0, or 1 where the
+ * norms' weights are stored around zero. */
 typedef struct gh_stream_step
 {
   const void* bias;
@@ -349,6 +353,7 @@ typedef struct gh_stream_step
   uint64_t out_stride; /* elements from row to row of `out` */
   float eps;
   int accumulate;
+  float norm_base;
 } gh_stream_step;
 /* y = in (rows, s) . w (width, s)^T */
 int gh_matmul_stream( float* x, const void* in, const void* w, uint64_t s, uint64_t width, uint64_t rows, const gh_stream_step* step, gh_dtype dt,
@@ -365,7 +370,10 @@ int gh_gather_rows( float* out, const float* x, const uint32_t* rows_dev, uint64
 
 /* Attention over a sliding window with kept first tokens and a bias by distance: position i sees j <= i with i - j < window or
  * j < keep_first, score = (q . k) * scale + distance_bias[h][min(i - j, n_dist - 1)], ordinary softmax.  window 0: no window.
- * Query head h uses kv head h / (heads / kv_heads).  Head sizes up to 512. */
+ * Query head h uses kv head h / (heads / kv_heads).  Head sizes up to 512.
+ * values_are_keys: values are the keys as projected, and a key is its value over its root mean square (vdim equals dim).  The cache then
+ * holds a head once, and beside the cache rows a second run of rows (gh_window_factor_bytes a token, in groups of
+ * GH_WINDOW_FACTOR_GROUP tokens) holds 1 / rms of every kv head in fp32. */
 typedef struct gh_window_attn
 {
   uint32_t heads;
@@ -376,18 +384,40 @@ typedef struct gh_window_attn
   uint32_t keep_first;
   uint32_t n_dist;
   float scale;
+  uint32_t values_are_keys;
 } gh_window_attn;
+enum { GH_WINDOW_FACTOR_GROUP = 32 };
 uint64_t gh_window_row_bytes( const gh_window_attn* a, gh_dtype dt );  /* one token's cache row (heads padded to 8 elements) */
+uint64_t gh_window_factor_bytes( const gh_window_attn* a );            /* one token's share of the key factors; 0 without them */
 uint64_t gh_window_query_elements( const gh_window_attn* a );          /* one row of q as the ops below exchange it */
 /* wqkv = rows of q, k, v; bias (may be NULL) alike.  q and k are normed over their whole projection (NULL: not), then q goes to `q`
- * and [k | v] to the context's cache row at the token's position. */
+ * and [k | v] to the context's cache row at the token's position.  (Not for values_are_keys.) */
 int gh_matmul_window_append( void* q, const void* x, const void* wqkv, const void* bias, uint64_t width, const gh_window_attn* a, const void* q_norm,
                              const void* k_norm, float eps, void* const* context_rows_dev, uint64_t cache_offset, const uint32_t* start_pos_dev, uint64_t batch,
                              uint32_t n_tokens, gh_dtype dt, gh_stream stream );
-/* out (rows, heads * vdim); the rows of this call are in the cache already.  distance_bias_dev (heads, n_dist) fp32 or NULL;
- * max_start_pos: host-side upper bound of the start positions */
-int gh_attn_window( void* out, const void* q, const gh_window_attn* a, const float* distance_bias_dev, void* const* context_rows_dev, uint64_t cache_offset,
-                    const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, uint32_t max_start_pos, gh_dtype dt, gh_stream stream );
+/* out (heads * vdim, rows out_stride elements apart); the rows of this call are in the cache already.  head_gates (rows, heads) fp32 or
+ * NULL: factor of each head's output.  distance_bias_dev (heads, n_dist) fp32 or NULL; factor_offset: where the key factors of
+ * values_are_keys begin in a context; max_start_pos: host-side upper bound of the start positions */
+int gh_attn_window( void* out, uint64_t out_stride, const float* head_gates, const void* q, const gh_window_attn* a, const float* distance_bias_dev,
+                    void* const* context_rows_dev, uint64_t cache_offset, uint64_t factor_offset, const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens,
+                    uint32_t max_start_pos, gh_dtype dt, gh_stream stream );
+
+/* Every projection of a parallel layer's input x in one product: the attention of values_are_keys and the gated feed-forward read the
+ * same x.  Query heads are divided by their root mean square and multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) at
+ * position p (temp_every 0: not), keys go to the context's cache rows as projected, 1 / rms of each beside them.
+ *   w: rows of q (heads * dim), k (kv_heads * dim), g (heads; only with head_gates), zeros up to ff_row, gate, up (ff each), zeros up to the
+ *   end (gh_parallel_weight_rows gives the row count and ff_row)
+ *   head_gates (rows, heads) = sigmoid(x . g^T), or NULL;  hidden (ff, rows hidden_stride elements apart) = DType( act(x . gate^T) * (x . up^T) ) */
+typedef struct gh_unit_heads
+{
+  float eps;
+  float temp_coef;
+  uint32_t temp_every;
+} gh_unit_heads;
+uint64_t gh_parallel_weight_rows( const gh_window_attn* a, int gated, uint64_t ff, uint64_t* ff_row );
+int gh_matmul_parallel( void* q, float* head_gates, void* hidden, uint64_t hidden_stride, const void* x, const void* w, uint64_t width, const gh_window_attn* a,
+                        const gh_unit_heads* u, uint64_t ff, int activation, void* const* context_rows_dev, uint64_t cache_offset, uint64_t factor_offset,
+                        const uint32_t* start_pos_dev, uint64_t batch, uint32_t n_tokens, gh_dtype dt, gh_stream stream );
 
 /* Matrix-memory LSTM mixer up to its output projection: projections, log gates, recurrence, norm of each head, output gate.
  *   w: rows of q, k (heads * dim each), v, g (heads * vdim each), zeros up to gate_row, rows of i, f (heads each), zeros up to the end
