@@ -28,21 +28,27 @@ def query_temperature(p, coef, every):
     return 1 + coef * np.log((p + 1) // every + 1)
 
 
+def softmax(score):
+    w = np.exp(score - score.max())
+    return w / w.sum()
+
+
+def read_keys(query, k, eps, scale):
+    """query (d) as it meets the keys, k (n, d) the visible keys as projected: their mean under the softmax of the scores, taken of the
+    keys before their norm."""
+    return softmax((unit_rms(k, eps) @ query) * scale) @ k
+
+
 def attention(q, k, scale, coef, every, eps, first=0):
-    """q (T, H, d) of positions first .. first + T - 1, k (first + T, G, d) of the whole sequence, both as projected.  Values are the
-    keys before their norm.  Returns (T, H, d)."""
-    T, H, d = q.shape
+    """q (T, H, d) of positions first .. first + T - 1, k (first + T, G, d) of the whole sequence, both as projected.  Returns (T, H, d)."""
+    T, H, _ = q.shape
     per = H // k.shape[1]
     out = np.zeros_like(q)
-    keys = unit_rms(k, eps)
     for t in range(T):
         p = first + t
         for h in range(H):
-            g = h // per
             query = unit_rms(q[t, h], eps) * query_temperature(p, coef, every)
-            score = (keys[: p + 1, g] @ query) * scale
-            weight = np.exp(score - score.max())
-            out[t, h] = (weight / weight.sum()) @ k[: p + 1, g]
+            out[t, h] = read_keys(query, k[: p + 1, h // per], eps, scale)
     return out
 
 
