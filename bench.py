@@ -109,6 +109,10 @@ DESIGNS = {
     "famidra-w8192": dict(
         llama=("llama2-70b-4k", 10, 4), batch=64, context=2048, prefill=(4, 2048),
         config=dict(width=8192, ff=28672, heads=64, kv_heads=8, dim=128, window=2048, mlstm=dict(heads=16, dim=256, vdim=512))),
+    "dirozen-w4096": dict(
+        llama=("llama2-7b", 8, 4), batch=32, context=1024, prefill=(8, 1024), config=dict(width=4096, ff=11008, heads=32, kv_heads=32, dim=128, layers=4)),
+    "dirozen-w8192": dict(
+        llama=("llama2-70b-4k", 10, 4), batch=64, context=2048, prefill=(4, 2048), config=dict(width=8192, ff=28672, heads=64, kv_heads=8, dim=128, layers=4)),
 }
 LAYER_TENSORS = ("rms_att_weight", "wq", "wkv", "wo", "rms_ffn_weight", "w1", "w2", "w3")
 
@@ -636,6 +640,14 @@ def famidra_config(c, positions):
             "layers": [mlstm, attention, mlstm, attention], "loop": {"start": 1, "stop": 3, "times": 2}}
 
 
+def dirozen_config(c):
+    """config.json of a Dirozen model of these layer sizes."""
+    layer = {"type": "attention", "mlp": {"kind": "dense", "ff": c["ff"]},
+             "mixer": {"heads": c["heads"], "kv_heads": c["kv_heads"], "dim": c["dim"], "vdim": c["dim"], "scale": c["dim"] ** -0.5,
+                       "q_temp": {"coef": 0.1, "every": 512}}}
+    return {"architecture": "Dirozen", "width": c["width"], "vocab": 32000, "norm": {"eps": 1e-5}, "layers": [layer] * c["layers"]}
+
+
 def design_bench(name, steps, warmup):
     """Prefill and decode of a run-time sized design (random weights) and of the closest Llama2 stage of equal layer sizes: decode of
     `batch` contexts at `context` keys, prefill of `prefill` prompts x tokens, both through the drivers' own entry points."""
@@ -662,10 +674,10 @@ def design_bench(name, steps, warmup):
         return (time.perf_counter() - t0) * 1e3 / n
 
     with tempfile.TemporaryDirectory() as tmp:
-        cfg = famidra_config(d["config"], positions)
+        cfg = famidra_config(d["config"], positions) if name.startswith("famidra") else dirozen_config(d["config"])
         with open(os.path.join(tmp, "config.json"), "w") as f:
             json.dump(cfg, f)
-        st = S.DesignStage(tmp, "bf16", batch, batch, random_weights=True)
+        st = S.DesignStage(tmp, "bf16", batch, batch, random_weights=True, max_positions=positions)
     ids = list(range(batch))
     prompts = rng.integers(0, cfg["vocab"], (n_prompts, T))
 

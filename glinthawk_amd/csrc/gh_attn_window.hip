@@ -315,23 +315,23 @@ constexpr float NO_KEY = -1e30f; // running maximum before the first key: exp(NO
 // partial result of one split of one (row, head): vpad weighted sums, then the sum of the weights and the maximum
 __host__ __device__ inline uint64_t partial_stride( const WindowShape& s ) { return s.vpad + 2; }
 
-// The results of a work-group's four waves for the query heads h0 .. h0 + nh - 1 of a row, wave w's for head h at
+// The results of a work-group's NW waves for the query heads h0 .. h0 + nh - 1 of a row, wave w's for head h at
 // lds[(w * hq + h) * (vpad + 2)]: added up and stored, as the output or as the partial result of a split.
-template<typename E>
+template<typename E, int NW>
 __device__ __forceinline__ void finish_split( const WindowOut<E>& out, float* partial, const float* lds, uint32_t hq, uint32_t nh, uint64_t row, uint32_t h0, uint32_t split,
                                               uint32_t splits, const WindowShape& s )
 {
   const uint32_t stride = s.vpad + 2;
-  for ( uint32_t i = threadIdx.x; i < nh * s.vpad; i += 256 ) {
+  for ( uint32_t i = threadIdx.x; i < nh * s.vpad; i += 64 * NW ) {
     const uint32_t h = i / s.vpad, e = i % s.vpad;
     float m = NO_KEY;
 #pragma unroll
-    for ( int w = 0; w < 4; w++ ) {
+    for ( int w = 0; w < NW; w++ ) {
       m = fmaxf( m, lds[( w * hq + h ) * stride + s.vpad + 1] );
     }
     float a = 0.0f, sm = 0.0f;
 #pragma unroll
-    for ( int w = 0; w < 4; w++ ) {
+    for ( int w = 0; w < NW; w++ ) {
       const float* src = lds + ( w * hq + h ) * stride;
       const float f = __expf( src[s.vpad + 1] - m );
       a += src[e] * f;
@@ -508,7 +508,7 @@ __global__ __launch_bounds__( 256 ) void window_rows_kernel( WindowOut<E> out,
     }
   }
   __syncthreads();
-  finish_split<E>( out, partial, lds, HQ, nh, row, h0, split, splits, s );
+  finish_split<E, 4>( out, partial, lds, HQ, nh, row, h0, split, splits, s );
 }
 
 // one wave per (row, head)
@@ -849,29 +849,44 @@ __global__ __launch_bounds__( 256, 2 ) void window_tiles_kernel( WindowOut<__bf1
 
 // ---- few tokens: one query row at a time on the matrix cores (bf16, head sizes up to 128) ---------------------------------------
 //
-// The products of the tile kernel with the query heads of a group as the columns (most of the 32 stay empty: the kernel streams keys, and
-// the matrix cores keep up with that many times over).  A wave takes every fourth tile of 32 of the row's visible keys, numbered as
-// in the rows kernel, so nothing needs a mask but the end; its tiles pass through LDS of its own, the next one's rows on their way
-// into registers meanwhile, without a barrier.  Adjacent work-groups read adjacent heads of the same cache rows.
+// The products of the tile kernel in 16 x 16 blocks, with the query heads of a group as the columns (where the group is small most of them
+// stay empty: the kernel streams keys, and the matrix cores keep up with that many times over).  A wave takes every NW-th tile of 32 of the
+// row's visible keys, numbered as in the rows kernel, so nothing needs a mask but the end; its tiles pass through LDS of its own, the next
+// one's rows on their way into registers meanwhile, without a barrier.  Two blocks of scores are, as they lie, the right operand of
+// the product with the values: slot 8 g + e of its 32 keys is key 4 g + e for e < 4, else key 16 + 4 g + e - 4 (g = lane / 16).
 constexpr uint32_t STEP_KEYS = 32;
 constexpr uint32_t STEP_COLS = 16; // query heads of a work-group
 // LDS of a work-group in 16-byte units: the waves' tiles, and the factors of their keys behind them; the results of the waves take its place
 // at the end
-constexpr uint32_t step_lds( bool shared ) { return 4 * STEP_KEYS * ( shared ? 16 : 32 ) + ( shared ? STEP_KEYS : 0 ); }
-static_assert( step_lds( true ) * 16 >= 4 * STEP_COLS * ( 128 + 2 ) * sizeof( float ), "results of four waves, heads of up to 128" );
+constexpr uint32_t step_lds( int waves, bool shared ) { return waves * ( STEP_KEYS * ( shared ? 16 : 32 ) + ( shared ? STEP_KEYS / 4 : 0 ) ); }
+static_assert( step_lds( 1, true ) * 16 >= STEP_COLS * ( 128 + 2 ) * sizeof( float ), "the results of a wave, heads of up to 128" );
+// 16-byte chunks of a key's 256 bytes are XORed with this: 16 rows at one chunk (plain reads) and 8 rows at one pair of chunks (transposing
+// reads) lie in different banks
+__device__ __forceinline__ uint32_t step_swizzle( uint32_t row ) { return ( ( row & 7 ) << 1 ) | ( ( row >> 3 ) & 1 ); }
 
-template<int KS, int VB, bool SHARED>
-__global__ __launch_bounds__( 256, SHARED && VB <= 2 ? 3 : 2 ) void window_decode_kernel( WindowOut<__bf16> out,
-                                                                  float* __restrict__ partial,
-                                                                  const __bf16* __restrict__ q,
-                                                                  const float* __restrict__ bias,
-                                                                  WindowRows wr,
-                                                                  WindowShape s,
-                                                                  uint32_t head_cols,
-                                                                  uint32_t keys_per_split,
-                                                                  uint32_t splits )
+// maximum over the four lanes of a column (lane, lane ^ 16, lane ^ 32, lane ^ 48), in all of them
+__device__ __forceinline__ float column_max( float v )
 {
-  __shared__ uint4 tiles[step_lds( SHARED )]; // K and V of each wave, 256 bytes a key
+  const unsigned bits = __builtin_bit_cast( unsigned, v );
+  const auto rows = __builtin_amdgcn_permlane16_swap( bits, bits, false, false );
+  const unsigned even = rows[0], odd = rows[1];
+  return half_wave_max( fmaxf( __builtin_bit_cast( float, even ), __builtin_bit_cast( float, odd ) ) );
+}
+
+// D: head size up to which the kernel goes; NW waves
+template<int D, bool SHARED, int NW>
+__global__ __launch_bounds__( 64 * NW, SHARED ? 4 : 2 ) void window_decode_kernel( WindowOut<__bf16> out,
+                                                                                         float* __restrict__ partial,
+                                                                                         const __bf16* __restrict__ q,
+                                                                                         const float* __restrict__ bias,
+                                                                                         WindowRows wr,
+                                                                                         WindowShape s,
+                                                                                         uint32_t head_cols,
+                                                                                         uint32_t keys_per_split,
+                                                                                         uint32_t splits )
+{
+  constexpr int KS = D / 32, VB = D / 16; // steps of 32 of the query/key size, blocks of 16 of the value size
+  __shared__ uint4 tiles[step_lds( NW, SHARED )]; // K and V of each wave, 256 bytes a key
   const uint32_t head_blocks = s.heads / head_cols;
   const uint32_t hb = blockIdx.x % head_blocks, split = blockIdx.x / head_blocks % splits;
   const uint64_t row = blockIdx.x / head_blocks / splits;
@@ -886,131 +901,137 @@ __global__ __launch_bounds__( 256, SHARED && VB <= 2 ? 3 : 2 ) void window_decod
   const Visible vis = visible_keys( pos, s );
   const uint32_t k_begin = split * keys_per_split, k_end = min( vis.count, k_begin + keys_per_split );
   const uint32_t wave = __builtin_amdgcn_readfirstlane( threadIdx.x >> 6 );
-  const uint32_t lane = threadIdx.x & 63, r = lane & 31, g2 = lane >> 5;
+  const uint32_t lane = threadIdx.x & 63, r = lane & 15, g4 = lane >> 4;
   const uint32_t hc = min( r, head_cols - 1 ); // columns beyond do as the last one and are not stored
   uint4* s_k = tiles + wave * STEP_KEYS * ( SHARED ? 16 : 32 );
   uint4* s_v = SHARED ? s_k : s_k + STEP_KEYS * 16;
-  float* s_factor = reinterpret_cast<float*>( tiles + 4 * STEP_KEYS * ( SHARED ? 16 : 32 ) ) + wave * STEP_KEYS; // times scale and log2(e)
+  float* s_factor = reinterpret_cast<float*>( tiles + NW * STEP_KEYS * ( SHARED ? 16 : 32 ) ) + wave * STEP_KEYS; // times scale and log2(e)
 
   bf16x8 qb[KS];
 #pragma unroll
   for ( int k = 0; k < KS; k++ ) {
-    const uint32_t ch = 2 * k + g2;
+    const uint32_t ch = 4 * k + g4;
     u32x4_t v = { 0, 0, 0, 0 };
     if ( ch * 8 < s.dpad ) {
       v = *(global_u32x4_t*)( q + ( row * s.heads + h0 + hc ) * s.dpad + ch * 8 );
     }
     qb[k] = __builtin_bit_cast( bf16x8, v );
   }
-  const uint32_t ld_chunk = lane & 15, ld_row = lane >> 4;
-  const bool k_chunk = ld_chunk * 8 < s.dpad && ld_chunk < 2 * KS, v_chunk = ld_chunk * 8 < s.vpad && ld_chunk < 4 * VB;
-  const uint32_t at_k = g * s.dpad + ld_chunk * 8, at_v = s.k_elems() + g * s.vpad + ld_chunk * 8;
-  u32x4_t rk[8], rv[SHARED ? 1 : 8];
+  const bool k_chunk = r * 8 < s.dpad && r < D / 8, v_chunk = r * 8 < s.vpad && r < D / 8;
+  const uint32_t row_bytes = s.row_elems() * sizeof( __bf16 );
+  const uint32_t at_k = ( g * s.dpad + r * 8 ) * sizeof( __bf16 ), at_v = ( s.k_elems() + g * s.vpad + r * 8 ) * sizeof( __bf16 );
+  u32x4_t rk[8], rv[SHARED ? 1 : 8]; // chunks beyond a head's size stay zero
+#pragma unroll
+  for ( int k = 0; k < 8; k++ ) {
+    rk[k] = u32x4_t { 0, 0, 0, 0 };
+    rv[SHARED ? 0 : k] = u32x4_t { 0, 0, 0, 0 };
+  }
   const float* factors = reinterpret_cast<const float*>( base + wr.factors );
   float rf = 0.0f;
-  auto load = [&]( uint32_t i0 ) {
-    if constexpr ( SHARED ) {
-      rf = factors[factor_index( vis.key( min( i0 + r, k_end - 1 ) ), g, s.kv_heads )];
+  auto load_row = [&]( int k, const char* row_k, uint32_t off ) {
+    if ( k_chunk ) {
+      rk[k] = __builtin_nontemporal_load( (global_u32x4_t*)( row_k + ( off + at_k ) ) );
     }
-#pragma unroll
-    for ( int k = 0; k < 8; k++ ) {
-      const uint32_t j = vis.key( min( i0 + ld_row + 4 * k, k_end - 1 ) ); // past the end: the last key again, without weight
-      const __bf16* p = cache + (uint64_t)j * s.row_elems();
-      rk[k] = u32x4_t { 0, 0, 0, 0 };
-      if ( k_chunk ) {
-        rk[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_k ) );
-      }
-      if constexpr ( !SHARED ) {
-        rv[k] = u32x4_t { 0, 0, 0, 0 };
-        if ( v_chunk ) {
-          rv[k] = __builtin_nontemporal_load( (global_u32x4_t*)( p + at_v ) );
-        }
+    if constexpr ( !SHARED ) {
+      if ( v_chunk ) {
+        rv[k] = __builtin_nontemporal_load( (global_u32x4_t*)( row_k + ( off + at_v ) ) );
       }
     }
   };
-  const uint32_t tr_e = ( lane & 15 ) >> 2, tr_q = lane & 3, tr_grp = ( lane >> 4 ) & 1;
-  const uint32_t v_lane = ( 4 * g2 + tr_e ) * 256 + ( ( ( 2 * tr_grp + ( tr_q >> 1 ) ) ^ ( 4 * tr_e ) ^ ( SHARED ? g2 : 0 ) ) * 16 ) + ( tr_q & 1 ) * 8;
+  auto load = [&]( uint32_t i0 ) {
+    if constexpr ( SHARED ) {
+      rf = factors[factor_index( vis.key( min( i0 + ( lane & 31 ), k_end - 1 ) ), g, s.kv_heads )];
+    }
+    if ( i0 + STEP_KEYS <= k_end && ( i0 >= vis.kept || i0 + STEP_KEYS <= vis.kept ) ) { // neighbouring rows: one address for the wave
+      const char* tile = reinterpret_cast<const char*>( cache ) + (uint64_t)vis.key( i0 ) * row_bytes;
+#pragma unroll
+      for ( int k = 0; k < 8; k++ ) {
+        load_row( k, tile + 4 * k * row_bytes, g4 * row_bytes );
+      }
+    } else {
+#pragma unroll
+      for ( int k = 0; k < 8; k++ ) {
+        const uint32_t j = vis.key( min( i0 + g4 + 4 * k, k_end - 1 ) ); // past the end: the last key again, without weight
+        load_row( k, reinterpret_cast<const char*>( cache ) + (uint64_t)j * row_bytes, 0 );
+      }
+    }
+  };
+  // a lane's bytes in a tile: of the row it writes first, of the key it reads for the scores, and of the transposing reads (16 lanes bring
+  // 4 keys of 16 value columns, lane i gets column i).  The other places are a few bits and rows away.
+  const uint32_t w_home = g4 * 256 + ( r ^ step_swizzle( g4 ) ) * 16;
+  const uint32_t k_home = r * 256 + ( g4 ^ step_swizzle( r ) ) * 16;
+  const uint32_t v_row = 4 * g4 + ( r >> 2 );
+  const uint32_t v_home = v_row * 256 + ( ( ( ( r & 3 ) >> 1 ) ^ step_swizzle( v_row ) ) * 16 ) + ( r & 1 ) * 8;
   const float scale_log2e = s.scale * LOG2E;
   const float* my_bias = bias != nullptr ? bias + (uint64_t)( h0 + hc ) * s.n_dist : nullptr;
   const float far_bias = bias != nullptr ? my_bias[s.n_dist - 1] * LOG2E : 0.0f;
 
-  mfma_f32x16 acc[VB];
+  mfma_f32x4 acc[VB];
 #pragma unroll
   for ( int vb = 0; vb < VB; vb++ ) {
-#pragma unroll
-    for ( int v = 0; v < 16; v++ ) {
-      acc[vb][v] = 0.0f;
-    }
+    acc[vb] = mfma_f32x4 { 0.0f, 0.0f, 0.0f, 0.0f };
   }
   float m = NO_KEY, l = 0.0f;
   uint32_t i0 = k_begin + wave * STEP_KEYS;
   if ( i0 < k_end ) {
     load( i0 );
   }
-  for ( ; i0 < k_end; i0 += 4 * STEP_KEYS ) {
+  for ( ; i0 < k_end; i0 += NW * STEP_KEYS ) {
+    uint32_t w_lane = w_home, k_lane = k_home, v_lane = v_home;
+    asm( "" : "+v"( w_lane ), "+v"( k_lane ), "+v"( v_lane ) ); // the addresses beside these are made where they are used, not kept in registers
 #pragma unroll
     for ( int k = 0; k < 8; k++ ) {
-      const uint32_t krow = ld_row + 4 * k;
-      s_k[krow * 16 + ( ld_chunk ^ ( SHARED ? shared_swizzle( krow ) : krow & 15 ) )] = __builtin_bit_cast( uint4, rk[k] );
+      const uint32_t at = ( w_lane ^ ( 16 * step_swizzle( 4 * k ) ) ) + 4 * k * 256;
+      *reinterpret_cast<uint4*>( reinterpret_cast<char*>( s_k ) + at ) = __builtin_bit_cast( uint4, rk[k] );
       if constexpr ( !SHARED ) {
-        s_v[krow * 16 + ( ld_chunk ^ ( 4 * ( krow & 3 ) ) )] = __builtin_bit_cast( uint4, rv[k] );
+        *reinterpret_cast<uint4*>( reinterpret_cast<char*>( s_v ) + at ) = __builtin_bit_cast( uint4, rv[k] );
       }
     }
-    if ( SHARED && g2 == 0 ) {
-      s_factor[r] = rf * scale_log2e;
+    if ( SHARED && lane < STEP_KEYS ) {
+      s_factor[lane] = rf * scale_log2e;
     }
-    if ( i0 + 4 * STEP_KEYS < k_end ) {
-      load( i0 + 4 * STEP_KEYS );
+    if ( i0 + NW * STEP_KEYS < k_end ) {
+      load( i0 + NW * STEP_KEYS );
     }
     __builtin_amdgcn_fence( __ATOMIC_RELEASE, "wavefront" );
-    mfma_f32x16 st;
+    float st[8]; // of key i0 + 16 (e / 4) + 4 g4 + e % 4
 #pragma unroll
-    for ( int v = 0; v < 16; v++ ) {
-      st[v] = 0.0f;
-    }
+    for ( int t = 0; t < 2; t++ ) {
+      mfma_f32x4 d = { 0.0f, 0.0f, 0.0f, 0.0f };
 #pragma unroll
-    for ( int k = 0; k < KS; k++ ) {
-      st = Mfma<__bf16>::k16( __builtin_bit_cast( bf16x8, s_k[r * 16 + ( ( 2 * k + g2 ) ^ ( SHARED ? shared_swizzle( r ) : r & 15 ) )] ), qb[k], st );
-    }
-    float factor[16];
-#pragma unroll
-    for ( int q4 = 0; q4 < 4; q4++ ) {
+      for ( int k = 0; k < KS; k++ ) {
+        const uint4 a = *reinterpret_cast<const uint4*>( reinterpret_cast<const char*>( s_k ) + ( k_lane ^ ( 64 * k ) ) + 16 * t * 256 );
+        d = Mfma<__bf16>::k32( __builtin_bit_cast( bf16x8, a ), qb[k], d );
+      }
       float4 f = make_float4( scale_log2e, scale_log2e, scale_log2e, scale_log2e );
       if constexpr ( SHARED ) {
-        f = *reinterpret_cast<const float4*>( s_factor + 8 * q4 + 4 * g2 );
+        f = *reinterpret_cast<const float4*>( s_factor + 16 * t + 4 * g4 );
       }
-      factor[4 * q4] = f.x, factor[4 * q4 + 1] = f.y, factor[4 * q4 + 2] = f.z, factor[4 * q4 + 3] = f.w;
+      st[4 * t] = d[0] * f.x, st[4 * t + 1] = d[1] * f.y, st[4 * t + 2] = d[2] * f.z, st[4 * t + 3] = d[3] * f.w;
     }
-    // every distance of the tile in the bias table's last row?
-    const uint32_t nearest = vis.key( min( i0 + STEP_KEYS, k_end ) - 1 );
-    if ( bias == nullptr || pos - nearest >= s.n_dist - 1 ) {
+    if ( bias != nullptr ) {
+      // every distance of the tile in the bias table's last row?
+      const uint32_t nearest = vis.key( min( i0 + STEP_KEYS, k_end ) - 1 );
+      if ( pos - nearest >= s.n_dist - 1 ) {
 #pragma unroll
-      for ( int v = 0; v < 16; v++ ) {
-        st[v] = st[v] * factor[v] + far_bias;
-      }
-    } else {
+        for ( int e = 0; e < 8; e++ ) {
+          st[e] += far_bias;
+        }
+      } else {
 #pragma unroll
-      for ( int v = 0; v < 16; v++ ) {
-        const uint32_t j = vis.key( min( i0 + 8 * ( v / 4 ) + 4 * g2 + v % 4, k_end - 1 ) );
-        st[v] = st[v] * factor[v] + my_bias[min( pos - j, s.n_dist - 1 )] * LOG2E;
+        for ( int e = 0; e < 8; e++ ) {
+          const uint32_t j = vis.key( min( i0 + 16 * ( e / 4 ) + 4 * g4 + e % 4, k_end - 1 ) );
+          st[e] += my_bias[min( pos - j, s.n_dist - 1 )] * LOG2E;
+        }
       }
     }
     if ( i0 + STEP_KEYS > k_end ) {
 #pragma unroll
-      for ( int v = 0; v < 16; v++ ) {
-        st[v] = i0 + 8 * ( v / 4 ) + 4 * g2 + v % 4 < k_end ? st[v] : -INFINITY;
+      for ( int e = 0; e < 8; e++ ) {
+        st[e] = i0 + 16 * ( e / 4 ) + 4 * g4 + e % 4 < k_end ? st[e] : -INFINITY;
       }
     }
-    float mx2[2];
-#pragma unroll
-    for ( int c = 0; c < 2; c++ ) {
-      mx2[c] = st[8 * c];
-#pragma unroll
-      for ( int e = 1; e < 8; e++ ) {
-        mx2[c] = fmaxf( mx2[c], st[8 * c + e] );
-      }
-    }
-    const float mx = half_wave_max( fmaxf( mx2[0], mx2[1] ) );
+    const float mx = column_max( fmaxf( fmaxf( fmaxf( st[0], st[1] ), fmaxf( st[2], st[3] ) ), fmaxf( fmaxf( st[4], st[5] ), fmaxf( st[6], st[7] ) ) ) );
     if ( __builtin_amdgcn_ballot_w64( mx > m + LAZY ) != 0 ) {
       const float m_new = fmaxf( m, mx );
       const float alpha = __builtin_amdgcn_exp2f( m - m_new );
@@ -1019,38 +1040,36 @@ __global__ __launch_bounds__( 256, SHARED && VB <= 2 ? 3 : 2 ) void window_decod
 #pragma unroll
       for ( int vb = 0; vb < VB; vb++ ) {
 #pragma unroll
-        for ( int v = 0; v < 16; v++ ) {
+        for ( int v = 0; v < 4; v++ ) {
           acc[vb][v] *= alpha;
         }
       }
     }
+    bf16x8 hi, lo;
 #pragma unroll
-    for ( int kk = 0; kk < 2; kk++ ) {
-      bf16x8 hi, lo;
+    for ( int e = 0; e < 8; e++ ) {
+      const float p = __builtin_amdgcn_exp2f( st[e] - m );
+      l += p;
+      hi[e] = (__bf16)p;
+      lo[e] = (__bf16)( p - (float)hi[e] );
+    }
 #pragma unroll
-      for ( int e = 0; e < 8; e++ ) {
-        const float p = __builtin_amdgcn_exp2f( st[8 * kk + e] - m );
-        l += p;
-        hi[e] = (__bf16)p;
-        lo[e] = (__bf16)( p - (float)hi[e] );
+    for ( int vb = 0; vb < VB; vb++ ) {
+      union
+      {
+        v4s half[2];
+        bf16x8 x;
+      } a;
+#pragma unroll
+      for ( int t = 0; t < 2; t++ ) {
+        a.half[t] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 32 * vb ) ) + 16 * t * 256 ) );
       }
-#pragma unroll
-      for ( int vb = 0; vb < VB; vb++ ) {
-        union
-        {
-          v4s half[2];
-          bf16x8 x;
-        } a;
-#pragma unroll
-        for ( int hf = 0; hf < 2; hf++ ) {
-          a.half[hf] = __builtin_amdgcn_ds_read_tr16_b64_v4i16( (lds_v4s)( (lds_char*)s_v + ( v_lane ^ ( 64 * vb ) ^ ( SHARED ? 32 * hf : 0 ) ) + ( 16 * kk + 8 * hf ) * 256 ) );
-        }
-        acc[vb] = Mfma<__bf16>::k16( a.x, lo, acc[vb] );
-        acc[vb] = Mfma<__bf16>::k16( a.x, hi, acc[vb] );
-      }
+      acc[vb] = Mfma<__bf16>::k32( a.x, lo, acc[vb] );
+      acc[vb] = Mfma<__bf16>::k32( a.x, hi, acc[vb] );
     }
     __builtin_amdgcn_fence( __ATOMIC_ACQUIRE, "wavefront" );
   }
+  l += __shfl_xor( l, 16 );
   l += __shfl_xor( l, 32 );
   __syncthreads(); // the tiles' LDS takes the waves' results
   float* results = reinterpret_cast<float*>( tiles );
@@ -1059,20 +1078,20 @@ __global__ __launch_bounds__( 256, SHARED && VB <= 2 ? 3 : 2 ) void window_decod
 #pragma unroll
     for ( int vb = 0; vb < VB; vb++ ) {
 #pragma unroll
-      for ( int v = 0; v < 16; v++ ) {
-        const uint32_t d = 32 * vb + 8 * ( v / 4 ) + 4 * g2 + v % 4;
+      for ( int v = 0; v < 4; v++ ) {
+        const uint32_t d = 16 * vb + 4 * g4 + v;
         if ( d < s.vpad ) {
           mine[d] = acc[vb][v];
         }
       }
     }
-    if ( g2 == 0 ) {
+    if ( g4 == 0 ) {
       mine[s.vpad] = l;
       mine[s.vpad + 1] = m * ( 1.0f / LOG2E ); // the sums are joined in natural units
     }
   }
   __syncthreads();
-  finish_split<__bf16>( out, partial, results, head_cols, head_cols, row, h0, split, splits, s );
+  finish_split<__bf16, NW>( out, partial, results, head_cols, head_cols, row, h0, split, splits, s );
 }
 
 template<typename E, int NC, bool SHARED>
@@ -1141,23 +1160,29 @@ int attend_decode( const WindowOut<__bf16>& out, const __bf16* q, const float* b
     head_cols--;
   }
   const uint64_t head_blocks = s.heads / head_cols;
+  // keys of a row over eight waves where work-groups of four would leave room on the CUs and each wave still has a few tiles
+  const bool wide = s.values_are_keys && rows * head_blocks < 4ull * cu_count() && max_pos >= 16 * STEP_KEYS;
   SplitPlan plan;
-  if ( int rc = plan_splits( s, rows, head_blocks, max_pos, 4 * STEP_KEYS, st, &plan ) ) {
+  if ( int rc = plan_splits( s, rows, head_blocks, max_pos, ( wide ? 8 : 4 ) * STEP_KEYS, st, &plan ) ) {
     return rc;
   }
   const uint64_t grid = rows * head_blocks * plan.splits;
   GH_REQUIRE( grid < ( 1ull << 31 ), "gh_attn_window: grid too large" );
-#define GH_WINDOW_DECODE( KS, VB, SHARED ) \
-  window_decode_kernel<KS, VB, SHARED><<<(unsigned)grid, 256, 0, st>>>( out, plan.partial, q, bias, wr, s, head_cols, plan.keys, plan.splits )
+#define GH_WINDOW_DECODE( D, SHARED, NW ) \
+  window_decode_kernel<D, SHARED, NW><<<(unsigned)grid, 64 * NW, 0, st>>>( out, plan.partial, q, bias, wr, s, head_cols, plan.keys, plan.splits )
   const bool small = s.dpad <= 64 && s.vpad <= 64;
-  if ( small && s.values_are_keys ) {
-    GH_WINDOW_DECODE( 4, 2, true );
+  if ( !s.values_are_keys && small ) {
+    GH_WINDOW_DECODE( 64, false, 4 );
+  } else if ( !s.values_are_keys ) {
+    GH_WINDOW_DECODE( 128, false, 4 );
+  } else if ( small && wide ) {
+    GH_WINDOW_DECODE( 64, true, 8 );
   } else if ( small ) {
-    GH_WINDOW_DECODE( 4, 2, false );
-  } else if ( s.values_are_keys ) {
-    GH_WINDOW_DECODE( 8, 4, true );
+    GH_WINDOW_DECODE( 64, true, 4 );
+  } else if ( wide ) {
+    GH_WINDOW_DECODE( 128, true, 8 );
   } else {
-    GH_WINDOW_DECODE( 8, 4, false );
+    GH_WINDOW_DECODE( 128, true, 4 );
   }
 #undef GH_WINDOW_DECODE
   GH_LAUNCH_CHECK();

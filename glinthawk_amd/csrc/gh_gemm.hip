@@ -25,8 +25,9 @@ int gemm_stream_launch( E* xout, float* partial, const E* x, const E* w, uint64_
                         uint32_t k_per_split, uint32_t rows_per_wg, bool write_partials, hipStream_t st );
 void gemm_stream_tuning( int target_wgs, int depth );
 void gemm_stream_gate_waves( int waves );
-bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const void* x, const void* w13, const void* hb );
-int gemm_stream_gate_launch( __half* hb, const __half* x, const __half* w13, uint64_t s, uint64_t hidden, uint64_t b, hipStream_t st );
+bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const void* x, const void* w13, const void* hb, uint64_t hb_stride );
+template<typename E>
+int gemm_stream_gate_launch( E* hb, uint64_t hb_stride, const E* x, const E* w13, uint64_t s, uint64_t hidden, uint64_t b, hipStream_t st );
 // 256 x 256 tile kernel for products with enough tiles (gh_gemm_tile256.hip)
 bool gemm_tile256_applicable( uint64_t s, uint64_t r, uint64_t b, const void* x, const void* w, const void* xout );
 template<typename E>
@@ -306,14 +307,18 @@ namespace gh {
 // otherwise the kernel may store DType results straight into `xout` (*splits_out == 0 then).
 // w1, w3 and the SiLU gate in one launch of the streaming kernel, where gemm_partials() would pick that
 // kernel without a K split.  *done = false: nothing was launched, the caller takes the two-kernel route.
-int gemm_gate_one_launch( void* hb, const void* x, const void* w13, uint64_t s, uint64_t hidden, uint64_t b, gh_dtype dt, hipStream_t st, bool* done )
+int gemm_gate_one_launch( void* hb, uint64_t hb_stride, const void* x, const void* w13, uint64_t s, uint64_t hidden, uint64_t b, gh_dtype dt, hipStream_t st,
+                          bool* done )
 {
   *done = false;
-  if ( dt != GH_F16 || ( g_force_kernel != 0 && g_force_kernel != 2 ) || b > 64 || !gemm_stream_gate_applicable( s, hidden, b, x, w13, hb ) ) {
+  if ( !is_half_type( dt ) || ( g_force_kernel != 0 && g_force_kernel != 2 ) || b > 64 || !gemm_stream_gate_applicable( s, hidden, b, x, w13, hb, hb_stride ) ) {
     return GH_OK;
   }
   *done = true;
-  return gemm_stream_gate_launch( static_cast<__half*>( hb ), static_cast<const __half*>( x ), static_cast<const __half*>( w13 ), s, hidden, b, st );
+  return with_half_type( dt, [&]( auto* e ) {
+    using E = std::remove_pointer_t<decltype( e )>;
+    return gemm_stream_gate_launch<E>( static_cast<E*>( hb ), hb_stride, static_cast<const E*>( x ), static_cast<const E*>( w13 ), s, hidden, b, st );
+  } );
 }
 
 // Tokens of the first part when a many-row product is better run as two products along the tokens (see

@@ -10,7 +10,7 @@ namespace gh {
 
 int gemm_partials( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, hipStream_t st, bool want_partials,
                    float** partial_out, uint32_t* splits_out );
-int gemm_gate_one_launch( void* hb, const void* x, const void* w13, uint64_t s, uint64_t hidden, uint64_t b, gh_dtype dt, hipStream_t st, bool* done );
+int gemm_gate_one_launch( void* hb, uint64_t hb_stride, const void* x, const void* w13, uint64_t s, uint64_t hidden, uint64_t b, gh_dtype dt, hipStream_t st, bool* done );
 uint64_t gemm_token_split( uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, const void* x, const void* w, const void* xout );
 bool gemm_tile_epilogue_applicable( uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, const void* x, const void* w, const void* xout );
 int gemm_tile_epilogue_launch( void* xout, const void* x, const void* w, uint64_t s, uint64_t r, uint64_t b, gh_dtype dt, int epilogue, hipStream_t st,
@@ -521,7 +521,7 @@ int gh_matmul_silu_gate( void* hb, const void* x, const void* w13, uint64_t s, u
   GH_REQUIRE( hb != nullptr, "gh_matmul_silu_gate: NULL output" );
   hipStream_t st = as_stream( stream );
   bool done = false;
-  if ( int rc = gemm_gate_one_launch( hb, x, w13, s, hidden_dim, b, dt, st, &done ) ) {
+  if ( int rc = gemm_gate_one_launch( hb, hidden_dim, x, w13, s, hidden_dim, b, dt, st, &done ) ) {
     return rc;
   }
   if ( done ) {

@@ -145,7 +145,8 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
                                                              uint32_t b,
                                                              uint32_t k_per_split,
                                                              uint32_t n_col_slabs,
-                                                             uint32_t rows_per_wave )
+                                                             uint32_t rows_per_wave,
+                                                             uint64_t gate_stride = 0 ) // MODE_GATE: elements from row to row of xout
 {
   __shared__ uint4 s_x[2][COLS * 16]; // 2 x 16 KiB
   __shared__ uint4 s_w[W][32 * 16];   // 8 KiB per wave
@@ -276,7 +277,7 @@ __global__ __launch_bounds__( 64 * W, W == 4 ? 2 : 1 ) void gemm_stream_kernel( 
           o.h[i] = from_f32<E>( y1 / ( 1.0f + __expf( -y1 ) ) * y3 );
         }
         if ( col < b && 8 * q4 + 4 * g2 < rows_per_wave ) {
-          E* dst = xout + (uint64_t)col * r + row;
+          E* dst = xout + (uint64_t)col * gate_stride + row;
           if ( row + 3 < r ) {
             *reinterpret_cast<uint2*>( dst ) = o.raw;
           } else {
@@ -422,11 +423,11 @@ int gemm_stream_launch( E* xout, float* partial, const E* x, const E* w, uint64_
   return GH_OK;
 }
 
-// hb(b, hidden) = DType(silu(DType(x . w1^T)) * DType(x . w3^T)), w13 = w1 rows then w3 rows, in one launch.
-// Only without a K split: the caller checks gemm_stream_gate_applicable first.
-bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const void* x, const void* w13, const void* hb )
+// hb(b, hidden) = DType(silu(DType(x . w1^T)) * DType(x . w3^T)), w13 = w1 rows then w3 rows, in one launch; rows of hb are hb_stride
+// elements apart.  Only without a K split: the caller checks gemm_stream_gate_applicable first.
+bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const void* x, const void* w13, const void* hb, uint64_t hb_stride )
 {
-  if ( hidden % 4 != 0 || !gemm_stream_applicable( s, 2 * hidden, b, x, w13, hb ) ) { // 8-byte output stores
+  if ( hidden % 4 != 0 || hb_stride % 4 != 0 || !gemm_stream_applicable( s, 2 * hidden, b, x, w13, hb ) ) { // 8-byte output stores
     return false;
   }
   uint32_t splits = 1, k_per_split = 0, rows = 0;
@@ -434,7 +435,8 @@ bool gemm_stream_gate_applicable( uint64_t s, uint64_t hidden, uint64_t b, const
   return splits == 1;
 }
 
-int gemm_stream_gate_launch( __half* hb, const __half* x, const __half* w13, uint64_t s, uint64_t hidden, uint64_t b, hipStream_t st )
+template<typename E>
+int gemm_stream_gate_launch( E* hb, uint64_t hb_stride, const E* x, const E* w13, uint64_t s, uint64_t hidden, uint64_t b, hipStream_t st )
 {
   uint32_t splits = 1, k_per_split = 0, rows = 0;
   gemm_stream_plan( s, 2 * hidden, b, &splits, &k_per_split, &rows );
@@ -451,16 +453,18 @@ int gemm_stream_gate_launch( __half* hb, const __half* x, const __half* w13, uin
   const uint64_t gx = col_slabs == 1 ? row_blocks : ( row_blocks + 7 ) / 8 * 8 * col_slabs;
   GH_REQUIRE( gx < ( 1ull << 31 ), "gh_matmul_silu_gate: grid too large" );
   if ( waves == 8 ) {
-    gemm_stream_kernel<__half, MODE_GATE, 8><<<dim3( (unsigned)gx, 1, 1 ), 512, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
-                                                                              (uint32_t)col_slabs, rows_per_wave );
+    gemm_stream_kernel<E, MODE_GATE, 8><<<dim3( (unsigned)gx, 1, 1 ), 512, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
+                                                                              (uint32_t)col_slabs, rows_per_wave, hb_stride );
   } else {
-    gemm_stream_kernel<__half, MODE_GATE><<<dim3( (unsigned)gx, 1, 1 ), 256, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
-                                                                           (uint32_t)col_slabs, rows_per_wave );
+    gemm_stream_kernel<E, MODE_GATE><<<dim3( (unsigned)gx, 1, 1 ), 256, 0, st>>>( hb, nullptr, x, w13, (uint32_t)s, (uint32_t)hidden, (uint32_t)b, (uint32_t)s,
+                                                                           (uint32_t)col_slabs, rows_per_wave, hb_stride );
   }
   GH_LAUNCH_CHECK();
   return GH_OK;
 }
 
+template int gemm_stream_gate_launch<__half>( __half*, uint64_t, const __half*, const __half*, uint64_t, uint64_t, uint64_t, hipStream_t );
+template int gemm_stream_gate_launch<__bf16>( __bf16*, uint64_t, const __bf16*, const __bf16*, uint64_t, uint64_t, uint64_t, hipStream_t );
 template int gemm_stream_launch<__half>( __half*, float*, const __half*, const __half*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, uint32_t, bool,
                                          hipStream_t );
 template int gemm_stream_launch<__bf16>( __bf16*, float*, const __bf16*, const __bf16*, uint64_t, uint64_t, uint64_t, uint32_t, uint32_t, uint32_t, bool,

@@ -1,5 +1,7 @@
 // Input side of a parallel layer: one product of the layer's input with everything that reads it (queries, keys that are also the values,
-// a gate per head, gate and up of the feed-forward), and one kernel behind it that brings each part to where it is read.
+// a gate per head, gate and up of the feed-forward), and one kernel behind it that brings each part to where it is read.  Where the
+// feed-forward is so large that its product fills the chip without a split of K, few rows take the launch that applies the gate itself for
+// it, and the product and the kernel serve the heads alone.
 //
 // work-group  256 threads on one row: first the heads, L lanes a head with V neighbouring elements each, then the feed-forward's columns
 // heads       a query is divided by its root mean square and multiplied by its position's temperature; a key goes to the cache as it is,
@@ -11,6 +13,10 @@
 #include <type_traits>
 
 namespace gh {
+
+// gh_gemm.hip: gate, up and SiLU in one launch where the streaming kernel runs without a K split; *done = false: nothing was launched
+int gemm_gate_one_launch( void* hb, uint64_t hb_stride, const void* x, const void* w13, uint64_t s, uint64_t hidden, uint64_t b, gh_dtype dt, hipStream_t st, bool* done );
+
 namespace {
 
 struct ParallelCols
@@ -246,8 +252,18 @@ int gh_matmul_parallel( void* q, float* head_gates, void* hidden, uint64_t hidde
               "gh_matmul_parallel: bad shape" );
   GH_REQUIRE( activation == GH_ACT_SILU || activation == GH_ACT_GELU_TANH, "gh_matmul_parallel: unknown activation %d", activation );
   const WindowShape s = window_shape( a );
-  const ParallelCols cols = parallel_cols( a, head_gates != nullptr, ff );
+  ParallelCols cols = parallel_cols( a, head_gates != nullptr, ff );
   hipStream_t st = as_stream( stream );
+  if ( ff > 0 && dt == GH_BF16 && activation == GH_ACT_SILU ) {
+    bool done = false;
+    if ( int rc = gemm_gate_one_launch( hidden, hidden_stride, x, static_cast<const __bf16*>( w ) + cols.ff * width, width, ff, rows, dt, st, &done ) ) {
+      return rc;
+    }
+    if ( done ) {
+      ff = 0;
+      cols.r = cols.ff;
+    }
+  }
   Product y;
   if ( int rc = make_product( x, w, width, cols.r, rows, dt, false, st, &y ) ) {
     return rc;

@@ -10,6 +10,8 @@
 namespace gh {
 namespace {
 
+bool aligned16( const void* p ) { return ( reinterpret_cast<uintptr_t>( p ) & 15u ) == 0; }
+
 // ---- embedding ---------------------------------------------------------------------------------
 template<typename E>
 __global__ __launch_bounds__( 256 ) void embed_positions_kernel( float* __restrict__ x,
@@ -33,6 +35,29 @@ __global__ __launch_bounds__( 256 ) void embed_positions_kernel( float* __restri
     x[(uint64_t)row * width + c] = v;
     if ( copy != nullptr ) {
       copy[(uint64_t)row * copy_stride + c] = from_f32<E>( v );
+    }
+  }
+}
+
+// four columns a thread: width, strides and tables in groups of four
+template<typename E>
+__global__ __launch_bounds__( 256 ) void embed_positions4_kernel( float* __restrict__ x, const uint32_t* __restrict__ tokens, const uint32_t* __restrict__ start_pos,
+                                                                  uint32_t n_tokens, const E* __restrict__ embed, const E* __restrict__ pos_table, uint32_t width,
+                                                                  uint32_t vocab, uint32_t max_pos, E* __restrict__ copy, uint64_t copy_stride )
+{
+  const uint32_t row = blockIdx.x;
+  const uint64_t token = min( tokens[row], vocab - 1 );
+  const E* p = pos_table != nullptr ? pos_table + (uint64_t)min( start_pos[row / n_tokens] + row % n_tokens, max_pos - 1 ) * width : nullptr;
+  for ( uint32_t c = 4 * threadIdx.x; c < width; c += 4 * blockDim.x ) {
+    float4 v = ProductView<E>::load4( embed + token * width + c );
+    if ( p != nullptr ) {
+      const float4 a = ProductView<E>::load4( p + c );
+      v = make_float4( v.x + a.x, v.y + a.y, v.z + a.z, v.w + a.w );
+    }
+    *reinterpret_cast<float4*>( x + (uint64_t)row * width + c ) = v;
+    if ( copy != nullptr ) {
+      E* to = copy + (uint64_t)row * copy_stride + c;
+      to[0] = from_f32<E>( v.x ), to[1] = from_f32<E>( v.y ), to[2] = from_f32<E>( v.z ), to[3] = from_f32<E>( v.w );
     }
   }
 }
@@ -218,8 +243,6 @@ __global__ __launch_bounds__( 256 ) void stream_step_any_kernel( float* __restri
   }
 }
 
-bool aligned16( const void* p ) { return ( reinterpret_cast<uintptr_t>( p ) & 15u ) == 0; }
-
 template<typename E, bool PRODUCT, typename View>
 int launch_step( float* x, const View& y, uint64_t width, uint64_t rows, const StepPtrs& p, hipStream_t st )
 {
@@ -350,14 +373,18 @@ int gh_embed_positions( float* x, const uint32_t* tokens_dev, const uint32_t* st
   GH_REQUIRE( x && tokens_dev && start_pos_dev && embed && width > 0 && vocab > 0 && max_pos > 0, "gh_embed_positions: bad argument" );
   GH_REQUIRE( dt == GH_BF16 || dt == GH_F32, "gh_embed_positions: unsupported dtype %d", (int)dt );
   GH_REQUIRE( rows < ( 1ull << 31 ) && width < ( 1ull << 31 ), "gh_embed_positions: too large" );
+  auto launch = [&]( auto tag ) {
+    using E = decltype( tag );
+    const E *e = static_cast<const E*>( embed ), *p = static_cast<const E*>( pos_table );
+    const bool vec = width % 4 == 0 && aligned16( x ) && aligned16( embed ) && aligned16( pos_table );
+    const uint32_t threads = vec ? (uint32_t)std::min<uint64_t>( 256, ( width / 4 + 63 ) / 64 * 64 ) : 256;
+    ( vec ? embed_positions4_kernel<E> : embed_positions_kernel<E> )<<<(unsigned)rows, threads, 0, as_stream( stream )>>>(
+      x, tokens_dev, start_pos_dev, n_tokens, e, p, (uint32_t)width, (uint32_t)vocab, (uint32_t)max_pos, static_cast<E*>( copy ), copy_stride );
+  };
   if ( dt == GH_F32 ) {
-    embed_positions_kernel<float><<<(unsigned)rows, 256, 0, as_stream( stream )>>>( x, tokens_dev, start_pos_dev, n_tokens, static_cast<const float*>( embed ),
-                                                                                   static_cast<const float*>( pos_table ), (uint32_t)width, (uint32_t)vocab,
-                                                                                   (uint32_t)max_pos, static_cast<float*>( copy ), copy_stride );
+    launch( float {} );
   } else {
-    embed_positions_kernel<__bf16><<<(unsigned)rows, 256, 0, as_stream( stream )>>>( x, tokens_dev, start_pos_dev, n_tokens, static_cast<const __bf16*>( embed ),
-                                                                                    static_cast<const __bf16*>( pos_table ), (uint32_t)width, (uint32_t)vocab,
-                                                                                    (uint32_t)max_pos, static_cast<__bf16*>( copy ), copy_stride );
+    launch( __bf16 {} );
   }
   GH_LAUNCH_CHECK();
   return GH_OK;

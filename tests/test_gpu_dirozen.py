@@ -75,6 +75,33 @@ def test_norms_around_zero(dtype, rows, s, width):
     assert_rows(back(out), P.rms_norm_around_zero(x0.astype(np.float64), nxt.astype(np.float64), eps), tol, "norm alone")
 
 
+@pytest.mark.parametrize("n_tokens", [1, 20, 70])
+def test_projections_with_a_large_feed_forward(n_tokens):
+    """Sizes at which few rows take the feed-forward's gate in the launch of its own product, into rows that lie apart."""
+    import torch
+    from glinthawk_amd import ops
+    heads, kv, d, ff, width = 4, 2, 64, 28672, 256
+    a = ops.window_attn(heads, kv, d, d, 1.0, values_are_keys=True)
+    rows, ff_row = ops.parallel_weight_rows(a, True, ff)
+    g = torch.Generator().manual_seed(n_tokens)
+    w = (torch.randn((rows, width), generator=g) / 16).cuda().bfloat16()
+    x = torch.randn((n_tokens, width), generator=g).cuda().bfloat16()
+    keys = torch.zeros((-(-(n_tokens + 4) // 32) * 32, kv * d), dtype=torch.bfloat16, device="cuda")
+    at = keys.numel() * 2
+    region = torch.cat([keys.reshape(-1).view(torch.uint8), torch.zeros(keys.shape[0] * kv * 4, dtype=torch.uint8, device="cuda")])
+    wide = torch.full((n_tokens, ff + 48), 5.0, dtype=torch.bfloat16, device="cuda")
+    q, gates = ops.matmul_parallel(x, w, a, ops.row_table([region.data_ptr()]), positions([4]), n_tokens, 1e-3, 0.5, 8, True, wide[:, 40:40 + ff], factor_offset=at)
+    y = x.float() @ w.float().T
+    h = torch.nn.functional.silu(y[:, ff_row:ff_row + ff]) * y[:, ff_row + ff:ff_row + 2 * ff]
+    assert_rows(back(wide[:, 40:40 + ff]), back(h), 1e-2, "hidden")
+    assert bool((wide[:, :40] == 5).all()) and bool((wide[:, 40 + ff:] == 5).all())
+    y = back(y)
+    temp = np.array([P.query_temperature(p, 0.5, 8) for p in range(4, 4 + n_tokens)])[:, None, None]
+    assert_rows(back(q), (P.unit_rms(y[:, :256].reshape(-1, heads, d), 1e-3) * temp).reshape(n_tokens, -1), 1e-2, "q")
+    assert_rows(back(gates), P.sigmoid(y[:, 384:388]), 1e-2, "head gates")
+    assert_rows(back(region[:at].view(torch.bfloat16)).reshape(-1, kv * d)[4:4 + n_tokens], y[:, 256:384], 1e-2, "keys")
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("n_tokens", [1, 4, 250, 600])
 @pytest.mark.parametrize("heads,kv,d,ff,gated,every", [(6, 3, 20, 44, True, 7), (4, 1, 64, 0, True, 1), (5, 5, 96, 72, False, 33), (3, 1, 136, 21, True, 64), (2, 2, 300, 40, True, 0),
@@ -230,14 +257,14 @@ def test_one_key_stands_out(name, dtype):
     """Every key in turn made the one its queries' scores pick, among hundreds: read from its own position on by every later query, near or
     far, and by none before it.  One head long and one short, which their norms make alike."""
     heads, kv, d = shape = ATTENTIONS[name]
-    T, scale, eps = 420, 14.0 / d, 1e-4
+    T, scale, eps = 700, 14.0 / d, 1e-4
     rng = np.random.default_rng(4)
     q0 = rng.standard_normal((kv, d))
     q0 /= np.sqrt((q0 ** 2).mean(-1, keepdims=True))
     q = M.to_bf16(np.broadcast_to(np.repeat(q0, heads // kv, axis=0), (T, heads, d)))
     tol = 2e-5 if dtype == "f32" else 1e-2
     base = M.to_bf16(rng.standard_normal((T, kv, d)))
-    for j in (0, 1, 30, 31, 32, 63, 64, 127, 128, 255, 256, 300, T - 2):
+    for j in (0, 1, 31, 32, 63, 64, 127, 128, 255, 256, 300, 511, 513, T - 2):
         k = base.copy()
         k[j] = M.to_bf16(q0 * (0.2 if j % 2 else 3.0))
         want = np.stack([[P.read_keys(q[t, h].astype(np.float64), k[: t + 1, h // (heads // kv)].astype(np.float64), eps, scale) for h in range(0, heads, heads // kv)] for t in range(T)])
@@ -245,7 +272,7 @@ def test_one_key_stands_out(name, dtype):
         assert_rows(got.reshape(T, -1), want.reshape(T, -1), tol, f"key {j} in a prompt")
         seen = np.array([np.corrcoef(got[t, 0], q0[0])[0, 1] > 0.95 for t in range(T)])
         assert seen[j:].all() and not seen[:j].any(), f"key {j}"
-        for p in sorted({j, j + 1, 64, 300, T - 1}):
+        for p in sorted({j, j + 1, 64, 300, 511, 512, 640, T - 1}):
             if p < T:
                 one = attend(shape, [q], [k], [p], 1, dtype, eps, scale)[0][:, ::heads // kv]
                 assert_rows(one.reshape(1, -1), want[p].reshape(1, -1), tol, f"key {j} decoded at {p}")

@@ -62,15 +62,18 @@ def test_profile_stage_log(tmp_path, ctx, stage, text):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("ctx", ["static", "paged"])
-def test_profile_of_a_design(tmp_path, ctx):
-    import famidra_models as M
+@pytest.mark.parametrize("design,positions", [("Famidra", 300), ("Dirozen", 4096)])      # what config.json names, and the host layer's default
+def test_profile_of_a_design(tmp_path, design, positions, ctx):
+    import dirozen_models
+    import famidra_models
+    M = {"Famidra": famidra_models, "Dirozen": dirozen_models}[design]
     M.write_model(tmp_path, M.CONFIGS["odd"], {})            # sizes only: the weights are drawn
-    log = tmp_path / f"famidra_all_{ctx}_297_0_3.csv"
-    r = run([STAGE, str(tmp_path), "Famidra", ctx, "all", "3", "297", "0", str(log)])
+    log = tmp_path / f"{design.lower()}_all_{ctx}_297_0_3.csv"
+    r = run([STAGE, str(tmp_path), design, ctx, "all", "3", "297", "0", str(log)])
     assert r.returncode == 0, r.stderr
-    assert open(log).readline().strip() == "# model='Famidra', stage=Pre+Att+Post+Cls, batch_size=3, token_pos=297, duration_s=0"
+    assert open(log).readline().strip() == f"# model='{design}', stage=Pre+Att+Post+Cls, batch_size=3, token_pos=297, duration_s=0"
     assert (pd.read_csv(log, skiprows=1)["duration_us"] > 0).all()
-    r = run([STAGE, str(tmp_path), "Famidra", ctx, "all", "3", "300", "0", str(log)])
+    r = run([STAGE, str(tmp_path), design, ctx, "all", "3", str(positions), "0", str(log)])
     assert r.returncode != 0 and "out of range" in r.stderr
 
 

@@ -46,6 +46,7 @@ def test_host_layer_under_asan_and_ubsan():
     if not os.path.exists(build.LIB):
         pytest.skip("libglint_hip.so is not built")
     lib = build.build_host_sanitized()
-    files = ["tests/test_host_book.py", "tests/test_host_state.py", "tests/test_host_loader.py", "tests/test_host_kernel.py", "tests/test_famidra_host.py"]
+    files = ["tests/test_host_book.py", "tests/test_host_state.py", "tests/test_host_loader.py", "tests/test_host_kernel.py", "tests/test_famidra_host.py",
+             "tests/test_dirozen_host.py"]
     tail = run_suite(files, {"GLINT_HOST_LIB": lib}, runtime)
     assert "failed" not in tail
