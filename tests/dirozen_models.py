@@ -6,7 +6,7 @@ import numpy as np
 from famidra_models import to_bf16, write_model  # noqa: F401  (the model directory's format is the designs' common one)
 
 
-def layer(heads, kv_heads, dim, every, coef=0.3, ff=None, scale=None):
+def layer(heads, kv_heads, dim, every, coef=0.35, ff=None, scale=None):
     return {"type": "attention", "mlp": None if ff is None else {"kind": "dense", "ff": ff},
             "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": 1.1 * dim ** -0.5 if scale is None else scale,
                       "q_temp": {"coef": coef, "every": every}}}
@@ -25,7 +25,7 @@ CONFIGS = {
     # one head, one layer with and one without a feed-forward of its width
     "plain": config(64, 200, [layer(1, 1, 128, 24, 0.0, ff=64), layer(1, 1, 64, 100, 1.2)], eps=1e-6),
     # head sizes between the kernels' steps
-    "between": config(80, 150, [layer(12, 3, 88, 20, 0.4, ff=72), layer(6, 6, 72, 9, 0.2, ff=40), layer(32, 1, 104, 64, 0.3, ff=88)]),
+    "between": config(80, 150, [layer(12, 3, 88, 20, 0.4, ff=72), layer(6, 6, 72, 9, 0.2, ff=40), layer(32, 1, 104, 64, 0.8, ff=88)]),
     # heads wider than the common kernels, a group of ten
     "wide": config(96, 150, [layer(10, 1, 136, 12, ff=52), layer(2, 2, 300, 33, 0.7, ff=48), layer(4, 2, 260, 5)], eps=1e-3),
 }
